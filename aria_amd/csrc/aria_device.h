@@ -437,12 +437,10 @@ __device__ __forceinline__ float rcp_fast(float x) {
 // x * sigmoid(x) (SiLU): x / (1 + e^-x) on v_exp_f32 + v_rcp_f32.  ONE definition for the fused GEMM epilogue, the stand-alone SwiGLU
 // kernels and the decode path, so that all of them round identically.
 __device__ __forceinline__ float silu_fast(float a) { return a * rcp_fast(1.f + exp2_fast(-1.4426950408889634f * a)); }
-// ---- r06: the two activation formulas whose evaluation sits in GEMM epilogues are written ON PAIRS of values, as explicit operation sequences
-// (every fused multiply-add spelled out, no sum of products left to the compiler's contraction): the compiler then emits v_pk_mul / v_pk_fma /
-// v_pk_add for everything but the two quarter-rate transcendentals, and every caller -- fused epilogue, stand-alone kernel, the scalar wrappers
-// below -- executes the same IEEE operations in the same order, i.e. rounds identically.  (The scalar forms left to the auto-vectorizer packed
-// only part of the work: 36 full-rate instructions per four GELU values against 22 now; the ViT fc1 launch spends ~10 us of a ~42 us tile in
-// this epilogue, the SwiGLU backward ~15 of ~83.)
+// The two activation formulas whose evaluation sits in GEMM epilogues are written ON PAIRS of values, as explicit operation sequences (every
+// fused multiply-add spelled out, no sum of products left to the compiler's contraction), so that every caller -- fused epilogue, stand-alone
+// kernel, the scalar wrappers below -- executes the same IEEE operations in the same order, i.e. rounds identically.  The build compiles them to
+// scalar fp32 instructions (packed fp32 is switched off in the Makefile).
 typedef float f32x2 __attribute__((ext_vector_type(2)));
 __device__ __forceinline__ f32x2 fma2(f32x2 a, f32x2 b, f32x2 c) {
 #ifdef ARIA_EMU

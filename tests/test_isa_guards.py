@@ -23,7 +23,7 @@ _ISA = {}
 
 def isa(src):
     if src not in _ISA:
-        r = subprocess.run([HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", "-Iinclude", "-Iaria_amd/csrc", "-S", "--cuda-device-only",
+        r = subprocess.run([HIPCC, "--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-O3", "-std=c++17", "-Iinclude", "-Iaria_amd/csrc", "-S", "--cuda-device-only",
                             os.path.join("aria_amd", "csrc", src), "-o", "-"], cwd=ROOT, capture_output=True, text=True)
         assert r.returncode == 0, r.stderr[-2000:]
         _ISA[src] = r.stdout.split("\n")

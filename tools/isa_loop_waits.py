@@ -3,7 +3,7 @@ path).  A full drain (vmcnt(0)) inside a loop whose next consumer is not the sta
 belongs to a value loaded in front of the loop lands at its first use inside it and then drains the loop's own prefetch every iteration."""
 import re, subprocess, sys
 src = sys.argv[1]
-asm = subprocess.run(["hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-Iinclude", "-Iaria_amd/csrc", "-S", "--cuda-device-only", src, "-o", "-"],
+asm = subprocess.run(["hipcc", "--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-O3", "-std=c++17", "-Iinclude", "-Iaria_amd/csrc", "-S", "--cuda-device-only", src, "-o", "-"],
                      capture_output=True, text=True).stdout.split("\n")
 kernel, in_loop_labels, loop_depth = None, set(), {}
 out = {}

@@ -12,7 +12,7 @@ print("# per-kernel resource usage of libaria_hip.so (hipcc -Rpass-analysis=kern
 print("# occ = waves/SIMD the register budget allows; LDS = STATIC bytes/block (the tiled GEMM / attention kernels take theirs dynamically)")
 print(f"{'file':10s} {'VGPR':>5s} {'AGPR':>5s} {'SGPR':>5s} {'vspill':>6s} {'scratch':>7s} {'LDS':>6s} {'occ':>3s}  kernel")
 for src in sorted(glob.glob("aria_amd/csrc/*.hip")):
-    out = subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Iinclude", "-Iaria_amd/csrc", "-c", src, "-o",
+    out = subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-O3", "-std=c++17", "-fPIC", "-Iinclude", "-Iaria_amd/csrc", "-c", src, "-o",
                           "/dev/null", "-Rpass-analysis=kernel-resource-usage"], capture_output=True, text=True).stderr
     cur = {}
     for line in out.split("\n"):
@@ -32,7 +32,7 @@ for src in sorted(glob.glob("aria_amd/csrc/*.hip")):
             name = name.replace("(anonymous namespace)::", "").split("(")[0][:70]
             print(f"{os.path.basename(src):10s} {cur.get('VGPRs', '?'):>5s} {cur.get('AGPRs', '?'):>5s} {cur.get('TotalSGPRs', '?'):>5s} "
                   f"{cur.get('VGPRs Spill', '?'):>6s} {cur.get('ScratchSize [bytes/lane]', '?'):>7s} {val:>6s} {cur.get('Occupancy [waves/SIMD]', '?'):>3s}  {name}")
-asm = subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-Iinclude", "-Iaria_amd/csrc", "-S", "--cuda-device-only",
+asm = subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-O3", "-std=c++17", "-Iinclude", "-Iaria_amd/csrc", "-S", "--cuda-device-only",
                       "aria_amd/csrc/gemm3.hip", "-o", "-"], capture_output=True, text=True).stdout.split("\n")
 starts = [(i, re.match(r"^_ZN12_GLOBAL__N_112gemm3_kernelI(\w+?)EEv10GemmParams:", l).group(1)) for i, l in enumerate(asm)
           if re.match(r"^_ZN12_GLOBAL__N_112gemm3_kernelI\w+EEv10GemmParams:", l)]

@@ -6,7 +6,7 @@ cd "$(dirname "$0")/../.."; mkdir -p build/abl
 MACRO=$1; TAG=$2; shift 2
 OTHERS=$(ls build/*.o | grep -v attn.o)
 for v in "$@"; do
-  ( /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -Iinclude -Iaria_amd/csrc -D$MACRO=$v -c aria_amd/csrc/attn.hip -o build/abl/${TAG}_$v.o \
+  ( /opt/rocm/bin/hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -fPIC -Iinclude -Iaria_amd/csrc -D$MACRO=$v -c aria_amd/csrc/attn.hip -o build/abl/${TAG}_$v.o \
     && /opt/rocm/bin/hipcc --offload-arch=gfx950 -shared -fPIC build/abl/${TAG}_$v.o $OTHERS -o build/abl/libaria_${TAG}_$v.so && rm build/abl/${TAG}_$v.o ) &
   while [ $(jobs -r | wc -l) -ge 4 ]; do sleep 1; done
 done

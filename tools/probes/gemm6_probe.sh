@@ -6,7 +6,7 @@
 cd "$GRAFT_REPO_ROOT"; export TMPDIR=/tmp; mkdir -p gpurun_out build/abl
 tag=${1:-r06}
 BIN=build/abl/gemm6_4wave
-[ -x $BIN ] || /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -Iaria_amd/csrc -Iinclude tools/probes/src/gemm6_4wave.hip -o $BIN -ldl
+[ -x $BIN ] || /opt/rocm/bin/hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -Iaria_amd/csrc -Iinclude tools/probes/src/gemm6_4wave.hip -o $BIN -ldl
 for shape in "16384 3328 2560 0" "16384 3328 2560 1" "8192 8192 8192 0" "16384 2560 3328 0" "78336 4352 1152 0" "78336 1280 4352 0" "16384 7680 2560 0"; do
   name=$(echo $shape | tr ' ' 'x')
   timeout 300 $BIN $shape ${ITERS:-100} 3 > gpurun_out/${tag}_gemm6_$name.json 2> gpurun_out/${tag}_gemm6_$name.err
