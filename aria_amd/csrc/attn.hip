@@ -81,9 +81,7 @@ __device__ __forceinline__ s16x8 pack_frag(const f32x16& p, int u) {
 
 __device__ __forceinline__ int acc_row(int r, int l) { return (r & 3) + 8 * (r >> 2) + 4 * (l >> 5); }
 
-// (a0 * b + c, a1 * b + c) as ONE v_pk_fma_f32 (two fp32 lanes per instruction at the plain-VALU rate; each lane is a fused multiply-add,
-// the same rounding as two v_fma_f32): the softmax's score scaling is 32 of a key tile's ~100 vector instructions in the forward kernels,
-// which are vector-ALU-bound as much as matrix-bound (profiles/r04_attn_fwd_ablate.json)
+// (a0 * b + c, a1 * b + c), each a fused multiply-add: the softmax's score scaling
 typedef float f32x2 __attribute__((ext_vector_type(2)));
 __device__ __forceinline__ f32x2 fma2(float a0, float a1, float b, float c) {
     const f32x2 a = {a0, a1}, bb = {b, b}, cc = {c, c};
@@ -1282,14 +1280,12 @@ __global__ __launch_bounds__(512) void attn_bwd5_dq_kernel(const bf16_t* Q, cons
 //     16 banks apart.
 // Same arithmetic in the same order as v2: results are bit-identical (tests compare the two).
 
-template <int HD>
-struct FwdFmt;
-template <>
-struct FwdFmt<128> {
-    static constexpr int KS = 8, DT = 4, KTILE = 16384, VTILE = 16384;
+// A tile format F: QD / VD = columns of a query (key) head and of a value head in memory, the images of the two 64-row tiles and how 8 waves
+// fill them by LDS-DMA.  PAD: the head holds fewer columns than KS * 16 (Q's missing chunks read as zeros).
+struct Fmt128 {
+    static constexpr int QD = 128, VD = 128, KS = 8, DT = 4, KTILE = 16384, VTILE = 16384;
     static constexpr bool ROWSUM_IN_MFMA = false;
-    int dummy;
-    __device__ __forceinline__ void init(int, int, int) {}  // (tile_dma3: 8 waves x 2 pieces)
+    __device__ __forceinline__ void init(int, int) {}  // (tile_dma3: 8 waves x 2 pieces)
     __device__ __forceinline__ void dma_k(const bf16_t* base, long long ld, int row0, int row_last, char* s, int w, int l) const {
         tile_dma3<128>(base, int(ld), row0, row_last, s, w, l);
     }
@@ -1299,21 +1295,79 @@ struct FwdFmt<128> {
     static __device__ __forceinline__ s16x8 kfrag(const char* s, int row, int kk, int l) { return frag_rc3<128>(s, row, kk, l); }
     static __device__ __forceinline__ s16x8 vfrag(const char* s, int rb, int d0, int l) { return frag_tr3<128>(s, rb, d0, l); }
 };
-template <int HD>
+// Query / key heads of QD columns beside value heads of VD columns (multiples of 64): latent attention expanded to per-head keys and values,
+// where a head's key is [unrotated | rotated | zero pad].  A row is CPR 16-byte chunks; image slot s of row r holds source chunk s ^ f(r).
+// f spreads the rows of a fragment read over the banks: 16-chunk multiples take the 4-bit swizzle of the 128-column image, the others 3 bits
+// (row >> 1 where consecutive rows already lie 32 banks apart).
+template <int COLS>
+struct TileImg {
+    static constexpr int CPR = COLS / 8, ROW = COLS * 2, BYTES = 64 * ROW, PIECES = CPR / 8;   // 1 KiB pieces per wave
+    static_assert(COLS % 64 == 0, "8 waves deal whole pieces");
+    static __device__ __forceinline__ int swz(int row) { return CPR % 16 == 0 ? swz3(row) : (CPR % 16 == 8 && CPR > 8) ? (row >> 1) & 7 : row & 7; }
+    int row[PIECES], col[PIECES];   // this lane's source row inside the tile and source column, per piece
+    __device__ __forceinline__ void init(int w, int l) {
+#pragma unroll
+        for (int i = 0; i < PIECES; ++i) {
+            const int c = (w + 8 * i) * 64 + l;
+            row[i] = c / CPR;
+            col[i] = ((c % CPR) ^ swz(row[i])) * 8;
+        }
+    }
+    __device__ __forceinline__ void dma(const bf16_t* base, long long ld, int row0, int row_last, char* s, int w) const {
+#pragma unroll
+        for (int i = 0; i < PIECES; ++i) glds16_raw(base + (long long)min(row0 + row[i], row_last) * ld + col[i], s + (w + 8 * i) * 1024);
+    }
+    static __device__ __forceinline__ s16x8 rows(const char* s, int r, int kk, int l) {
+        return *reinterpret_cast<const s16x8*>(s + r * ROW + (((2 * kk + (l >> 5)) ^ swz(r)) << 4));
+    }
+    static __device__ __forceinline__ s16x8 columns(const char* s, int rb, int d0, int l) {   // frag_tr3's contract
+        const int r = rb + 4 * (l >> 5) + ((l & 15) >> 2);
+        const int c = d0 + 16 * ((l >> 4) & 1) + 4 * (l & 3);
+        const int ch = c >> 3, within = (c & 7) * 2;
+        const s16x4 a0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(s + r * ROW + ((ch ^ swz(r)) << 4) + within));
+        const s16x4 a1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(s + (r + 8) * ROW + ((ch ^ swz(r + 8)) << 4) + within));
+        s16x8 f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            f[e] = a0[e];
+            f[4 + e] = a1[e];
+        }
+        return f;
+    }
+};
+template <int QD_, int VD_>
+struct FmtQV {
+    static constexpr int QD = QD_, VD = VD_, KS = QD / 16, DT = VD / 32, KTILE = TileImg<QD>::BYTES, VTILE = TileImg<VD>::BYTES;
+    static constexpr bool ROWSUM_IN_MFMA = false;
+    TileImg<QD> ki;
+    TileImg<VD> vi;
+    __device__ __forceinline__ void init(int w, int l) {
+        ki.init(w, l);
+        vi.init(w, l);
+    }
+    __device__ __forceinline__ void dma_k(const bf16_t* base, long long ld, int row0, int row_last, char* s, int w, int) const {
+        ki.dma(base, ld, row0, row_last, s, w);
+    }
+    __device__ __forceinline__ void dma_v(const bf16_t* base, long long ld, int row0, int row_last, char* s, int w, int) const {
+        vi.dma(base, ld, row0, row_last, s, w);
+    }
+    static __device__ __forceinline__ s16x8 kfrag(const char* s, int row, int kk, int l) { return TileImg<QD>::rows(s, row, kk, l); }
+    static __device__ __forceinline__ s16x8 vfrag(const char* s, int rb, int d0, int l) { return TileImg<VD>::columns(s, rb, d0, l); }
+};
+template <class F>
 struct Fwd3Smem {
-    using F = FwdFmt<HD>;
     static constexpr int K0 = 0, V0 = 2 * F::KTILE, M0 = V0 + 2 * F::VTILE, FLAG0 = M0 + 3 * 64, BYTES = FLAG0 + 16;
 };
 
 // S^T tile of one key tile: rows = keys (two sub-tiles of 32), cols = this wave's 32 queries
-template <int HD>
-__device__ __forceinline__ void fwd3_qk(f32x16 (&st)[2], const char* cK, const s16x8 (&qf)[FwdFmt<HD>::KS], int l) {
+template <class F>
+__device__ __forceinline__ void fwd3_qk(f32x16 (&st)[2], const char* cK, const s16x8 (&qf)[F::KS], int l) {
     st[0] = zero_acc();
     st[1] = zero_acc();
 #pragma unroll
-    for (int kk = 0; kk < FwdFmt<HD>::KS; ++kk)
+    for (int kk = 0; kk < F::KS; ++kk)
 #pragma unroll
-        for (int i = 0; i < 2; ++i) st[i] = mfma32(FwdFmt<HD>::kfrag(cK, i * 32 + (l & 31), kk, l), qf[kk], st[i]);
+        for (int i = 0; i < 2; ++i) st[i] = mfma32(F::kfrag(cK, i * 32 + (l & 31), kk, l), qf[kk], st[i]);
 }
 
 // key-mask / length / causal mask of one score tile (edge, diagonal and padded tiles only)
@@ -1337,10 +1391,9 @@ __device__ __forceinline__ void fwd3_mask(f32x16 (&st)[2], const uint8_t* cM, bo
 //     a quarter of the next tile's score MFMAs | the group's 8 exponentials + packing | the group's P V MFMAs (one per 32 features)
 // -- independent matrix and vector work side by side in every sub-step; scheduling fences between the sub-steps keep the compiler from
 // hoisting all fragment reads of the tile to the top (256 VGPRs and spills without them).
-template <int HD, bool PIPE>
-__device__ __forceinline__ void fwd3_step(f32x16 (&st)[2], f32x16 (&sn)[2], f32x16 (&o)[FwdFmt<HD>::DT], float& m, float& lsum,
-                                          const s16x8 (&qf)[FwdFmt<HD>::KS], const char* cV, const char* nK, float scale2, int l) {
-    using F = FwdFmt<HD>;
+template <class F, bool PIPE>
+__device__ __forceinline__ void fwd3_step(f32x16 (&st)[2], f32x16 (&sn)[2], f32x16 (&o)[F::DT], float& m, float& lsum,
+                                          const s16x8 (&qf)[F::KS], const char* cV, const char* nK, float scale2, int l) {
     constexpr int KS = F::KS;
     float mx = st[0][0];
 #pragma unroll
@@ -1398,13 +1451,14 @@ __device__ __forceinline__ void fwd3_step(f32x16 (&st)[2], f32x16 (&sn)[2], f32x
 // 145 VGPRs, THREE waves per SIMD).  Measured for the ViT's shape (profiles/r04_attn_fwd3_ab.json): the third wave is worth more than the
 // in-wave overlap, and with it LDS-DMA staging into the conflict-free images (SQ_LDS_BANK_CONFLICT 0, was 8 % of the LDS cycles) is level
 // with v2's register staging -- so hd 72 stays on v2 by default and both v3 forms are kept selectable (ARIA_ATTN_FWD) as measurements.
-template <int HD, int NW, bool PIPE>
+// RAGGED: the sequences of the batch are rows cu[b] .. cu[b + 1] of the token axis (Sq = S = the longest), and every head's output is multiplied
+// by sigmoid(gate[token * ldg + head]) in the epilogue (gate may be NULL).
+template <class F, int NW, bool PIPE, bool RAGGED>
 __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, const bf16_t* K, const bf16_t* V, bf16_t* O, float* LSE,
                                                         const int32_t* kv_len, const uint8_t* key_mask, int Sq, int S, int H,
                                                         long long ldq, long long ldk, long long ldv, long long ldo, float scale,
-                                                        int causal, int nbatch) {
-    using F = FwdFmt<HD>;
-    using L = Fwd3Smem<HD>;
+                                                        int causal, int nbatch, const int32_t* cu, const bf16_t* gate, long long ldg) {
+    using L = Fwd3Smem<F>;
     constexpr int KS = F::KS, DT = F::DT;
     ARIA_DYN_SMEM(smem);
     char* sK = smem + L::K0;
@@ -1414,26 +1468,30 @@ __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, con
     const int t = threadIdx.x, l = t & 63, w = first_lane(t >> 6), h2 = l >> 5;
     int qblk, head, b;
     constexpr int QB = NW * 32, KA = PIPE ? 1 : 0;  // queries per workgroup; how many tiles K runs ahead of V in LDS
-    static_assert(HD != 128 || NW == 8, "tile_dma3 deals a tile's 16 pieces to 8 waves");
+    static_assert(NW == 8, "the tile images are dealt to 8 waves");
     if (!attn_block_coords((Sq + QB - 1) / QB, H, nbatch, causal, true, qblk, head, b)) return;
     const int q0 = qblk * QB;
-    const long long tok0 = (long long)b * S, tokq0 = (long long)b * Sq;
-    const bf16_t* Qb = Q + tokq0 * ldq + head * HD;
-    const bf16_t* Kb = K + tok0 * ldk + head * HD;
-    const bf16_t* Vb = V + tok0 * ldv + head * HD;
+    if (RAGGED) {
+        Sq = S = cu[b + 1] - cu[b];
+        if (q0 >= Sq) return;
+    }
+    const long long tok0 = RAGGED ? (long long)cu[b] : (long long)b * S, tokq0 = RAGGED ? tok0 : (long long)b * Sq;
+    const bf16_t* Qb = Q + tokq0 * ldq + head * F::QD;
+    const bf16_t* Kb = K + tok0 * ldk + head * F::QD;
+    const bf16_t* Vb = V + tok0 * ldv + head * F::VD;
     const uint8_t* kmb = key_mask ? key_mask + tok0 : nullptr;
     const int q_wmin = q0 + 32 * w, q_abs = q_wmin + (l & 31);
     const int klen = kv_len ? min(S, kv_len[b]) : S;
     const float scale2 = scale * 1.4426950408889634f;
     F fmt;
-    fmt.init(w, l, NW);
+    fmt.init(w, l);
 
     s16x8 qf[KS];
 #pragma unroll
     for (int kk = 0; kk < KS; ++kk) {
         u32x4 v = zero16();
         const int col = kk * 16 + h2 * 8;
-        if (q_abs < Sq && col < HD) v = ld16(Qb + (long long)q_abs * ldq + col);
+        if (q_abs < Sq) v = ld16(Qb + (long long)q_abs * ldq + col);
         qf[kk] = __builtin_bit_cast(s16x8, v);
     }
     f32x16 o[DT];
@@ -1452,10 +1510,6 @@ __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, con
         if (t == 0) sFlag[tile % 3] = int(all == ~0ull) | (int(all == 0ull) << 1);
     };
     if (ntiles > 0) {
-        if (HD == 72) {  // what the pad-column reads behind the last rows touch must hold finite values (0 x NaN = NaN)
-            if (t < 2) st16(sK + t * F::KTILE + F::KTILE - 16, zero16());
-            if (t >= 64 && t < 68) st16(sV + ((t - 64) >> 1) * F::VTILE + F::VTILE - 32 + 16 * (t & 1), zero16());
-        }
         fmt.dma_k(Kb, ldk, 0, S - 1, sK, w, l);
         fmt.dma_v(Vb, ldv, 0, S - 1, sV, w, l);
         if (PIPE && ntiles > 1) fmt.dma_k(Kb, ldk, 64, S - 1, sK + F::KTILE, w, l);
@@ -1489,14 +1543,14 @@ __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, con
     if (PIPE && ntiles > 0) {
         wait_vm<0>();
         sync();
-        if (nmine > 0) fwd3_qk<HD>(sa, sK, qf, l);
+        if (nmine > 0) fwd3_qk<F>(sa, sK, qf, l);
     }
     // one iteration: tile `it` (PIPE: its scores are in `cur`) -> softmax + P V; PIPE: tile it + 1 -> scores into `nxt`
     auto iterate = [&](int it, f32x16 (&cur)[2], f32x16 (&nxt)[2]) __attribute__((always_inline)) {
         duties(it);
-        if (!PIPE) fwd3_qk<HD>(cur, sK + (it & 1) * F::KTILE, qf, l);
+        if (!PIPE) fwd3_qk<F>(cur, sK + (it & 1) * F::KTILE, qf, l);
         if (tile_masked(it)) fwd3_mask(cur, sM + (it % 3) * 64, kmb != nullptr, it * 64, klen, causal, q_abs, l);
-        fwd3_step<HD, PIPE>(cur, nxt, o, m, lsum, qf, sV + (it & 1) * F::VTILE, sK + ((it + 1) & 1) * F::KTILE, scale2, l);
+        fwd3_step<F, PIPE>(cur, nxt, o, m, lsum, qf, sV + (it & 1) * F::VTILE, sK + ((it + 1) & 1) * F::KTILE, scale2, l);
         park(it);
     };
     int it = 0;
@@ -1518,17 +1572,18 @@ __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, con
     }
     // ROWSUM_IN_MFMA: feature row HD = 32 (DT-1) + 8 sits in accumulator register 4 of the lanes with h2 == 0
     const float ltot = F::ROWSUM_IN_MFMA ? shfl(o[DT - 1][4], l & 31) : lsum + shfl_xor(lsum, 32);
-    const float inv = ltot > 0.f ? 1.f / ltot : 0.f;
+    float inv = ltot > 0.f ? 1.f / ltot : 0.f;
+    if (RAGGED && gate && q_abs < Sq) inv *= 1.f / (1.f + expf(-bf2f(gate[(tokq0 + q_abs) * ldg + head])));
     if (q_abs < Sq) {
         if (h2 == 0 && LSE)
             LSE[((long long)b * H + head) * Sq + q_abs] = (ltot > 0.f) ? (m + log2f(ltot)) * 0.6931471805599453f : -INFINITY;
-        bf16_t* orow = O + (tokq0 + q_abs) * ldo + head * HD;
+        bf16_t* orow = O + (tokq0 + q_abs) * ldo + head * F::VD;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
             for (int rg = 0; rg < 4; ++rg) {
                 const int d0 = 32 * dt + 8 * rg + 4 * h2;
-                if (d0 < HD) {
+                if (d0 < F::VD) {
                     u32x2 v;
                     v[0] = pack2bf(o[dt][4 * rg] * inv, o[dt][4 * rg + 1] * inv);
                     v[1] = pack2bf(o[dt][4 * rg + 2] * inv, o[dt][4 * rg + 3] * inv);
@@ -1568,9 +1623,10 @@ int aria_attn_fwd(const void* q, const void* k, const void* v, void* o, float* l
     const bool v3 = !(fwdv && fwdv[0] == '2') && hd == 128 && Skv > 0;
     g_last_fwd_variant = v3 ? 3 : 2;
     if (v3)
-        ARIA_LAUNCH((attn_fwd3_kernel<128, 8, true>), dim3(attn_grid((Sq + 255) / 256, H, B)), dim3(512), size_t(Fwd3Smem<128>::BYTES), stream, Q, K, V,
+        ARIA_LAUNCH((attn_fwd3_kernel<Fmt128, 8, true, false>), dim3(attn_grid((Sq + 255) / 256, H, B)), dim3(512), size_t(Fwd3Smem<Fmt128>::BYTES), stream, Q, K, V,
                     static_cast<bf16_t*>(o), lse, kv_len, key_mask, int(Sq), int(Skv), int(H), (long long)ldq, (long long)ldk,
-                    (long long)ldv, (long long)ldo, scale, causal_arg, int(B));
+                    (long long)ldv, (long long)ldo, scale, causal_arg, int(B), static_cast<const int32_t*>(nullptr),
+                    static_cast<const bf16_t*>(nullptr), 0ll);
     else if (hd == 128)
         ARIA_LAUNCH((attn_fwd2_kernel<128, 8>), dim3(attn_grid((Sq + 255) / 256, H, B)), dim3(512), size_t(Cfg2<128>::SMEM), stream, Q, K, V,
                     static_cast<bf16_t*>(o), lse, kv_len, key_mask, int(Sq), int(Skv), int(H), (long long)ldq, (long long)ldk,
@@ -1587,6 +1643,37 @@ int aria_attn_fwd(const void* q, const void* k, const void* v, void* o, float* l
         ARIA_LAUNCH((attn_fwd2_kernel<64, 8>), dim3(attn_grid((Sq + 255) / 256, H, B)), dim3(512), size_t(Cfg2<64>::SMEM), stream, Q, K, V,
                     static_cast<bf16_t*>(o), lse, kv_len, key_mask, int(Sq), int(Skv), int(H), (long long)ldq, (long long)ldk,
                     (long long)ldv, (long long)ldo, scale, causal, int(B));
+    return aria_check_launch();
+}
+
+int aria_attn_varlen_fwd(const void* q, const void* k, const void* v, void* o, const int32_t* cu, const void* gate, int64_t B, int64_t S_max,
+                         int64_t H, int64_t qd, int64_t vd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t ldg, float scale,
+                         void* stream) {
+    if (!q || !k || !v || !o || !cu || B < 0 || S_max < 0 || H <= 0) return ARIA_ERR_INVALID;
+    if (!al16(q) || !al16(k) || !al16(v) || (ldq & 7) || (ldk & 7) || (ldv & 7) || (ldo & 3) || (reinterpret_cast<uintptr_t>(o) & 7))
+        return ARIA_ERR_ALIGN;
+    const bool known = (qd == 64 && vd == 64) || (qd == 128 && vd == 128) || (qd == 192 && vd == 128) || (qd == 256 && vd == 256);
+    if (!known) return ARIA_ERR_UNSUPPORTED;
+    if (B == 0 || S_max == 0) return ARIA_OK;
+    const int causal = S_max >= 32768 ? 2 : 1;   // (2: attn_block_coords' grouped order)
+#define ARIA_VARLEN(F, PIPE)                                                                                                                  \
+    ARIA_LAUNCH((attn_fwd3_kernel<F, 8, PIPE, true>), dim3(attn_grid((S_max + 255) / 256, H, B)), dim3(512), size_t(Fwd3Smem<F>::BYTES), stream, \
+                static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k), static_cast<const bf16_t*>(v), static_cast<bf16_t*>(o),           \
+                static_cast<float*>(nullptr), static_cast<const int32_t*>(nullptr), static_cast<const uint8_t*>(nullptr), int(S_max),           \
+                int(S_max), int(H), (long long)ldq, (long long)ldk, (long long)ldv, (long long)ldo, scale, causal, int(B), cu,                  \
+                static_cast<const bf16_t*>(gate), (long long)ldg)
+    using F64 = FmtQV<64, 64>;
+    using F192 = FmtQV<192, 128>;
+    using F256 = FmtQV<256, 256>;
+    if (qd == 64)
+        ARIA_VARLEN(F64, true);
+    else if (qd == 128)
+        ARIA_VARLEN(Fmt128, true);
+    else if (qd == 192)
+        ARIA_VARLEN(F192, true);
+    else
+        ARIA_VARLEN(F256, false);
+#undef ARIA_VARLEN
     return aria_check_launch();
 }
 

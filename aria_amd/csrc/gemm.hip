@@ -262,6 +262,54 @@ int launch_gemm(const GemmParams& p, int a_oc, int b_oc, int grid_x, int grid_y,
     return aria_check_launch();
 }
 
+// C = A W^T in true 32-bit: 64 x 64 tile, 4 x 4 outputs per thread, 16 reduction indices per stage, one rounding per multiply-add (the matrix pipe
+// is left alone).  offsets: rows grouped by expert, blockIdx.z = expert.
+__global__ __launch_bounds__(256) void gemm_f32_kernel(const float* A, const float* W, float* C, int M, int N, int K, long long lda, long long ldw,
+                                                       long long ldc, const int* offsets, long long strideW) {
+    ARIA_SMEM_STATIC float sA[16][68], sB[16][68];
+    int m0 = blockIdx.y * 64, m_end = M;
+    const int n0 = blockIdx.x * 64, t = threadIdx.x;
+    if (offsets) {
+        m_end = offsets[blockIdx.z + 1];
+        m0 += offsets[blockIdx.z];
+        W += (long long)blockIdx.z * strideW;
+    }
+    if (m0 >= m_end) return;
+    const int tx = t & 15, ty = t >> 4, lr = t >> 2, lk = (t & 3) * 4;
+    float acc[4][4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = 0.f;
+    for (int k0 = 0; k0 < K; k0 += 16) {
+        f32x4 a = {0.f, 0.f, 0.f, 0.f}, b = a;
+        if (k0 + lk < K) {   // (K % 4 == 0)
+            if (m0 + lr < m_end) a = *reinterpret_cast<const f32x4*>(A + (long long)(m0 + lr) * lda + k0 + lk);
+            if (n0 + lr < N) b = *reinterpret_cast<const f32x4*>(W + (long long)(n0 + lr) * ldw + k0 + lk);
+        }
+        sync();
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            sA[lk + e][lr] = a[e];
+            sB[lk + e][lr] = b[e];
+        }
+        sync();
+#pragma unroll
+        for (int kk = 0; kk < 16; ++kk)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(sA[kk][ty * 4 + i], sB[kk][tx * 4 + j], acc[i][j]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int m = m0 + ty * 4 + i, n = n0 + tx * 4 + j;
+            if (m < m_end && n < N) C[(long long)m * ldc + n] = acc[i][j];
+        }
+}
+
 thread_local int g_last_variant = 0;
 constexpr int GROUPED_V3_DEFAULT = 3;  // r02 in-bench A/B with the wide epilogue: v3 for both weight forms 702 ms/step, v2 for the [K,N] form 710
 bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
@@ -876,6 +924,17 @@ int aria_grouped_gemm_wgrad_bf16(const void* A, const void* dY, void* dW, const 
         return g_last_variant = 3, aria_launch_gemm3(p, 1, 1, int((K + 255) / 256), stream);
     if (use_v2(((K + 255) / 256) * ((N + 255) / 256) * E)) return g_last_variant = 2, aria_launch_gemm2(p, 1, 1, int((K + 255) / 256), int(E), stream);
     return g_last_variant = 1, launch_gemm(p, 1, 1, p.ntn * ntm, int(E), stream);
+}
+
+int aria_gemm_f32(const float* A, const float* W, float* C, int64_t M, int64_t N, int64_t K, int64_t lda, int64_t ldw, int64_t ldc,
+                  const int32_t* offsets, int64_t E, int64_t strideW, void* stream) {
+    if (!A || !W || !C || M < 0 || N < 0 || K <= 0 || (offsets && E <= 0)) return ARIA_ERR_INVALID;
+    if (!aligned16(A) || !aligned16(W) || (lda & 3) || (ldw & 3) || (K & 3) || (strideW & 3)) return ARIA_ERR_ALIGN;
+    if (M == 0 || N == 0) return ARIA_OK;
+    if ((M + 63) / 64 > 65535 || E > 65535) return ARIA_ERR_UNSUPPORTED;
+    ARIA_LAUNCH(gemm_f32_kernel, dim3(unsigned((N + 63) / 64), unsigned((M + 63) / 64), offsets ? unsigned(E) : 1u), dim3(256), 0, stream, A, W, C, int(M),
+                int(N), int(K), (long long)lda, (long long)ldw, (long long)ldc, (const int*)offsets, (long long)strideW);
+    return aria_check_launch();
 }
 
 }  // extern "C"

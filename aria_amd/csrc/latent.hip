@@ -1,0 +1,808 @@
+// Latent attention: every head's keys and values are linear images of one low-rank latent per token, so the cache holds the latent and one
+// rotated key part shared by the heads (R + dr numbers a token instead of 2 H hd).
+//
+// Prefill expands the latents of the new tokens to per-head keys and values (a GEMM on the packed cache rows whose weight carries identity rows for
+// the rotated part) and runs the flash kernel of attn.hip on unequal query / value head widths.  Decode -- and a prompt that continues on a cache --
+// never expands: the query moves into latent space once (q W_uk, per head), scores are dot products with the cache rows as they lie in memory, and
+// the weighted sum of latents is expanded through W_uv at the end.  A cache row is then read ONCE for 16 or 32 heads, which makes decode
+// attention a matrix product with the heads as rows (v_mfma_f32_16x16x32_bf16) whose operand streams from HBM.
+#include "elem.h"
+#include <cstdlib>
+
+namespace {
+using namespace ad;
+typedef AriaLatentShape Shape;
+
+// one cache row: RMS-normed latent | rotated key part | zeros.  One wave; src = the token's down-projection (R + dr columns).
+template <class T>
+__device__ __forceinline__ void latent_row(const T* src, const Shape& s, const float* cs, const float* wn, T* row, T* packed, int l) {
+    float ss = 0.f;
+    for (int i = l; i < s.R; i += 64) {
+        const float v = ldf(src + i);
+        ss += v * v;
+    }
+    ss = wave_sum_bcast(ss);
+    const float r = 1.f / sqrtf(ss / float(s.R) + s.eps);
+    const int half = int(s.rot) >> 1;
+    for (int i = l; i < s.cw; i += 64) {
+        float v = 0.f;
+        if (i < s.R) {
+            v = ldf(src + i) * r * wn[i];
+        } else if (i < s.R + s.dr) {
+            const int j = i - int(s.R);
+            v = ldf(src + i);
+            if (j < half)
+                v = v * cs[2 * j] - ldf(src + i + half) * cs[2 * j + 1];
+            else if (j < s.rot)
+                v = v * cs[2 * (j - half)] + ldf(src + i - half) * cs[2 * (j - half) + 1];
+        }
+        stf(row + i, v);
+        if (packed) stf(packed + i, v);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------- prefill: rotate q, write the cache
+template <class T>
+__global__ __launch_bounds__(256) void latent_rows_kernel(T* proj, Shape s, const int32_t* slot, const int32_t* pos, const float* rope,
+                                                          const float* wn, T* cache, T* packed, int n_tok) {
+    const int l = threadIdx.x & 63;
+    const int t = (blockIdx.x * blockDim.x + threadIdx.x) >> 6;
+    if (t >= n_tok) return;
+    T* p = proj + (long long)t * s.ldp;
+    const int ps = pos[t];
+    const float* cs = rope + (long long)ps * s.rot;
+    latent_row<T>(p + s.kv_off, s, cs, wn, cache + ((long long)slot[t] * s.S_cap + ps) * s.cw, packed + (long long)t * s.cw, l);
+    const int half = int(s.rot) >> 1;
+    for (int i = l; i < s.H * half; i += 64) {
+        const int h = i / half, j = i % half;
+        T* a = p + (long long)h * s.dq + s.dn + j;
+        const float u = ldf(a), v = ldf(a + half), c = cs[2 * j], sn = cs[2 * j + 1];
+        stf(a, u * c - v * sn);
+        stf(a + half, v * c + u * sn);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------- decode: queries into latent space
+// grid (H * RB + 1, token groups): workgroup (h, rb) computes 128 latent columns of head h for NB tokens (16 column groups of 8 x 16 slices of
+// the reduction over dn: every thread has its weights in flight at once); the last workgroup of a token group writes the cache rows and the
+// rotated query parts.
+constexpr int ABS_NB = 4;
+template <class T>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(const T* proj, Shape s, const int32_t* slot, const int32_t* pos, const float* rope,
+                                                            const float* wn, const T* uk, T* cache, T* qa, int n_tok) {
+    ARIA_SMEM_STATIC float red[16][ABS_NB][128];
+    const int t = threadIdx.x, l = t & 63, w = t >> 6;
+    const int RB = int(s.R + 127) / 128, unit = blockIdx.x, t0 = blockIdx.y * ABS_NB;
+    const int nb = min(ABS_NB, n_tok - t0);
+    if (unit == s.H * RB) {
+        const int half = int(s.rot) >> 1, extra = int(s.cw - s.R);
+        for (int b = w; b < nb; b += 4) {
+            const int tok = t0 + b, ps = pos[tok];
+            const T* p = proj + (long long)tok * s.ldp;
+            const float* cs = rope + (long long)ps * s.rot;
+            latent_row<T>(p + s.kv_off, s, cs, wn, cache + ((long long)slot[tok] * s.S_cap + ps) * s.cw, static_cast<T*>(nullptr), l);
+            for (int i = l; i < s.H * extra; i += 64) {
+                const int h = i / extra, j = i % extra;
+                const T* a = p + (long long)h * s.dq + s.dn + j;
+                float v = 0.f;
+                if (j < s.dr) {
+                    v = ldf(a);
+                    if (j < half)
+                        v = v * cs[2 * j] - ldf(a + half) * cs[2 * j + 1];
+                    else if (j < s.rot)
+                        v = v * cs[2 * (j - half)] + ldf(a - half) * cs[2 * (j - half) + 1];
+                }
+                stf(qa + ((long long)tok * s.H + h) * s.cw + s.R + j, v);
+            }
+        }
+        return;
+    }
+    const int h = unit / RB, r0 = (unit % RB) * 128, cg = t & 15, g = t >> 4;
+    const int col = r0 + cg * 8;
+    float acc[ABS_NB][8];
+#pragma unroll
+    for (int b = 0; b < ABS_NB; ++b)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[b][e] = 0.f;
+    if (col < s.rp) {
+        const T* wp = uk + (long long)h * s.dn * s.rp + col;
+        const T* qp = proj + (long long)t0 * s.ldp + (long long)h * s.dq;
+#pragma unroll 8
+        for (int d = g; d < s.dn; d += 16) {
+            float wv[8];
+            ld8(wp + (long long)d * s.rp, wv);
+#pragma unroll
+            for (int b = 0; b < ABS_NB; ++b) {
+                const float q = ldf(qp + (long long)min(b, nb - 1) * s.ldp + d);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) acc[b][e] += q * wv[e];
+            }
+        }
+    }
+#pragma unroll
+    for (int b = 0; b < ABS_NB; ++b)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) red[g][b][cg * 8 + e] = acc[b][e];
+    sync();
+    for (int i = t; i < nb * 128; i += 256) {
+        const int b = i >> 7, c = i & 127;
+        if (r0 + c >= s.R) continue;
+        float v = 0.f;
+#pragma unroll
+        for (int j = 0; j < 16; ++j) v += red[j][b][c];
+        stf(qa + ((long long)(t0 + b) * s.H + h) * s.cw + r0 + c, v);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------- decode attention, matrix pipe (bf16)
+// One workgroup: one token, NG groups of 16 heads, a contiguous range of 64-row cache tiles.  Tiles arrive by LDS-DMA, double-buffered, chunk
+// slot = chunk ^ (row & 7).  Wave w scores rows 16 w .. 16 w + 15 of a tile against all heads (cache rows are k-contiguous B fragments as they
+// lie); the row maxima and the probabilities (bf16) meet in LDS; wave w then accumulates DTW 16-column slices of the latent output for all
+// 64 rows (V fragments by transposing reads of the same tile).  Online softmax in the log2 domain, fp32.
+template <int NG, int DTW, int KTM>
+__global__ __launch_bounds__(256) void latent_attn_kernel(const bf16_t* qa, const bf16_t* cache, Shape s, const int32_t* slot, const int32_t* pos,
+                                                          float* part_o, float* part_ml, int splits) {
+    ARIA_DYN_SMEM(smem);
+    constexpr int PP = 72;   // pitch of the probability tile (elements)
+    const int t = threadIdx.x, l = t & 63, w = first_lane(t >> 6), q4 = l >> 4, c16 = l & 15;
+    const int CPR = int(s.cw) >> 3, KT = int(s.cw) >> 5, tile_bytes = 64 * int(s.cw) * 2;
+    bf16_t* sP = reinterpret_cast<bf16_t*>(smem + 2 * tile_bytes);                    // [NG * 16][PP]
+    float* sMax = reinterpret_cast<float*>(smem + 2 * tile_bytes + NG * 16 * PP * 2); // [4][NG * 16]
+    const int sp = blockIdx.x, hg = blockIdx.y, tok = blockIdx.z;
+    const int n_keys = pos[tok] + 1, ntiles = (n_keys + 63) / 64, per = (ntiles + splits - 1) / splits;
+    const int it0 = sp * per, it1 = min(ntiles, it0 + per);
+    const int head0 = hg * NG * 16;
+    float* ml = part_ml + ((long long)tok * splits + sp) * s.H * 2;
+    if (it0 >= it1) {   // nothing to see for this split
+        if (t < NG * 16 && head0 + t < s.H) {
+            ml[2 * (head0 + t)] = -INFINITY;
+            ml[2 * (head0 + t) + 1] = 0.f;
+        }
+        return;
+    }
+    const bf16_t* base = cache + (long long)slot[tok] * s.S_cap * s.cw;
+    // this lane's chunk of the wave's first DMA piece, and the step to its next one (4 pieces of 64 chunks further on)
+    const int row_i = (w * 64 + l) / CPR, slot_i = (w * 64 + l) % CPR, dr_ = 256 / CPR, ds_ = 256 % CPR;
+    auto dma = [&](int tile, char* dst) __attribute__((always_inline)) {
+        int row = row_i, sl = slot_i;
+        for (int pc = w; pc < CPR; pc += 4) {
+            const int ch = sl ^ (row & 7);
+            glds16_raw(base + (long long)min(tile * 64 + row, n_keys - 1) * s.cw + ch * 8, dst + pc * 1024);
+            row += dr_;
+            sl += ds_;
+            if (sl >= CPR) {
+                sl -= CPR;
+                row += 1;
+            }
+        }
+    };
+    dma(it0, smem);
+    s16x8 qf[NG][KTM];
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+        for (int kk = 0; kk < KTM; ++kk) {
+            u32x4 v = zero16();
+            const int head = head0 + g * 16 + c16;
+            if (head < s.H && kk < KT) v = ld16(qa + ((long long)tok * s.H + head) * s.cw + kk * 32 + q4 * 8);
+            qf[g][kk] = __builtin_bit_cast(s16x8, v);
+        }
+    f32x4 o[NG][DTW];
+    float m[NG][4], lsum[NG][4];
+#pragma unroll
+    for (int g = 0; g < NG; ++g) {
+#pragma unroll
+        for (int i = 0; i < DTW; ++i) o[g][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            m[g][r] = -INFINITY;
+            lsum[g][r] = 0.f;
+        }
+    }
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+        for (int kk = 0; kk < KTM; ++kk) settle(qf[g][kk]);
+    const float scale2 = s.scale * 1.4426950408889634f;
+    for (int it = it0; it < it1; ++it) {
+        const char* cur = smem + ((it - it0) & 1) * tile_bytes;
+        wait_vm<0>();
+        sync();   // tile `it` is complete; every wave is done with the other buffer, the probabilities and the maxima
+        if (it + 1 < it1) dma(it + 1, smem + ((it - it0 + 1) & 1) * tile_bytes);
+        // scores: C rows = heads 4 q4 + r of a group, columns = cache rows 16 w + c16
+        f32x4 sc[NG];
+#pragma unroll
+        for (int g = 0; g < NG; ++g) sc[g] = f32x4{0.f, 0.f, 0.f, 0.f};
+        const int krow = 16 * w + c16;
+        const char* kbase = cur + krow * CPR * 16;
+#pragma unroll
+        for (int kk = 0; kk < KTM; ++kk)
+            if (kk < KT) {
+                const s16x8 kf = *reinterpret_cast<const s16x8*>(kbase + (((kk * 4 + q4) ^ (krow & 7)) << 4));
+#pragma unroll
+                for (int g = 0; g < NG; ++g) sc[g] = mfma16(qf[g][kk], kf, sc[g]);
+            }
+        const bool dead = it * 64 + krow >= n_keys;
+#pragma unroll
+        for (int g = 0; g < NG; ++g)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                sc[g][r] = dead ? -INFINITY : sc[g][r] * scale2;
+                float mx = sc[g][r];
+#pragma unroll
+                for (int d = 1; d < 16; d <<= 1) mx = fmaxf(mx, shfl_xor(mx, d));
+                if (c16 == 0) sMax[w * NG * 16 + g * 16 + 4 * q4 + r] = mx;
+            }
+        sync();
+#pragma unroll
+        for (int g = 0; g < NG; ++g) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int hr = g * 16 + 4 * q4 + r;
+                float mn = m[g][r];
+#pragma unroll
+                for (int ww = 0; ww < 4; ++ww) mn = fmaxf(mn, sMax[ww * NG * 16 + hr]);   // finite: a tile holds at least one visible row
+                const float alpha = exp2_fast(m[g][r] - mn);
+                const float p = exp2_fast(sc[g][r] - mn);
+                m[g][r] = mn;
+                lsum[g][r] = lsum[g][r] * alpha + p;
+                sP[hr * PP + krow] = f2bf(p);
+#pragma unroll
+                for (int i = 0; i < DTW; ++i) o[g][i][r] *= alpha;
+            }
+        }
+        sync();
+        // latent output: A = probabilities (heads x 32 rows), B = the tile's columns
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            s16x8 pf[NG];
+#pragma unroll
+            for (int g = 0; g < NG; ++g) pf[g] = *reinterpret_cast<const s16x8*>(sP + (g * 16 + c16) * PP + kk * 32 + q4 * 8);
+            const int vr = kk * 32 + q4 * 8 + (c16 >> 2);
+#pragma unroll
+            for (int i = 0; i < DTW; ++i) {
+                const int d0 = (w * DTW + i) * 16;
+                if (d0 < s.R) {   // (wave-uniform)
+                    const int col = d0 + 4 * (c16 & 3), ch = col >> 3, within = (col & 7) * 2;
+                    const s16x4 a0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + vr * CPR * 16 + ((ch ^ (vr & 7)) << 4) + within));
+                    const s16x4 a1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + (vr + 4) * CPR * 16 + ((ch ^ ((vr + 4) & 7)) << 4) + within));
+                    s16x8 vf;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        vf[e] = a0[e];
+                        vf[4 + e] = a1[e];
+                    }
+#pragma unroll
+                    for (int g = 0; g < NG; ++g) o[g][i] = mfma16(pf[g], vf, o[g][i]);
+                }
+            }
+        }
+    }
+    // row sums: over the 16 columns a lane group holds, then over the waves
+    sync();
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const float v = group_sum<16>(lsum[g][r]);
+            if (c16 == 0) sMax[w * NG * 16 + g * 16 + 4 * q4 + r] = v;
+        }
+    sync();
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int hr = g * 16 + 4 * q4 + r, head = head0 + hr;
+            if (head >= s.H) continue;
+            if (w == 0 && c16 == 0) {
+                float v = 0.f;
+                for (int ww = 0; ww < 4; ++ww) v += sMax[ww * NG * 16 + hr];
+                ml[2 * head] = m[g][r];
+                ml[2 * head + 1] = v;
+            }
+            float* po = part_o + (((long long)tok * splits + sp) * s.H + head) * s.R;
+#pragma unroll
+            for (int i = 0; i < DTW; ++i) {
+                const int d = (w * DTW + i) * 16 + c16;
+                if (d < s.R) po[d] = o[g][i][r];
+            }
+        }
+}
+
+// ---------------------------------------------------------------------------------------------- decode attention, any size (fp32 or bf16)
+// One workgroup per (head, token), a thread per cache row of a 256-row tile, then a thread per latent column.
+constexpr int ANY_COLS = 8;   // latent columns per thread: R <= 2048
+template <class T>
+__global__ __launch_bounds__(256) void latent_attn_any_kernel(const T* qa, const T* cache, Shape s, const int32_t* slot, const int32_t* pos,
+                                                              float* part_o, float* part_ml) {
+    ARIA_DYN_SMEM(smem);
+    float* sq = reinterpret_cast<float*>(smem);   // [cw]
+    float* sp = sq + s.cw;                        // [256]
+    float* sr = sp + 256;                         // [8]
+    const int t = threadIdx.x, l = t & 63, w = t >> 6, h = blockIdx.x, tok = blockIdx.y;
+    const int n_keys = pos[tok] + 1, width = int(s.R + s.dr);
+    const T* base = cache + (long long)slot[tok] * s.S_cap * s.cw;
+    const T* q = qa + ((long long)tok * s.H + h) * s.cw;
+    for (int i = t; i < s.cw; i += 256) sq[i] = ldf(q + i);
+    float acc[ANY_COLS], m = -INFINITY, lsum = 0.f;
+#pragma unroll
+    for (int j = 0; j < ANY_COLS; ++j) acc[j] = 0.f;
+    const float scale2 = s.scale * 1.4426950408889634f;
+    sync();
+    for (int k0 = 0; k0 < n_keys; k0 += 256) {
+        float x = -INFINITY;
+        if (k0 + t < n_keys) {
+            const T* row = base + (long long)(k0 + t) * s.cw;
+            float d = 0.f;
+            for (int c = 0; c < width; c += 8) {   // (the row and the query are zero behind `width`)
+                float v[8];
+                ld8(row + c, v);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) d += v[e] * sq[c + e];
+            }
+            x = d * scale2;
+        }
+        float mx = wave_max(x);
+        if (l == 0) sr[w] = mx;
+        sync();
+        const float mn = fmaxf(m, fmaxf(fmaxf(sr[0], sr[1]), fmaxf(sr[2], sr[3])));
+        const float p = exp2f(x - mn), alpha = exp2f(m - mn);
+        sp[t] = p;
+        const float ws = wave_sum(p);
+        if (l == 0) sr[4 + w] = ws;
+        sync();
+        m = mn;
+        lsum = lsum * alpha + (sr[4] + sr[5] + sr[6] + sr[7]);
+        const int n = min(256, n_keys - k0);
+#pragma unroll
+        for (int j = 0; j < ANY_COLS; ++j) {
+            const int r = t + 256 * j;
+            if (r < s.R) {
+                float a = acc[j] * alpha;
+                const T* colp = base + (long long)k0 * s.cw + r;
+                for (int i = 0; i < n; ++i) a += sp[i] * ldf(colp + (long long)i * s.cw);
+                acc[j] = a;
+            }
+        }
+        sync();
+    }
+    float* po = part_o + ((long long)tok * s.H + h) * s.R;
+#pragma unroll
+    for (int j = 0; j < ANY_COLS; ++j)
+        if (t + 256 * j < s.R) po[t + 256 * j] = acc[j];
+    if (t == 0) {
+        part_ml[((long long)tok * s.H + h) * 2] = m;
+        part_ml[((long long)tok * s.H + h) * 2 + 1] = lsum;
+    }
+}
+
+// ---------------------------------------------------------------------------------------------- decode: merge, expand, gate
+constexpr int EXP_ROWS = 32;       // value columns per workgroup
+constexpr int MAX_SPLITS = 64;
+template <class T>
+__global__ __launch_bounds__(256) void latent_expand_kernel(const float* part_o, const float* part_ml, Shape s, const T* proj, const T* uv, T* out,
+                                                            int splits) {
+    ARIA_DYN_SMEM(smem);
+    float* lat = reinterpret_cast<float*>(smem);   // [rp], zero behind R
+    float* wt = lat + s.rp;                        // [MAX_SPLITS]
+    const int t = threadIdx.x, l = t & 63, w = t >> 6, h = blockIdx.x, v0 = blockIdx.y * EXP_ROWS, tok = blockIdx.z;
+    if (w == 0) {
+        float m = -INFINITY, sum = 0.f;
+        if (l < splits) {
+            const float* ml = part_ml + (((long long)tok * splits + l) * s.H + h) * 2;
+            m = ml[0];
+            sum = ml[1];
+        }
+        const float mx = wave_max(m);
+        const float f = sum > 0.f ? exp2f(m - mx) : 0.f;
+        const float tot = wave_sum(sum * f);
+        if (l < splits) wt[l] = f / tot;
+    }
+    sync();
+    for (int r = t; r < s.rp; r += 256) {
+        float v = 0.f;
+        if (r < s.R)
+            for (int j = 0; j < splits; ++j)
+                if (wt[j] != 0.f) v += wt[j] * part_o[(((long long)tok * splits + j) * s.H + h) * s.R + r];
+        lat[r] = v;
+    }
+    sync();
+    const float gate = sigmoid_exact(ldf(proj + (long long)tok * s.ldp + s.g_off + h));
+    T* orow = out + ((long long)tok * s.H + h) * s.dvp;
+    const int nch = int(s.rp) >> 3;
+    float acc[EXP_ROWS / 4];
+#pragma unroll
+    for (int i = 0; i < EXP_ROWS / 4; ++i) acc[i] = 0.f;
+    for (int c = l; c < nch; c += 64) {
+        float lv[8];
+        ld8(lat + c * 8, lv);
+#pragma unroll
+        for (int i = 0; i < EXP_ROWS / 4; ++i) {
+            const int v = min(v0 + w + 4 * i, int(s.dv) - 1);
+            float wv[8];
+            ld8(uv + ((long long)h * s.dv + v) * s.rp + c * 8, wv);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[i] += wv[e] * lv[e];
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < EXP_ROWS / 4; ++i) {
+        const float v = wave_sum_bcast(acc[i]);
+        const int col = v0 + w + 4 * i;
+        if (l == 0 && col < s.dvp) stf(orow + col, col < s.dv ? v * gate : 0.f);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------- decode: row-streaming projections (bf16)
+__device__ __forceinline__ u32x4 ldw16(const bf16_t* p) {   // a weight stream is read once: non-temporal
+#ifdef ARIA_EMU
+    return ld16(p);
+#else
+    return __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(p));
+#endif
+}
+// acc[r][b] += W[row r] . X[token b], a wave over two weight rows and NB token rows: four 16-byte chunks per row and lane requested before the
+// first use, the token rows come from the L1 / L2
+template <int NB>
+__device__ __forceinline__ void two_rows(float (&acc)[2][NB], const bf16_t* w0, const bf16_t* w1, const bf16_t* x, long long ldx, int nb, int K, int l) {
+    const int nch = K >> 3;
+    for (int c0 = l; c0 < nch; c0 += 256) {
+        u32x4 a[2][4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int c = min(c0 + 64 * u, nch - 1);
+            a[0][u] = ldw16(w0 + c * 8);
+            a[1][u] = ldw16(w1 + c * 8);
+        }
+#pragma unroll
+        for (int b = 0; b < NB; ++b) {
+            const bf16_t* xr = x + (long long)min(b, nb - 1) * ldx;
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                u32x4 v = ld16(xr + min(c0 + 64 * u, nch - 1) * 8);
+                const bool in = c0 + 64 * u < nch;
+#pragma unroll
+                for (int q = 0; q < 4; ++q) {
+                    const uint32_t xv = in ? v[q] : 0u;
+                    acc[0][b] = dot2bf(a[0][u][q], xv, acc[0][b]);
+                    acc[1][b] = dot2bf(a[1][u][q], xv, acc[1][b]);
+                }
+            }
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < 2; ++r)
+#pragma unroll
+        for (int b = 0; b < NB; ++b) acc[r][b] = wave_sum_bcast(acc[r][b]);
+}
+// the residual step of one stream element: x += post(v), and the next norm of the new x
+__device__ __forceinline__ void stream_step(float v, const AriaDyT& post, const AriaDyT& next, float* x, bf16_t* h, long long at, int n) {
+    const float xn = x[at] + dyt<bf16_t>(post, v, n);
+    x[at] = xn;
+    if (next.w) h[at] = f2bf(dyt<bf16_t>(next, xn, n));
+}
+enum { ROWS_BF16 = 0, ROWS_RELU2 = 1, ROWS_STREAM = 2, ROWS_F32 = 3 };
+struct RowsOut {
+    void* out;
+    long long ldo;
+    AriaDyT post, next;
+    float* x;
+    bf16_t* h;
+};
+template <int NB, int MODE>
+__global__ __launch_bounds__(256) void rows_kernel(const bf16_t* W, const bf16_t* X, long long ldx, int K, int N, int n_tok, RowsOut ro) {
+    const int l = threadIdx.x & 63, w = threadIdx.x >> 6;
+    const int row0 = (blockIdx.x * 4 + w) * 2, t0 = blockIdx.y * NB;
+    if (row0 >= N) return;
+    const int nb = min(NB, n_tok - t0);
+    float acc[2][NB];
+#pragma unroll
+    for (int r = 0; r < 2; ++r)
+#pragma unroll
+        for (int b = 0; b < NB; ++b) acc[r][b] = 0.f;
+    two_rows<NB>(acc, W + (long long)row0 * K, W + (long long)min(row0 + 1, N - 1) * K, X + (long long)t0 * ldx, ldx, nb, K, l);
+    float mine = 0.f;   // lane r * NB + b finishes element (row0 + r, t0 + b)
+#pragma unroll
+    for (int r = 0; r < 2; ++r)
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+            if (l == r * NB + b) mine = acc[r][b];
+    const int n = row0 + l / NB, b = l % NB;
+    if (l >= 2 * NB || n >= N || b >= nb) return;
+    const long long at = (long long)(t0 + b) * ro.ldo + n;
+    if (MODE == ROWS_BF16) static_cast<bf16_t*>(ro.out)[at] = f2bf(mine);
+    if (MODE == ROWS_RELU2) static_cast<bf16_t*>(ro.out)[at] = f2bf(relu_squared(mine));
+    if (MODE == ROWS_F32) static_cast<float*>(ro.out)[at] = mine;
+    if (MODE == ROWS_STREAM) stream_step(mine, ro.post, ro.next, ro.x, ro.h, at, n);
+}
+
+// routed up-projection of one (token, slot): act = silu(gate . h) * (up . h); the routing runs in front of the rows, workgroup x = 0 publishes it
+__global__ __launch_bounds__(256) void mix_up_kernel(const float* logits, const float* correction, int E, int ldl, int groups, int keep, int k,
+                                                     const bf16_t* Wg, const bf16_t* Wu, const bf16_t* X, int K, int F, bf16_t* act, float* weights,
+                                                     int32_t* idx) {
+    ARIA_SMEM_STATIC float lds[4][768];
+    const int l = threadIdx.x & 63, w = threadIdx.x >> 6, j = blockIdx.y, tok = blockIdx.z;
+    float my_w;
+    int my_e;
+    const int e = route_group_limited(logits + (long long)tok * ldl, correction, E, groups, keep, k, lds[w], l, j, my_w, my_e);
+    if (blockIdx.x == 0 && j == 0 && w == 0 && l < k) {
+        weights[tok * k + l] = my_w;
+        idx[tok * k + l] = my_e;
+    }
+    const int n = blockIdx.x * 4 + w;
+    if (n >= F) return;
+    float acc[2][1] = {{0.f}, {0.f}};
+    const long long row = ((long long)e * F + n) * K;
+    two_rows<1>(acc, Wg + row, Wu + row, X + (long long)tok * K, K, 1, K, l);
+    if (l == 0) act[((long long)tok * k + j) * F + n] = f2bf(silu_fast(acc[0][0]) * acc[1][0]);
+}
+// down-projections of a token's k experts for two stream columns, their weighted sum, residual and norms
+__global__ __launch_bounds__(256) void mix_down_kernel(const bf16_t* Wd, const float* weights, const int32_t* idx, int k, const bf16_t* act, int F, int D,
+                                                       RowsOut ro) {
+    const int l = threadIdx.x & 63, w = threadIdx.x >> 6, tok = blockIdx.y;
+    const int row0 = (blockIdx.x * 4 + w) * 2;
+    if (row0 >= D) return;
+    float y0 = 0.f, y1 = 0.f;
+    for (int j = 0; j < k; ++j) {
+        const bf16_t* base = Wd + (long long)idx[tok * k + j] * D * F;
+        float acc[2][1] = {{0.f}, {0.f}};
+        two_rows<1>(acc, base + (long long)row0 * F, base + (long long)min(row0 + 1, D - 1) * F, act + ((long long)tok * k + j) * F, F, 1, F, l);
+        const float wj = weights[tok * k + j];
+        y0 += wj * acc[0][0];
+        y1 += wj * acc[1][0];
+    }
+    if (l < 2 && row0 + l < D) stream_step(l ? y1 : y0, ro.post, ro.next, ro.x, ro.h, (long long)tok * D + row0 + l, row0 + l);
+}
+
+bool al16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+
+int shape_ok(const Shape* s) {
+    if (!s || s->H <= 0 || s->dn <= 0 || s->dr < 0 || s->dv <= 0 || s->R <= 0 || s->S_cap <= 0) return ARIA_ERR_INVALID;
+    if (s->rot < 0 || (s->rot & 1) || s->rot > s->dr || s->dq < s->dn + s->dr || s->dvp < s->dv || s->cw < s->R + s->dr || s->rp < s->R ||
+        s->kv_off < s->H * s->dq || s->g_off < s->kv_off + s->R + s->dr || s->ldp < s->g_off + s->H)
+        return ARIA_ERR_INVALID;
+    if ((s->cw & 63) || (s->rp & 7) || s->rp > s->cw || (s->ldp & 7)) return ARIA_ERR_ALIGN;
+    return ARIA_OK;
+}
+
+template <class T>
+int launch_any(const T* qa, const T* cache, const Shape& s, const int32_t* slot, const int32_t* pos, float* po, float* ml, int64_t n_tok, void* stream) {
+    if (s.R > 256 * ANY_COLS) return ARIA_ERR_UNSUPPORTED;
+    ARIA_LAUNCH((latent_attn_any_kernel<T>), dim3(unsigned(s.H), unsigned(n_tok)), dim3(256), size_t(s.cw + 264) * 4, stream, qa, cache, s, slot, pos,
+                po, ml);
+    return aria_check_launch();
+}
+// the matrix-pipe form's limits: cache row and latent width of one instantiation
+int mfma_class(const Shape& s) {
+    if (s.R <= 128 && s.cw <= 192) return 1;
+    if (s.R <= 256 && s.cw <= 320) return 2;
+    if (s.R <= 512 && s.cw <= 576) return 3;
+    return 0;
+}
+
+}  // namespace
+
+extern "C" {
+
+int aria_latent_rows(void* proj, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, const float* rope, const float* kv_norm, void* cache,
+                     void* packed, int64_t T, int f32, void* stream) {
+    if (!proj || !slot || !pos || !rope || !kv_norm || !cache || !packed || T < 0) return ARIA_ERR_INVALID;
+    if (const int rc = shape_ok(s)) return rc;
+    if (T == 0) return ARIA_OK;
+    const dim3 grid(unsigned((T + 3) / 4)), block(256);
+    if (f32)
+        ARIA_LAUNCH((latent_rows_kernel<float>), grid, block, 0, stream, static_cast<float*>(proj), *s, slot, pos, rope, kv_norm,
+                    static_cast<float*>(cache), static_cast<float*>(packed), int(T));
+    else
+        ARIA_LAUNCH((latent_rows_kernel<bf16_t>), grid, block, 0, stream, static_cast<bf16_t*>(proj), *s, slot, pos, rope, kv_norm,
+                    static_cast<bf16_t*>(cache), static_cast<bf16_t*>(packed), int(T));
+    return aria_check_launch();
+}
+
+int aria_latent_absorb(const void* proj, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, const float* rope, const float* kv_norm,
+                       const void* uk, void* cache, void* qa, int64_t T, int f32, void* stream) {
+    if (!proj || !slot || !pos || !rope || !kv_norm || !uk || !cache || !qa || T < 0) return ARIA_ERR_INVALID;
+    if (const int rc = shape_ok(s)) return rc;
+    if (!al16(uk)) return ARIA_ERR_ALIGN;
+    if (T == 0) return ARIA_OK;
+    const dim3 grid(unsigned(s->H * ((s->R + 127) / 128) + 1), unsigned((T + ABS_NB - 1) / ABS_NB)), block(256);
+    if (f32)
+        ARIA_LAUNCH((latent_absorb_kernel<float>), grid, block, 0, stream, static_cast<const float*>(proj), *s, slot, pos, rope, kv_norm,
+                    static_cast<const float*>(uk), static_cast<float*>(cache), static_cast<float*>(qa), int(T));
+    else
+        ARIA_LAUNCH((latent_absorb_kernel<bf16_t>), grid, block, 0, stream, static_cast<const bf16_t*>(proj), *s, slot, pos, rope, kv_norm,
+                    static_cast<const bf16_t*>(uk), static_cast<bf16_t*>(cache), static_cast<bf16_t*>(qa), int(T));
+    return aria_check_launch();
+}
+
+int64_t aria_latent_splits(const AriaLatentShape* s, int64_t T, int64_t max_len) {
+    if (!s || T <= 0 || !mfma_class(*s)) return 1;
+    const int64_t tiles = (max_len + 63) / 64, groups = (s->H + 15) / 16 <= 1 ? 1 : (s->H + 31) / 32;
+    int64_t n = (2 * 256 + T * groups - 1) / (T * groups);   // about two workgroups a CU
+    n = n < tiles ? n : tiles;
+    n = n < MAX_SPLITS ? n : MAX_SPLITS;
+    return n < 1 ? 1 : n;
+}
+
+int aria_latent_attn(const void* qa, const void* cache, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, float* part_o, float* part_ml,
+                     int64_t T, int64_t splits, int f32, void* stream) {
+    if (!qa || !cache || !slot || !pos || !part_o || !part_ml || T < 0 || splits < 1) return ARIA_ERR_INVALID;
+    if (const int rc = shape_ok(s)) return rc;
+    if (!al16(qa) || !al16(cache)) return ARIA_ERR_ALIGN;
+    if (T == 0) return ARIA_OK;
+    if (T > 65535 || splits > MAX_SPLITS) return ARIA_ERR_UNSUPPORTED;
+    const int cls = f32 ? 0 : mfma_class(*s);
+    if (cls == 0) {
+        if (splits != 1) return ARIA_ERR_UNSUPPORTED;
+        return f32 ? launch_any(static_cast<const float*>(qa), static_cast<const float*>(cache), *s, slot, pos, part_o, part_ml, T, stream)
+                   : launch_any(static_cast<const bf16_t*>(qa), static_cast<const bf16_t*>(cache), *s, slot, pos, part_o, part_ml, T, stream);
+    }
+    const bf16_t *q = static_cast<const bf16_t*>(qa), *c = static_cast<const bf16_t*>(cache);
+    const int NG = s->H <= 16 ? 1 : 2;
+    const dim3 grid(unsigned(splits), unsigned((s->H + 16 * NG - 1) / (16 * NG)), unsigned(T)), block(256);
+    const size_t lds = size_t(2) * 64 * s->cw * 2 + size_t(NG) * 16 * 72 * 2 + size_t(4) * NG * 16 * 4;
+#define ARIA_LATENT(G, D, K) ARIA_LAUNCH((latent_attn_kernel<G, D, K>), grid, block, lds, stream, q, c, *s, slot, pos, part_o, part_ml, int(splits))
+    if (NG == 1) {
+        if (cls == 1)
+            ARIA_LATENT(1, 2, 6);
+        else if (cls == 2)
+            ARIA_LATENT(1, 4, 10);
+        else
+            ARIA_LATENT(1, 8, 18);
+    } else {
+        if (cls == 1)
+            ARIA_LATENT(2, 2, 6);
+        else if (cls == 2)
+            ARIA_LATENT(2, 4, 10);
+        else
+            ARIA_LATENT(2, 8, 18);
+    }
+#undef ARIA_LATENT
+    return aria_check_launch();
+}
+
+int aria_latent_expand(const float* part_o, const float* part_ml, const AriaLatentShape* s, const void* proj, const void* uv, void* out, int64_t T,
+                       int64_t splits, int f32, void* stream) {
+    if (!part_o || !part_ml || !proj || !uv || !out || T < 0 || splits < 1) return ARIA_ERR_INVALID;
+    if (const int rc = shape_ok(s)) return rc;
+    if (!al16(uv)) return ARIA_ERR_ALIGN;
+    if (T == 0) return ARIA_OK;
+    if (T > 65535 || splits > MAX_SPLITS) return ARIA_ERR_UNSUPPORTED;
+    const dim3 grid(unsigned(s->H), unsigned((s->dvp + EXP_ROWS - 1) / EXP_ROWS), unsigned(T)), block(256);
+    const size_t lds = size_t(s->rp + MAX_SPLITS) * 4;
+    if (f32)
+        ARIA_LAUNCH((latent_expand_kernel<float>), grid, block, lds, stream, part_o, part_ml, *s, static_cast<const float*>(proj),
+                    static_cast<const float*>(uv), static_cast<float*>(out), int(splits));
+    else
+        ARIA_LAUNCH((latent_expand_kernel<bf16_t>), grid, block, lds, stream, part_o, part_ml, *s, static_cast<const bf16_t*>(proj),
+                    static_cast<const bf16_t*>(uv), static_cast<bf16_t*>(out), int(splits));
+    return aria_check_launch();
+}
+
+}  // extern "C"
+
+namespace {
+
+struct Scratch {
+    float *x, *part_o, *part_ml, *logits, *weights;
+    bf16_t *h, *proj, *qa, *ao, *act;
+    int32_t* idx;
+    int64_t bytes;
+};
+Scratch layout(const AriaLatentStack& st, const AriaLatentLayer* L, int64_t T, int64_t max_len, char* base) {
+    int64_t ldp = 0, qa = 0, ao = 0, act = 0, po = 0, ml = 0, E = 0, k = 0;
+    for (int64_t i = 0; i < st.n_layers; ++i) {
+        const Shape& s = L[i].mix;
+        const int64_t ns = aria_latent_splits(&s, T, max_len);
+        ldp = std::max(ldp, s.ldp);
+        qa = std::max(qa, s.H * s.cw);
+        ao = std::max(ao, s.H * s.dvp);
+        po = std::max(po, ns * s.H * s.R);
+        ml = std::max(ml, ns * s.H * 2);
+        if (L[i].mlp) act = std::max(act, L[i].ff * (L[i].mlp == 2 ? L[i].k : 1));
+        if (L[i].mlp == 2) {
+            E = std::max(E, (L[i].E + 7) & ~int64_t(7));
+            k = std::max(k, L[i].k);
+        }
+    }
+    Scratch z{};
+    int64_t at = 0;
+    auto take = [&](int64_t bytes) {
+        char* p = base + at;
+        at += (bytes + 255) & ~int64_t(255);
+        return p;
+    };
+    z.x = reinterpret_cast<float*>(take(4 * T * st.D));
+    z.h = reinterpret_cast<bf16_t*>(take(2 * T * st.D));
+    z.proj = reinterpret_cast<bf16_t*>(take(2 * T * ldp));
+    z.qa = reinterpret_cast<bf16_t*>(take(2 * T * qa));
+    z.ao = reinterpret_cast<bf16_t*>(take(2 * T * ao));
+    z.act = reinterpret_cast<bf16_t*>(take(2 * T * act));
+    z.part_o = reinterpret_cast<float*>(take(4 * T * po));
+    z.part_ml = reinterpret_cast<float*>(take(4 * T * ml));
+    z.logits = reinterpret_cast<float*>(take(4 * T * E));
+    z.weights = reinterpret_cast<float*>(take(4 * T * k));
+    z.idx = reinterpret_cast<int32_t*>(take(4 * T * k));
+    z.bytes = at;
+    return z;
+}
+
+template <int MODE>
+int rows(const void* W, const bf16_t* X, int64_t ldx, int64_t K, int64_t N, int64_t T, const RowsOut& ro, void* stream) {
+    const bf16_t* w = static_cast<const bf16_t*>(W);
+    const int nb = T >= 5 ? 8 : T >= 3 ? 4 : int(T);
+    const dim3 grid(unsigned((N + 7) / 8), unsigned((T + nb - 1) / nb)), block(256);
+#define ARIA_ROWS(B) ARIA_LAUNCH((rows_kernel<B, MODE>), grid, block, 0, stream, w, X, (long long)ldx, int(K), int(N), int(T), ro)
+    if (nb == 1)
+        ARIA_ROWS(1);
+    else if (nb == 2)
+        ARIA_ROWS(2);
+    else if (nb == 4)
+        ARIA_ROWS(4);
+    else
+        ARIA_ROWS(8);
+#undef ARIA_ROWS
+    return aria_check_launch();
+}
+
+}  // namespace
+
+extern "C" {
+
+int64_t aria_latent_decode_scratch(const AriaLatentStack* stack, const AriaLatentLayer* layers, int64_t T, int64_t max_len) {
+    if (!stack || !layers || T <= 0 || max_len <= 0) return 0;
+    return layout(*stack, layers, T, max_len, nullptr).bytes;
+}
+
+int aria_latent_decode(const AriaLatentStack* st, const AriaLatentLayer* L, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos,
+                       int64_t max_len, float* logits, void* scratch, int64_t scratch_bytes, void* stream) {
+    if (!st || !L || !ids || !slot || !pos || !logits || !scratch || T < 0 || max_len <= 0 || st->n_layers <= 0) return ARIA_ERR_INVALID;
+    if (T == 0) return ARIA_OK;
+    if ((st->D & 7) || !al16(scratch)) return ARIA_ERR_ALIGN;
+    const Scratch z = layout(*st, L, T, max_len, static_cast<char*>(scratch));
+    if (scratch_bytes < z.bytes) return ARIA_ERR_INVALID;
+    for (int64_t i = 0; i < st->n_layers; ++i) {
+        if (const int rc = shape_ok(&L[i].mix)) return rc;
+        if (max_len > L[i].mix.S_cap || (L[i].mix.H * L[i].mix.dvp & 7) || (L[i].mlp && (L[i].ff & 7))) return ARIA_ERR_INVALID;
+        if (L[i].mlp == 2 && (L[i].E > 256 || L[i].k > 64 || L[i].groups <= 0 || L[i].E % L[i].groups)) return ARIA_ERR_UNSUPPORTED;
+    }
+    const int64_t D = st->D;
+    const AriaDyT none{0.f, nullptr, nullptr};
+    int rc = aria_dyt_stream(ids, st->embed, nullptr, nullptr, nullptr, 0, &none, z.x, &st->first, z.h, T, D, 0, 0, stream);
+    for (int64_t i = 0; i < st->n_layers && rc == ARIA_OK; ++i) {
+        const AriaLatentLayer& y = L[i];
+        const Shape& s = y.mix;
+        const int64_t ns = aria_latent_splits(&s, T, max_len);
+        RowsOut plain{z.proj, (long long)s.ldp, none, none, nullptr, nullptr};
+        rc = rows<ROWS_BF16>(y.w_in, z.h, D, D, s.ldp, T, plain, stream);
+        if (rc == ARIA_OK) rc = aria_latent_absorb(z.proj, &s, slot, pos, y.rope, y.kv_norm, y.w_uk, y.cache, z.qa, T, 0, stream);
+        if (rc == ARIA_OK) rc = aria_latent_attn(z.qa, y.cache, &s, slot, pos, z.part_o, z.part_ml, T, ns, 0, stream);
+        if (rc == ARIA_OK) rc = aria_latent_expand(z.part_o, z.part_ml, &s, z.proj, y.w_uv, z.ao, T, ns, 0, stream);
+        RowsOut out{nullptr, (long long)D, y.norm1b, y.mlp ? y.norm2 : y.next, z.x, z.h};
+        if (rc == ARIA_OK) rc = rows<ROWS_STREAM>(y.w_o, z.ao, s.H * s.dvp, s.H * s.dvp, D, T, out, stream);
+        if (rc != ARIA_OK || y.mlp == 0) continue;
+        out.post = y.norm2b;
+        out.next = y.next;
+        if (y.mlp == 1) {
+            RowsOut up{z.act, (long long)y.ff, none, none, nullptr, nullptr};
+            rc = rows<ROWS_RELU2>(y.w_up, z.h, D, D, y.ff, T, up, stream);
+            if (rc == ARIA_OK) rc = rows<ROWS_STREAM>(y.w_down, z.act, y.ff, y.ff, D, T, out, stream);
+        } else {
+            const int64_t ldl = (y.E + 7) & ~int64_t(7);
+            RowsOut lg{z.logits, (long long)ldl, none, none, nullptr, nullptr};
+            rc = rows<ROWS_F32>(y.w_router, z.h, D, D, y.E, T, lg, stream);
+            if (rc != ARIA_OK) break;
+            ARIA_LAUNCH(mix_up_kernel, dim3(unsigned((y.ff + 3) / 4), unsigned(y.k), unsigned(T)), dim3(256), 0, stream, (const float*)z.logits,
+                        y.correction, int(y.E), int(ldl), int(y.groups), int(y.keep), int(y.k), static_cast<const bf16_t*>(y.w_gate),
+                        static_cast<const bf16_t*>(y.w_up), (const bf16_t*)z.h, int(D), int(y.ff), z.act, z.weights, z.idx);
+            ARIA_LAUNCH(mix_down_kernel, dim3(unsigned((D + 7) / 8), unsigned(T)), dim3(256), 0, stream, static_cast<const bf16_t*>(y.w_down),
+                        (const float*)z.weights, (const int32_t*)z.idx, int(y.k), (const bf16_t*)z.act, int(y.ff), int(D), out);
+            rc = aria_check_launch();
+        }
+    }
+    if (rc != ARIA_OK) return rc;
+    RowsOut lo{logits, (long long)st->V, none, none, nullptr, nullptr};
+    return rows<ROWS_F32>(st->head, z.h, D, D, st->V, T, lo, stream);
+}
+
+}  // extern "C"

@@ -1,7 +1,6 @@
 // MoE routing / token dispatch kernels (HBM-bound integer + byte work: coalesced 16-byte rows, wave
 // ballots for the stable sort, no host round trips).  Reference: aria/model/moe_lm.py:243-365, 505-507.
-#include "aria_device.h"
-#include "aria_hip.h"
+#include "elem.h"
 #include <cstdlib>
 #include <algorithm>
 
@@ -180,6 +179,35 @@ __global__ __launch_bounds__(256) void route_kernel(const void* logits_, void* s
         if (hist[i]) atomic_add(&counts[i], hist[i]);
 }
 
+// ------------------------------------------------------------------------------------------- group-limited route
+__global__ __launch_bounds__(256) void zero_i32_kernel(int32_t* p, int n) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) p[i] = 0;
+}
+// one wave per token (route_group_limited, elem.h); the histogram per workgroup in LDS like route_kernel
+__global__ __launch_bounds__(256) void route_groups_kernel(const float* logits, const float* correction, float* weights, int32_t* indices, int32_t* counts,
+                                                           int T, int E, int ldl, int groups, int keep, int k) {
+    ARIA_SMEM_STATIC int hist[256];
+    ARIA_SMEM_STATIC float lds[4][768];
+    for (int i = threadIdx.x; i < E; i += blockDim.x) hist[i] = 0;
+    sync();
+    const int l = threadIdx.x & 63, w = threadIdx.x >> 6;
+    const int nwaves = (gridDim.x * blockDim.x) >> 6;
+    for (int t = (blockIdx.x * blockDim.x + threadIdx.x) >> 6; t < T; t += nwaves) {
+        float my_w;
+        int my_e;
+        route_group_limited(logits + (long long)t * ldl, correction, E, groups, keep, k, lds[w], l, 0, my_w, my_e);
+        if (l < k) {
+            weights[(long long)t * k + l] = my_w;
+            indices[(long long)t * k + l] = my_e;
+            atomic_add(&hist[my_e], 1);
+        }
+    }
+    sync();
+    for (int i = threadIdx.x; i < E; i += blockDim.x)
+        if (hist[i]) atomic_add(&counts[i], hist[i]);
+}
+
 // ------------------------------------------------------------------------------------------- stable sort (E <= 64)
 constexpr int SORT_CHUNK = 2048;
 
@@ -251,6 +279,30 @@ __global__ __launch_bounds__(64) void sort_scatter_kernel(const int32_t* idx, co
             inv[i] = pos;
         }
         counter += __builtin_popcountll(match_mask(l, bal, vm));
+    }
+}
+
+// more than 64 experts: one workgroup, thread e owns expert e and walks the indices (staged through LDS, read as broadcasts) in order
+constexpr int SORT_WIDE_E = 256;
+__global__ __launch_bounds__(SORT_WIDE_E) void sort_wide_kernel(const int32_t* idx, const int32_t* counts, int32_t* offsets, int32_t* sorted_src,
+                                                                int32_t* inv, int E, int M) {
+    ARIA_SMEM_STATIC int buf[SORT_WIDE_E], cnt[SORT_WIDE_E];
+    const int t = threadIdx.x;
+    cnt[t] = t < E ? counts[t] : 0;
+    sync();
+    int at = 0;
+    for (int e = 0; e < t; ++e) at += cnt[e];
+    if (t < E) offsets[t] = at;
+    if (t == E - 1) offsets[E] = at + cnt[t];
+    for (int i0 = 0; i0 < M; i0 += SORT_WIDE_E) {
+        sync();
+        buf[t] = i0 + t < M ? idx[i0 + t] : -1;
+        sync();
+        for (int i = 0; i < SORT_WIDE_E; ++i)
+            if (buf[i] == t) {
+                sorted_src[at] = i0 + i;
+                inv[i0 + i] = at++;
+            }
     }
 }
 
@@ -554,6 +606,20 @@ __global__ __launch_bounds__(256) void swiglu_fwd_kernel(const bf16_t* h, const 
     }
 }
 
+// act = relu(u)^2, or silu(gate) u, on rows with leading dimensions (bf16 and 32-bit)
+template <class T>
+__global__ __launch_bounds__(256) void act_rows_kernel(const T* gate, const T* u, T* act, long long nitems, int nch, long long ld_in, long long ld_act) {
+    for (long long i = blockIdx.x * (long long)blockDim.x + threadIdx.x; i < nitems; i += (long long)gridDim.x * blockDim.x) {
+        const long long m = i / nch, n0 = (i % nch) * 8;
+        float v[8], g[8];
+        ld8(u + m * ld_in + n0, v);
+        if (gate) ld8(gate + m * ld_in + n0, g);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = gate ? g[e] * sigmoid_exact(g[e]) * v[e] : relu_squared(v[e]);
+        st8(act + m * ld_act + n0, v);
+    }
+}
+
 __global__ __launch_bounds__(256) void swiglu_bwd_kernel(const bf16_t* h, const bf16_t* h2, const bf16_t* dact, bf16_t* dh,
                                                          bf16_t* dh2, long long nchunks, int I, long long lda, long long ldb) {
     const int cpr = I >> 3;
@@ -663,8 +729,12 @@ int aria_moe_router_fused(const void* x, const void* w, void* logits, void* scor
 int aria_moe_sort(const int32_t* indices, const int32_t* counts, int32_t* offsets, int32_t* sorted_src, int32_t* inv,
                   int32_t* workspace, int64_t T, int64_t E, int64_t k, void* stream) {
     if (!indices || !counts || !offsets || !sorted_src || !inv || !workspace || T < 0 || E <= 0 || k <= 0) return ARIA_ERR_INVALID;
-    if (E > 64) return ARIA_ERR_UNSUPPORTED;
+    if (E > SORT_WIDE_E) return ARIA_ERR_UNSUPPORTED;
     const int M = int(T * k);
+    if (E > 64) {
+        ARIA_LAUNCH(sort_wide_kernel, dim3(1), dim3(SORT_WIDE_E), 0, stream, indices, counts, offsets, sorted_src, inv, int(E), M);
+        return aria_check_launch();
+    }
     const int nchunks = (M + SORT_CHUNK - 1) / SORT_CHUNK;
     int32_t* chunk_counts = workspace;
     int32_t* chunk_base = workspace + (size_t)nchunks * 64;
@@ -790,6 +860,32 @@ int aria_embedding_bwd(const void* dy, const int32_t* ids, void* dw, int64_t T, 
     if (T == 0) return ARIA_OK;
     ARIA_LAUNCH(embedding_bwd_kernel, dim3(grid_for_waves(T)), dim3(256), 0, stream, static_cast<const bf16_t*>(dy), ids,
                 static_cast<bf16_t*>(dw), int(T), int(D));
+    return aria_check_launch();
+}
+
+int aria_moe_route_groups(const float* logits, const float* correction, float* weights, int32_t* indices, int32_t* counts, int64_t T, int64_t E,
+                          int64_t ldl, int64_t groups, int64_t keep, int64_t k, void* stream) {
+    if (!logits || !correction || !weights || !indices || !counts || T < 0 || E <= 0 || k <= 0 || groups <= 0 || keep <= 0 || ldl < E) return ARIA_ERR_INVALID;
+    if (E > 256 || k > 64 || E % groups || keep > groups || k > keep * (E / groups)) return ARIA_ERR_UNSUPPORTED;
+    ARIA_LAUNCH(zero_i32_kernel, dim3(1), dim3(256), 0, stream, counts, int(E));   // (a kernel: the call may be captured into a graph)
+    if (T == 0) return aria_check_launch();
+    ARIA_LAUNCH(route_groups_kernel, dim3(std::min(grid_for_waves(T), 512)), dim3(256), 0, stream, logits, correction, weights, indices, counts, int(T),
+                int(E), int(ldl), int(groups), int(keep), int(k));
+    return aria_check_launch();
+}
+
+int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int f32, void* stream) {
+    if (!u || !act || M < 0 || n_cols <= 0) return ARIA_ERR_INVALID;
+    if ((n_cols & 7) || (ld_in & 7) || (ld_act & 7)) return ARIA_ERR_ALIGN;
+    if (M == 0) return ARIA_OK;
+    const long long nitems = M * (n_cols / 8);
+    const dim3 grid(unsigned(std::min<long long>((nitems + 255) / 256, 256 * 16))), block(256);
+    if (f32)
+        ARIA_LAUNCH((act_rows_kernel<float>), grid, block, 0, stream, static_cast<const float*>(gate), static_cast<const float*>(u), static_cast<float*>(act),
+                    nitems, int(n_cols / 8), (long long)ld_in, (long long)ld_act);
+    else
+        ARIA_LAUNCH((act_rows_kernel<bf16_t>), grid, block, 0, stream, static_cast<const bf16_t*>(gate), static_cast<const bf16_t*>(u),
+                    static_cast<bf16_t*>(act), nitems, int(n_cols / 8), (long long)ld_in, (long long)ld_act);
     return aria_check_launch();
 }
 

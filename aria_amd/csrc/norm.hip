@@ -1,9 +1,7 @@
 // RMSNorm (+ fused residual add), RoPE, small elementwise kernels: all HBM-bound, 16-byte accesses,
 // one wave per row.  Reference: transformers/models/llama/modeling_llama.py:62-67, 130-160, 295-325
 // (inherited by aria/model/moe_lm.py:580-602); gptfast/model.py:461-472.
-#include "aria_device.h"
-#include "aria_hip.h"
-#include <cmath>
+#include "elem.h"
 
 namespace {
 using namespace ad;
@@ -349,6 +347,45 @@ int grid1d(long long n, int per_block, int cap = 4096) {
     return int(g);
 }
 
+// One pass over the fp32 residual stream with the dynamic-tanh norms around it: source (embedding row | sublayer output | weighted sum of a token's
+// expert rows) -> x (+)= post(source) -> h = next(x).  Elementwise in the columns (these norms have no statistics): a thread owns 8 of them.
+template <class T>
+__global__ __launch_bounds__(256) void dyt_stream_kernel(const int32_t* ids, const T* table, const T* y, const int32_t* inv, const float* weights, int k,
+                                                         AriaDyT post, float* x, AriaDyT next, T* h, long long nitems, int nch, long long ldy) {
+    for (long long i = blockIdx.x * (long long)blockDim.x + threadIdx.x; i < nitems; i += (long long)gridDim.x * blockDim.x) {
+        const long long t = i / nch;
+        const int n0 = int(i % nch) * 8;
+        float v[8], xv[8];
+        float* xr = x + (t * nch) * 8 + n0;
+        if (ids) {
+            ld8(table + (long long)ids[t] * nch * 8 + n0, xv);
+        } else {
+            if (inv) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) v[e] = 0.f;
+                for (int j = 0; j < k; ++j) {
+                    float r[8];
+                    ld8(y + (long long)inv[t * k + j] * ldy + n0, r);
+                    const float w = weights[t * k + j];
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) v[e] += w * r[e];
+                }
+            } else {
+                ld8(y + t * ldy + n0, v);
+            }
+            ld8(xr, xv);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) xv[e] += dyt<T>(post, v[e], n0 + e);
+        }
+        st8(xr, xv);
+        if (next.w) {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] = dyt<T>(next, xv[e], n0 + e);
+            st8(h + (t * nch) * 8 + n0, v);
+        }
+    }
+}
+
 }  // namespace
 
 extern "C" {
@@ -459,6 +496,24 @@ int aria_adamw_step(void* param, const void* grad, float* master, float* m, floa
     const float bc1 = 1.f - powf(beta1, float(step)), bc2 = 1.f - powf(beta2, float(step));
     ARIA_LAUNCH(adamw_kernel, dim3(grid1d(n / 2, 256)), dim3(256), 0, stream, static_cast<bf16_t*>(param),
                 static_cast<const bf16_t*>(grad), master, m, v, (long long)n, lr, beta1, beta2, eps, weight_decay, bc1, bc2, grad_scale);
+    return aria_check_launch();
+}
+
+
+int aria_dyt_stream(const int32_t* ids, const void* table, const void* y, const int32_t* inv, const float* weights, int64_t k, const AriaDyT* post,
+                    float* x, const AriaDyT* next, void* h, int64_t T, int64_t D, int64_t ldy, int f32, void* stream) {
+    if (!x || !post || !next || T < 0 || D <= 0 || (ids ? !table : !y) || (!ids && !post->w) || (next->w && !h) || (inv && (!weights || k <= 0)))
+        return ARIA_ERR_INVALID;
+    if ((D & 7) || (!ids && (ldy & 7))) return ARIA_ERR_ALIGN;
+    if (T == 0) return ARIA_OK;
+    const long long nitems = T * (D / 8);
+    const dim3 grid(unsigned(std::min<long long>((nitems + 255) / 256, 256 * 16))), block(256);
+    if (f32)
+        ARIA_LAUNCH((dyt_stream_kernel<float>), grid, block, 0, stream, ids, static_cast<const float*>(table), static_cast<const float*>(y), inv, weights,
+                    int(k), *post, x, *next, static_cast<float*>(h), nitems, int(D / 8), (long long)ldy);
+    else
+        ARIA_LAUNCH((dyt_stream_kernel<bf16_t>), grid, block, 0, stream, ids, static_cast<const bf16_t*>(table), static_cast<const bf16_t*>(y), inv,
+                    weights, int(k), *post, x, *next, static_cast<bf16_t*>(h), nitems, int(D / 8), (long long)ldy);
     return aria_check_launch();
 }
 

@@ -23,7 +23,8 @@ ERRORS = {
 
 P, I64, I32, F32 = c_void_p, c_int64, c_int, c_float
 RESTYPES = {"aria_gemm_workspace_bytes": c_int64, "aria_decode_scratch_bytes": c_int64, "aria_decode_graph_create": c_void_p,
-            "aria_decode_graph_destroy": None, "aria_decode_attn_workspace_bytes": c_int64}  # everything else returns an int status
+            "aria_decode_graph_destroy": None, "aria_decode_attn_workspace_bytes": c_int64,
+            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64}  # everything else returns an int status
 
 # name -> argtypes (all return int).  Kept in one table so tests can check that the shared
 # library exports every symbol the header declares.
@@ -100,10 +101,42 @@ SIGNATURES = {
     "aria_gather_add_rows": [P, P, P, I64, I64, P],
     "aria_colsum_bf16": [P, P, I64, I64, I64, I64, P],
     "aria_cross_entropy": [P, P, P, P, P, F32, P, I64, I64, I64, P],
+    "aria_attn_varlen_fwd": [P, P, P, P, P, P, I64, I64, I64, I64, I64, I64, I64, I64, I64, I64, F32, P],
+    "aria_dyt_stream": [P, P, P, P, P, I64, P, P, P, P, I64, I64, I64, I32, P],
+    "aria_act_rows": [P, P, P, I64, I64, I64, I64, I32, P],
+    "aria_gemm_f32": [P, P, P, I64, I64, I64, I64, I64, I64, P, I64, I64, P],
+    "aria_moe_route_groups": [P, P, P, P, P, I64, I64, I64, I64, I64, I64, P],
+    "aria_latent_rows": [P, P, P, P, P, P, P, P, I64, I32, P],
+    "aria_latent_absorb": [P, P, P, P, P, P, P, P, P, I64, I32, P],
+    "aria_latent_attn": [P, P, P, P, P, P, P, I64, I64, I32, P],
+    "aria_latent_expand": [P, P, P, P, P, P, I64, I64, I32, P],
+    "aria_latent_splits": [P, I64, I64],
+    "aria_latent_decode_scratch": [P, P, I64, I64],
+    "aria_latent_decode": [P, P, I64, P, P, P, I64, P, P, I64, P],
 }
 
 
-ABI_VERSION = 3   # include/aria_hip.h ARIA_ABI_VERSION this host code was written against
+class DyTParams(ctypes.Structure):      # AriaDyT
+    _fields_ = [("alpha", c_float), ("w", c_void_p), ("b", c_void_p)]
+
+
+class LatentShape(ctypes.Structure):    # AriaLatentShape
+    _fields_ = [(n, c_int64) for n in ("H", "dn", "dr", "dv", "R", "rot", "dq", "dvp", "cw", "rp", "ldp", "kv_off", "g_off", "S_cap")] + \
+               [("scale", c_float), ("eps", c_float)]
+
+
+class LatentLayer(ctypes.Structure):    # AriaLatentLayer
+    _fields_ = [("mix", LatentShape)] + [(n, DyTParams) for n in ("norm1b", "norm2", "norm2b", "next")] + \
+               [(n, c_void_p) for n in ("w_in", "w_uk", "w_uv", "w_o", "kv_norm", "rope", "cache")] + \
+               [(n, c_int64) for n in ("mlp", "ff", "E", "groups", "keep", "k")] + \
+               [(n, c_void_p) for n in ("w_gate", "w_up", "w_down", "w_router", "correction")]
+
+
+class LatentStack(ctypes.Structure):    # AriaLatentStack
+    _fields_ = [("n_layers", c_int64), ("D", c_int64), ("V", c_int64), ("first", DyTParams), ("embed", c_void_p), ("head", c_void_p)]
+
+
+ABI_VERSION = 4   # include/aria_hip.h ARIA_ABI_VERSION this host code was written against
 
 
 class AriaHipError(RuntimeError):

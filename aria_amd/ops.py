@@ -986,6 +986,161 @@ def decode_attention(qkv: torch.Tensor, freqs_cis: torch.Tensor, pos: torch.Tens
     return out
 
 
+# ----------------------------------------------------------------------------- latent attention, dynamic-tanh stream, group-limited routing
+# Every op below exists in two forms, chosen by the activations' dtype: bf16 (matrix pipe, fp32 accumulation) and float32 (vector ALU throughout).
+def _f32(t: torch.Tensor) -> int:
+    if t.dtype not in (bf16, torch.float32):
+        raise TypeError(f"expected bf16 or float32, got {t.dtype}")
+    return int(t.dtype == torch.float32)
+
+
+def linear_any(a: torch.Tensor, w: torch.Tensor, out_dtype=None) -> torch.Tensor:
+    """a [M, K] w^T for a weight [N, K] of the same dtype: the MFMA GEMM for bf16, the 32-bit kernel for float32."""
+    if not _f32(a):
+        return gemm(a, w, out_dtype=out_dtype or bf16)
+    _chk(w, torch.float32, "w")
+    M, K = a.shape
+    out = torch.empty((M, w.shape[0]), dtype=torch.float32, device=a.device)
+    if w.shape[1] != K:
+        raise ValueError("linear_any: reduction sizes differ")
+    hip.get_lib().call("aria_gemm_f32", _p(a), _p(w), _p(out), M, w.shape[0], K, _rowmajor_2d(a, "a"), _rowmajor_2d(w, "w"), w.shape[0], None, 0, 0,
+                       _stream(a))
+    return out
+
+
+def grouped_linear_any(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor) -> torch.Tensor:
+    """Rows grouped by expert times w[e]^T, w [E, N, K]."""
+    if not _f32(a):
+        return grouped_gemm(a, w, offsets, w_is_kn=False)
+    _chk(w, torch.float32, "w"), _chk(offsets, torch.int32, "offsets")
+    M, K = a.shape
+    E, N, Kw = w.shape
+    if Kw != K or not w.is_contiguous() or offsets.numel() != E + 1:
+        raise ValueError("grouped_linear_any: w must be a contiguous [E, N, K] tensor, offsets [E + 1]")
+    out = torch.empty((M, N), dtype=torch.float32, device=a.device)
+    hip.get_lib().call("aria_gemm_f32", _p(a), _p(w), _p(out), M, N, K, _rowmajor_2d(a, "a"), K, N, _p(offsets), E, N * K, _stream(a))
+    return out
+
+
+def permute_any(x: torch.Tensor, rows_src: torch.Tensor, k: int) -> torch.Tensor:
+    """``moe_permute`` on rows of either width (a float32 row moves as twice as many 16-bit words)."""
+    if not _f32(x):
+        return moe_permute(x, rows_src, k)
+    return moe_permute(x.view(bf16), rows_src, k).view(torch.float32)
+
+
+def act_rows(u: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """relu(u)^2, or silu(gate) u."""
+    assert u.is_contiguous() and (gate is None or (gate.is_contiguous() and gate.shape == u.shape and gate.dtype == u.dtype))
+    out = torch.empty_like(u)
+    hip.get_lib().call("aria_act_rows", _p(gate), _p(u), _p(out), u.shape[0], u.shape[1], u.shape[1], u.shape[1], _f32(u), _stream(u))
+    return out
+
+
+def dyt_stream(x: torch.Tensor, post, nxt, *, ids: Optional[torch.Tensor] = None, table: Optional[torch.Tensor] = None,
+               y: Optional[torch.Tensor] = None, inv: Optional[torch.Tensor] = None, weights: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """One pass over the residual stream x [T, D] fp32 (in place): x = table[ids], or x += post(y), or x += post(weighted sum of a token's expert
+    rows y[inv]); -> next(x), or None without ``nxt``.  post / nxt: hip.DyTParams (their tensors are kept alive by the caller)."""
+    import ctypes
+
+    _chk(x, torch.float32, "x")
+    T, D = x.shape
+    assert x.is_contiguous()
+    src = table if ids is not None else y
+    h = torch.empty((T, D), dtype=src.dtype, device=x.device) if nxt is not None else None
+    if ids is not None:
+        _chk(ids, torch.int32, "ids")
+        assert ids.is_contiguous() and ids.numel() == T and table.is_contiguous() and table.shape[1] == D
+    elif inv is not None:
+        _chk(inv, torch.int32, "inv"), _chk(weights, torch.float32, "weights")
+        assert inv.is_contiguous() and weights.is_contiguous() and weights.shape[0] == T and inv.numel() == weights.numel() == y.shape[0]
+    else:
+        assert y.shape[0] == T
+    if ids is None:
+        assert y.shape[1] == D
+    none = hip.DyTParams(0.0, None, None)
+    hip.get_lib().call("aria_dyt_stream", _p(ids), _p(table) if ids is not None else None, _p(y), _p(inv), _p(weights),
+                       weights.shape[1] if inv is not None else 0, ctypes.byref(post if post is not None else none), _p(x),
+                       ctypes.byref(nxt if nxt is not None else none), _p(h), T, D, _rowmajor_2d(y, "y") if ids is None else 0, _f32(src), _stream(x))
+    return h
+
+
+def moe_route_groups(logits: torch.Tensor, correction: torch.Tensor, groups: int, keep: int, k: int):
+    """Group-limited top-k routing: logits fp32 [T, >= E] (leading dimension = its columns), correction fp32 [E] -> (weights fp32 [T, k], indices
+    int32 [T, k], counts int32 [E])."""
+    _chk(logits, torch.float32, "logits"), _chk(correction, torch.float32, "correction")
+    T, E = logits.shape[0], correction.numel()
+    dev = logits.device
+    weights = torch.empty((T, k), dtype=torch.float32, device=dev)
+    idx = torch.empty((T, k), dtype=torch.int32, device=dev)
+    counts = torch.empty((E,), dtype=torch.int32, device=dev)
+    hip.get_lib().call("aria_moe_route_groups", _p(logits), _p(correction), _p(weights), _p(idx), _p(counts), T, E, _rowmajor_2d(logits, "logits"), groups,
+                       keep, k, _stream(logits))
+    return weights, idx, counts
+
+
+VARLEN_HEADS = ((64, 64), (128, 128), (192, 128), (256, 256))   # (query, value) head columns of aria_attn_varlen_fwd
+
+
+def varlen_head(qd: int, vd: int) -> Optional[Tuple[int, int]]:
+    """The smallest padded head pair of ``attention_varlen`` that holds (qd, vd), or None."""
+    return next(((a, b) for a, b in VARLEN_HEADS if a >= qd and b >= vd), None)
+
+
+def attention_varlen(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu: torch.Tensor, S_max: int, H: int, qd: int, vd: int, scale: float,
+                     gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Causal attention of packed sequences (sequence b = rows cu[b] .. cu[b + 1)): q, k [T, >= H qd], v [T, >= H vd] views, gate [T, >= H] logits of
+    a per-head sigmoid gate -> [T, H vd]."""
+    for t, n in ((q, "q"), (k, "k"), (v, "v")):
+        _chk(t, name=n)
+    _chk(cu, torch.int32, "cu")
+    out = torch.empty((q.shape[0], H * vd), dtype=bf16, device=q.device)
+    hip.get_lib().call("aria_attn_varlen_fwd", _p(q), _p(k), _p(v), _p(out), _p(cu), _p(gate), cu.numel() - 1, S_max, H, qd, vd, _rowmajor_2d(q, "q"),
+                       _rowmajor_2d(k, "k"), _rowmajor_2d(v, "v"), H * vd, _rowmajor_2d(gate, "gate") if gate is not None else 0, float(scale), _stream(q))
+    return out
+
+
+def _chk_latent(shape, proj: torch.Tensor, slot: torch.Tensor, pos: torch.Tensor, rope: torch.Tensor, cache: torch.Tensor) -> int:
+    _chk(slot, torch.int32, "slot"), _chk(pos, torch.int32, "pos"), _chk(rope, torch.float32, "rope")
+    T = slot.numel()
+    if pos.numel() != T or (proj is not None and (proj.shape != (T, shape.ldp) or not proj.is_contiguous())):
+        raise ValueError("latent attention: slot / pos / proj rows differ")
+    if cache.shape[1:] != (shape.S_cap, shape.cw) or not cache.is_contiguous() or rope.shape[0] < shape.S_cap or not rope.is_contiguous():
+        raise ValueError("latent attention: the cache or the rotation table does not fit the shape")
+    return T
+
+
+def latent_rows(shape, proj, slot, pos, rope, kv_norm, cache) -> torch.Tensor:
+    """Rotates the queries of ``proj`` in place and writes the latent cache rows; -> the same rows packed [T, cw]."""
+    import ctypes
+
+    T = _chk_latent(shape, proj, slot, pos, rope, cache)
+    packed = torch.empty((T, shape.cw), dtype=proj.dtype, device=proj.device)
+    hip.get_lib().call("aria_latent_rows", _p(proj), ctypes.byref(shape), _p(slot), _p(pos), _p(rope), _p(kv_norm), _p(cache), _p(packed), T, _f32(proj),
+                       _stream(proj))
+    return packed
+
+
+def latent_decode_attention(shape, proj, slot, pos, rope, kv_norm, uk, uv, cache, max_len: int) -> torch.Tensor:
+    """Tokens against their cached latents (absorbed form; their own rows are written first): -> gated head outputs [T, H dvp].  ``max_len`` >= the
+    largest position + 1."""
+    import ctypes
+
+    T = _chk_latent(shape, proj, slot, pos, rope, cache)
+    if max_len > shape.S_cap:
+        raise ValueError(f"{max_len} positions do not fit a cache of {shape.S_cap}")
+    f32, dev, lib, ref = _f32(proj), proj.device, hip.get_lib(), ctypes.byref(shape)
+    qa = torch.empty((T, shape.H, shape.cw), dtype=proj.dtype, device=dev)
+    lib.call("aria_latent_absorb", _p(proj), ref, _p(slot), _p(pos), _p(rope), _p(kv_norm), _p(uk), _p(cache), _p(qa), T, f32, _stream(proj))
+    splits = 1 if f32 else int(lib.cdll.aria_latent_splits(ref, T, max_len))
+    part_o = torch.empty((T, splits, shape.H, shape.R), dtype=torch.float32, device=dev)
+    part_ml = torch.empty((T, splits, shape.H, 2), dtype=torch.float32, device=dev)
+    lib.call("aria_latent_attn", _p(qa), _p(cache), ref, _p(slot), _p(pos), _p(part_o), _p(part_ml), T, splits, f32, _stream(proj))
+    out = torch.empty((T, shape.H * shape.dvp), dtype=proj.dtype, device=dev)
+    lib.call("aria_latent_expand", _p(part_o), _p(part_ml), ref, _p(proj), _p(uv), _p(out), T, splits, f32, _stream(proj))
+    return out
+
+
 # ----------------------------------------------------------------------------- loss
 def cross_entropy(logits: torch.Tensor, labels: torch.Tensor, grad_scale: Optional[float] = None,
                   dlogits: Optional[torch.Tensor] = None, count_in: Optional[torch.Tensor] = None):

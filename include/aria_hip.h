@@ -26,10 +26,10 @@ extern "C" {
 #define ARIA_ERR_UNSUPPORTED 3 /* shape outside what the kernels implement (e.g. > 256 experts) */
 #define ARIA_ERR_LAUNCH 4      /* hipGetLastError() != hipSuccess after the launch */
 
-/* Library / ABI version: bumped whenever an entry point is added or a signature changes (3 = round 5's additions: aria_moe_router_fused,
+/* Library / ABI version: bumped whenever an entry point is added or a signature changes (4 added the latent-attention family; 3: aria_moe_router_fused,
  * aria_attn_bwd_rope, aria_moe_unpermute_res, aria_scale_bf16, aria_gemm_qkv_rope_hf_bf16, the *_lora_* family).  The Python host
  * (aria_amd/hip.py) refuses a library whose version is not the one it was written against. */
-#define ARIA_ABI_VERSION 3
+#define ARIA_ABI_VERSION 4
 int aria_abi_version(void);
 /* Test/diagnostic aid: which GEMM kernel family the calling thread's last aria_*gemm* call dispatched to
  * (1 = 128x128 tile, 2 = 256x256 register-staged, 3 = 256x256 LDS-DMA phase-scheduled; 0 = none yet). */
@@ -339,6 +339,14 @@ int aria_attn_bwd_rope(const void* q, const void* k, const void* v, const void* 
                        int64_t H, int64_t hd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t lddq, int64_t lddk,
                        int64_t lddv, float scale, int causal, const void* rope_cos, const void* rope_sin, int64_t rope_S, void* stream);
 
+/* Causal attention over a batch of sequences of unequal length packed on the token axis (sequence b = rows cu[b] .. cu[b + 1), S_max = the
+ * longest), with query / key heads of qd columns beside value heads of vd columns (zero-padded by the caller to one of 64 / 64, 128 / 128,
+ * 192 / 128, 256 / 256), and -- gate != NULL -- every head's output multiplied by sigmoid(gate[token * ldg + head]) in the epilogue.  The kernel
+ * is aria_attn_fwd's LDS-DMA form on other tile images.  q [T, H, qd], k [T, H, qd], v [T, H, vd] -> o [T, H, vd] as views with row strides ld*. */
+int aria_attn_varlen_fwd(const void* q, const void* k, const void* v, void* o, const int32_t* cu, const void* gate, int64_t B, int64_t S_max,
+                         int64_t H, int64_t qd, int64_t vd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t ldg, float scale,
+                         void* stream);
+
 /* which backward the calling thread's last aria_attn_bwd ran: 2 = padded-tile pair (hd 64 / 72), 5 = role-split dK/dV + dQ v5 (hd 128) */
 int aria_last_attn_bwd_variant(void);
 /* which forward the calling thread's last aria_attn_fwd launched: 3 = attn_fwd3 (hd 128 / 72: software-pipelined score tiles, K / V by
@@ -433,6 +441,91 @@ int aria_decode_attn(const void* qkv, const void* freqs_cis, const int32_t* pos,
 void* aria_decode_graph_create(const void* const* ptrs, const int64_t* dims, float eps);
 int aria_decode_graph_launch(void* graph, void* stream);
 void aria_decode_graph_destroy(void* graph);
+
+/* ------------------------------------------------------------------------------------------------
+ * Latent attention, dynamic-tanh norms, group-limited routing: the mechanisms of the Duguzen design, each with its sizes and constants as
+ * arguments.  `f32` selects the form: 0 = weights and activations bf16 (fp32 accumulation), 1 = everything in 32-bit (no matrix pipe).
+ * The residual stream, norms, routing, rotation angles, scores and softmax are fp32 in both.
+ * ------------------------------------------------------------------------------------------------ */
+typedef struct {
+    float alpha;
+    const float* w; /* [D]; NULL: no norm at this place */
+    const float* b; /* [D] */
+} AriaDyT;
+
+/* One pass over the residual stream x [T, D] fp32 (D % 8 == 0):
+ *   ids != NULL:  x = table[ids[t], :]                                       (table [V, D])
+ *   inv != NULL:  x += post(sum_j weights[t, j] y[inv[t k + j], :])          (y: expert rows, aria_moe_sort's inv; weights fp32 [T, k])
+ *   otherwise  :  x += post(y[t, :])
+ * then, next.w != NULL: h[t, :] = next(x[t, :]).  post / next: tanh(alpha v) w + b. */
+int aria_dyt_stream(const int32_t* ids, const void* table, const void* y, const int32_t* inv, const float* weights, int64_t k, const AriaDyT* post,
+                    float* x, const AriaDyT* next, void* h, int64_t T, int64_t D, int64_t ldy, int f32, void* stream);
+
+/* act[m, n] = relu(u[m, n])^2 (gate == NULL) or silu(gate[m, n]) u[m, n]; rows of n_cols (% 8 == 0), leading dimensions in elements. */
+int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int f32, void* stream);
+
+/* C [M, N] = A [M, K] W^T (W [N, K]) in true 32-bit on the vector ALU.  offsets != NULL: rows offsets[e] .. offsets[e + 1] of A use W + e strideW
+ * (int32 [E + 1] on the device).  K % 4 == 0, 16-byte aligned rows. */
+int aria_gemm_f32(const float* A, const float* W, float* C, int64_t M, int64_t N, int64_t K, int64_t lda, int64_t ldw, int64_t ldc,
+                  const int32_t* offsets, int64_t E, int64_t strideW, void* stream);
+
+/* Group-limited top-k routing: s = sigmoid(logits), choice = s + correction; of the `keep` groups (of `groups` equal groups of neighbours) with the
+ * largest sum of two best choice scores, the k experts with the largest choice scores; weights = s of the chosen, not renormalised.
+ * logits fp32 [T, ldl] -> weights fp32 [T, k], indices int32 [T, k], counts int32 [E].  E <= 256, E % groups == 0, k <= keep E / groups. */
+int aria_moe_route_groups(const float* logits, const float* correction, float* weights, int32_t* indices, int32_t* counts, int64_t T, int64_t E,
+                          int64_t ldl, int64_t groups, int64_t keep, int64_t k, void* stream);
+
+/* Shape of a latent-attention layer's fused input projection and cache.  A row of `proj` holds H query heads of dq columns ([dn unrotated |
+ * dr rotated | pad]), at kv_off the R + dr columns of the key / value down-projection, at g_off the H output-gate logits.  A cache row (cw columns,
+ * cw % 64 == 0) is [latent, RMS-normed (R) | rotated key part (dr) | zeros]; sequence slots are S_cap rows apart.  `rot` of the dr columns turn,
+ * component i with i + rot / 2; rope fp32 [positions, rot / 2, 2] = (cos, sin).  uk [H dn, rp] and uv [H dv, rp] hold the up-projections with
+ * rows padded to rp = R rounded up to 8. */
+typedef struct {
+    int64_t H, dn, dr, dv, R, rot, dq, dvp, cw, rp, ldp, kv_off, g_off, S_cap;
+    float scale, eps;
+} AriaLatentShape;
+
+/* Prefill: rotates the query heads of `proj` in place; normalises the latent, rotates the key part and writes the row both to the cache (row
+ * slot[t] S_cap + pos[t]) and to packed [T, cw] (the operand of the per-head key / value expansion). */
+int aria_latent_rows(void* proj, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, const float* rope, const float* kv_norm, void* cache,
+                     void* packed, int64_t T, int f32, void* stream);
+/* Decode / continuation: the same cache row, and per head the query moved into latent space, qa [T, H, cw] = [q_unrotated W_uk | rotated q | 0]. */
+int aria_latent_absorb(const void* proj, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, const float* rope, const float* kv_norm,
+                       const void* uk, void* cache, void* qa, int64_t T, int f32, void* stream);
+/* softmax(qa . cache row) over cache rows 0 .. pos[t] of slot[t], split over `splits` workgroups per (token, head group): part_o fp32
+ * [T, splits, H, R] unnormalised latent outputs, part_ml fp32 [T, splits, H, 2] (running maximum in log2 units, sum). */
+int aria_latent_attn(const void* qa, const void* cache, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, float* part_o, float* part_ml,
+                     int64_t T, int64_t splits, int f32, void* stream);
+/* Merges the splits, expands through uv and gates: out [T, H, dvp] (columns dv .. dvp are zeros). */
+int aria_latent_expand(const float* part_o, const float* part_ml, const AriaLatentShape* s, const void* proj, const void* uv, void* out, int64_t T,
+                       int64_t splits, int f32, void* stream);
+
+/* A decoder stack of latent-attention layers (bf16), for the one-call decode step. */
+typedef struct {
+    AriaLatentShape mix;
+    AriaDyT norm1b, norm2, norm2b, next; /* next: the following layer's norm1, or the model's final norm */
+    const void *w_in, *w_uk, *w_uv, *w_o; /* [ldp, D], [H dn, rp], [H dv, rp], [D, H dvp] */
+    const float *kv_norm, *rope;
+    void* cache;
+    int64_t mlp; /* 0 none, 1 dense (relu squared), 2 mixture */
+    int64_t ff, E, groups, keep, k;
+    const void *w_gate, *w_up, *w_down, *w_router; /* dense: up [ff, D], down [D, ff]; mixture: gate, up [E, ff, D], down [E, D, ff], router [E, D] */
+    const float* correction;
+} AriaLatentLayer;
+typedef struct {
+    int64_t n_layers, D, V; /* V: rows of the head (padded) */
+    AriaDyT first;          /* norm1 of the first layer */
+    const void *embed, *head;
+} AriaLatentStack;
+/* bytes of scratch aria_latent_decode needs for T rows over at most max_len cache rows */
+int64_t aria_latent_decode_scratch(const AriaLatentStack* stack, const AriaLatentLayer* layers, int64_t T, int64_t max_len);
+/* One step of T single tokens (token ids, cache slots, positions: int32 on the device; max_len >= largest position + 1, known to the host): enqueues
+ * every kernel of every layer, logits fp32 [T, V].  Projections are row-streaming kernels with squared relu, residual and norms in their
+ * epilogues: meant for T up to 16. */
+int aria_latent_decode(const AriaLatentStack* stack, const AriaLatentLayer* layers, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos,
+                       int64_t max_len, float* logits, void* scratch, int64_t scratch_bytes, void* stream);
+/* how many splits aria_latent_decode / a caller of aria_latent_attn should use */
+int64_t aria_latent_splits(const AriaLatentShape* s, int64_t T, int64_t max_len);
 
 #ifdef __cplusplus
 }
