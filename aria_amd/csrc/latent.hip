@@ -13,32 +13,16 @@ namespace {
 using namespace ad;
 typedef AriaLatentShape Shape;
 
-// one cache row: RMS-normed latent | rotated key part | zeros.  One wave; src = the token's down-projection (R + dr columns).
+// column i of a cache row: RMS-normed latent | rotated key part | zeros.  src = the token's down-projection (R + dr columns), r = 1 / rms
 template <class T>
-__device__ __forceinline__ void latent_row(const T* src, const Shape& s, const float* cs, const float* wn, T* row, T* packed, int l) {
-    float ss = 0.f;
-    for (int i = l; i < s.R; i += 64) {
-        const float v = ldf(src + i);
-        ss += v * v;
-    }
-    ss = wave_sum_bcast(ss);
-    const float r = 1.f / sqrtf(ss / float(s.R) + s.eps);
-    const int half = int(s.rot) >> 1;
-    for (int i = l; i < s.cw; i += 64) {
-        float v = 0.f;
-        if (i < s.R) {
-            v = ldf(src + i) * r * wn[i];
-        } else if (i < s.R + s.dr) {
-            const int j = i - int(s.R);
-            v = ldf(src + i);
-            if (j < half)
-                v = v * cs[2 * j] - ldf(src + i + half) * cs[2 * j + 1];
-            else if (j < s.rot)
-                v = v * cs[2 * (j - half)] + ldf(src + i - half) * cs[2 * (j - half) + 1];
-        }
-        stf(row + i, v);
-        if (packed) stf(packed + i, v);
-    }
+__device__ __forceinline__ float latent_column(const T* src, const Shape& s, const float* cs, const float* wn, float r, int i) {
+    if (i < s.R) return ldf(src + i) * r * wn[i];
+    if (i >= s.R + s.dr) return 0.f;
+    const int j = i - int(s.R), half = int(s.rot) >> 1;
+    const float v = ldf(src + i);
+    if (j < half) return v * cs[2 * j] - ldf(src + i + half) * cs[2 * j + 1];
+    if (j < s.rot) return v * cs[2 * (j - half)] + ldf(src + i - half) * cs[2 * (j - half) + 1];
+    return v;
 }
 
 // ---------------------------------------------------------------------------------------------- prefill: rotate q, write the cache
@@ -51,7 +35,19 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(T* proj, Shape s, cons
     T* p = proj + (long long)t * s.ldp;
     const int ps = pos[t];
     const float* cs = rope + (long long)ps * s.rot;
-    latent_row<T>(p + s.kv_off, s, cs, wn, cache + ((long long)slot[t] * s.S_cap + ps) * s.cw, packed + (long long)t * s.cw, l);
+    const T* src = p + s.kv_off;
+    float ss = 0.f;
+    for (int i = l; i < s.R; i += 64) {
+        const float v = ldf(src + i);
+        ss += v * v;
+    }
+    const float r = 1.f / sqrtf(wave_sum_bcast(ss) / float(s.R) + s.eps);
+    T *row = cache + ((long long)slot[t] * s.S_cap + ps) * s.cw, *prow = packed + (long long)t * s.cw;
+    for (int i = l; i < s.cw; i += 64) {
+        const float v = latent_column<T>(src, s, cs, wn, r, i);
+        stf(row + i, v);
+        stf(prow + i, v);
+    }
     const int half = int(s.rot) >> 1;
     for (int i = l; i < s.H * half; i += 64) {
         const int h = i / half, j = i % half;
@@ -63,91 +59,130 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(T* proj, Shape s, cons
 }
 
 // ---------------------------------------------------------------------------------------------- decode: queries into latent space
-// grid (H * RB + 1, token groups): workgroup (h, rb) computes 128 latent columns of head h for NB tokens (16 column groups of 8 x 16 slices of
-// the reduction over dn: every thread has its weights in flight at once); the last workgroup of a token group writes the cache rows and the
-// rotated query parts.
-constexpr int ABS_NB = 4;
+// grid (H * RB + 1, token groups): workgroup (h, rb) computes 128 latent columns of head h for NB tokens -- 16 column groups of 8 x 16 slices of the
+// reduction over dn, a thread's eight weight rows requested before the queries are staged -- and, at rb = 0, the head's rotated query part; the last
+// workgroup of a token group writes the cache rows.
 template <class T>
+struct Pack8 {   // 8 elements in registers as they came from memory
+    u32x4 v[sizeof(T) / 2];
+    __device__ __forceinline__ void load(const T* p) {
+#pragma unroll
+        for (int i = 0; i < int(sizeof(T) / 2); ++i) v[i] = ld16(reinterpret_cast<const char*>(p) + 16 * i);
+    }
+    __device__ __forceinline__ float at(int e) const {
+        if (sizeof(T) == 2) return e & 1 ? bfhi(v[0][e >> 1]) : bflo(v[0][e >> 1]);
+        const uint32_t bits = v[(sizeof(T) / 4) * (e >> 2)][e & 3];   // (a bit_cast of the element itself reads element 0)
+        return __builtin_bit_cast(float, bits);
+    }
+};
+template <class T, int NB>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(const T* proj, Shape s, const int32_t* slot, const int32_t* pos, const float* rope,
                                                             const float* wn, const T* uk, T* cache, T* qa, int n_tok) {
-    ARIA_SMEM_STATIC float red[16][ABS_NB][128];
+    ARIA_DYN_SMEM(smem);
+    float* red = reinterpret_cast<float*>(smem);   // [16][NB][128]
+    float* sq = red + 16 * NB * 128;               // [NB][dn]
     const int t = threadIdx.x, l = t & 63, w = t >> 6;
-    const int RB = int(s.R + 127) / 128, unit = blockIdx.x, t0 = blockIdx.y * ABS_NB;
-    const int nb = min(ABS_NB, n_tok - t0);
-    if (unit == s.H * RB) {
-        const int half = int(s.rot) >> 1, extra = int(s.cw - s.R);
-        for (int b = w; b < nb; b += 4) {
+    const int RB = int(s.R + 127) / 128, unit = blockIdx.x, t0 = blockIdx.y * NB;
+    const int nb = min(NB, n_tok - t0), half = int(s.rot) >> 1;
+    if (unit == s.H * RB) {   // cache rows: the whole workgroup on one token at a time
+        for (int b = 0; b < nb; ++b) {
             const int tok = t0 + b, ps = pos[tok];
-            const T* p = proj + (long long)tok * s.ldp;
-            const float* cs = rope + (long long)ps * s.rot;
-            latent_row<T>(p + s.kv_off, s, cs, wn, cache + ((long long)slot[tok] * s.S_cap + ps) * s.cw, static_cast<T*>(nullptr), l);
-            for (int i = l; i < s.H * extra; i += 64) {
-                const int h = i / extra, j = i % extra;
-                const T* a = p + (long long)h * s.dq + s.dn + j;
-                float v = 0.f;
-                if (j < s.dr) {
-                    v = ldf(a);
-                    if (j < half)
-                        v = v * cs[2 * j] - ldf(a + half) * cs[2 * j + 1];
-                    else if (j < s.rot)
-                        v = v * cs[2 * (j - half)] + ldf(a - half) * cs[2 * (j - half) + 1];
-                }
-                stf(qa + ((long long)tok * s.H + h) * s.cw + s.R + j, v);
+            const T* src = proj + (long long)tok * s.ldp + s.kv_off;
+            float ss = 0.f;
+            for (int i = t; i < s.R; i += 256) {
+                const float v = ldf(src + i);
+                ss += v * v;
             }
+            ss = wave_sum_bcast(ss);
+            sync();
+            if (l == 0) red[w] = ss;
+            sync();
+            const float r = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / float(s.R) + s.eps);
+            T* row = cache + ((long long)slot[tok] * s.S_cap + ps) * s.cw;
+            for (int i = t; i < s.cw; i += 256) stf(row + i, latent_column<T>(src, s, rope + (long long)ps * s.rot, wn, r, i));
         }
         return;
     }
     const int h = unit / RB, r0 = (unit % RB) * 128, cg = t & 15, g = t >> 4;
-    const int col = r0 + cg * 8;
-    float acc[ABS_NB][8];
+    const int col = r0 + cg * 8, dn = int(s.dn);
+    const T* wp = uk + (long long)h * dn * s.rp + (col < s.rp ? col : 0);
+    float acc[NB][8];
 #pragma unroll
-    for (int b = 0; b < ABS_NB; ++b)
+    for (int b = 0; b < NB; ++b)
 #pragma unroll
         for (int e = 0; e < 8; ++e) acc[b][e] = 0.f;
-    if (col < s.rp) {
-        const T* wp = uk + (long long)h * s.dn * s.rp + col;
-        const T* qp = proj + (long long)t0 * s.ldp + (long long)h * s.dq;
-#pragma unroll 8
-        for (int d = g; d < s.dn; d += 16) {
-            float wv[8];
-            ld8(wp + (long long)d * s.rp, wv);
+    for (int d0 = 0; d0 < dn; d0 += 128) {
+        Pack8<T> wv[8];
 #pragma unroll
-            for (int b = 0; b < ABS_NB; ++b) {
-                const float q = ldf(qp + (long long)min(b, nb - 1) * s.ldp + d);
+        for (int i = 0; i < 8; ++i) wv[i].load(wp + (long long)min(d0 + 16 * i + g, dn - 1) * s.rp);
+        if (d0 == 0) {
+            for (int i = t; i < NB * dn; i += 256) {
+                const int b = i / dn;
+                sq[i] = ldf(proj + (long long)(t0 + min(b, nb - 1)) * s.ldp + (long long)h * s.dq + i % dn);
+            }
+            sync();
+        }
 #pragma unroll
-                for (int e = 0; e < 8; ++e) acc[b][e] += q * wv[e];
+        for (int i = 0; i < 8; ++i) {
+            const int d = d0 + 16 * i + g;
+#pragma unroll
+            for (int b = 0; b < NB; ++b) {
+                const float q = d < dn ? sq[b * dn + d] : 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) acc[b][e] += q * wv[i].at(e);
             }
         }
     }
 #pragma unroll
-    for (int b = 0; b < ABS_NB; ++b)
+    for (int b = 0; b < NB; ++b)
 #pragma unroll
-        for (int e = 0; e < 8; ++e) red[g][b][cg * 8 + e] = acc[b][e];
+        for (int e = 0; e < 8; ++e) red[(g * NB + b) * 128 + cg * 8 + e] = acc[b][e];
     sync();
     for (int i = t; i < nb * 128; i += 256) {
         const int b = i >> 7, c = i & 127;
         if (r0 + c >= s.R) continue;
         float v = 0.f;
 #pragma unroll
-        for (int j = 0; j < 16; ++j) v += red[j][b][c];
+        for (int j = 0; j < 16; ++j) v += red[(j * NB + b) * 128 + c];
         stf(qa + ((long long)(t0 + b) * s.H + h) * s.cw + r0 + c, v);
+    }
+    if (r0 == 0) {   // the head's rotated part, zeros behind it
+        const int extra = int(s.cw - s.R);
+        for (int i = t; i < nb * extra; i += 256) {
+            const int b = i / extra, j = i % extra, tok = t0 + b;
+            const T* a = proj + (long long)tok * s.ldp + (long long)h * s.dq + s.dn + j;
+            const float* cs = rope + (long long)pos[tok] * s.rot;
+            float v = 0.f;
+            if (j < s.dr) {
+                v = ldf(a);
+                if (j < half)
+                    v = v * cs[2 * j] - ldf(a + half) * cs[2 * j + 1];
+                else if (j < s.rot)
+                    v = v * cs[2 * (j - half)] + ldf(a - half) * cs[2 * (j - half) + 1];
+            }
+            stf(qa + ((long long)tok * s.H + h) * s.cw + s.R + j, v);
+        }
     }
 }
 
 // ---------------------------------------------------------------------------------------------- decode attention, matrix pipe (bf16)
-// One workgroup: one token, NG groups of 16 heads, a contiguous range of 64-row cache tiles.  Tiles arrive by LDS-DMA, double-buffered, chunk
-// slot = chunk ^ (row & 7).  Wave w scores rows 16 w .. 16 w + 15 of a tile against all heads (cache rows are k-contiguous B fragments as they
-// lie); the row maxima and the probabilities (bf16) meet in LDS; wave w then accumulates DTW 16-column slices of the latent output for all
-// 64 rows (V fragments by transposing reads of the same tile).  Online softmax in the log2 domain, fp32.
+// One workgroup of 8 waves: one token, NG groups of 16 heads, a contiguous range of 64-row cache tiles.  Tiles arrive by LDS-DMA, double-buffered,
+// chunk slot = chunk ^ (row & 7).  Per tile: wave w scores rows 16 (w & 3) .. against head group w >> 2 (NG = 1: against the half of the reduction
+// w >> 2; cache rows are k-contiguous B fragments as they lie) and parks the scores in LDS; wave w then owns the softmax of 2 NG heads, a lane per
+// row (DPP reductions, running maximum and sum in registers), and publishes probabilities (bf16) and rescale factors; last, wave w accumulates DTW
+// 16-column slices of the latent output over all 64 rows (V fragments by transposing reads of the same tile).  Softmax in the log2 domain, fp32.
 template <int NG, int DTW, int KTM>
-__global__ __launch_bounds__(256) void latent_attn_kernel(const bf16_t* qa, const bf16_t* cache, Shape s, const int32_t* slot, const int32_t* pos,
+__global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, const bf16_t* cache, Shape s, const int32_t* slot, const int32_t* pos,
                                                           float* part_o, float* part_ml, int splits) {
     ARIA_DYN_SMEM(smem);
-    constexpr int PP = 72;   // pitch of the probability tile (elements)
+    constexpr int PP = 72, SPI = 66;   // pitches of the probability tile (bf16) and of the score tile (fp32)
+    constexpr int NP = NG == 1 ? 2 : 1;   // partial score tiles (halves of the reduction)
+    constexpr int KW = (KTM + NP - 1) / NP, HW = 2 * NG;
     const int t = threadIdx.x, l = t & 63, w = first_lane(t >> 6), q4 = l >> 4, c16 = l & 15;
     const int CPR = int(s.cw) >> 3, KT = int(s.cw) >> 5, tile_bytes = 64 * int(s.cw) * 2;
-    bf16_t* sP = reinterpret_cast<bf16_t*>(smem + 2 * tile_bytes);                    // [NG * 16][PP]
-    float* sMax = reinterpret_cast<float*>(smem + 2 * tile_bytes + NG * 16 * PP * 2); // [4][NG * 16]
+    float* sS = reinterpret_cast<float*>(smem + 2 * tile_bytes);                 // [NP][NG * 16][SPI]
+    bf16_t* sP = reinterpret_cast<bf16_t*>(sS + NP * NG * 16 * SPI);             // [NG * 16][PP]
+    float* sA = reinterpret_cast<float*>(sP + NG * 16 * PP);                     // [NG * 16]
     const int sp = blockIdx.x, hg = blockIdx.y, tok = blockIdx.z;
     const int n_keys = pos[tok] + 1, ntiles = (n_keys + 63) / 64, per = (ntiles + splits - 1) / splits;
     const int it0 = sp * per, it1 = min(ntiles, it0 + per);
@@ -161,11 +196,11 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const bf16_t* qa, cons
         return;
     }
     const bf16_t* base = cache + (long long)slot[tok] * s.S_cap * s.cw;
-    // this lane's chunk of the wave's first DMA piece, and the step to its next one (4 pieces of 64 chunks further on)
-    const int row_i = (w * 64 + l) / CPR, slot_i = (w * 64 + l) % CPR, dr_ = 256 / CPR, ds_ = 256 % CPR;
+    // this lane's chunk of the wave's first DMA piece, and the step to its next one (8 pieces of 64 chunks further on)
+    const int row_i = (w * 64 + l) / CPR, slot_i = (w * 64 + l) % CPR, dr_ = 512 / CPR, ds_ = 512 % CPR;
     auto dma = [&](int tile, char* dst) __attribute__((always_inline)) {
         int row = row_i, sl = slot_i;
-        for (int pc = w; pc < CPR; pc += 4) {
+        for (int pc = w; pc < CPR; pc += 8) {
             const int ch = sl ^ (row & 7);
             glds16_raw(base + (long long)min(tile * 64 + row, n_keys - 1) * s.cw + ch * 8, dst + pc * 1024);
             row += dr_;
@@ -177,87 +212,78 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const bf16_t* qa, cons
         }
     };
     dma(it0, smem);
-    s16x8 qf[NG][KTM];
+    const int g = NG == 1 ? 0 : w >> 2, k_first = NG == 1 ? (w >> 2) * KW : 0, krow = 16 * (w & 3) + c16;
+    s16x8 qf[KW];
 #pragma unroll
-    for (int g = 0; g < NG; ++g)
-#pragma unroll
-        for (int kk = 0; kk < KTM; ++kk) {
-            u32x4 v = zero16();
-            const int head = head0 + g * 16 + c16;
-            if (head < s.H && kk < KT) v = ld16(qa + ((long long)tok * s.H + head) * s.cw + kk * 32 + q4 * 8);
-            qf[g][kk] = __builtin_bit_cast(s16x8, v);
-        }
+    for (int kk = 0; kk < KW; ++kk) {
+        u32x4 v = zero16();
+        const int head = head0 + g * 16 + c16;
+        if (head < s.H && k_first + kk < KT) v = ld16(qa + ((long long)tok * s.H + head) * s.cw + (k_first + kk) * 32 + q4 * 8);
+        qf[kk] = __builtin_bit_cast(s16x8, v);
+    }
     f32x4 o[NG][DTW];
-    float m[NG][4], lsum[NG][4];
 #pragma unroll
-    for (int g = 0; g < NG; ++g) {
+    for (int gg = 0; gg < NG; ++gg)
 #pragma unroll
-        for (int i = 0; i < DTW; ++i) o[g][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int i = 0; i < DTW; ++i) o[gg][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m[HW], lsum[HW];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            m[g][r] = -INFINITY;
-            lsum[g][r] = 0.f;
-        }
+    for (int j = 0; j < HW; ++j) {
+        m[j] = -INFINITY;
+        lsum[j] = 0.f;
     }
 #pragma unroll
-    for (int g = 0; g < NG; ++g)
-#pragma unroll
-        for (int kk = 0; kk < KTM; ++kk) settle(qf[g][kk]);
+    for (int kk = 0; kk < KW; ++kk) settle(qf[kk]);
     const float scale2 = s.scale * 1.4426950408889634f;
     for (int it = it0; it < it1; ++it) {
         const char* cur = smem + ((it - it0) & 1) * tile_bytes;
         wait_vm<0>();
-        sync();   // tile `it` is complete; every wave is done with the other buffer, the probabilities and the maxima
+        sync();   // tile `it` is complete; every wave is done with the other buffer and the probabilities
         if (it + 1 < it1) dma(it + 1, smem + ((it - it0 + 1) & 1) * tile_bytes);
-        // scores: C rows = heads 4 q4 + r of a group, columns = cache rows 16 w + c16
-        f32x4 sc[NG];
+        {   // scores: C rows = heads 4 q4 + r of group g, columns = cache rows
+            f32x4 sc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+            const char* kbase = cur + krow * CPR * 16;
 #pragma unroll
-        for (int g = 0; g < NG; ++g) sc[g] = f32x4{0.f, 0.f, 0.f, 0.f};
-        const int krow = 16 * w + c16;
-        const char* kbase = cur + krow * CPR * 16;
+            for (int kk = 0; kk < KW; ++kk)
+                if (k_first + kk < KT) {
+                    const s16x8 kf = *reinterpret_cast<const s16x8*>(kbase + ((((k_first + kk) * 4 + q4) ^ (krow & 7)) << 4));
+                    sc[kk & 1] = mfma16(qf[kk], kf, sc[kk & 1]);
+                }
+            float* dst = sS + ((NG == 1 ? w >> 2 : 0) * NG * 16 + g * 16 + 4 * q4) * SPI + krow;
 #pragma unroll
-        for (int kk = 0; kk < KTM; ++kk)
-            if (kk < KT) {
-                const s16x8 kf = *reinterpret_cast<const s16x8*>(kbase + (((kk * 4 + q4) ^ (krow & 7)) << 4));
-#pragma unroll
-                for (int g = 0; g < NG; ++g) sc[g] = mfma16(qf[g][kk], kf, sc[g]);
-            }
-        const bool dead = it * 64 + krow >= n_keys;
-#pragma unroll
-        for (int g = 0; g < NG; ++g)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                sc[g][r] = dead ? -INFINITY : sc[g][r] * scale2;
-                float mx = sc[g][r];
-#pragma unroll
-                for (int d = 1; d < 16; d <<= 1) mx = fmaxf(mx, shfl_xor(mx, d));
-                if (c16 == 0) sMax[w * NG * 16 + g * 16 + 4 * q4 + r] = mx;
-            }
+            for (int r = 0; r < 4; ++r) dst[r * SPI] = sc[0][r] + sc[1][r];
+        }
         sync();
+        // softmax: lane = row of the tile
+        const bool dead = it * 64 + l >= n_keys;
 #pragma unroll
-        for (int g = 0; g < NG; ++g) {
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int hr = g * 16 + 4 * q4 + r;
-                float mn = m[g][r];
-#pragma unroll
-                for (int ww = 0; ww < 4; ++ww) mn = fmaxf(mn, sMax[ww * NG * 16 + hr]);   // finite: a tile holds at least one visible row
-                const float alpha = exp2_fast(m[g][r] - mn);
-                const float p = exp2_fast(sc[g][r] - mn);
-                m[g][r] = mn;
-                lsum[g][r] = lsum[g][r] * alpha + p;
-                sP[hr * PP + krow] = f2bf(p);
-#pragma unroll
-                for (int i = 0; i < DTW; ++i) o[g][i][r] *= alpha;
-            }
+        for (int j = 0; j < HW; ++j) {
+            const int hr = w * HW + j;
+            float x = sS[hr * SPI + l];
+            if (NP == 2) x += sS[(NG * 16 + hr) * SPI + l];
+            x = dead ? -INFINITY : x * scale2;
+            const float mn = fmaxf(m[j], wave_max_bcast(x));   // finite: a tile holds at least one visible row
+            const float alpha = exp2_fast(m[j] - mn), p = exp2_fast(x - mn);
+            m[j] = mn;
+            lsum[j] = lsum[j] * alpha + p;
+            sP[hr * PP + l] = f2bf(p);
+            if (l == 0) sA[hr] = alpha;
         }
         sync();
         // latent output: A = probabilities (heads x 32 rows), B = the tile's columns
 #pragma unroll
+        for (int gg = 0; gg < NG; ++gg) {
+            const f32x4 al = *reinterpret_cast<const f32x4*>(sA + gg * 16 + 4 * q4);
+#pragma unroll
+            for (int i = 0; i < DTW; ++i)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[gg][i][r] *= al[r];
+        }
+#pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
             s16x8 pf[NG];
 #pragma unroll
-            for (int g = 0; g < NG; ++g) pf[g] = *reinterpret_cast<const s16x8*>(sP + (g * 16 + c16) * PP + kk * 32 + q4 * 8);
+            for (int gg = 0; gg < NG; ++gg) pf[gg] = *reinterpret_cast<const s16x8*>(sP + (gg * 16 + c16) * PP + kk * 32 + q4 * 8);
             const int vr = kk * 32 + q4 * 8 + (c16 >> 2);
 #pragma unroll
             for (int i = 0; i < DTW; ++i) {
@@ -273,38 +299,31 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const bf16_t* qa, cons
                         vf[4 + e] = a1[e];
                     }
 #pragma unroll
-                    for (int g = 0; g < NG; ++g) o[g][i] = mfma16(pf[g], vf, o[g][i]);
+                    for (int gg = 0; gg < NG; ++gg) o[gg][i] = mfma16(pf[gg], vf, o[gg][i]);
                 }
             }
         }
     }
-    // row sums: over the 16 columns a lane group holds, then over the waves
-    sync();
 #pragma unroll
-    for (int g = 0; g < NG; ++g)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const float v = group_sum<16>(lsum[g][r]);
-            if (c16 == 0) sMax[w * NG * 16 + g * 16 + 4 * q4 + r] = v;
+    for (int j = 0; j < HW; ++j) {
+        const float v = wave_sum_bcast(lsum[j]);
+        const int head = head0 + w * HW + j;
+        if (l == 0 && head < s.H) {
+            ml[2 * head] = m[j];
+            ml[2 * head + 1] = v;
         }
-    sync();
+    }
 #pragma unroll
-    for (int g = 0; g < NG; ++g)
+    for (int gg = 0; gg < NG; ++gg)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int hr = g * 16 + 4 * q4 + r, head = head0 + hr;
+            const int head = head0 + gg * 16 + 4 * q4 + r;
             if (head >= s.H) continue;
-            if (w == 0 && c16 == 0) {
-                float v = 0.f;
-                for (int ww = 0; ww < 4; ++ww) v += sMax[ww * NG * 16 + hr];
-                ml[2 * head] = m[g][r];
-                ml[2 * head + 1] = v;
-            }
             float* po = part_o + (((long long)tok * splits + sp) * s.H + head) * s.R;
 #pragma unroll
             for (int i = 0; i < DTW; ++i) {
                 const int d = (w * DTW + i) * 16 + c16;
-                if (d < s.R) po[d] = o[g][i][r];
+                if (d < s.R) po[d] = o[gg][i][r];
             }
         }
 }
@@ -377,15 +396,21 @@ __global__ __launch_bounds__(256) void latent_attn_any_kernel(const T* qa, const
 }
 
 // ---------------------------------------------------------------------------------------------- decode: merge, expand, gate
-constexpr int EXP_ROWS = 32;       // value columns per workgroup
+constexpr int EXP_ROWS = 32;       // value columns per workgroup: 4 per wave
 constexpr int MAX_SPLITS = 64;
 template <class T>
-__global__ __launch_bounds__(256) void latent_expand_kernel(const float* part_o, const float* part_ml, Shape s, const T* proj, const T* uv, T* out,
+__global__ __launch_bounds__(512) void latent_expand_kernel(const float* part_o, const float* part_ml, Shape s, const T* proj, const T* uv, T* out,
                                                             int splits) {
     ARIA_DYN_SMEM(smem);
     float* lat = reinterpret_cast<float*>(smem);   // [rp], zero behind R
     float* wt = lat + s.rp;                        // [MAX_SPLITS]
     const int t = threadIdx.x, l = t & 63, w = t >> 6, h = blockIdx.x, v0 = blockIdx.y * EXP_ROWS, tok = blockIdx.z;
+    const int nch = int(s.rp) >> 3;
+    // the wave's weight rows (their first 512 columns) are requested before the latent is merged
+    Pack8<T> wv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) wv[i].load(uv + ((long long)h * s.dv + min(v0 + w * 4 + i, int(s.dv) - 1)) * s.rp + min(l, nch - 1) * 8);
+    const float gate_logit = ldf(proj + (long long)tok * s.ldp + s.g_off + h);
     if (w == 0) {
         float m = -INFINITY, sum = 0.f;
         if (l < splits) {
@@ -393,42 +418,50 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(const float* part_o,
             m = ml[0];
             sum = ml[1];
         }
-        const float mx = wave_max(m);
+        const float mx = wave_max_bcast(m);
         const float f = sum > 0.f ? exp2f(m - mx) : 0.f;
-        const float tot = wave_sum(sum * f);
+        const float tot = wave_sum_bcast(sum * f);
         if (l < splits) wt[l] = f / tot;
     }
     sync();
-    for (int r = t; r < s.rp; r += 256) {
+    for (int r = t; r < s.rp; r += 512) {
         float v = 0.f;
-        if (r < s.R)
-            for (int j = 0; j < splits; ++j)
-                if (wt[j] != 0.f) v += wt[j] * part_o[(((long long)tok * splits + j) * s.H + h) * s.R + r];
+        if (r < s.R) {
+            const float* p = part_o + (((long long)tok * splits) * s.H + h) * s.R + r;
+            const long long step = s.H * s.R;
+            for (int j = 0; j < splits; j += 8) {   // (a split without rows left its slab unwritten: selected away, not multiplied)
+                float x[8];
+#pragma unroll
+                for (int u = 0; u < 8; ++u) x[u] = p[min(j + u, splits - 1) * step];
+#pragma unroll
+                for (int u = 0; u < 8; ++u) {
+                    const float f = j + u < splits ? wt[min(j + u, splits - 1)] : 0.f;
+                    v += f != 0.f ? f * x[u] : 0.f;
+                }
+            }
+        }
         lat[r] = v;
     }
     sync();
-    const float gate = sigmoid_exact(ldf(proj + (long long)tok * s.ldp + s.g_off + h));
+    const float gate = sigmoid_exact(gate_logit);
     T* orow = out + ((long long)tok * s.H + h) * s.dvp;
-    const int nch = int(s.rp) >> 3;
-    float acc[EXP_ROWS / 4];
+    float acc[4];
 #pragma unroll
-    for (int i = 0; i < EXP_ROWS / 4; ++i) acc[i] = 0.f;
+    for (int i = 0; i < 4; ++i) acc[i] = 0.f;
     for (int c = l; c < nch; c += 64) {
         float lv[8];
         ld8(lat + c * 8, lv);
 #pragma unroll
-        for (int i = 0; i < EXP_ROWS / 4; ++i) {
-            const int v = min(v0 + w + 4 * i, int(s.dv) - 1);
-            float wv[8];
-            ld8(uv + ((long long)h * s.dv + v) * s.rp + c * 8, wv);
+        for (int i = 0; i < 4; ++i) {
+            if (c != l) wv[i].load(uv + ((long long)h * s.dv + min(v0 + w * 4 + i, int(s.dv) - 1)) * s.rp + c * 8);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) acc[i] += wv[e] * lv[e];
+            for (int e = 0; e < 8; ++e) acc[i] += wv[i].at(e) * lv[e];
         }
     }
 #pragma unroll
-    for (int i = 0; i < EXP_ROWS / 4; ++i) {
+    for (int i = 0; i < 4; ++i) {
         const float v = wave_sum_bcast(acc[i]);
-        const int col = v0 + w + 4 * i;
+        const int col = v0 + w * 4 + i;
         if (l == 0 && col < s.dvp) stf(orow + col, col < s.dv ? v * gate : 0.f);
     }
 }
@@ -489,31 +522,63 @@ struct RowsOut {
     float* x;
     bf16_t* h;
 };
-template <int NB, int MODE>
-__global__ __launch_bounds__(256) void rows_kernel(const bf16_t* W, const bf16_t* X, long long ldx, int K, int N, int n_tok, RowsOut ro) {
+template <int MODE>
+__device__ __forceinline__ void rows_finish(const RowsOut& ro, float v, int tok, int n) {
+    const long long at = (long long)tok * ro.ldo + n;
+    if (MODE == ROWS_BF16) static_cast<bf16_t*>(ro.out)[at] = f2bf(v);
+    if (MODE == ROWS_RELU2) static_cast<bf16_t*>(ro.out)[at] = f2bf(relu_squared(v));
+    if (MODE == ROWS_F32) static_cast<float*>(ro.out)[at] = v;
+    if (MODE == ROWS_STREAM) stream_step(v, ro.post, ro.next, ro.x, ro.h, at, n);
+}
+// one token: a wave per two weight rows
+template <int MODE>
+__global__ __launch_bounds__(256) void row_kernel(const bf16_t* W, const bf16_t* X, int K, int N, RowsOut ro) {
     const int l = threadIdx.x & 63, w = threadIdx.x >> 6;
-    const int row0 = (blockIdx.x * 4 + w) * 2, t0 = blockIdx.y * NB;
+    const int row0 = (blockIdx.x * 4 + w) * 2;
     if (row0 >= N) return;
-    const int nb = min(NB, n_tok - t0);
-    float acc[2][NB];
+    float acc[2][1] = {{0.f}, {0.f}};
+    two_rows<1>(acc, W + (long long)row0 * K, W + (long long)min(row0 + 1, N - 1) * K, X, 0, 1, K, l);
+    if (l < 2 && row0 + l < N) rows_finish<MODE>(ro, l ? acc[1][0] : acc[0][0], 0, row0 + l);
+}
+// 2 .. 16 tokens: a workgroup per 16 weight rows, its NW waves on interleaved 128-column blocks of the reduction.  Tokens are the rows of A, weight
+// rows the columns of B: both k-contiguous in memory, so fragments come straight from global memory (every weight byte once), and the matrix pipe
+// takes the multiply-adds of all tokens at the price of one.
+template <int NW, int MODE>
+__global__ __launch_bounds__(NW * 64) void rows_kernel(const bf16_t* W, const bf16_t* X, long long ldx, int K, int N, int n_tok, RowsOut ro) {
+    ARIA_SMEM_STATIC float red[NW][16][17];
+    const int t = threadIdx.x, l = t & 63, w = t >> 6, q4 = l >> 4, c16 = l & 15;
+    const int n0 = blockIdx.x * 16, t0 = blockIdx.y * 16;
+    const bf16_t* wp = W + (long long)min(n0 + c16, N - 1) * K;
+    const bf16_t* xp = X + (long long)min(t0 + c16, n_tok - 1) * ldx;
+    f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+    for (int k0 = w * 128; k0 < K; k0 += 2 * NW * 128) {   // two blocks in flight: eight weight fragments before the first use
+        u32x4 a[8], b[8];
 #pragma unroll
-    for (int r = 0; r < 2; ++r)
+        for (int u = 0; u < 8; ++u) {
+            const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
+            b[u] = ldw16(wp + (k < K ? k : 0));
+        }
 #pragma unroll
-        for (int b = 0; b < NB; ++b) acc[r][b] = 0.f;
-    two_rows<NB>(acc, W + (long long)row0 * K, W + (long long)min(row0 + 1, N - 1) * K, X + (long long)t0 * ldx, ldx, nb, K, l);
-    float mine = 0.f;   // lane r * NB + b finishes element (row0 + r, t0 + b)
+        for (int u = 0; u < 8; ++u) {
+            const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
+            a[u] = ld16(xp + (k < K ? k : 0));
 #pragma unroll
-    for (int r = 0; r < 2; ++r)
+            for (int q = 0; q < 4; ++q) a[u][q] = k < K ? a[u][q] : 0u;
+        }
 #pragma unroll
-        for (int b = 0; b < NB; ++b)
-            if (l == r * NB + b) mine = acc[r][b];
-    const int n = row0 + l / NB, b = l % NB;
-    if (l >= 2 * NB || n >= N || b >= nb) return;
-    const long long at = (long long)(t0 + b) * ro.ldo + n;
-    if (MODE == ROWS_BF16) static_cast<bf16_t*>(ro.out)[at] = f2bf(mine);
-    if (MODE == ROWS_RELU2) static_cast<bf16_t*>(ro.out)[at] = f2bf(relu_squared(mine));
-    if (MODE == ROWS_F32) static_cast<float*>(ro.out)[at] = mine;
-    if (MODE == ROWS_STREAM) stream_step(mine, ro.post, ro.next, ro.x, ro.h, at, n);
+        for (int u = 0; u < 8; ++u) acc[u & 1] = mfma16(__builtin_bit_cast(s16x8, a[u]), __builtin_bit_cast(s16x8, b[u]), acc[u & 1]);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) red[w][4 * q4 + r][c16] = acc[0][r] + acc[1][r];
+    sync();
+    for (int i = t; i < 256; i += NW * 64) {
+        const int tok = i >> 4, n = i & 15;
+        if (t0 + tok >= n_tok || n0 + n >= N) continue;
+        float v = 0.f;
+#pragma unroll
+        for (int ww = 0; ww < NW; ++ww) v += red[ww][tok][n];
+        rows_finish<MODE>(ro, v, t0 + tok, n0 + n);
+    }
 }
 
 // routed up-projection of one (token, slot): act = silu(gate . h) * (up . h); the routing runs in front of the rows, workgroup x = 0 publishes it
@@ -605,13 +670,25 @@ int aria_latent_absorb(const void* proj, const AriaLatentShape* s, const int32_t
     if (const int rc = shape_ok(s)) return rc;
     if (!al16(uk)) return ARIA_ERR_ALIGN;
     if (T == 0) return ARIA_OK;
-    const dim3 grid(unsigned(s->H * ((s->R + 127) / 128) + 1), unsigned((T + ABS_NB - 1) / ABS_NB)), block(256);
-    if (f32)
-        ARIA_LAUNCH((latent_absorb_kernel<float>), grid, block, 0, stream, static_cast<const float*>(proj), *s, slot, pos, rope, kv_norm,
-                    static_cast<const float*>(uk), static_cast<float*>(cache), static_cast<float*>(qa), int(T));
-    else
-        ARIA_LAUNCH((latent_absorb_kernel<bf16_t>), grid, block, 0, stream, static_cast<const bf16_t*>(proj), *s, slot, pos, rope, kv_norm,
-                    static_cast<const bf16_t*>(uk), static_cast<bf16_t*>(cache), static_cast<bf16_t*>(qa), int(T));
+    const int NB = T == 1 ? 1 : 4;
+    const size_t lds = (size_t(16) * NB * 128 + size_t(NB) * s->dn) * 4;
+    if (lds > 160 * 1024) return ARIA_ERR_UNSUPPORTED;
+    const dim3 grid(unsigned(s->H * ((s->R + 127) / 128) + 1), unsigned((T + NB - 1) / NB)), block(256);
+#define ARIA_ABSORB(T_, B_)                                                                                                                          \
+    ARIA_LAUNCH((latent_absorb_kernel<T_, B_>), grid, block, lds, stream, static_cast<const T_*>(proj), *s, slot, pos, rope, kv_norm,                \
+                static_cast<const T_*>(uk), static_cast<T_*>(cache), static_cast<T_*>(qa), int(T))
+    if (f32) {
+        if (NB == 1)
+            ARIA_ABSORB(float, 1);
+        else
+            ARIA_ABSORB(float, 4);
+    } else {
+        if (NB == 1)
+            ARIA_ABSORB(bf16_t, 1);
+        else
+            ARIA_ABSORB(bf16_t, 4);
+    }
+#undef ARIA_ABSORB
     return aria_check_launch();
 }
 
@@ -639,23 +716,23 @@ int aria_latent_attn(const void* qa, const void* cache, const AriaLatentShape* s
     }
     const bf16_t *q = static_cast<const bf16_t*>(qa), *c = static_cast<const bf16_t*>(cache);
     const int NG = s->H <= 16 ? 1 : 2;
-    const dim3 grid(unsigned(splits), unsigned((s->H + 16 * NG - 1) / (16 * NG)), unsigned(T)), block(256);
-    const size_t lds = size_t(2) * 64 * s->cw * 2 + size_t(NG) * 16 * 72 * 2 + size_t(4) * NG * 16 * 4;
+    const dim3 grid(unsigned(splits), unsigned((s->H + 16 * NG - 1) / (16 * NG)), unsigned(T)), block(512);
+    const size_t lds = size_t(2) * 64 * s->cw * 2 + size_t(32) * 66 * 4 + size_t(NG) * 16 * (72 * 2 + 4);
 #define ARIA_LATENT(G, D, K) ARIA_LAUNCH((latent_attn_kernel<G, D, K>), grid, block, lds, stream, q, c, *s, slot, pos, part_o, part_ml, int(splits))
     if (NG == 1) {
         if (cls == 1)
-            ARIA_LATENT(1, 2, 6);
+            ARIA_LATENT(1, 1, 6);
         else if (cls == 2)
-            ARIA_LATENT(1, 4, 10);
+            ARIA_LATENT(1, 2, 10);
         else
-            ARIA_LATENT(1, 8, 18);
+            ARIA_LATENT(1, 4, 18);
     } else {
         if (cls == 1)
-            ARIA_LATENT(2, 2, 6);
+            ARIA_LATENT(2, 1, 6);
         else if (cls == 2)
-            ARIA_LATENT(2, 4, 10);
+            ARIA_LATENT(2, 2, 10);
         else
-            ARIA_LATENT(2, 8, 18);
+            ARIA_LATENT(2, 4, 18);
     }
 #undef ARIA_LATENT
     return aria_check_launch();
@@ -668,7 +745,7 @@ int aria_latent_expand(const float* part_o, const float* part_ml, const AriaLate
     if (!al16(uv)) return ARIA_ERR_ALIGN;
     if (T == 0) return ARIA_OK;
     if (T > 65535 || splits > MAX_SPLITS) return ARIA_ERR_UNSUPPORTED;
-    const dim3 grid(unsigned(s->H), unsigned((s->dvp + EXP_ROWS - 1) / EXP_ROWS), unsigned(T)), block(256);
+    const dim3 grid(unsigned(s->H), unsigned((s->dvp + EXP_ROWS - 1) / EXP_ROWS), unsigned(T)), block(512);
     const size_t lds = size_t(s->rp + MAX_SPLITS) * 4;
     if (f32)
         ARIA_LAUNCH((latent_expand_kernel<float>), grid, block, lds, stream, part_o, part_ml, *s, static_cast<const float*>(proj),
@@ -730,18 +807,14 @@ Scratch layout(const AriaLatentStack& st, const AriaLatentLayer* L, int64_t T, i
 template <int MODE>
 int rows(const void* W, const bf16_t* X, int64_t ldx, int64_t K, int64_t N, int64_t T, const RowsOut& ro, void* stream) {
     const bf16_t* w = static_cast<const bf16_t*>(W);
-    const int nb = T >= 5 ? 8 : T >= 3 ? 4 : int(T);
-    const dim3 grid(unsigned((N + 7) / 8), unsigned((T + nb - 1) / nb)), block(256);
-#define ARIA_ROWS(B) ARIA_LAUNCH((rows_kernel<B, MODE>), grid, block, 0, stream, w, X, (long long)ldx, int(K), int(N), int(T), ro)
-    if (nb == 1)
-        ARIA_ROWS(1);
-    else if (nb == 2)
-        ARIA_ROWS(2);
-    else if (nb == 4)
-        ARIA_ROWS(4);
+    if (T == 1)
+        ARIA_LAUNCH((row_kernel<MODE>), dim3(unsigned((N + 7) / 8)), dim3(256), 0, stream, w, X, int(K), int(N), ro);
+    else if (N <= 16 * 1024)   // few row groups: more waves per group
+        ARIA_LAUNCH((rows_kernel<8, MODE>), dim3(unsigned((N + 15) / 16), unsigned((T + 15) / 16)), dim3(512), 0, stream, w, X, (long long)ldx, int(K), int(N),
+                    int(T), ro);
     else
-        ARIA_ROWS(8);
-#undef ARIA_ROWS
+        ARIA_LAUNCH((rows_kernel<4, MODE>), dim3(unsigned((N + 15) / 16), unsigned((T + 15) / 16)), dim3(256), 0, stream, w, X, (long long)ldx, int(K), int(N),
+                    int(T), ro);
     return aria_check_launch();
 }
 

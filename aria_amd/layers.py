@@ -27,7 +27,7 @@ def up8(n: int) -> int:
 
 def padded(t: torch.Tensor, *shape: int) -> torch.Tensor:
     """``t`` in the corner of a zero tensor of ``shape``."""
-    out = torch.zeros(shape, dtype=t.dtype)
+    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
     out[tuple(slice(0, n) for n in t.shape)] = t
     return out
 
@@ -81,13 +81,13 @@ class LatentAttention(nn.Module):
         ldp = g_off + up8(H)
         self.geometry = dict(H=H, dn=dim, dr=rot_dim, dv=vdim, R=kv_rank, rot=rot_dims, dq=dq, dvp=dvp, cw=cw, rp=rp, ldp=ldp, kv_off=kv_off, g_off=g_off,
                              scale=scale, eps=eps)
-        D = w["q"].shape[1]
-        w_in = torch.zeros((ldp, width), dtype=w["q"].dtype)
+        D, like = w["q"].shape[1], dict(dtype=w["q"].dtype, device=w["q"].device)
+        w_in = torch.zeros((ldp, width), **like)
         w_in[:kv_off].view(H, dq, width)[:, :qd, :D] = w["q"].view(H, qd, D)
         w_in[kv_off:kv_off + kv_rank + rot_dim, :D] = w["dkv"]
         w_in[g_off:g_off + H, :D] = w["g"]
         uk, uv = w["uk"].view(H, dim, kv_rank), w["uv"].view(H, vdim, kv_rank)
-        w_o = torch.zeros((width, H, dvp), dtype=w["o"].dtype)
+        w_o = torch.zeros((width, H, dvp), **like)
         w_o[:w["o"].shape[0], :, :vdim] = w["o"].view(-1, H, vdim)
         self.w_in, self.w_o = _frozen(w_in, dtype), _frozen(w_o.view(width, H * dvp), dtype)
         self.w_uk, self.w_uv = _frozen(padded(uk, H, dim, rp).view(H * dim, rp), dtype), _frozen(padded(uv, H, vdim, rp).view(H * vdim, rp), dtype)
@@ -95,10 +95,10 @@ class LatentAttention(nn.Module):
         self.w_kv: Optional[nn.Parameter] = None
         if self.flash:
             # one cache row -> every head's padded key and value: the rotated part passes through identity rows
-            kv = torch.zeros((H * (dq + dvp), cw), dtype=w["uk"].dtype)
+            kv = torch.zeros((H * (dq + dvp), cw), **like)
             keys, vals = kv[:H * dq].view(H, dq, cw), kv[H * dq:].view(H, dvp, cw)
             keys[:, :dim, :kv_rank], vals[:, :vdim, :kv_rank] = uk, uv
-            keys[:, dim:qd, kv_rank:kv_rank + rot_dim] = torch.eye(rot_dim, dtype=kv.dtype)
+            keys[:, dim:qd, kv_rank:kv_rank + rot_dim] = torch.eye(rot_dim, **like)
             self.w_kv = _frozen(kv, dtype)
 
     def shape(self, S_cap: int) -> hip.LatentShape:
