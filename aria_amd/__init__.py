@@ -6,6 +6,7 @@ _EXPORTS = {
     "AriaConfig": "modeling_aria", "AriaForConditionalGeneration": "modeling_aria",
     "AriaMoELMForCausalLM": "moe_lm", "GroupedGEMM": "moe_lm", "MoEAuxLossAutoScaler": "moe_lm", "AriaMoELMConfig": "moe_lm",
     "AriaProcessor": "processing", "AriaVisionProcessor": "processing",
+    "DuguzenForCausalLM": "duguzen", "DuguzenConfig": "duguzen", "load_model": "registry", "Scheduler": "serving",
     "AriaProjector": "vision", "AriaVisionModel": "vision", "AriaVisionConfig": "vision",
 }
 __all__ = sorted(_EXPORTS)

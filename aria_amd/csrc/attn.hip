@@ -1670,7 +1670,7 @@ int aria_attn_varlen_fwd(const void* q, const void* k, const void* v, void* o, c
     else if (qd == 128)
         ARIA_VARLEN(Fmt128, true);
     else if (qd == 192)
-        ARIA_VARLEN(F192, true);
+        ARIA_VARLEN(F192, false);   // (the pipelined form holds 18 registers too many and spills: 643 against 736 TF/s, 8192 tokens x 20 heads)
     else
         ARIA_VARLEN(F256, false);
 #undef ARIA_VARLEN

@@ -36,6 +36,28 @@ __device__ __forceinline__ void st8(float* p, const float (&v)[8]) {
     *reinterpret_cast<f32x4*>(p + 4) = f32x4{v[4], v[5], v[6], v[7]};
 }
 
+// wave_max_bcast of N values, their DPP ladders in step (one ladder alone is a chain of dependent instructions)
+template <int N>
+__device__ __forceinline__ void wave_max_bcast_n(float (&v)[N]) {
+#ifdef ARIA_EMU
+    for (int j = 0; j < N; ++j) v[j] = wave_max_bcast(v[j]);
+#else
+    const int ninf = int(0xff800000u);
+#define ARIA_DPP_MAXN(ctrl, rows)        \
+    _Pragma("unroll") for (int j = 0; j < N; ++j) v[j] = \
+        fmaxf(v[j], __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(ninf, __builtin_bit_cast(int, v[j]), ctrl, rows, 0xF, false)))
+    ARIA_DPP_MAXN(0x111, 0xF);  // row_shr:1, 2, 4, 8: lane 15 of every row holds the row's maximum
+    ARIA_DPP_MAXN(0x112, 0xF);
+    ARIA_DPP_MAXN(0x114, 0xF);
+    ARIA_DPP_MAXN(0x118, 0xF);
+    ARIA_DPP_MAXN(0x142, 0xA);  // row_bcast:15, 31
+    ARIA_DPP_MAXN(0x143, 0xC);
+#undef ARIA_DPP_MAXN
+#pragma unroll
+    for (int j = 0; j < N; ++j) v[j] = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v[j]), 63));
+#endif
+}
+
 // tanh: the 32-bit form is libm's; beside bfloat16 activations 1 - 2 / (1 + e^2z) on v_exp_f32 + v_rcp_f32 (absolute error ~1e-7)
 template <class T>
 __device__ __forceinline__ float tanh_for(float z);

@@ -167,10 +167,13 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const T* proj, Shape
 
 // ---------------------------------------------------------------------------------------------- decode attention, matrix pipe (bf16)
 // One workgroup of 8 waves: one token, NG groups of 16 heads, a contiguous range of 64-row cache tiles.  Tiles arrive by LDS-DMA, double-buffered,
-// chunk slot = chunk ^ (row & 7).  Per tile: wave w scores rows 16 (w & 3) .. against head group w >> 2 (NG = 1: against the half of the reduction
+// chunk slot = chunk ^ tile_swz(row).  Per tile: wave w scores rows 16 (w & 3) .. against head group w >> 2 (NG = 1: against the half of the reduction
 // w >> 2; cache rows are k-contiguous B fragments as they lie) and parks the scores in LDS; wave w then owns the softmax of 2 NG heads, a lane per
 // row (DPP reductions, running maximum and sum in registers), and publishes probabilities (bf16) and rescale factors; last, wave w accumulates DTW
 // 16-column slices of the latent output over all 64 rows (V fragments by transposing reads of the same tile).  Softmax in the log2 domain, fp32.
+// XOR of a chunk index inside its group of 8: a row is an odd multiple of 32 banks (or an even one) behind its neighbour, so the 16 rows of a score
+// fragment (8 of either parity) need 8 different values, and the 16 (row, 32-byte) pairs of a transposing read need all four upper-bit values twice
+__device__ __forceinline__ int tile_swz(int row) { return ((((row >> 1) ^ (row >> 3)) & 3) << 1) | ((row >> 3) & 1); }
 template <int NG, int DTW, int KTM>
 __global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, const bf16_t* cache, Shape s, const int32_t* slot, const int32_t* pos,
                                                           float* part_o, float* part_ml, int splits) {
@@ -201,7 +204,7 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, cons
     auto dma = [&](int tile, char* dst) __attribute__((always_inline)) {
         int row = row_i, sl = slot_i;
         for (int pc = w; pc < CPR; pc += 8) {
-            const int ch = sl ^ (row & 7);
+            const int ch = sl ^ tile_swz(row);
             glds16_raw(base + (long long)min(tile * 64 + row, n_keys - 1) * s.cw + ch * 8, dst + pc * 1024);
             row += dr_;
             sl += ds_;
@@ -241,14 +244,29 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, cons
         sync();   // tile `it` is complete; every wave is done with the other buffer and the probabilities
         if (it + 1 < it1) dma(it + 1, smem + ((it - it0 + 1) & 1) * tile_bytes);
         {   // scores: C rows = heads 4 q4 + r of group g, columns = cache rows
+            // (no branch on the row's width: blocks past it read the last chunk against zero query fragments; the next group's fragments are
+            // requested in front of this group's multiply-adds)
+            constexpr int GQ = KW % 3 == 0 ? 3 : 5;
             f32x4 sc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
             const char* kbase = cur + krow * CPR * 16;
+            const int fx = tile_swz(krow);
+            s16x8 kf[2][GQ];
+            auto fetch = [&](int kk, s16x8& f) __attribute__((always_inline)) {
+                f = *reinterpret_cast<const s16x8*>(kbase + ((min((k_first + kk) * 4 + q4, CPR - 1) ^ fx) << 4));
+            };
 #pragma unroll
-            for (int kk = 0; kk < KW; ++kk)
-                if (k_first + kk < KT) {
-                    const s16x8 kf = *reinterpret_cast<const s16x8*>(kbase + ((((k_first + kk) * 4 + q4) ^ (krow & 7)) << 4));
-                    sc[kk & 1] = mfma16(qf[kk], kf, sc[kk & 1]);
+            for (int u = 0; u < GQ; ++u) fetch(u, kf[0][u]);
+#pragma unroll
+            for (int k0 = 0; k0 < KW; k0 += GQ) {
+                if (k0 + GQ < KW) {
+#pragma unroll
+                    for (int u = 0; u < GQ; ++u) fetch(k0 + GQ + u, kf[(k0 / GQ + 1) & 1][u]);
                 }
+                sched_fence();
+#pragma unroll
+                for (int u = 0; u < GQ; ++u) sc[u & 1] = mfma16(qf[k0 + u], kf[(k0 / GQ) & 1][u], sc[u & 1]);
+                sched_fence();
+            }
             float* dst = sS + ((NG == 1 ? w >> 2 : 0) * NG * 16 + g * 16 + 4 * q4) * SPI + krow;
 #pragma unroll
             for (int r = 0; r < 4; ++r) dst[r * SPI] = sc[0][r] + sc[1][r];
@@ -256,18 +274,23 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, cons
         sync();
         // softmax: lane = row of the tile
         const bool dead = it * 64 + l >= n_keys;
+        float x[HW], mx[HW];
 #pragma unroll
         for (int j = 0; j < HW; ++j) {
-            const int hr = w * HW + j;
-            float x = sS[hr * SPI + l];
-            if (NP == 2) x += sS[(NG * 16 + hr) * SPI + l];
-            x = dead ? -INFINITY : x * scale2;
-            const float mn = fmaxf(m[j], wave_max_bcast(x));   // finite: a tile holds at least one visible row
-            const float alpha = exp2_fast(m[j] - mn), p = exp2_fast(x - mn);
+            x[j] = sS[(w * HW + j) * SPI + l];
+            if (NP == 2) x[j] += sS[(NG * 16 + w * HW + j) * SPI + l];
+        }
+#pragma unroll
+        for (int j = 0; j < HW; ++j) mx[j] = x[j] = dead ? -INFINITY : x[j] * scale2;
+        wave_max_bcast_n<HW>(mx);
+#pragma unroll
+        for (int j = 0; j < HW; ++j) {
+            const float mn = fmaxf(m[j], mx[j]);   // finite: a tile holds at least one visible row
+            const float alpha = exp2_fast(m[j] - mn), p = exp2_fast(x[j] - mn);
             m[j] = mn;
             lsum[j] = lsum[j] * alpha + p;
-            sP[hr * PP + l] = f2bf(p);
-            if (l == 0) sA[hr] = alpha;
+            sP[(w * HW + j) * PP + l] = f2bf(p);
+            if (l == 0) sA[w * HW + j] = alpha;
         }
         sync();
         // latent output: A = probabilities (heads x 32 rows), B = the tile's columns
@@ -279,29 +302,34 @@ __global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, cons
 #pragma unroll
                 for (int r = 0; r < 4; ++r) o[gg][i][r] *= al[r];
         }
+        s16x8 pf[2][NG], vf[2][DTW];
+        auto fetch_v = [&](int kk) __attribute__((always_inline)) {
 #pragma unroll
-        for (int kk = 0; kk < 2; ++kk) {
-            s16x8 pf[NG];
-#pragma unroll
-            for (int gg = 0; gg < NG; ++gg) pf[gg] = *reinterpret_cast<const s16x8*>(sP + (gg * 16 + c16) * PP + kk * 32 + q4 * 8);
+            for (int gg = 0; gg < NG; ++gg) pf[kk][gg] = *reinterpret_cast<const s16x8*>(sP + (gg * 16 + c16) * PP + kk * 32 + q4 * 8);
             const int vr = kk * 32 + q4 * 8 + (c16 >> 2);
 #pragma unroll
             for (int i = 0; i < DTW; ++i) {
-                const int d0 = (w * DTW + i) * 16;
-                if (d0 < s.R) {   // (wave-uniform)
-                    const int col = d0 + 4 * (c16 & 3), ch = col >> 3, within = (col & 7) * 2;
-                    const s16x4 a0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + vr * CPR * 16 + ((ch ^ (vr & 7)) << 4) + within));
-                    const s16x4 a1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + (vr + 4) * CPR * 16 + ((ch ^ ((vr + 4) & 7)) << 4) + within));
-                    s16x8 vf;
+                const int d0 = min((w * DTW + i) * 16, int(s.cw) - 16);   // (slices past the row: any columns, their results are dropped)
+                const int col = d0 + 4 * (c16 & 3), ch = col >> 3, within = (col & 7) * 2;
+                const s16x4 a0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + vr * CPR * 16 + ((ch ^ tile_swz(vr)) << 4) + within));
+                const s16x4 a1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + (vr + 4) * CPR * 16 + ((ch ^ tile_swz(vr + 4)) << 4) + within));
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        vf[e] = a0[e];
-                        vf[4 + e] = a1[e];
-                    }
-#pragma unroll
-                    for (int gg = 0; gg < NG; ++gg) o[gg][i] = mfma16(pf[gg], vf, o[gg][i]);
+                for (int e = 0; e < 4; ++e) {
+                    vf[kk][i][e] = a0[e];
+                    vf[kk][i][4 + e] = a1[e];
                 }
             }
+        };
+        fetch_v(0);
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            if (kk == 0) fetch_v(1);
+            sched_fence();
+#pragma unroll
+            for (int i = 0; i < DTW; ++i)
+#pragma unroll
+                for (int gg = 0; gg < NG; ++gg) o[gg][i] = mfma16(pf[kk][gg], vf[kk][i], o[gg][i]);
+            sched_fence();
         }
     }
 #pragma unroll
@@ -429,12 +457,12 @@ __global__ __launch_bounds__(512) void latent_expand_kernel(const float* part_o,
         if (r < s.R) {
             const float* p = part_o + (((long long)tok * splits) * s.H + h) * s.R + r;
             const long long step = s.H * s.R;
-            for (int j = 0; j < splits; j += 8) {   // (a split without rows left its slab unwritten: selected away, not multiplied)
-                float x[8];
+            for (int j = 0; j < splits; j += 16) {   // (a split without rows left its slab unwritten: selected away, not multiplied)
+                float x[16];
 #pragma unroll
-                for (int u = 0; u < 8; ++u) x[u] = p[min(j + u, splits - 1) * step];
+                for (int u = 0; u < 16; ++u) x[u] = p[min(j + u, splits - 1) * step];
 #pragma unroll
-                for (int u = 0; u < 8; ++u) {
+                for (int u = 0; u < 16; ++u) {
                     const float f = j + u < splits ? wt[min(j + u, splits - 1)] : 0.f;
                     v += f != 0.f ? f * x[u] : 0.f;
                 }
@@ -541,8 +569,9 @@ __global__ __launch_bounds__(256) void row_kernel(const bf16_t* W, const bf16_t*
     if (l < 2 && row0 + l < N) rows_finish<MODE>(ro, l ? acc[1][0] : acc[0][0], 0, row0 + l);
 }
 // 2 .. 16 tokens: a workgroup per 16 weight rows, its NW waves on interleaved 128-column blocks of the reduction.  Tokens are the rows of A, weight
-// rows the columns of B: both k-contiguous in memory, so fragments come straight from global memory (every weight byte once), and the matrix pipe
-// takes the multiply-adds of all tokens at the price of one.
+// rows the columns of B: both k-contiguous in memory, so fragments come straight from global memory, and the matrix pipe takes the multiply-adds of all
+// tokens at the price of one.  (Plain loads: a fragment touches half a cache line of 16 rows and the next one the other half, which a non-temporal
+// hint fetches twice -- 157 against 123 us for a 514 MB head at 8 tokens.)
 template <int NW, int MODE>
 __global__ __launch_bounds__(NW * 64) void rows_kernel(const bf16_t* W, const bf16_t* X, long long ldx, int K, int N, int n_tok, RowsOut ro) {
     ARIA_SMEM_STATIC float red[NW][16][17];
@@ -556,7 +585,7 @@ __global__ __launch_bounds__(NW * 64) void rows_kernel(const bf16_t* W, const bf
 #pragma unroll
         for (int u = 0; u < 8; ++u) {
             const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
-            b[u] = ldw16(wp + (k < K ? k : 0));
+            b[u] = ld16(wp + (k < K ? k : 0));
         }
 #pragma unroll
         for (int u = 0; u < 8; ++u) {

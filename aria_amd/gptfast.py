@@ -116,6 +116,12 @@ class KVCache:
         self.k = torch.zeros((max_batch_size, max_seq_length, n_heads * head_dim), dtype=bf16, device=device)
         self.v = torch.zeros_like(self.k)
 
+    def row(self, i: int) -> "KVCache":
+        """sequence slot ``i`` as a one-sequence cache on the same memory"""
+        r = KVCache.__new__(KVCache)
+        r.k, r.v = self.k[i:i + 1], self.v[i:i + 1]
+        return r
+
 
 class Attention(nn.Module):
     def __init__(self, config: ModelArgs):
@@ -329,6 +335,46 @@ class Transformer(nn.Module):
             return ops.gemm(h, self.output.weight).view(B, 1, -1)
         return ops.gemm(h, self.output.weight).view(B, S, -1)
 
+    # ---- the serving protocol (serving.py): sequences of a batch run one after the other, each on its own cache slot with its own decode engine
+    @property
+    def vocab(self) -> int:
+        return self.config.vocab_size
+
+    @property
+    def device(self):
+        return self.output.weight.device
+
+    @torch.no_grad()
+    def step(self, batch) -> torch.Tensor:
+        """Run a ``serving.StepBatch`` -> float32 logits [wanted rows, vocab]."""
+        whole = [b.attention.kv_cache for b in self.layers]
+        key = tuple(c.k.data_ptr() for c in whole)
+        if getattr(self, "_slot_key", None) != key:
+            self._slot_key, self._slot_state = key, {}      # slot -> (per-layer cache rows, decode engine)
+        out, at, engine = [], 0, self._engine
+        ids = batch.ids.long()
+        try:
+            for n, start, slot, want in zip(batch.lengths, batch.starts, batch.slots, batch.wanted_by_sequence()):
+                rows, self._engine = self._slot_state.get(slot) or ([c.row(slot) for c in whole], None)
+                for b, r in zip(self.layers, rows):
+                    b.attention.kv_cache = r
+                toks = ids[at:at + n].view(1, n)
+                at += n
+                if start == 0 and n > 1:
+                    last = list(want) == [n - 1]
+                    logits = self.forward(toks, last_only=last)[0].float()
+                    out.append(logits if last else logits[list(want)])
+                else:
+                    for j in range(n):      # (on a cache: token by token)
+                        logits = self.forward(toks[:, j:j + 1], torch.tensor([start + j], dtype=torch.int32, device=ids.device))
+                        out += [logits[0].float().clone()] * list(want).count(j)
+                self._slot_state[slot] = (rows, self._engine)
+        finally:
+            for b, c in zip(self.layers, whole):
+                b.attention.kv_cache = c
+            self._engine = engine
+        return torch.cat(out) if out else torch.empty((0, self.vocab), dtype=torch.float32, device=ids.device)
+
 
 class DecodeEngine:
     """One-call-per-token decode (aria_decode_token, csrc/decode.hip) for batch 1: builds the pointer / dims tables the C entry point
@@ -467,6 +513,12 @@ class Aria(nn.Module):
 
     def forward(self, idx, input_pos=None, input_embeds=None, last_only=False):
         return self.llm(idx, input_pos, input_embeds, last_only=last_only)
+
+    vocab = property(lambda self: self.llm.vocab)        # text-only serving (serving.py)
+    device = property(lambda self: self.llm.device)
+
+    def step(self, batch):
+        return self.llm.step(batch)
 
 
 # ------------------------------------------------------------------------------------------------- generate.py

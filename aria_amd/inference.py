@@ -2,7 +2,10 @@
 MI355X path: same flags, same four steps (``load_model`` with an optional LoRA adapter, ``prepare_input`` through the chat template and the
 processor, ``inference`` = sample until ``<|im_end|>``, decode).  Differences that follow from the path, not the interface: the checkpoint
 is a local HF directory (no hub access), the adapter is the ``adapter_model.safetensors`` a ``use_peft`` run of ``aria_amd.train`` writes
-and is folded into the base weights (``merge_and_unload``) so generation runs the fused prefill kernels and the native decode engine."""
+and is folded into the base weights (``merge_and_unload``) so generation runs the fused prefill kernels and the native decode engine.
+
+``--prompt_ids 5,17,3`` (repeatable) is the text-only form for any registered architecture (registry.py), also those without a tokenizer: the
+prompts run as one batch through the serving scheduler, one line of new token ids each."""
 from __future__ import annotations
 
 import argparse
@@ -12,14 +15,34 @@ def parse_arguments(argv=None):
     parser = argparse.ArgumentParser(description="Aria inference on MI355X")
     parser.add_argument("--base_model_path", required=True, help="HF checkpoint directory (config.json + safetensors shards)")
     parser.add_argument("--peft_model_path", help="directory with adapter_config.json + adapter_model.safetensors (optional)")
-    parser.add_argument("--tokenizer_path", required=True, help="tokenizer directory")
-    parser.add_argument("--image_path", required=True)
-    parser.add_argument("--prompt", required=True)
+    parser.add_argument("--tokenizer_path", help="tokenizer directory")
+    parser.add_argument("--image_path")
+    parser.add_argument("--prompt")
+    parser.add_argument("--prompt_ids", action="append", help="token ids with commas between them (repeat for a batch): text-only generation, no tokenizer")
+    parser.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="with --prompt_ids")
+    parser.add_argument("--top_k", type=int, default=200, help="with --prompt_ids")
+    parser.add_argument("--stop_token", type=int, help="with --prompt_ids")
     parser.add_argument("--max_image_size", type=int, default=980)
     parser.add_argument("--split_image", action="store_true", default=False)
     parser.add_argument("--max_new_tokens", type=int, default=500)
     parser.add_argument("--temperature", type=float, default=0.9)
-    return parser.parse_args(argv)
+    args = parser.parse_args(argv)
+    if not args.prompt_ids:
+        missing = [n for n in ("tokenizer_path", "image_path", "prompt") if getattr(args, n) is None]
+        if missing:
+            parser.error("the following arguments are required: " + ", ".join("--" + n for n in missing))
+    return args
+
+
+def generate_ids(args, device="cuda"):
+    """The ``--prompt_ids`` form: new token ids of every prompt."""
+    import torch
+
+    from . import registry, serving
+
+    model = registry.serving_model(registry.load_model(args.base_model_path, device, getattr(torch, args.dtype)))
+    prompts = [[int(t) for t in p.split(",")] for p in args.prompt_ids]
+    return serving.generate(model, prompts, args.max_new_tokens, temperature=args.temperature, top_k=args.top_k, stop_token=args.stop_token)
 
 
 def load_model(base_model_path: str, peft_model_path: str = None, device="cuda"):
@@ -57,6 +80,10 @@ def inference(image_path: str, prompt: str, model, processor, max_image_size: in
 
 def main(argv=None):
     args = parse_arguments(argv)
+    if args.prompt_ids:
+        for ids in generate_ids(args):
+            print(",".join(map(str, ids)))
+        return
     from .processing import AriaProcessor
 
     processor = AriaProcessor.from_pretrained(args.base_model_path, tokenizer_path=args.tokenizer_path)   # aria/inference.py:137-139

@@ -11,10 +11,9 @@ import torch
 # architecture name -> (module, class); every class has ``from_pretrained(path, device=..., dtype=...)`` and ``dtypes``, the formats it computes in
 MODELS = {
     "AriaForConditionalGeneration": ("modeling_aria", "AriaForConditionalGeneration"),
-    "AriaMoELMForCausalLM": ("moe_lm", "AriaMoELMForCausalLM"),
     "Duguzen": ("duguzen", "DuguzenForCausalLM"),
 }
-MODEL_TYPES = {"aria": "AriaForConditionalGeneration", "aria_moe_lm": "AriaMoELMForCausalLM"}   # Hugging Face configs without an architecture name
+MODEL_TYPES = {"aria": "AriaForConditionalGeneration"}   # Hugging Face configs without an architecture name
 
 
 def read_config(path: str) -> dict:

@@ -5,9 +5,9 @@ that ends leaves its cache slot to a later batch.  A model serves through three 
 
 * ``setup_caches(slots, max_len)`` -- static caches for that many sequences;
 * ``step(batch) -> float32 [wanted, vocab]`` -- run the batch's tokens from and into the caches, logits at the wanted rows;
-* ``vocab`` -- columns of the logits.
+* ``vocab``, ``device`` -- columns of the logits, where tensors live.
 
-The same ``step`` is what ``generate`` and the trace runner (bin/trace_run) drive."""
+``duguzen.DuguzenForCausalLM`` runs a batch as one; ``gptfast.Transformer`` (Aria) runs its sequences one after the other on the slots' caches.  The same ``step`` is what ``generate`` and the trace runner (bin/trace_run) drive."""
 from __future__ import annotations
 
 from dataclasses import dataclass
@@ -31,6 +31,15 @@ class StepBatch:
     lengths: List[int]
     starts: List[int]
     slots: List[int]
+    rows: Optional[List[int]] = None   # the host's copy of ``wanted``
+
+    def wanted_by_sequence(self) -> List[List[int]]:
+        """per sequence: the wanted places among its own tokens, in order"""
+        out, first = [], 0
+        for n in self.lengths:
+            out.append(list(range(n)) if self.rows is None else [r - first for r in self.rows if first <= r < first + n])
+            first += n
+        return out
 
     @property
     def fresh(self) -> bool:
@@ -71,11 +80,13 @@ class StepBatch:
             return buf[at - n:at]
 
         ids = tokens if on_device else take(T)
-        return cls(ids, take(T), take(T), take(len(slots) + 1), take(len(wanted)) if wanted is not None else None, lengths, list(starts), list(slots))
+        return cls(ids, take(T), take(T), take(len(slots) + 1), take(len(wanted)) if wanted is not None else None, lengths, list(starts), list(slots),
+                   list(wanted) if wanted is not None else None)
 
 
 class Scheduler:
-    """Slots and positions of the live requests of one model."""
+    """Slots and positions of the live requests of one model.  A batch claims the free slots it needs; when there are too few and nothing is running the
+    caches are set up again for it (a larger batch), when something is running that is an error: batches do not grow."""
 
     def __init__(self, model, max_tokens: int):
         self.model, self.max_len = model, int(max_tokens)
