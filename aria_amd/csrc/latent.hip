@@ -724,7 +724,10 @@ int aria_latent_absorb(const void* proj, const AriaLatentShape* s, const int32_t
 int64_t aria_latent_splits(const AriaLatentShape* s, int64_t T, int64_t max_len) {
     if (!s || T <= 0 || !mfma_class(*s)) return 1;
     const int64_t tiles = (max_len + 63) / 64, groups = (s->H + 15) / 16 <= 1 ? 1 : (s->H + 31) / 32;
-    int64_t n = (2 * 256 + T * groups - 1) / (T * groups);   // about two workgroups a CU
+    // one round of workgroups: as many as the 256 CUs hold at a time (a workgroup's LDS is two cache tiles), no more -- a workgroup's start and end cost
+    // as much as two tiles
+    const int64_t per_cu = (2 * 64 * s->cw * 2 + 16 * 1024) * 2 <= 160 * 1024 ? 2 : 1;
+    int64_t n = 256 * per_cu / (T * groups);
     n = n < tiles ? n : tiles;
     n = n < MAX_SPLITS ? n : MAX_SPLITS;
     return n < 1 ? 1 : n;

@@ -47,13 +47,14 @@ class DuguzenConfig:
             mlp = e.get("mlp")
             if mlp is not None and mlp["kind"] not in ("dense", "moe"):
                 raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
-            src = e.get("weights_of")
-            src = i if src is None else int(src)
-            if src != i:
-                if not 0 <= src < len(c["layers"]) or c["layers"][src].get("weights_of") is not None:
-                    raise ValueError(f"layer {i}: weights_of {src} names no layer with tensors")
-                if c["layers"][src]["mixer"] != e["mixer"] or c["layers"][src].get("mlp") != mlp:
-                    raise ValueError(f"layer {i} differs from layer {src}, whose weights it uses")
+            src, seen = i, set()
+            while c["layers"][src].get("weights_of") is not None:      # (a borrowed layer may itself name a borrowed one)
+                seen.add(src)
+                src = int(c["layers"][src]["weights_of"])
+                if src in seen or not 0 <= src < len(c["layers"]):
+                    raise ValueError(f"layer {i}: weights_of leads to no layer with tensors")
+            if c["layers"][src]["mixer"] != e["mixer"] or c["layers"][src].get("mlp") != mlp:
+                raise ValueError(f"layer {i} differs from layer {src}, whose weights it uses")
             layers.append(DuguzenLayerConfig(e["mixer"], mlp, src))
         return cls(int(c["vocab"]), int(c["width"]), float(c["norm"]["eps"]), layers)
 

@@ -68,6 +68,9 @@ def parse():
                     "region with HIP events around every large launch class -> `roofline.worst_large_launch`)")
     ap.add_argument("--no-lora-record", action="store_true", help="skip the `lora_config` sub-record (N = 1 only: recipes/config_lora.yaml's adapter set "
                     "on the same model and micro-batch, three timed steps + the frozen-base forward + input-gradient reference)")
+    ap.add_argument("--design", choices=["duguzen"], help="serving throughput of that design instead of the training workload: prefill and decode at a few "
+                    "real layer sizes (random weights) beside the gptfast decoder at equal width, heads, experts and vocabulary; one GPU, one JSON line; "
+                    "--steps / --warmup count timed / untimed prefills (decode steps: 10 x)")
     ap.add_argument("--ep", action="store_true", help="BASELINE config #5 instead of #3: routed experts sharded over the N ranks (all-to-all "
                                                       "dispatch over xGMI), everything else data-parallel; not what the driver runs")
     args = ap.parse_args()
@@ -585,6 +588,110 @@ def self_launch(args):
     os.execv(sys.executable, cmd)
 
 
+DESIGN_SIZES = {   # width: heads, latent rank, dense ff, experts, top-k, expert ff, (groups, kept), vocabulary
+    2560: (20, 512, 6656, 64, 6, 1664, (8, 4), 100352),
+    1536: (12, 384, 4096, 32, 4, 1024, (4, 2), 64000),
+    1024: (8, 256, 2816, 16, 2, 768, (4, 2), 32000),
+}
+
+
+def duguzen_random(width, layers, dev):
+    """config + random device tensors of a Duguzen stack with ``width``'s sizes: one dense layer, then mixtures (heads 128 + 64 / 128)."""
+    H, R, ff, E, top, ffe, (G, keep), V = DESIGN_SIZES[width]
+    mix = dict(heads=H, dim=128, rot_dim=64, vdim=128, kv_rank=R, scale=192 ** -0.5, rot=dict(base=500000.0, dims=64))
+    moe = dict(kind="moe", expert=dict(ff=ffe), router=dict(experts=E, top=top, groups=dict(count=G, keep=keep)))
+    cfg = dict(architecture="Duguzen", width=width, vocab=V, norm=dict(eps=1e-6),
+               layers=[dict(type="latent_attention", mixer=mix, mlp=dict(kind="dense", ff=ff) if i == 0 else moe) for i in range(layers)])
+    g = torch.Generator(device=dev).manual_seed(0)
+    w = {}
+
+    def t(name, *shape, scale=None):
+        w[name] = torch.empty(shape, dtype=bf16, device=dev).normal_(0.0, scale or shape[-1] ** -0.5, generator=g)
+
+    def norm(name):
+        w[name], w[name + ".b"] = torch.ones(width, dtype=bf16, device=dev), torch.zeros(width, dtype=bf16, device=dev)
+        w[name + ".alpha"] = torch.tensor(0.7)
+
+    t("embed", V, width, scale=1.0), t("head", V, width), norm("final.norm")
+    for i, L in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            norm(p + n)
+        t(p + "mix.q", H * 192, width), t(p + "mix.dkv", R + 64, width), t(p + "mix.uk", H * 128, R), t(p + "mix.uv", H * 128, R)
+        t(p + "mix.g", H, width), t(p + "mix.o", width, H * 128)
+        w[p + "mix.dkv.norm"] = torch.ones(R, dtype=bf16, device=dev)
+        if i == 0:
+            t(p + "mlp.up", ff, width), t(p + "mlp.down", width, ff)
+            continue
+        for e in range(E):
+            t(f"{p}mlp.e{e}.gate", ffe, width), t(f"{p}mlp.e{e}.up", ffe, width), t(f"{p}mlp.e{e}.down", width, ffe)
+        t(p + "mlp.router", E, width)
+        w[p + "mlp.correction"] = torch.zeros(E, dtype=bf16, device=dev)
+    return cfg, w
+
+
+def design_bench(args, dev, json_out):
+    """``--design duguzen``: prefill and decode throughput of Duguzen and of the gptfast (Aria) decoder at equal sizes, both through the serving step
+    (``serving.StepBatch``) on this GPU."""
+    import gc
+
+    from aria_amd import gptfast as G
+    from aria_amd.duguzen import DuguzenForCausalLM
+    from aria_amd.serving import StepBatch
+
+    layers, steps, warmup = min(args.layers, 4), max(1, args.steps), max(1, args.warmup)
+
+    def timed(fn, n, w):
+        for _ in range(w):
+            fn()
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(n):
+            fn()
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t0) / n
+
+    def measure(model, vocab, batches, ctxs):
+        rec = {}
+        for T in (2048, 8192):
+            model.setup_caches(1, T)
+            ids = torch.randint(0, vocab, (T,)).tolist()
+            b = StepBatch.build([ids], [0], [0], [T - 1], dev)
+            s = timed(lambda: model.step(b), steps, warmup)
+            rec[f"prefill_{T}"] = {"ms": round(s * 1e3, 3), "tokens_per_s": round(T / s, 1)}
+        for B in batches:
+            model.setup_caches(B, max(ctxs))
+            for S in ctxs:
+                b = StepBatch.build([[7 + i] for i in range(B)], list(range(B)), [S - 1] * B, list(range(B)), dev)
+                s = timed(lambda: model.step(b), 10 * steps, 2 * warmup)
+                rec[f"decode_b{B}_ctx{S}"] = {"ms": round(s * 1e3, 3), "tokens_per_s": round(B / s, 1)}
+        return rec
+
+    out = {}
+    for width, (H, R, ff, E, top, ffe, groups, V) in DESIGN_SIZES.items():
+        cfg, w = duguzen_random(width, layers, dev)
+        m = DuguzenForCausalLM.from_tensors(cfg, w, dev)
+        del w
+        rec = {"duguzen": measure(m, V, (1, 8, 16), (512, 4096, 16384))}
+        del m
+        gc.collect(), torch.cuda.empty_cache()
+        torch.set_default_device(dev)
+        a = G.Transformer(G.ModelArgs(block_size=16384, vocab_size=V, n_layer=layers, n_head=H, dim=width, intermediate_size=ffe, num_experts=E,
+                                      router_topk=top, num_shared_experts=2))
+        torch.set_default_device("cpu")
+        init_params(a, seed=0)
+        rec["gptfast"] = measure(a.eval(), V, (1, 8), (512, 4096, 16384))
+        del a
+        gc.collect(), torch.cuda.empty_cache()
+        out[f"width_{width}"] = rec
+    head = out["width_2560"]["duguzen"]["prefill_8192"]
+    print(json.dumps({"metric": "Duguzen prefill tokens/s (width 2560, 8192-token prompt)", "value": head["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+                      "steps": steps, "warmup": warmup, "ms_per_step": head["ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+                      "dtype": "bf16", "data": "synthetic",
+                      "config": {"model": f"Duguzen, random weights, {layers} layers (1 dense + mixtures)", "global_batch": 1, "seq_len": 8192,
+                                 "parallelism": "single", "sizes": {str(k): v for k, v in DESIGN_SIZES.items()}}, "records": out}), file=json_out, flush=True)
+
+
 def main():
     args = parse()
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
@@ -602,6 +709,10 @@ def main():
         raise SystemExit("bench.py needs an MI355X: the hot path has no CPU fallback")
     torch.cuda.set_device(local)
     dev = torch.device("cuda", local)
+    if args.design:
+        if world != 1:
+            raise SystemExit("bench.py: --design measures one GPU")
+        return design_bench(args, dev, json_out)
     if world > 1 or args.ep:
         import torch.distributed as dist
 

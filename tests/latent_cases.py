@@ -563,3 +563,8 @@ def case_bad_inputs(dev):
         with pytest.raises(ValueError):
             DuguzenConfig.from_dict(bad)
     assert math.isclose(DuguzenConfig.from_dict(cfg).eps, cfg["norm"]["eps"])
+    one = cfg["layers"][0]
+    chain = DuguzenConfig.from_dict(dict(cfg, layers=[dict(one, weights_of=2), dict(one, weights_of=0), one]))
+    assert [l.source for l in chain.layers] == [2, 2, 2]
+    with pytest.raises(ValueError):
+        DuguzenConfig.from_dict(dict(cfg, layers=[dict(one, weights_of=1), dict(one, weights_of=0)]))
