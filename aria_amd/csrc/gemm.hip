@@ -358,7 +358,8 @@ int aria_gemm_bf16_ws(const void* A, const void* B, void* C, const void* bias, i
 int aria_gemm_act_bf16(const void* A, const void* B, void* C, const void* bias, int64_t M, int64_t N, int64_t K, int a_oc,
                        int b_oc, int64_t lda, int64_t ldb, int64_t ldc, int c_f32, int accumulate, int act, void* workspace,
                        int64_t workspace_bytes, void* stream) {
-    if (act != ARIA_ACT_NONE && act != ARIA_ACT_GELU_TANH) return ARIA_ERR_UNSUPPORTED;
+    if (act != ARIA_ACT_NONE && act != ARIA_ACT_GELU_TANH && act != ARIA_ACT_RELU2) return ARIA_ERR_UNSUPPORTED;
+    if (act == ARIA_ACT_RELU2 && (a_oc || b_oc)) return ARIA_ERR_UNSUPPORTED;   // (built for the forward form only)
     if (!A || !B || !C || M < 0 || N < 0 || K < 0) return ARIA_ERR_INVALID;
     if (M == 0 || N == 0) return ARIA_OK;
     if (!aligned16(A) || !aligned16(B) || (lda & 7) || (ldb & 7) || (N & 1) || (ldc & 1)) return ARIA_ERR_ALIGN;

@@ -1075,6 +1075,8 @@ __global__ __launch_bounds__(512) void gemm3_kernel(GemmParams p) {
         store_tile3_glu(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
     else if (p.act == 1)  // (one wave-uniform branch here instead of one per value inside the unrolled epilogues)
         store_any3<1>(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
+    else if (!A_OC && !B_OC && VER == 3 && p.act == 2)
+        store_any3<2>(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
     else
         store_any3<0>(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
 }

@@ -14,7 +14,7 @@ struct GemmParams {
     int E;
     long long strideB, strideC;
     int c_f32, accumulate;
-    int act;  // epilogue activation applied to the bf16-ROUNDED (acc + bias), before any accumulate: 0 none, 1 gelu_tanh
+    int act;  // epilogue activation applied to the bf16-ROUNDED (acc + bias), before any accumulate: 0 none, 1 gelu_tanh, 2 squared relu
     int ntn, ntm;  // column / row tile counts of the launch (256-wide tiles for v2/v3)
     // v3 remainder split-K (mode 0): tile-list positions >= split_first are each computed by `split` workgroups over disjoint K
     // ranges into fp32 slabs (ws), which a second kernel sums in a fixed order.  split <= 1: off.
@@ -247,20 +247,23 @@ inline int aria_tile_grid(const GemmParams& p) {
 }
 
 // the epilogue value of every GEMM kernel: bias added by the caller; activation exactly as a separate elementwise kernel would see it
-template <class P>
-__device__ __forceinline__ float aria_epilogue_act(const P& p, float v) {
-    return p.act == 1 ? ad::gelu_tanh(ad::rbf(v)) : v;
-}
-// the same with the activation as a compile-time constant: inside an unrolled epilogue the run-time form costs one branch PER VALUE
 template <int ACT>
 __device__ __forceinline__ float aria_epilogue_act_c(float v) {
-    return ACT == 1 ? ad::gelu_tanh(ad::rbf(v)) : v;
+    if (ACT == 0) return v;
+    v = ad::rbf(v);
+    if (ACT == 1) return ad::gelu_tanh(v);
+    v = fmaxf(v, 0.f);
+    return v * v;
 }
-
-// the same on a pair (r06: packed arithmetic in the GELU epilogue of the ViT's fc1)
+template <class P>
+__device__ __forceinline__ float aria_epilogue_act(const P& p, float v) {
+    return p.act == 1 ? aria_epilogue_act_c<1>(v) : p.act == 2 ? aria_epilogue_act_c<2>(v) : v;
+}
+// the compile-time form (inside an unrolled epilogue the run-time form costs one branch PER VALUE) on a pair
 template <int ACT>
 __device__ __forceinline__ ad::f32x2 aria_epilogue_act2(ad::f32x2 v) {
-    return ACT == 1 ? ad::gelu_tanh2(ad::rbf2(v)) : v;
+    if (ACT == 1) return ad::gelu_tanh2(ad::rbf2(v));
+    return ad::f32x2{aria_epilogue_act_c<ACT>(v.x), aria_epilogue_act_c<ACT>(v.y)};
 }
 
 // (internal to the library: hidden, not part of the C ABI)

@@ -132,7 +132,7 @@ class SquaredReluFeedForward(nn.Module):
         self.up, self.down = _frozen(padded(up, self.ff, width), dtype), _frozen(padded(down, width, self.ff), dtype)
 
     def forward(self, h: torch.Tensor):
-        return dict(y=ops.linear_any(ops.act_rows(ops.linear_any(h, self.up)), self.down))
+        return dict(y=ops.linear_any(ops.linear_any(h, self.up, relu_squared=True), self.down))
 
 
 class GroupLimitedMixture(nn.Module):

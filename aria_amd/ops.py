@@ -41,7 +41,7 @@ def _rowmajor_2d(t: torch.Tensor, name="tensor") -> int:
 
 
 # ----------------------------------------------------------------------------- GEMM
-ACTIVATIONS = {None: 0, "gelu_tanh": 1}
+ACTIVATIONS = {None: 0, "gelu_tanh": 1, "relu_squared": 2}
 
 
 def gemm(a: torch.Tensor, b: torch.Tensor, *, a_oc: bool = False, b_oc: bool = False, bias: Optional[torch.Tensor] = None,
@@ -994,10 +994,11 @@ def _f32(t: torch.Tensor) -> int:
     return int(t.dtype == torch.float32)
 
 
-def linear_any(a: torch.Tensor, w: torch.Tensor, out_dtype=None) -> torch.Tensor:
-    """a [M, K] w^T for a weight [N, K] of the same dtype: the MFMA GEMM for bf16, the 32-bit kernel for float32."""
+def linear_any(a: torch.Tensor, w: torch.Tensor, out_dtype=None, relu_squared: bool = False) -> torch.Tensor:
+    """a [M, K] w^T (then max(z, 0)^2) for a weight [N, K] of the same dtype: the MFMA GEMM for bf16 (the activation in its epilogue), the 32-bit
+    kernel for float32."""
     if not _f32(a):
-        return gemm(a, w, out_dtype=out_dtype or bf16)
+        return gemm(a, w, out_dtype=out_dtype or bf16, act="relu_squared" if relu_squared else None)
     _chk(w, torch.float32, "w")
     M, K = a.shape
     out = torch.empty((M, w.shape[0]), dtype=torch.float32, device=a.device)
@@ -1005,7 +1006,7 @@ def linear_any(a: torch.Tensor, w: torch.Tensor, out_dtype=None) -> torch.Tensor
         raise ValueError("linear_any: reduction sizes differ")
     hip.get_lib().call("aria_gemm_f32", _p(a), _p(w), _p(out), M, w.shape[0], K, _rowmajor_2d(a, "a"), _rowmajor_2d(w, "w"), w.shape[0], None, 0, 0,
                        _stream(a))
-    return out
+    return act_rows(out) if relu_squared else out
 
 
 def grouped_linear_any(a: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor) -> torch.Tensor:

@@ -62,6 +62,7 @@ int aria_gemm_bf16_ws(const void* A, const void* B, void* C, const void* bias, i
  * modeling_idefics2.py MLP / ACT2FN).  The activation is applied before `accumulate` adds the old C. */
 #define ARIA_ACT_NONE 0
 #define ARIA_ACT_GELU_TANH 1
+#define ARIA_ACT_RELU2 2 /* max(z, 0)^2; a_oc = b_oc = 0 only */
 int aria_gemm_act_bf16(const void* A, const void* B, void* C, const void* bias, int64_t M, int64_t N, int64_t K, int a_oc,
                        int b_oc, int64_t lda, int64_t ldb, int64_t ldc, int c_f32, int accumulate, int act, void* workspace,
                        int64_t workspace_bytes, void* stream);

@@ -197,6 +197,16 @@ def case_activations(dev, dtype):
     assert rel(ops.act_rows(u.to(dev), gate=g.to(dev)), O.silu(g.double()) * u.double()) < tol
 
 
+def case_gemm_relu_squared(dev, M, N, K):
+    """The activation in the GEMM epilogue equals the GEMM followed by the elementwise pass, bit for bit."""
+    from aria_amd import ops
+
+    a, w = rnd(M, K, seed=3).to(dev), rnd(N, K, seed=4, scale=0.3).to(dev)
+    got = ops.linear_any(a, w, relu_squared=True)
+    assert torch.equal(got, ops.act_rows(ops.gemm(a, w)))
+    assert rel(got, O.relu_squared(a.cpu().double() @ w.cpu().double().T)) < 1e-2
+
+
 def case_gemm_f32(dev, M, N, K):
     from aria_amd import ops
 

@@ -28,6 +28,11 @@ def test_activations(dtype):
     C.case_activations(DEV, dtype)
 
 
+@pytest.mark.parametrize("M,N,K", [(5, 24, 16), (70, 136, 72)])
+def test_gemm_relu_squared(M, N, K):
+    C.case_gemm_relu_squared(DEV, M, N, K)
+
+
 @pytest.mark.parametrize("M,N,K", [(5, 9, 4), (70, 66, 20)])
 def test_gemm_f32(M, N, K):
     C.case_gemm_f32(DEV, M, N, K)

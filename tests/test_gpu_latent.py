@@ -32,6 +32,11 @@ def test_activations(dtype):
     C.case_activations(DEV, dtype)
 
 
+@pytest.mark.parametrize("M,N,K", [(5, 24, 16), (300, 520, 264), (512, 768, 1024), (4096, 3080, 256), (1024, 2560, 4096)])   # every kernel family, split tiles
+def test_gemm_relu_squared(M, N, K):
+    C.case_gemm_relu_squared(DEV, M, N, K)
+
+
 @pytest.mark.parametrize("M,N,K", [(5, 9, 4), (70, 66, 20), (300, 257, 516)])
 def test_gemm_f32(M, N, K):
     C.case_gemm_f32(DEV, M, N, K)
