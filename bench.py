@@ -598,7 +598,7 @@ DESIGN_SIZES = {   # width: heads, latent rank, dense ff, experts, top-k, expert
 def duguzen_random(width, layers, dev):
     """config + random device tensors of a Duguzen stack with ``width``'s sizes: one dense layer, then mixtures (heads 128 + 64 / 128)."""
     H, R, ff, E, top, ffe, (G, keep), V = DESIGN_SIZES[width]
-    mix = dict(heads=H, dim=128, rot_dim=64, vdim=128, kv_rank=R, scale=192 ** -0.5, rot=dict(base=500000.0, dims=64))
+    mix = dict(heads=H, dim=128, rot_dim=64, vdim=128, kv_rank=R, scale=192 ** -0.5, rot=dict(base=10000.0, dims=64))
     moe = dict(kind="moe", expert=dict(ff=ffe), router=dict(experts=E, top=top, groups=dict(count=G, keep=keep)))
     cfg = dict(architecture="Duguzen", width=width, vocab=V, norm=dict(eps=1e-6),
                layers=[dict(type="latent_attention", mixer=mix, mlp=dict(kind="dense", ff=ff) if i == 0 else moe) for i in range(layers)])

@@ -64,7 +64,7 @@ def test_one_key_stands_out(dtype):
     C.case_one_key_stands_out(DEV, dtype, [0, 1, 63, 64, 65], 68)
 
 
-@pytest.mark.parametrize("dtype,name", [(bf16, "odd"), (f32, "odd"), (f32, "mixed")])
+@pytest.mark.parametrize("dtype,name", [(bf16, "odd"), (f32, "odd"), (f32, "mixed"), (bf16, "broad"), (bf16, "vocabulary")])
 def test_model(dtype, name):
     C.case_model(DEV, dtype, name, lens=(4, 1, 2), tail=2)
 

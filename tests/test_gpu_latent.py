@@ -99,8 +99,9 @@ def test_continuation_beside_decode(dtype):
 
 
 @both
-def test_rows_do_not_depend_on_company(dtype):
-    C.case_rows_do_not_depend_on_company(DEV, dtype)
+@pytest.mark.parametrize("name", ["mixed", "vocabulary", "broad"])
+def test_rows_do_not_depend_on_company(dtype, name):
+    C.case_rows_do_not_depend_on_company(DEV, dtype, name)
 
 
 @both
