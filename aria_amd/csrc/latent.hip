@@ -568,12 +568,12 @@ __global__ __launch_bounds__(256) void row_kernel(const bf16_t* W, const bf16_t*
     two_rows<1>(acc, W + (long long)row0 * K, W + (long long)min(row0 + 1, N - 1) * K, X, 0, 1, K, l);
     if (l < 2 && row0 + l < N) rows_finish<MODE>(ro, l ? acc[1][0] : acc[0][0], 0, row0 + l);
 }
-// 2 .. 16 tokens: a workgroup per 16 RG weight rows, its NW waves on interleaved 128-column blocks of the reduction, U blocks in flight.  Tokens are the
+// 2 .. 16 tokens: a workgroup per 16 RG weight rows, its NW waves on interleaved 128-column blocks of the reduction.  Tokens are the
 // rows of A, weight rows the columns of B: both k-contiguous in memory, so fragments come straight from global memory, and the matrix pipe takes the
 // multiply-adds of all tokens at the price of one.  RG = 2 reads the tokens once for 32 weight rows: at 16 tokens they are as many bytes as 16 rows.
 // (Plain loads: a fragment touches half a cache line of 16 rows and the next one the other half, which a non-temporal hint fetches twice -- 157
 // against 123 us for a 514 MB head at 8 tokens.)
-template <int NW, int RG, int U, int MODE>
+template <int NW, int RG, int MODE>
 __global__ __launch_bounds__(NW * 64) void rows_kernel(const bf16_t* W, const bf16_t* X, long long ldx, int K, int N, int n_tok, RowsOut ro) {
     ARIA_SMEM_STATIC float red[NW][16][16 * RG + 1];
     const int t = threadIdx.x, l = t & 63, w = t >> 6, q4 = l >> 4, c16 = l & 15;
@@ -585,24 +585,24 @@ __global__ __launch_bounds__(NW * 64) void rows_kernel(const bf16_t* W, const bf
     f32x4 acc[RG][2];
 #pragma unroll
     for (int g = 0; g < RG; ++g) acc[g][0] = acc[g][1] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k0 = w * 128; k0 < K; k0 += U * NW * 128) {   // every weight fragment of the U blocks before the first use
-        u32x4 a[4 * U], b[RG][4 * U];
+    for (int k0 = w * 128; k0 < K; k0 += 2 * NW * 128) {   // two blocks in flight: every weight fragment before the first use
+        u32x4 a[8], b[RG][8];
 #pragma unroll
         for (int g = 0; g < RG; ++g)
 #pragma unroll
-            for (int u = 0; u < 4 * U; ++u) {
+            for (int u = 0; u < 8; ++u) {
                 const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
                 b[g][u] = ld16(wp[g] + (k < K ? k : 0));
             }
 #pragma unroll
-        for (int u = 0; u < 4 * U; ++u) {
+        for (int u = 0; u < 8; ++u) {
             const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
             a[u] = ld16(xp + (k < K ? k : 0));
 #pragma unroll
             for (int q = 0; q < 4; ++q) a[u][q] = k < K ? a[u][q] : 0u;
         }
 #pragma unroll
-        for (int u = 0; u < 4 * U; ++u)
+        for (int u = 0; u < 8; ++u)
 #pragma unroll
             for (int g = 0; g < RG; ++g) acc[g][u & 1] = mfma16(__builtin_bit_cast(s16x8, a[u]), __builtin_bit_cast(s16x8, b[g][u]), acc[g][u & 1]);
     }
@@ -853,13 +853,10 @@ int rows(const void* W, const bf16_t* X, int64_t ldx, int64_t K, int64_t N, int6
     if (T == 1)
         ARIA_LAUNCH((row_kernel<MODE>), dim3(unsigned((N + 7) / 8)), dim3(256), 0, stream, w, X, int(K), int(N), ro);
     else if (N > 16 * 1024)
-        ARIA_LAUNCH((rows_kernel<4, 2, 2, MODE>), dim3(unsigned((N + 31) / 32), unsigned((T + 15) / 16)), dim3(256), 0, stream, w, X, (long long)ldx, int(K),
+        ARIA_LAUNCH((rows_kernel<4, 2, MODE>), dim3(unsigned((N + 31) / 32), unsigned((T + 15) / 16)), dim3(256), 0, stream, w, X, (long long)ldx, int(K),
                     int(N), int(T), ro);
-    else if (K > 2048 && K <= 3072)   // few row groups: more waves per group, and all of K in one round of requests
-        ARIA_LAUNCH((rows_kernel<8, 1, 3, MODE>), dim3(unsigned((N + 15) / 16), unsigned((T + 15) / 16)), dim3(512), 0, stream, w, X, (long long)ldx, int(K),
-                    int(N), int(T), ro);
-    else
-        ARIA_LAUNCH((rows_kernel<8, 1, 2, MODE>), dim3(unsigned((N + 15) / 16), unsigned((T + 15) / 16)), dim3(512), 0, stream, w, X, (long long)ldx, int(K),
+    else   // few row groups: more waves per group
+        ARIA_LAUNCH((rows_kernel<8, 1, MODE>), dim3(unsigned((N + 15) / 16), unsigned((T + 15) / 16)), dim3(512), 0, stream, w, X, (long long)ldx, int(K),
                     int(N), int(T), ro);
     return aria_check_launch();
 }

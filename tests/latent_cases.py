@@ -108,7 +108,7 @@ CONFIGS = {
     "equal": config([(mixer(heads=4, dim=16, rot_dim=16, vdim=32, kv_rank=32), moe(ff=32, experts=4, top=4, count=4, keep=4))] * 2, width=32, vocab=32),
     # sharp scores: a softmax that is close to one-hot
     "sharp": config([(mixer(heads=2, dim=16, rot_dim=8, vdim=16, kv_rank=32, scale=0.7), dense(ff=40))] * 2, width=40, vocab=64),
-    # a head of more than 16384 rows, and a reduction of 2049 .. 3072: forms of the batched decode projections of their own
+    # a head of more than 16384 rows (the 32-row form of the batched decode projections), and a reduction of several rounds of its waves
     "vocabulary": config([(mixer(heads=2, dim=16, rot_dim=8, vdim=16, kv_rank=32), dense(ff=24))], width=24, vocab=16411),
     "broad": config([(mixer(heads=2, dim=16, rot_dim=8, vdim=16, kv_rank=32), dense(ff=24))], width=2061, vocab=45),
     # wider than the 64-expert sort, more heads than one group of 16, fused expert launch shapes (ff % 128 == 0, width % 64 == 0)
