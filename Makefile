@@ -20,9 +20,16 @@ aria_amd/libaria_hip.so: $(OBJ)
 
 # test infrastructure: same sources, SIMT emulator instead of a GPU
 emu: tests/emu/libaria_emu.so
-tests/emu/libaria_emu.so: $(SRC) $(HDR) tests/emu/hip_emu.cpp tests/emu/hip_emu.h
-	$(HOSTCXX) -x c++ -std=c++17 -O3 -g -fPIC -shared -DARIA_EMU -Wno-unknown-attributes -Wno-unused-value -Wno-psabi \
-	    -Iinclude -Iaria_amd/csrc -Itests/emu $(SRC) tests/emu/hip_emu.cpp -o $@
+EMUOBJ := $(patsubst aria_amd/csrc/%.hip,build/emu_%.o,$(SRC)) build/emu_host.o
+EMUFLAGS := -x c++ -std=c++17 -O3 -g -fPIC -DARIA_EMU -Wno-unknown-attributes -Wno-unused-value -Wno-psabi -Iinclude -Iaria_amd/csrc -Itests/emu
+build/emu_host.o: tests/emu/hip_emu.cpp tests/emu/hip_emu.h Makefile
+	@mkdir -p build
+	$(HOSTCXX) $(EMUFLAGS) -c $< -o $@
+build/emu_%.o: aria_amd/csrc/%.hip $(HDR) tests/emu/hip_emu.h Makefile
+	@mkdir -p build
+	$(HOSTCXX) $(EMUFLAGS) -c $< -o $@
+tests/emu/libaria_emu.so: $(EMUOBJ)
+	$(HOSTCXX) -shared -fPIC $(EMUOBJ) -o $@
 
 # test infrastructure: hardware-semantics probes (lane layout of ds_read_b64_tr_b16, fp32 atomic rates) -- their own shared object
 probes: tests/probes/libaria_probe.so

@@ -71,6 +71,7 @@ template <class T>
 __device__ __forceinline__ float dyt(const AriaDyT& p, float v, int n) { return tanh_for<T>(p.alpha * v) * p.w[n] + p.b[n]; }
 
 __device__ __forceinline__ float sigmoid_exact(float z) { return 1.f / (1.f + expf(-z)); }
+__device__ __forceinline__ float softcap(float z, float cap) { return cap * tanhf(z / cap); }
 __device__ __forceinline__ float relu_squared(float z) {
     const float r = fmaxf(z, 0.f);
     return r * r;

@@ -606,16 +606,17 @@ __global__ __launch_bounds__(256) void swiglu_fwd_kernel(const bf16_t* h, const 
     }
 }
 
-// act = relu(u)^2, or silu(gate) u, on rows with leading dimensions (bf16 and 32-bit)
+// act = relu(u)^2, silu(gate) u or relu(gate) u, on rows with leading dimensions (bf16 and 32-bit)
 template <class T>
-__global__ __launch_bounds__(256) void act_rows_kernel(const T* gate, const T* u, T* act, long long nitems, int nch, long long ld_in, long long ld_act) {
+__global__ __launch_bounds__(256) void act_rows_kernel(const T* gate, const T* u, T* act, long long nitems, int nch, long long ld_in, long long ld_act,
+                                                       int relu_gate) {
     for (long long i = blockIdx.x * (long long)blockDim.x + threadIdx.x; i < nitems; i += (long long)gridDim.x * blockDim.x) {
         const long long m = i / nch, n0 = (i % nch) * 8;
         float v[8], g[8];
         ld8(u + m * ld_in + n0, v);
         if (gate) ld8(gate + m * ld_in + n0, g);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v[e] = gate ? g[e] * sigmoid_exact(g[e]) * v[e] : relu_squared(v[e]);
+        for (int e = 0; e < 8; ++e) v[e] = gate ? (relu_gate ? fmaxf(g[e], 0.f) : g[e] * sigmoid_exact(g[e])) * v[e] : relu_squared(v[e]);
         st8(act + m * ld_act + n0, v);
     }
 }
@@ -874,7 +875,8 @@ int aria_moe_route_groups(const float* logits, const float* correction, float* w
     return aria_check_launch();
 }
 
-int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int f32, void* stream) {
+int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int relu_gate, int f32,
+                  void* stream) {
     if (!u || !act || M < 0 || n_cols <= 0) return ARIA_ERR_INVALID;
     if ((n_cols & 7) || (ld_in & 7) || (ld_act & 7)) return ARIA_ERR_ALIGN;
     if (M == 0) return ARIA_OK;
@@ -882,10 +884,10 @@ int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t
     const dim3 grid(unsigned(std::min<long long>((nitems + 255) / 256, 256 * 16))), block(256);
     if (f32)
         ARIA_LAUNCH((act_rows_kernel<float>), grid, block, 0, stream, static_cast<const float*>(gate), static_cast<const float*>(u), static_cast<float*>(act),
-                    nitems, int(n_cols / 8), (long long)ld_in, (long long)ld_act);
+                    nitems, int(n_cols / 8), (long long)ld_in, (long long)ld_act, relu_gate);
     else
         ARIA_LAUNCH((act_rows_kernel<bf16_t>), grid, block, 0, stream, static_cast<const bf16_t*>(gate), static_cast<const bf16_t*>(u),
-                    static_cast<bf16_t*>(act), nitems, int(n_cols / 8), (long long)ld_in, (long long)ld_act);
+                    static_cast<bf16_t*>(act), nitems, int(n_cols / 8), (long long)ld_in, (long long)ld_act, relu_gate);
     return aria_check_launch();
 }
 

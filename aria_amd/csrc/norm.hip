@@ -386,6 +386,110 @@ __global__ __launch_bounds__(256) void dyt_stream_kernel(const int32_t* ids, con
     }
 }
 
+// One pass over the fp32 residual stream with the RMS norms around it, a workgroup per token: x (+)= mult (y, or the half-sum of two normed rows) and
+// embedding rows, then h = rms(x) w.  NC 8-column chunks per thread.
+__device__ __forceinline__ float block_sum(float v, float* red) {   // 4 waves; red: 4 floats that no earlier call still reads
+    v = wave_sum_bcast(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    sync();
+    return (red[0] + red[1]) + (red[2] + red[3]);
+}
+template <class T, int NC>
+__global__ __launch_bounds__(256) void rms_stream_kernel(AriaRmsStream a, int nch) {
+    ARIA_SMEM_STATIC float red[12];
+    const long long t = blockIdx.x, D = (long long)nch * 8;
+    float x[NC][8];
+    const T *y = static_cast<const T*>(a.y), *y2 = static_cast<const T*>(a.y2), *table = static_cast<const T*>(a.table);
+    float* xr = a.x + t * D;
+    const float inv_n = 1.f / float(a.n);
+    if (y) {
+        float v[NC][8], v2[NC][8], ss = 0.f, ss2 = 0.f;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+            const int c = threadIdx.x + 256 * i;
+            if (c < nch) {
+                ld8(xr + c * 8, x[i]);
+                ld8(y + t * a.ldy + c * 8, v[i]);
+                if (a.y_w) ld8(y2 + t * a.ldy + c * 8, v2[i]);
+            }
+        }
+        if (a.y_w) {
+#pragma unroll
+            for (int i = 0; i < NC; ++i)
+                if (int(threadIdx.x) + 256 * i < nch) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        ss += v[i][e] * v[i][e];
+                        ss2 += v2[i][e] * v2[i][e];
+                    }
+                }
+            const float r = 0.5f / sqrtf(block_sum(ss, red) * inv_n + a.eps), r2 = 0.5f / sqrtf(block_sum(ss2, red + 4) * inv_n + a.eps);
+#pragma unroll
+            for (int i = 0; i < NC; ++i) {
+                const int c = threadIdx.x + 256 * i;
+                if (c < nch) {
+                    float w[8], w2[8];
+                    ld8(a.y_w + c * 8, w);
+                    ld8(a.y2_w + c * 8, w2);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) v[i][e] = v[i][e] * r * w[e] + v2[i][e] * r2 * w2[e];
+                }
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < NC; ++i)
+            if (int(threadIdx.x) + 256 * i < nch) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[i][e] += a.mult * v[i][e];
+            }
+    } else {
+#pragma unroll
+        for (int i = 0; i < NC; ++i)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[i][e] = 0.f;
+    }
+    if (a.ids) {
+        const T* row = table + (long long)a.ids[t] * D;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+            const int c = threadIdx.x + 256 * i;
+            if (c < nch) {
+                float v[8];
+                ld8(row + c * 8, v);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[i][e] += a.scale * v[e];
+            }
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+        const int c = threadIdx.x + 256 * i;
+        if (c < nch) {
+            st8(xr + c * 8, x[i]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss += x[i][e] * x[i][e];
+        }
+    }
+    if (!a.next_w) return;
+    const float r = 1.f / sqrtf(block_sum(ss, red + 8) * inv_n + a.eps);
+    T* h = static_cast<T*>(a.h) + t * D;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+        const int c = threadIdx.x + 256 * i;
+        if (c < nch) {
+            float w[8];
+            ld8(a.next_w + c * 8, w);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) w[e] = x[i][e] * r * w[e];
+            st8(h + c * 8, w);
+        }
+    }
+}
+__global__ __launch_bounds__(256) void softcap_kernel(float* x, long long n, float cap) {
+    for (long long i = blockIdx.x * (long long)blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x) x[i] = softcap(x[i], cap);
+}
+
 }  // namespace
 
 extern "C" {
@@ -514,6 +618,40 @@ int aria_dyt_stream(const int32_t* ids, const void* table, const void* y, const 
     else
         ARIA_LAUNCH((dyt_stream_kernel<bf16_t>), grid, block, 0, stream, ids, static_cast<const bf16_t*>(table), static_cast<const bf16_t*>(y), inv,
                     weights, int(k), *post, x, *next, static_cast<bf16_t*>(h), nitems, int(D / 8), (long long)ldy);
+    return aria_check_launch();
+}
+
+int aria_rms_stream(const AriaRmsStream* a, int64_t T, int64_t D, int f32, void* stream) {
+    if (!a || !a->x || T < 0 || D <= 0 || a->n <= 0 || a->n > D || (!a->ids && !a->y) || (a->ids && !a->table) || (a->y_w && (!a->y || !a->y2 || !a->y2_w)) ||
+        (a->next_w && !a->h))
+        return ARIA_ERR_INVALID;
+    if ((D & 7) || (a->y && (a->ldy & 7))) return ARIA_ERR_ALIGN;
+    if (D > 256 * 8 * 8) return ARIA_ERR_UNSUPPORTED;
+    if (T == 0) return ARIA_OK;
+    const int nch = int(D / 8);
+    const dim3 grid(static_cast<unsigned>(T)), block(256);
+#define ARIA_RMS_STREAM(N)                                                              \
+    if (f32)                                                                            \
+        ARIA_LAUNCH((rms_stream_kernel<float, N>), grid, block, 0, stream, *a, nch);    \
+    else                                                                                \
+        ARIA_LAUNCH((rms_stream_kernel<bf16_t, N>), grid, block, 0, stream, *a, nch)
+    if (nch <= 256) {
+        ARIA_RMS_STREAM(1);
+    } else if (nch <= 512) {
+        ARIA_RMS_STREAM(2);
+    } else if (nch <= 1024) {
+        ARIA_RMS_STREAM(4);
+    } else {
+        ARIA_RMS_STREAM(8);
+    }
+#undef ARIA_RMS_STREAM
+    return aria_check_launch();
+}
+
+int aria_softcap(float* x, int64_t n, float cap, void* stream) {
+    if (!x || n < 0 || !(cap > 0.f)) return ARIA_ERR_INVALID;
+    if (n == 0) return ARIA_OK;
+    ARIA_LAUNCH(softcap_kernel, dim3(grid1d(n, 256)), dim3(256), 0, stream, x, (long long)n, cap);
     return aria_check_launch();
 }
 

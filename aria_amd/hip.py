@@ -103,7 +103,7 @@ SIGNATURES = {
     "aria_cross_entropy": [P, P, P, P, P, F32, P, I64, I64, I64, P],
     "aria_attn_varlen_fwd": [P, P, P, P, P, P, I64, I64, I64, I64, I64, I64, I64, I64, I64, I64, F32, P],
     "aria_dyt_stream": [P, P, P, P, P, I64, P, P, P, P, I64, I64, I64, I32, P],
-    "aria_act_rows": [P, P, P, I64, I64, I64, I64, I32, P],
+    "aria_act_rows": [P, P, P, I64, I64, I64, I64, I32, I32, P],
     "aria_gemm_f32": [P, P, P, I64, I64, I64, I64, I64, I64, P, I64, I64, P],
     "aria_moe_route_groups": [P, P, P, P, P, I64, I64, I64, I64, I64, I64, P],
     "aria_latent_rows": [P, P, P, P, P, P, P, P, I64, I32, P],
@@ -113,6 +113,12 @@ SIGNATURES = {
     "aria_latent_splits": [P, I64, I64],
     "aria_latent_decode_scratch": [P, P, I64, I64],
     "aria_latent_decode": [P, P, I64, P, P, P, I64, P, P, I64, P],
+    "aria_rms_stream": [P, I64, I64, I32, P],
+    "aria_softcap": [P, I64, F32, P],
+    "aria_chunk_attn_any": [P, P, P, P, P, P, P, P, I64, I32, P],
+    "aria_chunk_rows": [P, P, P, P, P, P, P, I64, I32, P],
+    "aria_linear_step": [P, P, P, P, P, P, I64, P, I32, P],
+    "aria_norm_gate": [P, P, I64, P, I64, P, I64, I64, I64, I64, F32, I32, I32, P],
 }
 
 
@@ -136,7 +142,21 @@ class LatentStack(ctypes.Structure):    # AriaLatentStack
     _fields_ = [("n_layers", c_int64), ("D", c_int64), ("V", c_int64), ("first", DyTParams), ("embed", c_void_p), ("head", c_void_p)]
 
 
-ABI_VERSION = 4   # include/aria_hip.h ARIA_ABI_VERSION this host code was written against
+class RmsStream(ctypes.Structure):      # AriaRmsStream
+    _fields_ = [("ids", c_void_p), ("table", c_void_p), ("scale", c_float), ("mult", c_float), ("eps", c_float), ("n", c_int64), ("ldy", c_int64)] + \
+               [(n, c_void_p) for n in ("y", "y2", "y_w", "y2_w", "x", "next_w", "h")]
+
+
+class ChunkShape(ctypes.Structure):     # AriaChunkShape
+    _fields_ = [(n, c_int64) for n in ("H", "G", "dq", "dvp", "ldp", "q_off", "k_off", "v_off", "size", "cap")] + [("scale", c_float)]
+
+
+class LinearShape(ctypes.Structure):    # AriaLinearShape
+    _fields_ = [(n, c_int64) for n in ("H", "d", "dv", "dp", "dvp", "ldp", "q_off", "k_off", "v_off", "a_off", "rank", "silu")] + \
+               [("q_scale", c_float), ("inv_tau", c_float)] + [(n, c_void_p) for n in ("decay", "a2", "a_bias")]
+
+
+ABI_VERSION = 5   # include/aria_hip.h ARIA_ABI_VERSION this host code was written against
 
 
 class AriaHipError(RuntimeError):

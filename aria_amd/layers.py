@@ -4,13 +4,18 @@
   (``ops.dyt_stream``) or a projection's epilogue, never as a launch of its own;
 * ``LatentAttention`` + ``LatentCache`` -- keys and values as images of one low-rank latent per token, a rotated key part shared by the heads, a
   sigmoid output gate per head;
-* ``SquaredReluFeedForward``; ``GroupLimitedMixture`` -- sigmoid router with a choice correction and group-limited top-k.
+* ``SquaredReluFeedForward``; ``GroupLimitedMixture`` -- sigmoid router with a choice correction and group-limited top-k;
+* ``RmsNorm`` -- its weight as a factor, evaluated inside a pass over the residual stream (``ops.rms_stream``);
+* ``ChunkAttention`` + ``ChunkCache`` -- grouped-query attention inside chunks of positions; ``LinearAttention`` + ``LinearState`` -- a decaying matrix
+  state per head, the decay constant or gated; ``MixerGroup`` -- mixers that read the same input side by side, their projections one matrix;
+* ``ReluGatedFeedForward``.
 
 Weights are held the way the kernels read them (padded, projections that share an input in one matrix) and packed once at load.  Modules exist in
 bf16 and in float32 (``dtype``); the float32 form runs the 32-bit kernels throughout."""
 from __future__ import annotations
 
-from typing import List, Optional
+import math
+from typing import List, Optional, Sequence
 
 import torch
 import torch.nn as nn
@@ -172,3 +177,157 @@ class GroupLimitedMixture(nn.Module):
             rows = ops.permute_any(h, sorted_src, self.top)
             act = ops.act_rows(ops.grouped_linear_any(rows, u, offsets), gate=ops.grouped_linear_any(rows, g, offsets))
         return dict(y=ops.grouped_linear_any(act, self.down, offsets), inv=inv, weights=weights)
+
+
+class RmsNorm(nn.Module):
+    """x / sqrt(mean(x^2) + eps) (weight + offset): the factor in float32, zeros behind the true width."""
+
+    def __init__(self, weight: torch.Tensor, width: int, offset: float = 0.0):
+        super().__init__()
+        self.weight = _frozen(padded(weight.float() + offset, width), f32)
+
+
+class ChunkCache:
+    """One layer's static cache of chunk-local attention: [slots, kv heads, rows, key | value].  A sequence holds ONE chunk, position p in row p % size;
+    rows behind its position in the chunk are never read."""
+
+    def __init__(self, slots: int, max_len: int, heads: int, size: int, width: int, dtype, device):
+        self.rows = torch.zeros((slots, heads, min(size, max_len), width), dtype=dtype, device=device)
+
+
+class ChunkAttention(nn.Module):
+    """Grouped-query softmax attention without positions, position i seeing the j <= i of its own chunk of ``size``.  ``w``: the checkpoint's tensors
+    q, k, v, o.  The input projection's rows are ``w_in`` until a ``MixerGroup`` takes them."""
+
+    def __init__(self, w, *, heads: int, kv_heads: int, dim: int, vdim: int, size: int, scale: float, width: int, dtype=bf16):
+        super().__init__()
+        if heads % kv_heads or size < 1:
+            raise ValueError(f"{heads} query heads over {kv_heads} key heads in chunks of {size}")
+        fused = ops.varlen_head(dim, vdim) if dtype == bf16 else None
+        dq, dvp = fused or (up8(dim), up8(vdim))
+        self.flash, self.dtype = fused is not None, dtype
+        D = w["q"].shape[1]
+        self.w_in = [padded(w["q"].view(heads, dim, D), heads, dq, D).view(-1, D), padded(w["k"].view(kv_heads, dim, D), kv_heads, dq, D).view(-1, D),
+                     padded(w["v"].view(kv_heads, vdim, D), kv_heads, dvp, D).view(-1, D)]
+        self.geometry = dict(H=heads, G=kv_heads, dq=dq, dvp=dvp, size=size, scale=scale)
+        self.w_o = _frozen(padded(w["o"].view(-1, heads, vdim), width, heads, dvp).view(width, heads * dvp), dtype)
+
+    def placed(self, offsets: Sequence[int], ldp: int) -> None:
+        self.geometry.update(zip(("q_off", "k_off", "v_off"), offsets), ldp=ldp)
+
+    def shape(self, cache: ChunkCache) -> hip.ChunkShape:
+        return hip.ChunkShape(cap=cache.rows.shape[2], **self.geometry)
+
+    def new_cache(self, slots: int, max_len: int, device) -> ChunkCache:
+        g = self.geometry
+        return ChunkCache(slots, max_len, g["G"], g["size"], g["dq"] + g["dvp"], self.dtype, device)
+
+    def forward(self, proj: torch.Tensor, batch, cache: ChunkCache) -> torch.Tensor:
+        return ops.linear_any(ops.chunk_attention_any(self.shape(cache), proj, cache.rows, batch), self.w_o)
+
+
+class LinearState:
+    """One layer's recurrent states, float32 [slots, heads, key, value]; a sequence at position 0 starts from zeros whatever its slot holds."""
+
+    def __init__(self, slots: int, heads: int, dim: int, vdim: int, device):
+        self.rows = torch.zeros((slots, heads, dim, vdim), dtype=f32, device=device)
+
+
+class LinearAttention(nn.Module):
+    """S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = q_scale S_t^T q_t per head, then an RMS norm (per head with a shared weight, or over all heads) and an
+    output gate.  Decay: ``decay``, a constant per head; or, without it, gated per key channel: sigmoid(a2 (a1 h) + a2.b)^(1 / tau).  ``w``: the
+    checkpoint's tensors q, k, v, g, o, norm (a1, a2, a2.b)."""
+
+    def __init__(self, w, *, heads: int, dim: int, vdim: int, decay: Optional[Sequence[float]] = None, tau: float = 1.0, q_scale: float = 1.0, silu_inputs: bool = False,
+                 norm_heads: bool = True, gate: str = "silu", eps: float, width: int, dtype=bf16):
+        super().__init__()
+        self.chunked = dtype == bf16 and dim <= 256
+        dp = next(n for n in (64, 128, 256) if n >= dim) if self.chunked else up8(dim)
+        dvp = (vdim + 63) // 64 * 64 if self.chunked else up8(vdim)
+        self.eps, self.dtype, self.silu_gate = eps, dtype, {"silu": True, "sigmoid": False}[gate]
+        D = w["q"].shape[1]
+
+        def rows(name, n, to):
+            return padded(w[name].view(heads, n, D), heads, to, D).view(-1, D)
+
+        self.w_in = [rows("q", dim, dp), rows("k", dim, dp), rows("v", vdim, dvp), rows("g", vdim, dvp)]
+        self.geometry = dict(H=heads, d=dim, dv=vdim, dp=dp, dvp=dvp, rank=0, silu=int(silu_inputs), q_scale=q_scale, inv_tau=1.0 / tau)
+        self.decay = self.a2 = self.a_bias = None
+        if decay is not None:
+            if len(decay) != heads or min(decay) < 0:
+                raise ValueError(f"{len(decay)} decays for {heads} heads")
+            self.decay = _frozen(torch.tensor([[a, math.log2(a) if a > 0 else -math.inf] for a in decay], dtype=torch.float64), f32)
+        else:
+            rank = up8(w["a1"].shape[0])
+            self.w_in.append(padded(w["a1"], rank, D))
+            self.geometry["rank"] = rank
+            self.a2 = _frozen(padded(w["a2"].view(heads, dim, -1), heads, dp, rank).view(heads * dp, rank), dtype)
+            self.a_bias = _frozen(padded(w["a2.b"].view(heads, dim), heads, dp).view(-1), f32)
+        self.norm_groups, self.norm_n = (heads, vdim) if norm_heads else (1, heads * vdim)
+        norm = w["norm"].view(-1, vdim)
+        self.norm = _frozen(padded(norm, norm.shape[0], dvp).view(-1), f32)
+        self.w_o = _frozen(padded(w["o"].view(-1, heads, vdim), width, heads, dvp).view(width, heads * dvp), dtype)
+
+    def placed(self, offsets: Sequence[int], ldp: int) -> None:
+        self.geometry.update(zip(("q_off", "k_off", "v_off"), offsets), ldp=ldp, a_off=offsets[4] if len(offsets) > 4 else 0)
+        self.g_off = offsets[3]
+
+    def shape(self) -> hip.LinearShape:
+        ptr = {n: t.data_ptr() for n, t in (("decay", self.decay), ("a2", self.a2), ("a_bias", self.a_bias)) if t is not None}
+        return hip.LinearShape(**self.geometry, **ptr)
+
+    def new_cache(self, slots: int, max_len: int, device) -> LinearState:
+        g = self.geometry
+        return LinearState(slots, g["H"], g["dp"], g["dvp"], device)
+
+    def forward(self, proj: torch.Tensor, batch, cache: LinearState) -> torch.Tensor:
+        o = ops.linear_step(self.shape(), proj, cache.rows, batch)
+        o = ops.norm_gate(o, proj[:, self.g_off:self.g_off + o.shape[1]], self.norm, self.norm_groups, self.norm_n, self.eps, self.silu_gate)
+        return ops.linear_any(o, self.w_o)
+
+
+class MixerGroup(nn.Module):
+    """One mixer, or two side by side that read the same input: one input projection for all.  Two: the result is the half-sum of their outputs, each
+    RMS-normed with its plain weight -- a step of the stream pass that follows, so forward returns that pass's operands."""
+
+    def __init__(self, parts: Sequence[nn.Module], width: int, out_norms: Sequence[RmsNorm] = (), dtype=bf16):
+        super().__init__()
+        if len(parts) != max(1, len(out_norms)) or len(parts) > 2:
+            raise ValueError(f"{len(parts)} mixers with {len(out_norms)} output norms")
+        blocks = [b for p in parts for b in p.w_in]
+        starts = [0]
+        for b in blocks:
+            starts.append(starts[-1] + up8(b.shape[0]))
+        w_in = torch.zeros((starts[-1], width), dtype=blocks[0].dtype, device=blocks[0].device)
+        for b, at in zip(blocks, starts):
+            w_in[at:at + b.shape[0], :b.shape[1]] = b
+        for p in parts:
+            p.placed(starts[:len(p.w_in)], w_in.shape[0])
+            starts = starts[len(p.w_in):]
+            del p.w_in
+        self.w_in = _frozen(w_in, dtype)
+        self.parts, self.out_norms = nn.ModuleList(parts), nn.ModuleList(out_norms)
+
+    def new_cache(self, slots: int, max_len: int, device) -> list:
+        return [p.new_cache(slots, max_len, device) for p in self.parts]
+
+    def forward(self, h: torch.Tensor, batch, caches: list) -> dict:
+        proj = ops.linear_any(h, self.w_in)
+        y = [p(proj, batch, c) for p, c in zip(self.parts, caches)]
+        if len(y) == 1:
+            return dict(y=y[0])
+        return dict(y=y[0], pair=(y[1], self.out_norms[0].weight, self.out_norms[1].weight))
+
+
+class ReluGatedFeedForward(nn.Module):
+    """W_down (max(W_gate h, 0) * (W_up h)); gate and up rows in one matrix."""
+
+    def __init__(self, gate: torch.Tensor, up: torch.Tensor, down: torch.Tensor, width: int, dtype=bf16):
+        super().__init__()
+        self.ff = up8(up.shape[0])
+        self.gate_up = _frozen(torch.cat([padded(t, self.ff, width) for t in (gate, up)]), dtype)
+        self.down = _frozen(padded(down, width, self.ff), dtype)
+
+    def forward(self, h: torch.Tensor) -> dict:
+        gu = ops.linear_any(h, self.gate_up)
+        return dict(y=ops.linear_any(ops.act_rows(gu[:, self.ff:], gate=gu[:, :self.ff], relu=True), self.down))

@@ -1030,11 +1030,12 @@ def permute_any(x: torch.Tensor, rows_src: torch.Tensor, k: int) -> torch.Tensor
     return moe_permute(x.view(bf16), rows_src, k).view(torch.float32)
 
 
-def act_rows(u: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """relu(u)^2, or silu(gate) u."""
-    assert u.is_contiguous() and (gate is None or (gate.is_contiguous() and gate.shape == u.shape and gate.dtype == u.dtype))
-    out = torch.empty_like(u)
-    hip.get_lib().call("aria_act_rows", _p(gate), _p(u), _p(out), u.shape[0], u.shape[1], u.shape[1], u.shape[1], _f32(u), _stream(u))
+def act_rows(u: torch.Tensor, gate: Optional[torch.Tensor] = None, relu: bool = False) -> torch.Tensor:
+    """relu(u)^2, silu(gate) u or (``relu``) relu(gate) u; u and gate may be column ranges of one matrix."""
+    ld = _rowmajor_2d(u, "u")
+    assert gate is None or (gate.shape == u.shape and gate.dtype == u.dtype and _rowmajor_2d(gate, "gate") == ld)
+    out = torch.empty(u.shape, dtype=u.dtype, device=u.device)
+    hip.get_lib().call("aria_act_rows", _p(gate), _p(u), _p(out), u.shape[0], u.shape[1], ld, u.shape[1], int(relu), _f32(u), _stream(u))
     return out
 
 
@@ -1139,6 +1140,115 @@ def latent_decode_attention(shape, proj, slot, pos, rope, kv_norm, uk, uv, cache
     lib.call("aria_latent_attn", _p(qa), _p(cache), ref, _p(slot), _p(pos), _p(part_o), _p(part_ml), T, splits, f32, _stream(proj))
     out = torch.empty((T, shape.H * shape.dvp), dtype=proj.dtype, device=dev)
     lib.call("aria_latent_expand", _p(part_o), _p(part_ml), ref, _p(proj), _p(uv), _p(out), T, splits, f32, _stream(proj))
+    return out
+
+
+# ----------------------------------------------------------------------------- RMS-normed stream, chunk-local attention, linear attention
+def rms_stream(x: torch.Tensor, n: int, eps: float, nxt: Optional[torch.Tensor], *, dtype=None, ids: Optional[torch.Tensor] = None,
+               table: Optional[torch.Tensor] = None, scale: float = 1.0, y: Optional[torch.Tensor] = None, mult: float = 1.0,
+               pair: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor]] = None) -> Optional[torch.Tensor]:
+    """One pass over the residual stream x [T, D] fp32 (in place; the first ``n`` columns count): x = (y given: x + mult y) + (ids given: scale
+    table[ids]), with ``pair`` = (y2, w, w2) the half-sum of rms(y) w and rms(y2) w2 in y's place; -> rms(x) nxt in ``dtype``, or None without
+    ``nxt``."""
+    import ctypes
+
+    _chk(x, torch.float32, "x")
+    T, D = x.shape
+    assert x.is_contiguous() and (y is not None or ids is not None)
+    src = y if y is not None else table
+    dtype = dtype or src.dtype
+    if y is not None:
+        assert y.shape == (T, D) and y.dtype == dtype
+    if ids is not None:
+        _chk(ids, torch.int32, "ids")
+        assert ids.is_contiguous() and ids.numel() == T and table.is_contiguous() and table.shape[1] == D and table.dtype == dtype
+    y2, w, w2 = pair if pair is not None else (None, None, None)
+    if pair is not None:
+        assert y2.shape == y.shape and y2.dtype == dtype and _rowmajor_2d(y2, "y2") == _rowmajor_2d(y, "y")
+    for v in (nxt, w, w2):
+        assert v is None or (v.dtype == torch.float32 and v.numel() == D)
+    h = torch.empty((T, D), dtype=dtype, device=x.device) if nxt is not None else None
+    a = hip.RmsStream(_p(ids), _p(table) if ids is not None else None, float(scale), float(mult), float(eps), n, _rowmajor_2d(y, "y") if y is not None else 0,
+                      _p(y), _p(y2), _p(w), _p(w2), _p(x), _p(nxt), _p(h))
+    hip.get_lib().call("aria_rms_stream", ctypes.byref(a), T, D, int(dtype == torch.float32), _stream(x))
+    return h
+
+
+def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap tanh(x / cap) in place, fp32."""
+    _chk(x, torch.float32, "x")
+    assert x.is_contiguous()
+    hip.get_lib().call("aria_softcap", _p(x), x.numel(), float(cap), _stream(x))
+    return x
+
+
+def _chk_rows(proj, ldp: int, batch) -> int:
+    T = batch.ids.numel()
+    if proj.shape != (T, ldp) or not proj.is_contiguous():
+        raise ValueError("the projection's rows do not fit the shape")
+    for t in (batch.slot, batch.pos, batch.seq, batch.cu):
+        _chk(t, torch.int32)
+        assert t.is_contiguous()
+    return T
+
+
+def chunk_attention_any(shape, proj: torch.Tensor, cache: torch.Tensor, batch) -> torch.Tensor:
+    """Chunk-local attention of the batch's tokens, any widths and any cut: keys of earlier steps from the cache, the batch's own from ``proj``; the
+    batch's keys and values are then written to the cache.  -> [T, H dvp]"""
+    import ctypes
+
+    T, ref, lib = _chk_rows(proj, shape.ldp, batch), ctypes.byref(shape), hip.get_lib()
+    _chk_ring(shape, cache, proj, batch)
+    out = torch.empty((T, shape.H * shape.dvp), dtype=proj.dtype, device=proj.device)
+    lib.call("aria_chunk_attn_any", _p(proj), _p(cache), ref, _p(batch.slot), _p(batch.pos), _p(batch.seq), _p(batch.cu), _p(out), T, _f32(proj), _stream(proj))
+    chunk_rows(shape, proj, cache, batch)
+    return out
+
+
+def _chk_ring(shape, cache: torch.Tensor, proj: torch.Tensor, batch) -> None:
+    if cache.shape[1:] != (shape.G, shape.cap, shape.dq + shape.dvp) or not cache.is_contiguous() or cache.dtype != proj.dtype:
+        raise ValueError("the cache does not fit the shape")
+    if min(shape.size, batch.max_len) > shape.cap or max(batch.slots) >= cache.shape[0]:
+        raise ValueError("the batch does not fit the cache")
+
+
+def chunk_rows(shape, proj: torch.Tensor, cache: torch.Tensor, batch) -> None:
+    """Keys and values of the batch's tokens into the chunk cache."""
+    import ctypes
+
+    T = _chk_rows(proj, shape.ldp, batch)
+    _chk_ring(shape, cache, proj, batch)
+    hip.get_lib().call("aria_chunk_rows", _p(proj), _p(cache), ctypes.byref(shape), _p(batch.slot), _p(batch.pos), _p(batch.seq), _p(batch.cu), T, _f32(proj),
+                       _stream(proj))
+
+
+def linear_step(shape, proj: torch.Tensor, state: torch.Tensor, batch) -> torch.Tensor:
+    """The linear-attention recurrence over every sequence of the batch, token by token, from and into its state: -> [T, H dvp]."""
+    import ctypes
+
+    T = _chk_rows(proj, shape.ldp, batch)
+    _chk_state(shape, state, batch)
+    out = torch.empty((T, shape.H * shape.dvp), dtype=proj.dtype, device=proj.device)
+    hip.get_lib().call("aria_linear_step", _p(proj), ctypes.byref(shape), _p(state), _p(batch.slot), _p(batch.pos), _p(batch.cu), len(batch.lengths), _p(out),
+                       _f32(proj), _stream(proj))
+    return out
+
+
+def _chk_state(shape, state: torch.Tensor, batch) -> None:
+    _chk(state, torch.float32, "state")
+    if state.shape[1:] != (shape.H, shape.dp, shape.dvp) or not state.is_contiguous() or max(batch.slots) >= state.shape[0]:
+        raise ValueError("the state does not fit the shape")
+
+
+def norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, groups: int, n: int, eps: float, silu: bool) -> torch.Tensor:
+    """rms norm of every group of columns of o (``n`` of them count) times weight (one group's, shared, or all columns') times silu or sigmoid of gate."""
+    T, C = o.shape
+    cols = C // groups
+    _chk(weight, torch.float32, "weight")
+    assert o.is_contiguous() and gate.shape == o.shape and gate.dtype == o.dtype and weight.numel() in (cols, C)
+    out = torch.empty_like(o)
+    hip.get_lib().call("aria_norm_gate", _p(o), _p(gate), _rowmajor_2d(gate, "gate"), _p(weight), cols if weight.numel() == C else 0, _p(out), T, groups, cols, n,
+                       float(eps), int(silu), _f32(o), _stream(o))
     return out
 
 

@@ -12,6 +12,7 @@ import torch
 MODELS = {
     "AriaForConditionalGeneration": ("modeling_aria", "AriaForConditionalGeneration"),
     "Duguzen": ("duguzen", "DuguzenForCausalLM"),
+    "Kozipel": ("kozipel", "KozipelForCausalLM"),
 }
 MODEL_TYPES = {"aria": "AriaForConditionalGeneration"}   # Hugging Face configs without an architecture name
 

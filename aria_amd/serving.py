@@ -7,10 +7,10 @@ that ends leaves its cache slot to a later batch.  A model serves through three 
 * ``step(batch) -> float32 [wanted, vocab]`` -- run the batch's tokens from and into the caches, logits at the wanted rows;
 * ``vocab``, ``device`` -- columns of the logits, where tensors live.
 
-``duguzen.DuguzenForCausalLM`` runs a batch as one; ``gptfast.Transformer`` (Aria) runs its sequences one after the other on the slots' caches.  The same ``step`` is what ``generate`` and the trace runner (bin/trace_run) drive."""
+``duguzen.DuguzenForCausalLM`` and ``kozipel.KozipelForCausalLM`` run a batch as one; ``gptfast.Transformer`` (Aria) runs its sequences one after the other on the slots' caches.  The same ``step`` is what ``generate`` and the trace runner (bin/trace_run) drive."""
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Dict, List, Optional, Sequence
 
 import torch
@@ -32,6 +32,19 @@ class StepBatch:
     starts: List[int]
     slots: List[int]
     rows: Optional[List[int]] = None   # the host's copy of ``wanted``
+    seq: Optional[torch.Tensor] = None   # [T] which sequence every token belongs to
+    made: Dict[object, object] = field(default_factory=dict)   # tables derived from the lengths, by what they are for
+
+    def chunks(self, size: int):
+        """The sequences cut at the multiples of ``size`` from their first token, for a batch of whole prompts: (first row of every piece and the end,
+        int32 on the device; length of the longest piece)."""
+        assert self.fresh
+        if ("chunks", size) not in self.made:
+            cu = [0]
+            for n in self.lengths:
+                cu += [cu[-1] + min(at + size, n) for at in range(0, n, size)]
+            self.made["chunks", size] = (torch.tensor(cu, dtype=torch.int32).to(self.ids.device), min(size, self.longest))
+        return self.made["chunks", size]
 
     def wanted_by_sequence(self) -> List[List[int]]:
         """per sequence: the wanted places among its own tokens, in order"""
@@ -64,13 +77,14 @@ class StepBatch:
         """tokens: one list of ids per sequence, or an int32 device tensor with one id per sequence (a decode step whose ids never visited the host)."""
         on_device = isinstance(tokens, torch.Tensor)
         lengths = [1] * len(slots) if on_device else [len(t) for t in tokens]
-        cu, slot, pos = [0], [], []
-        for n, s, p in zip(lengths, slots, starts):
+        cu, slot, pos, seq = [0], [], [], []
+        for i, (n, s, p) in enumerate(zip(lengths, slots, starts)):
             cu.append(cu[-1] + n)
             slot += [s] * n
             pos += range(p, p + n)
+            seq += [i] * n
         T = cu[-1]
-        host = ([] if on_device else [i for t in tokens for i in t]) + slot + pos + cu + (list(wanted) if wanted is not None else [])
+        host = ([] if on_device else [i for t in tokens for i in t]) + slot + pos + seq + cu + (list(wanted) if wanted is not None else [])
         buf = torch.tensor(host, dtype=torch.int32).to(device)      # one copy to the device per step
         at = 0
 
@@ -80,8 +94,9 @@ class StepBatch:
             return buf[at - n:at]
 
         ids = tokens if on_device else take(T)
-        return cls(ids, take(T), take(T), take(len(slots) + 1), take(len(wanted)) if wanted is not None else None, lengths, list(starts), list(slots),
-                   list(wanted) if wanted is not None else None)
+        slot, pos, seq, cu = take(T), take(T), take(T), take(len(slots) + 1)
+        return cls(ids, slot, pos, cu, take(len(wanted)) if wanted is not None else None, lengths, list(starts), list(slots),
+                   list(wanted) if wanted is not None else None, seq)
 
 
 class Scheduler:

@@ -26,10 +26,11 @@ extern "C" {
 #define ARIA_ERR_UNSUPPORTED 3 /* shape outside what the kernels implement (e.g. > 256 experts) */
 #define ARIA_ERR_LAUNCH 4      /* hipGetLastError() != hipSuccess after the launch */
 
-/* Library / ABI version: bumped whenever an entry point is added or a signature changes (4 added the latent-attention family; 3: aria_moe_router_fused,
+/* Library / ABI version: bumped whenever an entry point is added or a signature changes (5 added
+ * the linear-attention family; 4: the latent-attention family; 3: aria_moe_router_fused,
  * aria_attn_bwd_rope, aria_moe_unpermute_res, aria_scale_bf16, aria_gemm_qkv_rope_hf_bf16, the *_lora_* family).  The Python host
  * (aria_amd/hip.py) refuses a library whose version is not the one it was written against. */
-#define ARIA_ABI_VERSION 4
+#define ARIA_ABI_VERSION 5
 int aria_abi_version(void);
 /* Test/diagnostic aid: which GEMM kernel family the calling thread's last aria_*gemm* call dispatched to
  * (1 = 128x128 tile, 2 = 256x256 register-staged, 3 = 256x256 LDS-DMA phase-scheduled; 0 = none yet). */
@@ -462,8 +463,10 @@ typedef struct {
 int aria_dyt_stream(const int32_t* ids, const void* table, const void* y, const int32_t* inv, const float* weights, int64_t k, const AriaDyT* post,
                     float* x, const AriaDyT* next, void* h, int64_t T, int64_t D, int64_t ldy, int f32, void* stream);
 
-/* act[m, n] = relu(u[m, n])^2 (gate == NULL) or silu(gate[m, n]) u[m, n]; rows of n_cols (% 8 == 0), leading dimensions in elements. */
-int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int f32, void* stream);
+/* act[m, n] = relu(u[m, n])^2 (gate == NULL), silu(gate[m, n]) u[m, n], or (relu_gate) relu(gate[m, n]) u[m, n]; rows of n_cols (% 8 == 0),
+ * leading dimensions in elements. */
+int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int relu_gate, int f32,
+                  void* stream);
 
 /* C [M, N] = A [M, K] W^T (W [N, K]) in true 32-bit on the vector ALU.  offsets != NULL: rows offsets[e] .. offsets[e + 1] of A use W + e strideW
  * (int32 [E + 1] on the device).  K % 4 == 0, 16-byte aligned rows. */
@@ -527,6 +530,67 @@ int aria_latent_decode(const AriaLatentStack* stack, const AriaLatentLayer* laye
                        int64_t max_len, float* logits, void* scratch, int64_t scratch_bytes, void* stream);
 /* how many splits aria_latent_decode / a caller of aria_latent_attn should use */
 int64_t aria_latent_splits(const AriaLatentShape* s, int64_t T, int64_t max_len);
+
+/* ------------------------------------------------------------------------------------------------
+ * Chunk-local grouped-query attention, linear attention, RMS-normed stream: the mechanisms of the Kozipel design.  `f32` as above.  Residual stream,
+ * norms, scores and softmax, decays, recurrent states are fp32 in both forms.
+ * ------------------------------------------------------------------------------------------------ */
+/* One pass over the residual stream x [T, D] fp32 (D % 8 == 0, the first n columns count, the others stay zero):
+ *   x = (y ? x + mult src : 0) + (ids ? scale table[ids[t], :] : 0)
+ *   src = y[t, :], or (y_w != NULL) the half-sum of rms(y[t, :]) y_w and rms(y2[t, :]) y2_w
+ * then, next_w != NULL: h[t, :] = rms(x[t, :]) next_w, where rms(v) = v / sqrt(mean(v^2) + eps).  D <= 16384. */
+typedef struct {
+    const int32_t* ids;
+    const void* table; /* [V, D] */
+    float scale, mult, eps;
+    int64_t n, ldy;
+    const void *y, *y2;
+    const float *y_w, *y2_w; /* [D] */
+    float* x;
+    const float* next_w; /* [D] */
+    void* h;
+} AriaRmsStream;
+int aria_rms_stream(const AriaRmsStream* a, int64_t T, int64_t D, int f32, void* stream);
+
+/* x[i] = cap tanh(x[i] / cap), fp32, in place. */
+int aria_softcap(float* x, int64_t n, float cap, void* stream);
+
+/* Shape of a chunk-local attention layer: positions of a sequence form chunks of `size` from position 0, a query sees the keys of its own chunk up to
+ * itself.  A row of `proj` (ldp columns) holds H query heads of dq columns at q_off, G key heads of dq at k_off, G value heads of dvp at v_off (query
+ * head h reads key / value head h / (H / G)); columns behind the true widths are zeros.  Cache: [slots, G, cap, dq + dvp] rows key | value, position p
+ * in row p % size, cap >= min(size, longest sequence). */
+typedef struct {
+    int64_t H, G, dq, dvp, ldp, q_off, k_off, v_off, size, cap;
+    float scale;
+} AriaChunkShape;
+/* Any widths, any cut of the sequences: out [T, H dvp].  Sequence seq[t] holds rows cu[seq[t]] .. of this call; keys of earlier calls come from the
+ * cache, the call's own from proj (call aria_chunk_rows afterwards). */
+int aria_chunk_attn_any(const void* proj, const void* cache, const AriaChunkShape* s, const int32_t* slot, const int32_t* pos, const int32_t* seq,
+                        const int32_t* cu, void* out, int64_t T, int f32, void* stream);
+/* Writes the call's keys and values to the cache (of the positions that share a row, the last one). */
+int aria_chunk_rows(const void* proj, void* cache, const AriaChunkShape* s, const int32_t* slot, const int32_t* pos, const int32_t* seq, const int32_t* cu,
+                    int64_t T, int f32, void* stream);
+
+/* Shape of a linear-attention layer: per head a state S [d, dv] (fp32, cache [slots, H, dp, dvp]), S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.
+ * A row of `proj` holds q and k (H heads of dp columns, zeros behind d), v (H heads of dvp, zeros behind dv) and, for the gated form, the rank columns
+ * a1 (padded with zeros to a multiple of 8).  silu != 0: q, k, v pass through silu.  Decay: decay != NULL: one constant per head, pairs (a, log2 a);
+ * else a = sigmoid(a2 a1 + a_bias)^inv_tau per key channel, a2 [H dp, rank], a_bias fp32 [H dp]. */
+typedef struct {
+    int64_t H, d, dv, dp, dvp, ldp, q_off, k_off, v_off, a_off, rank, silu;
+    float q_scale, inv_tau;
+    const float* decay;
+    const void* a2;
+    const float* a_bias;
+} AriaLinearShape;
+/* Token by token, any widths (dp <= 1024): sequence i = rows cu[i] .. cu[i + 1], a sequence at position 0 starts from a zero state whatever its slot
+ * holds; out [T, H dvp]. */
+int aria_linear_step(const void* proj, const AriaLinearShape* s, float* state, const int32_t* slot, const int32_t* pos, const int32_t* cu, int64_t n_seq,
+                     void* out, int f32, void* stream);
+
+/* y = o / sqrt(sum(o^2) / n + eps) w act(gate) per (row, group of cols columns): act = silu, or sigmoid (silu == 0); w [groups, cols] with w_stride
+ * between groups (0: shared).  o [T, groups cols], gate rows ldg apart.  cols % 8 == 0; y may be o. */
+int aria_norm_gate(const void* o, const void* gate, int64_t ldg, const float* w, int64_t w_stride, void* y, int64_t T, int64_t groups, int64_t cols, int64_t n,
+                   float eps, int silu, int f32, void* stream);
 
 #ifdef __cplusplus
 }

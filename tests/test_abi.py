@@ -30,8 +30,8 @@ def test_library_exports_every_declared_symbol():
         g.build()
     lib = hip.HipLibrary(hip.LIB_PATH)
     assert lib.missing == []
-    assert lib.cdll.aria_abi_version() == hip.ABI_VERSION == 4
-    assert "#define ARIA_ABI_VERSION 4" in open(os.path.join(ROOT, "include", "aria_hip.h")).read()
+    assert lib.cdll.aria_abi_version() == hip.ABI_VERSION == 5
+    assert "#define ARIA_ABI_VERSION 5" in open(os.path.join(ROOT, "include", "aria_hip.h")).read()
     # the library's own `aria_*` exports are exactly the header's entry points (internal helpers such as aria_check_launch are hidden)
     import subprocess
 
