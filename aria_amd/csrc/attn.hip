@@ -18,6 +18,7 @@
 //  * tensors are [B, S, H, hd] views of token-major activations (row stride ld*): no head transposes in HBM.
 #include "aria_device.h"
 #include "aria_hip.h"
+#include "tile.h"
 #include <cstdlib>
 
 namespace {
@@ -71,28 +72,11 @@ __device__ __forceinline__ s16x8 frag_rc(const bf16_t* s, int row, int kk, int l
     return *reinterpret_cast<const s16x8*>(s + row * Cfg<HD>::PITCH + kk * 16 + (l >> 5) * 8);
 }
 
-// accumulator regs 8u..8u+7 of a 32x32 tile -> bf16 fragment (lane-local)
-__device__ __forceinline__ s16x8 pack_frag(const f32x16& p, int u) {
-    u32x4 v;
-#pragma unroll
-    for (int j = 0; j < 4; ++j) v[j] = pack2bf(p[8 * u + 2 * j], p[8 * u + 2 * j + 1]);
-    return __builtin_bit_cast(s16x8, v);
-}
-
-__device__ __forceinline__ int acc_row(int r, int l) { return (r & 3) + 8 * (r >> 2) + 4 * (l >> 5); }
-
 // (a0 * b + c, a1 * b + c), each a fused multiply-add: the softmax's score scaling
 typedef float f32x2 __attribute__((ext_vector_type(2)));
 __device__ __forceinline__ f32x2 fma2(float a0, float a1, float b, float c) {
     const f32x2 a = {a0, a1}, bb = {b, b}, cc = {c, c};
     return __builtin_elementwise_fma(a, bb, cc);
-}
-
-__device__ __forceinline__ f32x16 zero_acc() {
-    f32x16 z;
-#pragma unroll
-    for (int r = 0; r < 16; ++r) z[r] = 0.f;
-    return z;
 }
 
 // 1-D grid -> (block along the sequence, head, batch) for the 512-thread kernels.  Workgroup n runs on XCD n % 8 (own L2).
@@ -791,7 +775,6 @@ struct Cfg3 {
     static constexpr int KS = HD / 16, DT = HD / 32;
     static constexpr int SMEM_DKDV = 4 * TILE + 2 * 2 * 64 * 4 + 4 * 8 * 1024;  // Q,dO double-buffered + lse,delta + P exchange
 };
-__device__ __forceinline__ int swz3(int row) { return ((row & 3) << 2) | ((row >> 2) & 3); }
 
 template <int HD>
 __device__ __forceinline__ void tile_load3(u32x4 (&r)[Cfg3<HD>::NCH], const bf16_t* base, long long ld, int row0, int row_end, int t) {
@@ -1295,46 +1278,8 @@ struct Fmt128 {
     static __device__ __forceinline__ s16x8 kfrag(const char* s, int row, int kk, int l) { return frag_rc3<128>(s, row, kk, l); }
     static __device__ __forceinline__ s16x8 vfrag(const char* s, int rb, int d0, int l) { return frag_tr3<128>(s, rb, d0, l); }
 };
-// Query / key heads of QD columns beside value heads of VD columns (multiples of 64): latent attention expanded to per-head keys and values,
-// where a head's key is [unrotated | rotated | zero pad].  A row is CPR 16-byte chunks; image slot s of row r holds source chunk s ^ f(r).
-// f spreads the rows of a fragment read over the banks: 16-chunk multiples take the 4-bit swizzle of the 128-column image, the others 3 bits
-// (row >> 1 where consecutive rows already lie 32 banks apart).
-template <int COLS>
-struct TileImg {
-    static constexpr int CPR = COLS / 8, ROW = COLS * 2, BYTES = 64 * ROW, PIECES = CPR / 8;   // 1 KiB pieces per wave
-    static_assert(COLS % 64 == 0, "8 waves deal whole pieces");
-    static __device__ __forceinline__ int swz(int row) { return CPR % 16 == 0 ? swz3(row) : (CPR % 16 == 8 && CPR > 8) ? (row >> 1) & 7 : row & 7; }
-    int row[PIECES], col[PIECES];   // this lane's source row inside the tile and source column, per piece
-    __device__ __forceinline__ void init(int w, int l) {
-#pragma unroll
-        for (int i = 0; i < PIECES; ++i) {
-            const int c = (w + 8 * i) * 64 + l;
-            row[i] = c / CPR;
-            col[i] = ((c % CPR) ^ swz(row[i])) * 8;
-        }
-    }
-    __device__ __forceinline__ void dma(const bf16_t* base, long long ld, int row0, int row_last, char* s, int w) const {
-#pragma unroll
-        for (int i = 0; i < PIECES; ++i) glds16_raw(base + (long long)min(row0 + row[i], row_last) * ld + col[i], s + (w + 8 * i) * 1024);
-    }
-    static __device__ __forceinline__ s16x8 rows(const char* s, int r, int kk, int l) {
-        return *reinterpret_cast<const s16x8*>(s + r * ROW + (((2 * kk + (l >> 5)) ^ swz(r)) << 4));
-    }
-    static __device__ __forceinline__ s16x8 columns(const char* s, int rb, int d0, int l) {   // frag_tr3's contract
-        const int r = rb + 4 * (l >> 5) + ((l & 15) >> 2);
-        const int c = d0 + 16 * ((l >> 4) & 1) + 4 * (l & 3);
-        const int ch = c >> 3, within = (c & 7) * 2;
-        const s16x4 a0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(s + r * ROW + ((ch ^ swz(r)) << 4) + within));
-        const s16x4 a1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(s + (r + 8) * ROW + ((ch ^ swz(r + 8)) << 4) + within));
-        s16x8 f;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            f[e] = a0[e];
-            f[4 + e] = a1[e];
-        }
-        return f;
-    }
-};
+// Query / key heads of QD columns beside value heads of VD columns (multiples of 64; TileImg): latent attention expanded to per-head keys and values,
+// where a head's key is [unrotated | rotated | zero pad], and chunk-local attention.
 template <int QD_, int VD_>
 struct FmtQV {
     static constexpr int QD = QD_, VD = VD_, KS = QD / 16, DT = VD / 32, KTILE = TileImg<QD>::BYTES, VTILE = TileImg<VD>::BYTES;
@@ -1452,12 +1397,12 @@ __device__ __forceinline__ void fwd3_step(f32x16 (&st)[2], f32x16 (&sn)[2], f32x
 // in-wave overlap, and with it LDS-DMA staging into the conflict-free images (SQ_LDS_BANK_CONFLICT 0, was 8 % of the LDS cycles) is level
 // with v2's register staging -- so hd 72 stays on v2 by default and both v3 forms are kept selectable (ARIA_ATTN_FWD) as measurements.
 // RAGGED: the sequences of the batch are rows cu[b] .. cu[b + 1] of the token axis (Sq = S = the longest), and every head's output is multiplied
-// by sigmoid(gate[token * ldg + head]) in the epilogue (gate may be NULL).
+// by sigmoid(gate[token * ldg + head]) in the epilogue (gate may be NULL); `group` neighbouring query heads share a key / value head.
 template <class F, int NW, bool PIPE, bool RAGGED>
 __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, const bf16_t* K, const bf16_t* V, bf16_t* O, float* LSE,
                                                         const int32_t* kv_len, const uint8_t* key_mask, int Sq, int S, int H,
                                                         long long ldq, long long ldk, long long ldv, long long ldo, float scale,
-                                                        int causal, int nbatch, const int32_t* cu, const bf16_t* gate, long long ldg) {
+                                                        int causal, int nbatch, const int32_t* cu, const bf16_t* gate, long long ldg, int group) {
     using L = Fwd3Smem<F>;
     constexpr int KS = F::KS, DT = F::DT;
     ARIA_DYN_SMEM(smem);
@@ -1477,8 +1422,9 @@ __global__ __launch_bounds__(NW * 64) void attn_fwd3_kernel(const bf16_t* Q, con
     }
     const long long tok0 = RAGGED ? (long long)cu[b] : (long long)b * S, tokq0 = RAGGED ? tok0 : (long long)b * Sq;
     const bf16_t* Qb = Q + tokq0 * ldq + head * F::QD;
-    const bf16_t* Kb = K + tok0 * ldk + head * F::QD;
-    const bf16_t* Vb = V + tok0 * ldv + head * F::VD;
+    const int kv_head = RAGGED ? head / group : head;
+    const bf16_t* Kb = K + tok0 * ldk + kv_head * F::QD;
+    const bf16_t* Vb = V + tok0 * ldv + kv_head * F::VD;
     const uint8_t* kmb = key_mask ? key_mask + tok0 : nullptr;
     const int q_wmin = q0 + 32 * w, q_abs = q_wmin + (l & 31);
     const int klen = kv_len ? min(S, kv_len[b]) : S;
@@ -1626,7 +1572,7 @@ int aria_attn_fwd(const void* q, const void* k, const void* v, void* o, float* l
         ARIA_LAUNCH((attn_fwd3_kernel<Fmt128, 8, true, false>), dim3(attn_grid((Sq + 255) / 256, H, B)), dim3(512), size_t(Fwd3Smem<Fmt128>::BYTES), stream, Q, K, V,
                     static_cast<bf16_t*>(o), lse, kv_len, key_mask, int(Sq), int(Skv), int(H), (long long)ldq, (long long)ldk,
                     (long long)ldv, (long long)ldo, scale, causal_arg, int(B), static_cast<const int32_t*>(nullptr),
-                    static_cast<const bf16_t*>(nullptr), 0ll);
+                    static_cast<const bf16_t*>(nullptr), 0ll, 1);
     else if (hd == 128)
         ARIA_LAUNCH((attn_fwd2_kernel<128, 8>), dim3(attn_grid((Sq + 255) / 256, H, B)), dim3(512), size_t(Cfg2<128>::SMEM), stream, Q, K, V,
                     static_cast<bf16_t*>(o), lse, kv_len, key_mask, int(Sq), int(Skv), int(H), (long long)ldq, (long long)ldk,
@@ -1647,9 +1593,9 @@ int aria_attn_fwd(const void* q, const void* k, const void* v, void* o, float* l
 }
 
 int aria_attn_varlen_fwd(const void* q, const void* k, const void* v, void* o, const int32_t* cu, const void* gate, int64_t B, int64_t S_max,
-                         int64_t H, int64_t qd, int64_t vd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t ldg, float scale,
-                         void* stream) {
-    if (!q || !k || !v || !o || !cu || B < 0 || S_max < 0 || H <= 0) return ARIA_ERR_INVALID;
+                         int64_t H, int64_t G, int64_t qd, int64_t vd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t ldg,
+                         float scale, void* stream) {
+    if (!q || !k || !v || !o || !cu || B < 0 || S_max < 0 || H <= 0 || G <= 0 || H % G) return ARIA_ERR_INVALID;
     if (!al16(q) || !al16(k) || !al16(v) || (ldq & 7) || (ldk & 7) || (ldv & 7) || (ldo & 3) || (reinterpret_cast<uintptr_t>(o) & 7))
         return ARIA_ERR_ALIGN;
     const bool known = (qd == 64 && vd == 64) || (qd == 128 && vd == 128) || (qd == 192 && vd == 128) || (qd == 256 && vd == 256);
@@ -1661,7 +1607,7 @@ int aria_attn_varlen_fwd(const void* q, const void* k, const void* v, void* o, c
                 static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k), static_cast<const bf16_t*>(v), static_cast<bf16_t*>(o),           \
                 static_cast<float*>(nullptr), static_cast<const int32_t*>(nullptr), static_cast<const uint8_t*>(nullptr), int(S_max),           \
                 int(S_max), int(H), (long long)ldq, (long long)ldk, (long long)ldv, (long long)ldo, scale, causal, int(B), cu,                  \
-                static_cast<const bf16_t*>(gate), (long long)ldg)
+                static_cast<const bf16_t*>(gate), (long long)ldg, int(H / G))
     using F64 = FmtQV<64, 64>;
     using F192 = FmtQV<192, 128>;
     using F256 = FmtQV<256, 256>;

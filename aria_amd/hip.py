@@ -24,7 +24,7 @@ ERRORS = {
 P, I64, I32, F32 = c_void_p, c_int64, c_int, c_float
 RESTYPES = {"aria_gemm_workspace_bytes": c_int64, "aria_decode_scratch_bytes": c_int64, "aria_decode_graph_create": c_void_p,
             "aria_decode_graph_destroy": None, "aria_decode_attn_workspace_bytes": c_int64,
-            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64}  # everything else returns an int status
+            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64, "aria_linear_chunks_scratch": c_int64}  # everything else returns an int status
 
 # name -> argtypes (all return int).  Kept in one table so tests can check that the shared
 # library exports every symbol the header declares.
@@ -101,7 +101,7 @@ SIGNATURES = {
     "aria_gather_add_rows": [P, P, P, I64, I64, P],
     "aria_colsum_bf16": [P, P, I64, I64, I64, I64, P],
     "aria_cross_entropy": [P, P, P, P, P, F32, P, I64, I64, I64, P],
-    "aria_attn_varlen_fwd": [P, P, P, P, P, P, I64, I64, I64, I64, I64, I64, I64, I64, I64, I64, F32, P],
+    "aria_attn_varlen_fwd": [P, P, P, P, P, P, I64, I64, I64, I64, I64, I64, I64, I64, I64, I64, I64, F32, P],
     "aria_dyt_stream": [P, P, P, P, P, I64, P, P, P, P, I64, I64, I64, I32, P],
     "aria_act_rows": [P, P, P, I64, I64, I64, I64, I32, I32, P],
     "aria_gemm_f32": [P, P, P, I64, I64, I64, I64, I64, I64, P, I64, I64, P],
@@ -118,6 +118,8 @@ SIGNATURES = {
     "aria_chunk_attn_any": [P, P, P, P, P, P, P, P, I64, I32, P],
     "aria_chunk_rows": [P, P, P, P, P, P, P, I64, I32, P],
     "aria_linear_step": [P, P, P, P, P, P, I64, P, I32, P],
+    "aria_linear_chunks_scratch": [P, I64, I64, I64],
+    "aria_linear_chunks": [P, P, P, P, P, P, I64, P, I64, P, I64, P, I64, P, I64, P],
     "aria_norm_gate": [P, P, I64, P, I64, P, I64, I64, I64, I64, F32, I32, I32, P],
 }
 

@@ -18,6 +18,7 @@ from .layers import ChunkAttention, LinearAttention, MixerGroup, ReluGatedFeedFo
 from .registry import read_config
 
 bf16, f32 = torch.bfloat16, torch.float32
+DECODE_ROWS = 16
 
 
 @dataclass

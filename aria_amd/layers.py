@@ -223,7 +223,16 @@ class ChunkAttention(nn.Module):
         return ChunkCache(slots, max_len, g["G"], g["size"], g["dq"] + g["dvp"], self.dtype, device)
 
     def forward(self, proj: torch.Tensor, batch, cache: ChunkCache) -> torch.Tensor:
-        return ops.linear_any(ops.chunk_attention_any(self.shape(cache), proj, cache.rows, batch), self.w_o)
+        g, s = self.geometry, self.shape(cache)
+        if batch.fresh and batch.longest > 1 and self.flash:
+            # whole prompts: every chunk is a sequence of its own
+            cu, longest = batch.chunks(g["size"])
+            q, k, v = (proj[:, g[n]:] for n in ("q_off", "k_off", "v_off"))
+            o = ops.attention_varlen(q, k, v, cu, longest, g["H"], g["dq"], g["dvp"], g["scale"], kv_heads=g["G"])
+            ops.chunk_rows(s, proj, cache.rows, batch)
+        else:
+            o = ops.chunk_attention_any(s, proj, cache.rows, batch)
+        return ops.linear_any(o, self.w_o)
 
 
 class LinearState:
@@ -281,7 +290,8 @@ class LinearAttention(nn.Module):
         return LinearState(slots, g["H"], g["dp"], g["dvp"], device)
 
     def forward(self, proj: torch.Tensor, batch, cache: LinearState) -> torch.Tensor:
-        o = ops.linear_step(self.shape(), proj, cache.rows, batch)
+        run = ops.linear_chunks if self.chunked and batch.longest > 1 else ops.linear_step
+        o = run(self.shape(), proj, cache.rows, batch)
         o = ops.norm_gate(o, proj[:, self.g_off:self.g_off + o.shape[1]], self.norm, self.norm_groups, self.norm_n, self.eps, self.silu_gate)
         return ops.linear_any(o, self.w_o)
 

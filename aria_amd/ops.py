@@ -1090,14 +1090,14 @@ def varlen_head(qd: int, vd: int) -> Optional[Tuple[int, int]]:
 
 
 def attention_varlen(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu: torch.Tensor, S_max: int, H: int, qd: int, vd: int, scale: float,
-                     gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """Causal attention of packed sequences (sequence b = rows cu[b] .. cu[b + 1)): q, k [T, >= H qd], v [T, >= H vd] views, gate [T, >= H] logits of
-    a per-head sigmoid gate -> [T, H vd]."""
+                     gate: Optional[torch.Tensor] = None, kv_heads: Optional[int] = None) -> torch.Tensor:
+    """Causal attention of packed sequences (sequence b = rows cu[b] .. cu[b + 1)): q [T, >= H qd], k [T, >= G qd], v [T, >= G vd] views (G = ``kv_heads``,
+    default H), gate [T, >= H] logits of a per-head sigmoid gate -> [T, H vd]."""
     for t, n in ((q, "q"), (k, "k"), (v, "v")):
         _chk(t, name=n)
     _chk(cu, torch.int32, "cu")
     out = torch.empty((q.shape[0], H * vd), dtype=bf16, device=q.device)
-    hip.get_lib().call("aria_attn_varlen_fwd", _p(q), _p(k), _p(v), _p(out), _p(cu), _p(gate), cu.numel() - 1, S_max, H, qd, vd, _rowmajor_2d(q, "q"),
+    hip.get_lib().call("aria_attn_varlen_fwd", _p(q), _p(k), _p(v), _p(out), _p(cu), _p(gate), cu.numel() - 1, S_max, H, kv_heads or H, qd, vd, _rowmajor_2d(q, "q"),
                        _rowmajor_2d(k, "k"), _rowmajor_2d(v, "v"), H * vd, _rowmajor_2d(gate, "gate") if gate is not None else 0, float(scale), _stream(q))
     return out
 
@@ -1231,6 +1231,27 @@ def linear_step(shape, proj: torch.Tensor, state: torch.Tensor, batch) -> torch.
     out = torch.empty((T, shape.H * shape.dvp), dtype=proj.dtype, device=proj.device)
     hip.get_lib().call("aria_linear_step", _p(proj), ctypes.byref(shape), _p(state), _p(batch.slot), _p(batch.pos), _p(batch.cu), len(batch.lengths), _p(out),
                        _f32(proj), _stream(proj))
+    return out
+
+
+LINEAR_BLOCK = 64   # rows of a matrix-pipe step of aria_linear_chunks
+
+
+def linear_chunks(shape, proj: torch.Tensor, state: torch.Tensor, batch) -> torch.Tensor:
+    """``linear_step`` for prompts in bf16 on the matrix pipe, chunks of a sequence side by side.  Rewrites the q, k, v columns of ``proj``."""
+    import ctypes
+
+    T = _chk_rows(_chk(proj), shape.ldp, batch)
+    _chk_state(shape, state, batch)
+    # about one workgroup per compute unit: chunks x heads x 128-column blocks of the values
+    rows = max(1, T * shape.H * ((shape.dvp + 127) // 128) // 256)
+    blocks, chunks, seqs = batch.linear_tables(LINEAR_BLOCK, max(1, -(-rows // LINEAR_BLOCK)))
+    lib, ref = hip.get_lib(), ctypes.byref(shape)
+    nb, nc, ns = blocks.shape[0], chunks.shape[0], seqs.shape[0]
+    scratch = torch.empty(int(lib.cdll.aria_linear_chunks_scratch(ref, T, nb, nc)), dtype=torch.uint8, device=proj.device)
+    out = torch.empty((T, shape.H * shape.dvp), dtype=bf16, device=proj.device)
+    lib.call("aria_linear_chunks", _p(proj), ref, _p(state), _p(batch.slot), _p(batch.pos), _p(blocks), nb, _p(chunks), nc, _p(seqs), ns, _p(out), T,
+             _p(scratch), scratch.numel(), _stream(proj))
     return out
 
 

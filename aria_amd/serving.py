@@ -46,6 +46,23 @@ class StepBatch:
             self.made["chunks", size] = (torch.tensor(cu, dtype=torch.int32).to(self.ids.device), min(size, self.longest))
         return self.made["chunks", size]
 
+    def linear_tables(self, block: int, per_chunk: int):
+        """The sequences cut into blocks of up to ``block`` rows, ``per_chunk`` of them (the last ones of a sequence: fewer) a chunk; int32 on the device:
+        blocks (first row, rows), chunks (first block, blocks, first of its sequence, last of it), sequences (first chunk, chunks)."""
+        if ("linear", block, per_chunk) not in self.made:
+            blocks, chunks, seqs, row = [], [], [], 0
+            for n in self.lengths:
+                b0, c0 = len(blocks), len(chunks)
+                blocks += [(row + at, min(block, n - at)) for at in range(0, n, block)]
+                firsts = range(b0, len(blocks), per_chunk)
+                chunks += [(b, min(per_chunk, len(blocks) - b), int(b == b0), int(b == firsts[-1])) for b in firsts]
+                seqs.append((c0, len(chunks) - c0))
+                row += n
+            flat = torch.tensor([x for t in (blocks, chunks, seqs) for r in t for x in r], dtype=torch.int32).to(self.ids.device)
+            nb, nc = 2 * len(blocks), 4 * len(chunks)
+            self.made["linear", block, per_chunk] = (flat[:nb].view(-1, 2), flat[nb:nb + nc].view(-1, 4), flat[nb + nc:].view(-1, 2))
+        return self.made["linear", block, per_chunk]
+
     def wanted_by_sequence(self) -> List[List[int]]:
         """per sequence: the wanted places among its own tokens, in order"""
         out, first = [], 0

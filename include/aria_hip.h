@@ -344,9 +344,10 @@ int aria_attn_bwd_rope(const void* q, const void* k, const void* v, const void* 
 /* Causal attention over a batch of sequences of unequal length packed on the token axis (sequence b = rows cu[b] .. cu[b + 1), S_max = the
  * longest), with query / key heads of qd columns beside value heads of vd columns (zero-padded by the caller to one of 64 / 64, 128 / 128,
  * 192 / 128, 256 / 256), and -- gate != NULL -- every head's output multiplied by sigmoid(gate[token * ldg + head]) in the epilogue.  The kernel
- * is aria_attn_fwd's LDS-DMA form on other tile images.  q [T, H, qd], k [T, H, qd], v [T, H, vd] -> o [T, H, vd] as views with row strides ld*. */
+ * is aria_attn_fwd's LDS-DMA form on other tile images.  q [T, H, qd], k [T, G, qd], v [T, G, vd] -> o [T, H, vd] as views with row strides ld*; query
+ * head h reads key / value head h / (H / G). */
 int aria_attn_varlen_fwd(const void* q, const void* k, const void* v, void* o, const int32_t* cu, const void* gate, int64_t B, int64_t S_max,
-                         int64_t H, int64_t qd, int64_t vd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t ldg, float scale,
+                         int64_t H, int64_t G, int64_t qd, int64_t vd, int64_t ldq, int64_t ldk, int64_t ldv, int64_t ldo, int64_t ldg, float scale,
                          void* stream);
 
 /* which backward the calling thread's last aria_attn_bwd ran: 2 = padded-tile pair (hd 64 / 72), 5 = role-split dK/dV + dQ v5 (hd 128) */
@@ -586,6 +587,15 @@ typedef struct {
  * holds; out [T, H dvp]. */
 int aria_linear_step(const void* proj, const AriaLinearShape* s, float* state, const int32_t* slot, const int32_t* pos, const int32_t* cu, int64_t n_seq,
                      void* out, int f32, void* stream);
+
+/* Whole prompts and long portions in bf16 on the matrix pipe: dp 64, 128 or 256, dvp a multiple of 64 (else ARIA_ERR_UNSUPPORTED).  The sequences are cut into
+ * runs of up to 64 rows, blocks[i] = (first row, rows), and consecutive runs of a sequence form chunks, chunks[i] = (first run, runs, 1 for the
+ * first chunk of its sequence, 1 for the last); seqs[i] = (first chunk, chunks).  int32 on the device.  Rewrites the q and k (silu: and v) columns of
+ * proj.  scratch: aria_linear_chunks_scratch bytes, 16-byte aligned. */
+int64_t aria_linear_chunks_scratch(const AriaLinearShape* s, int64_t T, int64_t n_blocks, int64_t n_chunks);
+int aria_linear_chunks(void* proj, const AriaLinearShape* s, float* state, const int32_t* slot, const int32_t* pos, const int32_t* blocks, int64_t n_blocks,
+                       const int32_t* chunks, int64_t n_chunks, const int32_t* seqs, int64_t n_seq, void* out, int64_t T, void* scratch,
+                       int64_t scratch_bytes, void* stream);
 
 /* y = o / sqrt(sum(o^2) / n + eps) w act(gate) per (row, group of cols columns): act = silu, or sigmoid (silu == 0); w [groups, cols] with w_stride
  * between groups (0: shared).  o [T, groups cols], gate rows ldg apart.  cols % 8 == 0; y may be o. */
