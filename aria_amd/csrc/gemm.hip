@@ -483,6 +483,22 @@ int aria_gemm_swiglu_bf16(const void* A, const void* B, void* H, void* ACT, int6
     return g_last_variant = 3, aria_launch_gemm3(p, 0, 0, int((M + 255) / 256), stream);
 }
 
+int aria_gemm_relu_glu_bf16(const void* A, const void* B, void* ACT, int64_t M, int64_t N2, int64_t K, int64_t lda, int64_t ldb, int64_t ldact, void* stream) {
+    const int rc = glu_check(A, B, nullptr, ACT, M, N2, K, lda, ldb, 0, ldact);
+    if (rc != ARIA_OK) return rc;
+    if (2 * M * lda >= (1ll << 32) || 2 * N2 * ldb >= (1ll << 32)) return ARIA_ERR_UNSUPPORTED;
+    if (M == 0) return ARIA_OK;
+    GemmParams p{};
+    p.A = static_cast<const bf16_t*>(A);
+    p.B = static_cast<const bf16_t*>(B);   // [N2, K] row-major: gate rows, then up rows
+    p.C2 = ACT;
+    p.lda = lda, p.ldb = ldb, p.ldc2 = ldact;
+    p.M = int(M), p.N = int(N2), p.K = int(K);
+    p.mode = 0;
+    p.glu = 2;
+    return g_last_variant = 3, aria_launch_gemm3(p, 0, 0, int((M + 255) / 256), stream);
+}
+
 // gate / up weights as two [.., I, K] tensors of one allocation (gptfast's w1 / w3): rows of the up tensor as an offset from the gate tensor
 static int glu_split_rows(const void* Bg, const void* Bu, int64_t I, int64_t ldb, int64_t extra_rows, int* up_rows) {
     const long long diff = static_cast<const char*>(Bu) - static_cast<const char*>(Bg);

@@ -721,7 +721,8 @@ __device__ __forceinline__ int wave_blk_off(int row, int pair) { return row * 64
 // is given, the two halves of h -> C.
 __device__ __forceinline__ float silu3(float a) { return silu_fast(a); }
 
-template <class P>
+// RELU: the gate activation is max(z, 0) (the form has no use for the un-activated halves: C is ignored).
+template <bool RELU, class P>
 __device__ __forceinline__ void store_tile3_glu(const P& p, const f32x16 (&acc)[2][2][2], char* C, int m0, int m_end, int n0, int l, int w,
                                                 int wm, int wn, char* smem) {
     const int c = l & 31, h = l >> 5;
@@ -742,11 +743,13 @@ __device__ __forceinline__ void store_tile3_glu(const P& p, const f32x16 (&acc)[
                 for (int j = 0; j < 4; ++j) {
                     g[j] = rbf(acc[a][i][0][4 * q + j]);
                     u[j] = rbf(acc[a][i][1][4 * q + j]);
-                    y[j] = rbf(silu3(g[j])) * u[j];
+                    y[j] = (RELU ? fmaxf(g[j], 0.f) : rbf(silu3(g[j]))) * u[j];
                 }
                 const int off = wave_blk_off(i * 32 + c, q) + 8 * h;
-                *reinterpret_cast<u32x2*>(mine + off) = u32x2{pack2bf(g[0], g[1]), pack2bf(g[2], g[3])};
-                *reinterpret_cast<u32x2*>(mine + 4096 + off) = u32x2{pack2bf(u[0], u[1]), pack2bf(u[2], u[3])};
+                if (!RELU) {
+                    *reinterpret_cast<u32x2*>(mine + off) = u32x2{pack2bf(g[0], g[1]), pack2bf(g[2], g[3])};
+                    *reinterpret_cast<u32x2*>(mine + 4096 + off) = u32x2{pack2bf(u[0], u[1]), pack2bf(u[2], u[3])};
+                }
                 *reinterpret_cast<u32x2*>(mine + 8192 + off) = u32x2{pack2bf(y[0], y[1]), pack2bf(y[2], y[3])};
             }
         wave_barrier();
@@ -760,7 +763,7 @@ __device__ __forceinline__ void store_tile3_glu(const P& p, const f32x16 (&acc)[
             const u32x4 vu = *reinterpret_cast<const u32x4*>(mine + 4096 + off);
             const u32x4 vy = *reinterpret_cast<const u32x4*>(mine + 8192 + off);
             if (m < m_end) {
-                if (H) {
+                if (!RELU && H) {
                     *reinterpret_cast<u32x4*>(H + (long long)m * p.ldc + n) = vg;
                     *reinterpret_cast<u32x4*>(H + (long long)m * p.ldc + I + n) = vu;
                 }
@@ -1071,8 +1074,12 @@ __global__ __launch_bounds__(512) void gemm3_kernel(GemmParams p) {
         store_tile3_rows_rope_hf(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
         return;
     }
+    if (VER == 13) {  // relu-gated pair: its own instantiation
+        store_tile3_glu<true>(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
+        return;
+    }
     if (p.glu)
-        store_tile3_glu(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
+        store_tile3_glu<false>(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
     else if (p.act == 1)  // (one wave-uniform branch here instead of one per value inside the unrolled epilogues)
         store_any3<1>(p, acc, C, m0, m_end, n0, l, w, wm, wn, smem);
     else if (!A_OC && !B_OC && VER == 3 && p.act == 2)
@@ -1224,6 +1231,11 @@ int aria_launch_gemm3(const GemmParams& p, int a_oc, int b_oc, int ntm, void* st
             ARIA_LAUNCH((gemm3_kernel<false, false, 9>), grid, block, shmem, stream, q);
         else
             ARIA_LAUNCH((gemm3_kernel<false, true, 8>), grid, block, shmem, stream, q);
+        return aria_check_launch();
+    }
+    if (p.glu == 2) {  // relu gate: dense, [gate | up] rows
+        if (a_oc || b_oc || p.mode != 0 || p.glu_up_rows > 0 || p.ext_k) return ARIA_ERR_INVALID;
+        ARIA_LAUNCH((gemm3_kernel<false, false, 13>), grid, block, shmem, stream, q);
         return aria_check_launch();
     }
     if (p.glu && p.glu_up_rows > 0) {  // fused SwiGLU with gate / up weights in two tensors ([N, K] form): its own instantiation

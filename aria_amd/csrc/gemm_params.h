@@ -24,7 +24,7 @@ struct GemmParams {
     // operand holds [gate | up] columns (N = 2 I); a workgroup's two 128-column B halves are gate columns n0.. and up columns I + n0..,
     // so gate and up of one output element meet in one lane.  C2 [M, I] receives silu(gate) * up with the reference's rounding points;
     // C ([M, 2 I], may be null) the un-activated product.
-    int glu;
+    int glu;   // 1: silu gate, 2: relu gate (dense, [gate | up] rows, C2 only)
     void* C2;
     long long ldc2;
     int reserved0;   // (was the round-2 start-up stagger experiment; the field keeps the kernarg offsets of what follows)

@@ -6,7 +6,8 @@
 // never expands: the query moves into latent space once (q W_uk, per head), scores are dot products with the cache rows as they lie in memory, and
 // the weighted sum of latents is expanded through W_uv at the end.  A cache row is then read ONCE for 16 or 32 heads, which makes decode
 // attention a matrix product with the heads as rows (v_mfma_f32_16x16x32_bf16) whose operand streams from HBM.
-#include "elem.h"
+#include "rows.h"
+#include "tile_attn.h"
 #include <cstdlib>
 
 namespace {
@@ -165,197 +166,6 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const T* proj, Shape
     }
 }
 
-// ---------------------------------------------------------------------------------------------- decode attention, matrix pipe (bf16)
-// One workgroup of 8 waves: one token, NG groups of 16 heads, a contiguous range of 64-row cache tiles.  Tiles arrive by LDS-DMA, double-buffered,
-// chunk slot = chunk ^ tile_swz(row).  Per tile: wave w scores rows 16 (w & 3) .. against head group w >> 2 (NG = 1: against the half of the reduction
-// w >> 2; cache rows are k-contiguous B fragments as they lie) and parks the scores in LDS; wave w then owns the softmax of 2 NG heads, a lane per
-// row (DPP reductions, running maximum and sum in registers), and publishes probabilities (bf16) and rescale factors; last, wave w accumulates DTW
-// 16-column slices of the latent output over all 64 rows (V fragments by transposing reads of the same tile).  Softmax in the log2 domain, fp32.
-// XOR of a chunk index inside its group of 8: a row is an odd multiple of 32 banks (or an even one) behind its neighbour, so the 16 rows of a score
-// fragment (8 of either parity) need 8 different values, and the 16 (row, 32-byte) pairs of a transposing read need all four upper-bit values twice
-__device__ __forceinline__ int tile_swz(int row) { return ((((row >> 1) ^ (row >> 3)) & 3) << 1) | ((row >> 3) & 1); }
-template <int NG, int DTW, int KTM>
-__global__ __launch_bounds__(512) void latent_attn_kernel(const bf16_t* qa, const bf16_t* cache, Shape s, const int32_t* slot, const int32_t* pos,
-                                                          float* part_o, float* part_ml, int splits) {
-    ARIA_DYN_SMEM(smem);
-    constexpr int PP = 72, SPI = 66;   // pitches of the probability tile (bf16) and of the score tile (fp32)
-    constexpr int NP = NG == 1 ? 2 : 1;   // partial score tiles (halves of the reduction)
-    constexpr int KW = (KTM + NP - 1) / NP, HW = 2 * NG;
-    const int t = threadIdx.x, l = t & 63, w = first_lane(t >> 6), q4 = l >> 4, c16 = l & 15;
-    const int CPR = int(s.cw) >> 3, KT = int(s.cw) >> 5, tile_bytes = 64 * int(s.cw) * 2;
-    float* sS = reinterpret_cast<float*>(smem + 2 * tile_bytes);                 // [NP][NG * 16][SPI]
-    bf16_t* sP = reinterpret_cast<bf16_t*>(sS + NP * NG * 16 * SPI);             // [NG * 16][PP]
-    float* sA = reinterpret_cast<float*>(sP + NG * 16 * PP);                     // [NG * 16]
-    const int sp = blockIdx.x, hg = blockIdx.y, tok = blockIdx.z;
-    const int n_keys = pos[tok] + 1, ntiles = (n_keys + 63) / 64, per = (ntiles + splits - 1) / splits;
-    const int it0 = sp * per, it1 = min(ntiles, it0 + per);
-    const int head0 = hg * NG * 16;
-    float* ml = part_ml + ((long long)tok * splits + sp) * s.H * 2;
-    if (it0 >= it1) {   // nothing to see for this split
-        if (t < NG * 16 && head0 + t < s.H) {
-            ml[2 * (head0 + t)] = -INFINITY;
-            ml[2 * (head0 + t) + 1] = 0.f;
-        }
-        return;
-    }
-    const bf16_t* base = cache + (long long)slot[tok] * s.S_cap * s.cw;
-    // this lane's chunk of the wave's first DMA piece, and the step to its next one (8 pieces of 64 chunks further on)
-    const int row_i = (w * 64 + l) / CPR, slot_i = (w * 64 + l) % CPR, dr_ = 512 / CPR, ds_ = 512 % CPR;
-    auto dma = [&](int tile, char* dst) __attribute__((always_inline)) {
-        int row = row_i, sl = slot_i;
-        for (int pc = w; pc < CPR; pc += 8) {
-            const int ch = sl ^ tile_swz(row);
-            glds16_raw(base + (long long)min(tile * 64 + row, n_keys - 1) * s.cw + ch * 8, dst + pc * 1024);
-            row += dr_;
-            sl += ds_;
-            if (sl >= CPR) {
-                sl -= CPR;
-                row += 1;
-            }
-        }
-    };
-    dma(it0, smem);
-    const int g = NG == 1 ? 0 : w >> 2, k_first = NG == 1 ? (w >> 2) * KW : 0, krow = 16 * (w & 3) + c16;
-    s16x8 qf[KW];
-#pragma unroll
-    for (int kk = 0; kk < KW; ++kk) {
-        u32x4 v = zero16();
-        const int head = head0 + g * 16 + c16;
-        if (head < s.H && k_first + kk < KT) v = ld16(qa + ((long long)tok * s.H + head) * s.cw + (k_first + kk) * 32 + q4 * 8);
-        qf[kk] = __builtin_bit_cast(s16x8, v);
-    }
-    f32x4 o[NG][DTW];
-#pragma unroll
-    for (int gg = 0; gg < NG; ++gg)
-#pragma unroll
-        for (int i = 0; i < DTW; ++i) o[gg][i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    float m[HW], lsum[HW];
-#pragma unroll
-    for (int j = 0; j < HW; ++j) {
-        m[j] = -INFINITY;
-        lsum[j] = 0.f;
-    }
-#pragma unroll
-    for (int kk = 0; kk < KW; ++kk) settle(qf[kk]);
-    const float scale2 = s.scale * 1.4426950408889634f;
-    for (int it = it0; it < it1; ++it) {
-        const char* cur = smem + ((it - it0) & 1) * tile_bytes;
-        wait_vm<0>();
-        sync();   // tile `it` is complete; every wave is done with the other buffer and the probabilities
-        if (it + 1 < it1) dma(it + 1, smem + ((it - it0 + 1) & 1) * tile_bytes);
-        {   // scores: C rows = heads 4 q4 + r of group g, columns = cache rows
-            // (no branch on the row's width: blocks past it read the last chunk against zero query fragments; the next group's fragments are
-            // requested in front of this group's multiply-adds)
-            constexpr int GQ = KW % 3 == 0 ? 3 : 5;
-            f32x4 sc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
-            const char* kbase = cur + krow * CPR * 16;
-            const int fx = tile_swz(krow);
-            s16x8 kf[2][GQ];
-            auto fetch = [&](int kk, s16x8& f) __attribute__((always_inline)) {
-                f = *reinterpret_cast<const s16x8*>(kbase + ((min((k_first + kk) * 4 + q4, CPR - 1) ^ fx) << 4));
-            };
-#pragma unroll
-            for (int u = 0; u < GQ; ++u) fetch(u, kf[0][u]);
-#pragma unroll
-            for (int k0 = 0; k0 < KW; k0 += GQ) {
-                if (k0 + GQ < KW) {
-#pragma unroll
-                    for (int u = 0; u < GQ; ++u) fetch(k0 + GQ + u, kf[(k0 / GQ + 1) & 1][u]);
-                }
-                sched_fence();
-#pragma unroll
-                for (int u = 0; u < GQ; ++u) sc[u & 1] = mfma16(qf[k0 + u], kf[(k0 / GQ) & 1][u], sc[u & 1]);
-                sched_fence();
-            }
-            float* dst = sS + ((NG == 1 ? w >> 2 : 0) * NG * 16 + g * 16 + 4 * q4) * SPI + krow;
-#pragma unroll
-            for (int r = 0; r < 4; ++r) dst[r * SPI] = sc[0][r] + sc[1][r];
-        }
-        sync();
-        // softmax: lane = row of the tile
-        const bool dead = it * 64 + l >= n_keys;
-        float x[HW], mx[HW];
-#pragma unroll
-        for (int j = 0; j < HW; ++j) {
-            x[j] = sS[(w * HW + j) * SPI + l];
-            if (NP == 2) x[j] += sS[(NG * 16 + w * HW + j) * SPI + l];
-        }
-#pragma unroll
-        for (int j = 0; j < HW; ++j) mx[j] = x[j] = dead ? -INFINITY : x[j] * scale2;
-        wave_max_bcast_n<HW>(mx);
-#pragma unroll
-        for (int j = 0; j < HW; ++j) {
-            const float mn = fmaxf(m[j], mx[j]);   // finite: a tile holds at least one visible row
-            const float alpha = exp2_fast(m[j] - mn), p = exp2_fast(x[j] - mn);
-            m[j] = mn;
-            lsum[j] = lsum[j] * alpha + p;
-            sP[(w * HW + j) * PP + l] = f2bf(p);
-            if (l == 0) sA[w * HW + j] = alpha;
-        }
-        sync();
-        // latent output: A = probabilities (heads x 32 rows), B = the tile's columns
-#pragma unroll
-        for (int gg = 0; gg < NG; ++gg) {
-            const f32x4 al = *reinterpret_cast<const f32x4*>(sA + gg * 16 + 4 * q4);
-#pragma unroll
-            for (int i = 0; i < DTW; ++i)
-#pragma unroll
-                for (int r = 0; r < 4; ++r) o[gg][i][r] *= al[r];
-        }
-        s16x8 pf[2][NG], vf[2][DTW];
-        auto fetch_v = [&](int kk) __attribute__((always_inline)) {
-#pragma unroll
-            for (int gg = 0; gg < NG; ++gg) pf[kk][gg] = *reinterpret_cast<const s16x8*>(sP + (gg * 16 + c16) * PP + kk * 32 + q4 * 8);
-            const int vr = kk * 32 + q4 * 8 + (c16 >> 2);
-#pragma unroll
-            for (int i = 0; i < DTW; ++i) {
-                const int d0 = min((w * DTW + i) * 16, int(s.cw) - 16);   // (slices past the row: any columns, their results are dropped)
-                const int col = d0 + 4 * (c16 & 3), ch = col >> 3, within = (col & 7) * 2;
-                const s16x4 a0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + vr * CPR * 16 + ((ch ^ tile_swz(vr)) << 4) + within));
-                const s16x4 a1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(cur + (vr + 4) * CPR * 16 + ((ch ^ tile_swz(vr + 4)) << 4) + within));
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    vf[kk][i][e] = a0[e];
-                    vf[kk][i][4 + e] = a1[e];
-                }
-            }
-        };
-        fetch_v(0);
-#pragma unroll
-        for (int kk = 0; kk < 2; ++kk) {
-            if (kk == 0) fetch_v(1);
-            sched_fence();
-#pragma unroll
-            for (int i = 0; i < DTW; ++i)
-#pragma unroll
-                for (int gg = 0; gg < NG; ++gg) o[gg][i] = mfma16(pf[kk][gg], vf[kk][i], o[gg][i]);
-            sched_fence();
-        }
-    }
-#pragma unroll
-    for (int j = 0; j < HW; ++j) {
-        const float v = wave_sum_bcast(lsum[j]);
-        const int head = head0 + w * HW + j;
-        if (l == 0 && head < s.H) {
-            ml[2 * head] = m[j];
-            ml[2 * head + 1] = v;
-        }
-    }
-#pragma unroll
-    for (int gg = 0; gg < NG; ++gg)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int head = head0 + gg * 16 + 4 * q4 + r;
-            if (head >= s.H) continue;
-            float* po = part_o + (((long long)tok * splits + sp) * s.H + head) * s.R;
-#pragma unroll
-            for (int i = 0; i < DTW; ++i) {
-                const int d = (w * DTW + i) * 16 + c16;
-                if (d < s.R) po[d] = o[gg][i][r];
-            }
-        }
-}
-
 // ---------------------------------------------------------------------------------------------- decode attention, any size (fp32 or bf16)
 // One workgroup per (head, token), a thread per cache row of a 256-row tile, then a thread per latent column.
 constexpr int ANY_COLS = 8;   // latent columns per thread: R <= 2048
@@ -425,7 +235,7 @@ __global__ __launch_bounds__(256) void latent_attn_any_kernel(const T* qa, const
 
 // ---------------------------------------------------------------------------------------------- decode: merge, expand, gate
 constexpr int EXP_ROWS = 32;       // value columns per workgroup: 4 per wave
-constexpr int MAX_SPLITS = 64;
+constexpr int MAX_SPLITS = TILE_MAX_SPLITS;
 template <class T>
 __global__ __launch_bounds__(512) void latent_expand_kernel(const float* part_o, const float* part_ml, Shape s, const T* proj, const T* uv, T* out,
                                                             int splits) {
@@ -494,48 +304,7 @@ __global__ __launch_bounds__(512) void latent_expand_kernel(const float* part_o,
     }
 }
 
-// ---------------------------------------------------------------------------------------------- decode: row-streaming projections (bf16)
-__device__ __forceinline__ u32x4 ldw16(const bf16_t* p) {   // a weight stream is read once: non-temporal
-#ifdef ARIA_EMU
-    return ld16(p);
-#else
-    return __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(p));
-#endif
-}
-// acc[r][b] += W[row r] . X[token b], a wave over two weight rows and NB token rows: four 16-byte chunks per row and lane requested before the
-// first use, the token rows come from the L1 / L2
-template <int NB>
-__device__ __forceinline__ void two_rows(float (&acc)[2][NB], const bf16_t* w0, const bf16_t* w1, const bf16_t* x, long long ldx, int nb, int K, int l) {
-    const int nch = K >> 3;
-    for (int c0 = l; c0 < nch; c0 += 256) {
-        u32x4 a[2][4];
-#pragma unroll
-        for (int u = 0; u < 4; ++u) {
-            const int c = min(c0 + 64 * u, nch - 1);
-            a[0][u] = ldw16(w0 + c * 8);
-            a[1][u] = ldw16(w1 + c * 8);
-        }
-#pragma unroll
-        for (int b = 0; b < NB; ++b) {
-            const bf16_t* xr = x + (long long)min(b, nb - 1) * ldx;
-#pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                u32x4 v = ld16(xr + min(c0 + 64 * u, nch - 1) * 8);
-                const bool in = c0 + 64 * u < nch;
-#pragma unroll
-                for (int q = 0; q < 4; ++q) {
-                    const uint32_t xv = in ? v[q] : 0u;
-                    acc[0][b] = dot2bf(a[0][u][q], xv, acc[0][b]);
-                    acc[1][b] = dot2bf(a[1][u][q], xv, acc[1][b]);
-                }
-            }
-        }
-    }
-#pragma unroll
-    for (int r = 0; r < 2; ++r)
-#pragma unroll
-        for (int b = 0; b < NB; ++b) acc[r][b] = wave_sum_bcast(acc[r][b]);
-}
+// ---------------------------------------------------------------------------------------------- decode: epilogues of the projections (rows.h)
 // the residual step of one stream element: x += post(v), and the next norm of the new x
 __device__ __forceinline__ void stream_step(float v, const AriaDyT& post, const AriaDyT& next, float* x, bf16_t* h, long long at, int n) {
     const float xn = x[at] + dyt<bf16_t>(post, v, n);
@@ -551,75 +320,19 @@ struct RowsOut {
     bf16_t* h;
 };
 template <int MODE>
-__device__ __forceinline__ void rows_finish(const RowsOut& ro, float v, int tok, int n) {
-    const long long at = (long long)tok * ro.ldo + n;
-    if (MODE == ROWS_BF16) static_cast<bf16_t*>(ro.out)[at] = f2bf(v);
-    if (MODE == ROWS_RELU2) static_cast<bf16_t*>(ro.out)[at] = f2bf(relu_squared(v));
-    if (MODE == ROWS_F32) static_cast<float*>(ro.out)[at] = v;
-    if (MODE == ROWS_STREAM) stream_step(v, ro.post, ro.next, ro.x, ro.h, at, n);
-}
-// one token: a wave per two weight rows
-template <int MODE>
-__global__ __launch_bounds__(256) void row_kernel(const bf16_t* W, const bf16_t* X, int K, int N, RowsOut ro) {
-    const int l = threadIdx.x & 63, w = threadIdx.x >> 6;
-    const int row0 = (blockIdx.x * 4 + w) * 2;
-    if (row0 >= N) return;
-    float acc[2][1] = {{0.f}, {0.f}};
-    two_rows<1>(acc, W + (long long)row0 * K, W + (long long)min(row0 + 1, N - 1) * K, X, 0, 1, K, l);
-    if (l < 2 && row0 + l < N) rows_finish<MODE>(ro, l ? acc[1][0] : acc[0][0], 0, row0 + l);
-}
-// 2 .. 16 tokens: a workgroup per 16 RG weight rows, its NW waves on interleaved 128-column blocks of the reduction.  Tokens are the
-// rows of A, weight rows the columns of B: both k-contiguous in memory, so fragments come straight from global memory, and the matrix pipe takes the
-// multiply-adds of all tokens at the price of one.  RG = 2 reads the tokens once for 32 weight rows: at 16 tokens they are as many bytes as 16 rows.
-// (Plain loads: a fragment touches half a cache line of 16 rows and the next one the other half, which a non-temporal hint fetches twice -- 157
-// against 123 us for a 514 MB head at 8 tokens.)
-template <int NW, int RG, int MODE>
-__global__ __launch_bounds__(NW * 64) void rows_kernel(const bf16_t* W, const bf16_t* X, long long ldx, int K, int N, int n_tok, RowsOut ro) {
-    ARIA_SMEM_STATIC float red[NW][16][16 * RG + 1];
-    const int t = threadIdx.x, l = t & 63, w = t >> 6, q4 = l >> 4, c16 = l & 15;
-    const int n0 = blockIdx.x * 16 * RG, t0 = blockIdx.y * 16;
-    const bf16_t* wp[RG];
-#pragma unroll
-    for (int g = 0; g < RG; ++g) wp[g] = W + (long long)min(n0 + 16 * g + c16, N - 1) * K;
-    const bf16_t* xp = X + (long long)min(t0 + c16, n_tok - 1) * ldx;
-    f32x4 acc[RG][2];
-#pragma unroll
-    for (int g = 0; g < RG; ++g) acc[g][0] = acc[g][1] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k0 = w * 128; k0 < K; k0 += 2 * NW * 128) {   // two blocks in flight: every weight fragment before the first use
-        u32x4 a[8], b[RG][8];
-#pragma unroll
-        for (int g = 0; g < RG; ++g)
-#pragma unroll
-            for (int u = 0; u < 8; ++u) {
-                const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
-                b[g][u] = ld16(wp[g] + (k < K ? k : 0));
-            }
-#pragma unroll
-        for (int u = 0; u < 8; ++u) {
-            const int k = k0 + (u >> 2) * NW * 128 + (u & 3) * 32 + q4 * 8;
-            a[u] = ld16(xp + (k < K ? k : 0));
-#pragma unroll
-            for (int q = 0; q < 4; ++q) a[u][q] = k < K ? a[u][q] : 0u;
-        }
-#pragma unroll
-        for (int u = 0; u < 8; ++u)
-#pragma unroll
-            for (int g = 0; g < RG; ++g) acc[g][u & 1] = mfma16(__builtin_bit_cast(s16x8, a[u]), __builtin_bit_cast(s16x8, b[g][u]), acc[g][u & 1]);
+struct LatentRows {
+    static constexpr bool SUMSQ = false;
+    RowsOut ro;
+    float* sums = nullptr;
+    __device__ __forceinline__ float operator()(float v, int tok, int n, int) const {
+        const long long at = (long long)tok * ro.ldo + n;
+        if (MODE == ROWS_BF16) static_cast<bf16_t*>(ro.out)[at] = f2bf(v);
+        if (MODE == ROWS_RELU2) static_cast<bf16_t*>(ro.out)[at] = f2bf(relu_squared(v));
+        if (MODE == ROWS_F32) static_cast<float*>(ro.out)[at] = v;
+        if (MODE == ROWS_STREAM) stream_step(v, ro.post, ro.next, ro.x, ro.h, at, n);
+        return 0.f;
     }
-#pragma unroll
-    for (int g = 0; g < RG; ++g)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) red[w][4 * q4 + r][16 * g + c16] = acc[g][0][r] + acc[g][1][r];
-    sync();
-    for (int i = t; i < 256 * RG; i += NW * 64) {
-        const int tok = i / (16 * RG), n = i % (16 * RG);
-        if (t0 + tok >= n_tok || n0 + n >= N) continue;
-        float v = 0.f;
-#pragma unroll
-        for (int ww = 0; ww < NW; ++ww) v += red[ww][tok][n];
-        rows_finish<MODE>(ro, v, t0 + tok, n0 + n);
-    }
-}
+};
 
 // routed up-projection of one (token, slot): act = silu(gate . h) * (up . h); the routing runs in front of the rows, workgroup x = 0 publishes it
 __global__ __launch_bounds__(256) void mix_up_kernel(const float* logits, const float* correction, int E, int ldl, int groups, int keep, int k,
@@ -677,13 +390,7 @@ int launch_any(const T* qa, const T* cache, const Shape& s, const int32_t* slot,
                 po, ml);
     return aria_check_launch();
 }
-// the matrix-pipe form's limits: cache row and latent width of one instantiation
-int mfma_class(const Shape& s) {
-    if (s.R <= 128 && s.cw <= 192) return 1;
-    if (s.R <= 256 && s.cw <= 320) return 2;
-    if (s.R <= 512 && s.cw <= 576) return 3;
-    return 0;
-}
+int mfma_class(const Shape& s) { return tile_attn_class(s.cw, s.R, s.cw); }
 
 }  // namespace
 
@@ -734,14 +441,7 @@ int aria_latent_absorb(const void* proj, const AriaLatentShape* s, const int32_t
 
 int64_t aria_latent_splits(const AriaLatentShape* s, int64_t T, int64_t max_len) {
     if (!s || T <= 0 || !mfma_class(*s)) return 1;
-    const int64_t tiles = (max_len + 63) / 64, groups = (s->H + 15) / 16 <= 1 ? 1 : (s->H + 31) / 32;
-    // one round of workgroups: as many as the 256 CUs hold at a time (a workgroup's LDS is two cache tiles), no more -- a workgroup's start and end cost
-    // as much as two tiles
-    const int64_t per_cu = (2 * 64 * s->cw * 2 + 16 * 1024) * 2 <= 160 * 1024 ? 2 : 1;
-    int64_t n = 256 * per_cu / (T * groups);
-    n = n < tiles ? n : tiles;
-    n = n < MAX_SPLITS ? n : MAX_SPLITS;
-    return n < 1 ? 1 : n;
+    return tile_attn_splits(s->cw, s->H, s->H, T, max_len);
 }
 
 int aria_latent_attn(const void* qa, const void* cache, const AriaLatentShape* s, const int32_t* slot, const int32_t* pos, float* part_o, float* part_ml,
@@ -757,28 +457,9 @@ int aria_latent_attn(const void* qa, const void* cache, const AriaLatentShape* s
         return f32 ? launch_any(static_cast<const float*>(qa), static_cast<const float*>(cache), *s, slot, pos, part_o, part_ml, T, stream)
                    : launch_any(static_cast<const bf16_t*>(qa), static_cast<const bf16_t*>(cache), *s, slot, pos, part_o, part_ml, T, stream);
     }
-    const bf16_t *q = static_cast<const bf16_t*>(qa), *c = static_cast<const bf16_t*>(cache);
-    const int NG = s->H <= 16 ? 1 : 2;
-    const dim3 grid(unsigned(splits), unsigned((s->H + 16 * NG - 1) / (16 * NG)), unsigned(T)), block(512);
-    const size_t lds = size_t(2) * 64 * s->cw * 2 + size_t(32) * 66 * 4 + size_t(NG) * 16 * (72 * 2 + 4);
-#define ARIA_LATENT(G, D, K) ARIA_LAUNCH((latent_attn_kernel<G, D, K>), grid, block, lds, stream, q, c, *s, slot, pos, part_o, part_ml, int(splits))
-    if (NG == 1) {
-        if (cls == 1)
-            ARIA_LATENT(1, 1, 6);
-        else if (cls == 2)
-            ARIA_LATENT(1, 2, 10);
-        else
-            ARIA_LATENT(1, 4, 18);
-    } else {
-        if (cls == 1)
-            ARIA_LATENT(2, 1, 6);
-        else if (cls == 2)
-            ARIA_LATENT(2, 2, 10);
-        else
-            ARIA_LATENT(2, 4, 18);
-    }
-#undef ARIA_LATENT
-    return aria_check_launch();
+    const TileAttn a{static_cast<const bf16_t*>(qa), (long long)(s->H * s->cw), int(s->cw), static_cast<const bf16_t*>(cache), (long long)(s->S_cap * s->cw),
+                     0, int(s->cw), int(s->cw), 0, int(s->R), int(s->H), int(s->H), 0, s->scale};
+    return launch_tile_attn(a, slot, pos, part_o, part_ml, T, splits, stream);
 }
 
 int aria_latent_expand(const float* part_o, const float* part_ml, const AriaLatentShape* s, const void* proj, const void* uv, void* out, int64_t T,
@@ -849,16 +530,8 @@ Scratch layout(const AriaLatentStack& st, const AriaLatentLayer* L, int64_t T, i
 
 template <int MODE>
 int rows(const void* W, const bf16_t* X, int64_t ldx, int64_t K, int64_t N, int64_t T, const RowsOut& ro, void* stream) {
-    const bf16_t* w = static_cast<const bf16_t*>(W);
-    if (T == 1)
-        ARIA_LAUNCH((row_kernel<MODE>), dim3(unsigned((N + 7) / 8)), dim3(256), 0, stream, w, X, int(K), int(N), ro);
-    else if (N > 16 * 1024)
-        ARIA_LAUNCH((rows_kernel<4, 2, MODE>), dim3(unsigned((N + 31) / 32), unsigned((T + 15) / 16)), dim3(256), 0, stream, w, X, (long long)ldx, int(K),
-                    int(N), int(T), ro);
-    else   // few row groups: more waves per group
-        ARIA_LAUNCH((rows_kernel<8, 1, MODE>), dim3(unsigned((N + 15) / 16), unsigned((T + 15) / 16)), dim3(512), 0, stream, w, X, (long long)ldx, int(K),
-                    int(N), int(T), ro);
-    return aria_check_launch();
+    RowsIn in{static_cast<const bf16_t*>(W), nullptr, X, (long long)ldx, int(K), int(N)};
+    return launch_rows(RowsPair{{in, in}}, 1, T, LatentRows<MODE>{ro}, stream);
 }
 
 }  // namespace

@@ -24,7 +24,7 @@ ERRORS = {
 P, I64, I32, F32 = c_void_p, c_int64, c_int, c_float
 RESTYPES = {"aria_gemm_workspace_bytes": c_int64, "aria_decode_scratch_bytes": c_int64, "aria_decode_graph_create": c_void_p,
             "aria_decode_graph_destroy": None, "aria_decode_attn_workspace_bytes": c_int64,
-            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64, "aria_linear_chunks_scratch": c_int64}  # everything else returns an int status
+            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64, "aria_linear_chunks_scratch": c_int64, "aria_mix_decode_scratch": c_int64}  # everything else returns an int status
 
 # name -> argtypes (all return int).  Kept in one table so tests can check that the shared
 # library exports every symbol the header declares.
@@ -113,6 +113,7 @@ SIGNATURES = {
     "aria_latent_splits": [P, I64, I64],
     "aria_latent_decode_scratch": [P, P, I64, I64],
     "aria_latent_decode": [P, P, I64, P, P, P, I64, P, P, I64, P],
+    "aria_gemm_relu_glu_bf16": [P, P, P, I64, I64, I64, I64, I64, I64, P],
     "aria_rms_stream": [P, I64, I64, I32, P],
     "aria_softcap": [P, I64, F32, P],
     "aria_chunk_attn_any": [P, P, P, P, P, P, P, P, I64, I32, P],
@@ -120,6 +121,8 @@ SIGNATURES = {
     "aria_linear_step": [P, P, P, P, P, P, I64, P, I32, P],
     "aria_linear_chunks_scratch": [P, I64, I64, I64],
     "aria_linear_chunks": [P, P, P, P, P, P, I64, P, I64, P, I64, P, I64, P, I64, P],
+    "aria_mix_decode_scratch": [P, P, I64, I64],
+    "aria_mix_decode": [P, P, I64, P, P, P, P, I64, P, P, I64, P],
     "aria_norm_gate": [P, P, I64, P, I64, P, I64, I64, I64, I64, F32, I32, I32, P],
 }
 
@@ -156,6 +159,17 @@ class ChunkShape(ctypes.Structure):     # AriaChunkShape
 class LinearShape(ctypes.Structure):    # AriaLinearShape
     _fields_ = [(n, c_int64) for n in ("H", "d", "dv", "dp", "dvp", "ldp", "q_off", "k_off", "v_off", "a_off", "rank", "silu")] + \
                [("q_scale", c_float), ("inv_tau", c_float)] + [(n, c_void_p) for n in ("decay", "a2", "a_bias")]
+
+
+class MixLayer(ctypes.Structure):       # AriaMixLayer
+    _fields_ = [("kind", c_int64), ("left", ChunkShape), ("right", LinearShape), ("g_off", c_int64)] + \
+               [(n, c_void_p) for n in ("w_in", "w_o_left", "w_o", "norm", "out_left", "out_right", "ring", "state", "norm2")] + [("ff", c_int64)] + \
+               [(n, c_void_p) for n in ("w_gate", "w_up", "w_down", "next")] + [("next_embedding", c_int64)]
+
+
+class MixStack(ctypes.Structure):       # AriaMixStack
+    _fields_ = [(n, c_int64) for n in ("n_runs", "D", "n", "V")] + [(n, c_float) for n in ("embedding_scale", "mult", "eps", "cap")] + \
+               [(n, c_void_p) for n in ("first", "embed", "head")]
 
 
 ABI_VERSION = 5   # include/aria_hip.h ARIA_ABI_VERSION this host code was written against

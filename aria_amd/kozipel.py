@@ -3,16 +3,21 @@ by two mixers side by side, chunk-local softmax attention and gated linear atten
 embedding output added to the stream before every pass but the first; every pass has a cache and states of its own.
 
 This file reads the design's config.json and tensor names and assembles the mechanisms of ``layers.py`` into the serving protocol of ``serving.py``
-(caches, step function, scheduler, sampling and command line are the framework's)."""
+(caches, step function, scheduler, sampling and command line are the framework's).  A step runs in one of two ways:
+
+* prompts, large batches and float32: sublayer by sublayer from here (tile GEMMs, flash attention and linear attention on the matrix pipe, the fused stream
+  pass);
+* up to ``DECODE_ROWS`` single tokens in bf16: one C call (``aria_mix_decode``) that enqueues every kernel of every layer run."""
 from __future__ import annotations
 
+import ctypes
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional
 
 import torch
 import torch.nn as nn
 
-from . import ops
+from . import hip, ops
 from .checkpoint import load_checkpoint_dir
 from .layers import ChunkAttention, LinearAttention, MixerGroup, ReluGatedFeedForward, RmsNorm, _frozen, padded, up8
 from .registry import read_config
@@ -114,6 +119,7 @@ class KozipelForCausalLM(nn.Module):
         self.head = _frozen(padded(tensors["head"], up8(config.vocab), self.width), dtype)
         self.caches: List[list] = []
         self.geometry = None
+        self._decode: Optional["_DecodeTables"] = None
 
     @classmethod
     def from_tensors(cls, config: dict, tensors: Dict[str, torch.Tensor], device="cuda", dtype=bf16) -> "KozipelForCausalLM":
@@ -122,6 +128,10 @@ class KozipelForCausalLM(nn.Module):
     @classmethod
     def from_pretrained(cls, path: str, device="cuda", dtype=bf16) -> "KozipelForCausalLM":
         return cls.from_tensors(read_config(path), load_checkpoint_dir(path), device, dtype)
+
+    def _apply(self, fn, *a, **k):       # (the decode tables hold raw addresses)
+        self._decode = None
+        return super()._apply(fn, *a, **k)
 
     @property
     def device(self):
@@ -133,7 +143,7 @@ class KozipelForCausalLM(nn.Module):
         if self.geometry == geometry:
             return                           # a sequence reads nothing that it has not written itself
         self.caches = [self.layers[r.layer].mixer.new_cache(slots, up8(max_len), self.device) for r in self.config.runs]
-        self.geometry = geometry
+        self.geometry, self._decode = geometry, None
 
     def _stream(self, x, batch, i, nxt, **src):
         """the stream pass behind a sublayer of run i that ends it: the next run's pass opening included"""
@@ -156,6 +166,11 @@ class KozipelForCausalLM(nn.Module):
         if batch.max_len > max_len or max(batch.slots) >= slots:
             raise ValueError("the batch does not fit the caches")
         c, T = self.config, batch.ids.numel()
+        if self.dtype == bf16 and trace is None and batch.longest == 1 and T <= DECODE_ROWS and all(L.mixer.one_call for L in self.layers):
+            if self._decode is None:
+                self._decode = _DecodeTables(self)
+            logits = self._decode.run(batch)
+            return logits if batch.wanted is None or batch.wanted.numel() == T else logits[batch.wanted.long()]
         x = torch.empty((T, self.width), dtype=f32, device=self.device)
         h = ops.rms_stream(x, c.width, c.eps, self.layers[c.runs[0].layer].norm1.weight, ids=batch.ids, table=self.embed, scale=c.embedding_scale)
         for i, run in enumerate(c.runs):
@@ -173,3 +188,39 @@ class KozipelForCausalLM(nn.Module):
                 return torch.empty((0, self.vocab), dtype=f32, device=self.device)
             h = ops.permute_any(h, batch.wanted.contiguous(), 1)
         return ops.softcap_(ops.linear_any(h, self.head, out_dtype=f32), c.logit_softcap)[:, :self.vocab]
+
+
+class _DecodeTables:
+    """Pointer and size tables of ``aria_mix_decode`` for a model's weights and caches (re-made when either moves), scratch and logits buffers."""
+
+    def __init__(self, model: KozipelForCausalLM):
+        c = model.config
+        n = len(c.runs)
+        self.runs = (hip.MixLayer * n)()
+        self.scratch: Optional[torch.Tensor] = None
+        for i, run in enumerate(c.runs):
+            L, t = model.layers[run.layer], self.runs[i]
+            L.mixer.fill_table(t, model.caches[i])
+            if L.mlp is not None:
+                gate = L.mlp.gate_up[:L.mlp.ff]
+                t.norm2, t.ff, t.w_gate, t.w_up = L.norm2.weight.data_ptr(), L.mlp.ff, gate.data_ptr(), L.mlp.gate_up[L.mlp.ff:].data_ptr()
+                t.w_down = L.mlp.down.data_ptr()
+            t.next = model.next_norm(i).weight.data_ptr()
+            t.next_embedding = int(i + 1 < n and c.runs[i + 1].again)
+        self.stack = hip.MixStack(n, model.width, c.width, model.head.shape[0], c.embedding_scale, c.residual_mult, c.eps, c.logit_softcap,
+                                  model.layers[c.runs[0].layer].norm1.weight.data_ptr(), model.embed.data_ptr(), model.head.data_ptr())
+        self.device, self.rows, self.vocab = model.device, model.head.shape[0], model.vocab
+
+    def run(self, batch) -> torch.Tensor:
+        T, lib = batch.ids.numel(), hip.get_lib()
+        stack, runs = ctypes.byref(self.stack), ctypes.byref(self.runs)
+        need = int(lib.cdll.aria_mix_decode_scratch(stack, runs, T, batch.max_len))
+        if self.scratch is None or self.scratch.numel() < need:
+            self.scratch = torch.empty(need, dtype=torch.uint8, device=self.device)
+        logits = torch.empty((T, self.rows), dtype=f32, device=self.device)
+        for t in (batch.ids, batch.slot, batch.pos):
+            assert t.dtype == torch.int32 and t.is_contiguous() and t.numel() == T
+        assert batch.cu.dtype == torch.int32 and batch.cu.is_contiguous() and batch.cu.numel() == T + 1
+        lib.call("aria_mix_decode", stack, runs, T, batch.ids.data_ptr(), batch.slot.data_ptr(), batch.pos.data_ptr(), batch.cu.data_ptr(), batch.max_len,
+                 logits.data_ptr(), self.scratch.data_ptr(), self.scratch.numel(), ops._stream(logits))
+        return logits[:, :self.vocab]

@@ -321,6 +321,25 @@ class MixerGroup(nn.Module):
     def new_cache(self, slots: int, max_len: int, device) -> list:
         return [p.new_cache(slots, max_len, device) for p in self.parts]
 
+    @property
+    def one_call(self) -> bool:
+        """aria_mix_decode takes the group: linear attention alone (one norm over all heads, a sigmoid gate), or chunk attention beside linear attention (a
+        norm per head, a silu gate), in widths of its kernels."""
+        lin = self.parts[-1]
+        if self.w_in.dtype != bf16 or not isinstance(lin, LinearAttention) or lin.geometry["dp"] > 1024:
+            return False
+        if len(self.parts) == 1:
+            return lin.norm_groups == 1 and not lin.silu_gate
+        return isinstance(self.parts[0], ChunkAttention) and self.parts[0].flash and lin.norm.numel() == lin.geometry["dvp"] and lin.silu_gate
+
+    def fill_table(self, t: hip.MixLayer, caches: list) -> None:
+        lin = self.parts[-1]
+        t.kind, t.right, t.g_off, t.w_in, t.w_o = len(self.parts) - 1, lin.shape(), lin.g_off, self.w_in.data_ptr(), lin.w_o.data_ptr()
+        t.norm, t.state = lin.norm.data_ptr(), caches[-1].rows.data_ptr()
+        if len(self.parts) == 2:
+            t.left, t.w_o_left, t.ring = self.parts[0].shape(caches[0]), self.parts[0].w_o.data_ptr(), caches[0].rows.data_ptr()
+            t.out_left, t.out_right = (n.weight.data_ptr() for n in self.out_norms)
+
     def forward(self, h: torch.Tensor, batch, caches: list) -> dict:
         proj = ops.linear_any(h, self.w_in)
         y = [p(proj, batch, c) for p, c in zip(self.parts, caches)]
@@ -339,5 +358,4 @@ class ReluGatedFeedForward(nn.Module):
         self.down = _frozen(padded(down, width, self.ff), dtype)
 
     def forward(self, h: torch.Tensor) -> dict:
-        gu = ops.linear_any(h, self.gate_up)
-        return dict(y=ops.linear_any(ops.act_rows(gu[:, self.ff:], gate=gu[:, :self.ff], relu=True), self.down))
+        return dict(y=ops.linear_any(ops.relu_glu(h, self.gate_up), self.down))

@@ -1174,6 +1174,19 @@ def rms_stream(x: torch.Tensor, n: int, eps: float, nxt: Optional[torch.Tensor],
     return h
 
 
+def relu_glu(x: torch.Tensor, gate_up: torch.Tensor) -> torch.Tensor:
+    """max(x gate^T, 0) * (x up^T), gate_up [2 I, K] = gate rows, then up rows: one launch for bf16 in the tile kernel's sizes, else GEMM + pass."""
+    I, K = gate_up.shape[0] // 2, gate_up.shape[1]
+    if _f32(x) or I % 128 or K % 64 or x.shape[0] * K >= 1 << 31 or gate_up.numel() >= 1 << 31:
+        gu = linear_any(x, gate_up)
+        return act_rows(gu[:, I:], gate=gu[:, :I], relu=True)
+    _chk(gate_up, name="gate_up")
+    assert gate_up.is_contiguous() and x.shape[1] == K
+    act = torch.empty((x.shape[0], I), dtype=bf16, device=x.device)
+    hip.get_lib().call("aria_gemm_relu_glu_bf16", _p(x), _p(gate_up), _p(act), x.shape[0], 2 * I, K, _rowmajor_2d(x, "x"), K, I, _stream(x))
+    return act
+
+
 def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
     """cap tanh(x / cap) in place, fp32."""
     _chk(x, torch.float32, "x")

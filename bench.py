@@ -16,6 +16,7 @@ from __future__ import annotations
 
 import argparse
 import json
+import math
 import os
 import sys
 import time
@@ -68,7 +69,7 @@ def parse():
                     "region with HIP events around every large launch class -> `roofline.worst_large_launch`)")
     ap.add_argument("--no-lora-record", action="store_true", help="skip the `lora_config` sub-record (N = 1 only: recipes/config_lora.yaml's adapter set "
                     "on the same model and micro-batch, three timed steps + the frozen-base forward + input-gradient reference)")
-    ap.add_argument("--design", choices=["duguzen"], help="serving throughput of that design instead of the training workload: prefill and decode at a few "
+    ap.add_argument("--design", choices=["duguzen", "kozipel"], help="serving throughput of that design instead of the training workload: prefill and decode at a few "
                     "real layer sizes (random weights) beside the gptfast decoder at equal width, heads, experts and vocabulary; one GPU, one JSON line; "
                     "--steps / --warmup count timed / untimed prefills (decode steps: 10 x)")
     ap.add_argument("--ep", action="store_true", help="BASELINE config #5 instead of #3: routed experts sharded over the N ranks (all-to-all "
@@ -595,13 +596,15 @@ DESIGN_SIZES = {   # width: heads, latent rank, dense ff, experts, top-k, expert
 }
 
 
-def duguzen_random(width, layers, dev):
-    """config + random device tensors of a Duguzen stack with ``width``'s sizes: one dense layer, then mixtures (heads 128 + 64 / 128)."""
+def duguzen_random(width, layers, dev, dense_ff=0):
+    """config + random device tensors of a Duguzen stack with ``width``'s sizes: one dense layer, then mixtures (heads 128 + 64 / 128); ``dense_ff``: dense
+    layers of that size only."""
     H, R, ff, E, top, ffe, (G, keep), V = DESIGN_SIZES[width]
+    ff = dense_ff or ff
     mix = dict(heads=H, dim=128, rot_dim=64, vdim=128, kv_rank=R, scale=192 ** -0.5, rot=dict(base=10000.0, dims=64))
     moe = dict(kind="moe", expert=dict(ff=ffe), router=dict(experts=E, top=top, groups=dict(count=G, keep=keep)))
     cfg = dict(architecture="Duguzen", width=width, vocab=V, norm=dict(eps=1e-6),
-               layers=[dict(type="latent_attention", mixer=mix, mlp=dict(kind="dense", ff=ff) if i == 0 else moe) for i in range(layers)])
+               layers=[dict(type="latent_attention", mixer=mix, mlp=dict(kind="dense", ff=ff) if i == 0 or dense_ff else moe) for i in range(layers)])
     g = torch.Generator(device=dev).manual_seed(0)
     w = {}
 
@@ -620,7 +623,7 @@ def duguzen_random(width, layers, dev):
         t(p + "mix.q", H * 192, width), t(p + "mix.dkv", R + 64, width), t(p + "mix.uk", H * 128, R), t(p + "mix.uv", H * 128, R)
         t(p + "mix.g", H, width), t(p + "mix.o", width, H * 128)
         w[p + "mix.dkv.norm"] = torch.ones(R, dtype=bf16, device=dev)
-        if i == 0:
+        if L["mlp"]["kind"] == "dense":
             t(p + "mlp.up", ff, width), t(p + "mlp.down", width, ff)
             continue
         for e in range(E):
@@ -630,9 +633,52 @@ def duguzen_random(width, layers, dev):
     return cfg, w
 
 
+KOZIPEL_SIZES = {   # width: (heads, key / value heads, chunk), (gated linear heads, key, value columns), lightning heads, ff; attention and lightning heads 128 wide
+    2560: ((20, 4, 2048), (5, 256, 512), 20, 6656),
+    1536: ((12, 4, 1024), (3, 256, 512), 12, 4096),
+    1024: ((8, 2, 1024), (4, 128, 256), 8, 2816),
+}
+
+
+def kozipel_random(width, layers, dev):
+    """config + random device tensors of a Kozipel stack with ``width``'s sizes, layers of both kinds in turn (vocabulary as DESIGN_SIZES)."""
+    (H, G, size), (Hr, dk, dv), Hl, ff = KOZIPEL_SIZES[width]
+    V = DESIGN_SIZES[width][-1]
+    par = dict(left=dict(heads=H, kv_heads=G, dim=128, vdim=128, scale=128 ** -0.5, mask=dict(size=size)), right=dict(heads=Hr, dim=dk, vdim=dv, tau=16.0))
+    lig = dict(heads=Hl, dim=128, vdim=128, decay=[math.exp(-2.0 ** (-8.0 * (i + 1) / Hl)) for i in range(Hl)])
+    cfg = dict(architecture="Kozipel", width=width, vocab=V, norm=dict(eps=1e-6), embedding=dict(scale=1.0), residual_mult=0.5, logit_softcap=30.0,
+               layers=[dict(type="lightning" if i % 2 else "parallel", mixer=lig if i % 2 else par, mlp=dict(kind="dense", ff=ff)) for i in range(layers)])
+    g = torch.Generator(device=dev).manual_seed(0)
+    w = {}
+
+    def t(name, *shape, scale=None):
+        w[name] = torch.empty(shape, dtype=bf16, device=dev).normal_(0.0, scale or shape[-1] ** -0.5, generator=g)
+
+    def linear(p, heads, k, v):
+        t(p + "q", heads * k, width), t(p + "k", heads * k, width), t(p + "v", heads * v, width), t(p + "g", heads * v, width), t(p + "o", width, heads * v)
+
+    t("embed", V, width, scale=1.0), t("head", V, width), t("final.norm", width, scale=0.1)
+    for i, L in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        t(p + "norm1", width, scale=0.1), t(p + "norm2", width, scale=0.1)
+        t(p + "mlp.gate", ff, width), t(p + "mlp.up", ff, width), t(p + "mlp.down", width, ff)
+        if i % 2:
+            linear(p + "mix.", Hl, 128, 128)
+            w[p + "mix.norm"] = torch.ones(Hl * 128, dtype=bf16, device=dev)
+            continue
+        q = p + "mix.left."
+        t(q + "q", H * 128, width), t(q + "k", G * 128, width), t(q + "v", G * 128, width), t(q + "o", width, H * 128)
+        q = p + "mix.right."
+        linear(q, Hr, dk, dv)
+        t(q + "a1", 16, width), t(q + "a2", Hr * dk, 16), t(q + "a2.b", Hr * dk, scale=1.0)
+        w[q + "norm"] = torch.ones(dv, dtype=bf16, device=dev)
+        w[p + "mix.left.out"] = w[p + "mix.right.out"] = torch.ones(width, dtype=bf16, device=dev)
+    return cfg, w
+
+
 def design_bench(args, dev, json_out):
-    """``--design duguzen``: prefill and decode throughput of Duguzen and of the gptfast (Aria) decoder at equal sizes, both through the serving step
-    (``serving.StepBatch``) on this GPU."""
+    """Prefill and decode throughput through the serving step (``serving.StepBatch``) on this GPU.  ``--design duguzen``: Duguzen and the gptfast (Aria) decoder
+    at equal sizes; ``--design kozipel``: Kozipel and a Duguzen of dense layers with as many feed-forward weights."""
     import gc
 
     from aria_amd import gptfast as G
@@ -668,6 +714,27 @@ def design_bench(args, dev, json_out):
         return rec
 
     out = {}
+    if args.design == "kozipel":
+        from aria_amd.kozipel import KozipelForCausalLM
+
+        for width, (_, _, _, ff) in KOZIPEL_SIZES.items():
+            rec = {}
+            for name, cls, (cfg, w) in (("kozipel", KozipelForCausalLM, kozipel_random(width, layers, dev)),
+                                        ("duguzen_dense", DuguzenForCausalLM, duguzen_random(width, layers, dev, dense_ff=3 * ff // 2))):
+                m = cls.from_tensors(cfg, w, dev)
+                del w
+                rec[name] = measure(m, cfg["vocab"], (1, 8, 16), (512, 4096, 16384))
+                del m
+                gc.collect(), torch.cuda.empty_cache()
+            out[f"width_{width}"] = rec
+            print(json.dumps({width: rec}), file=sys.stderr, flush=True)
+        head = out["width_2560"]["kozipel"]["prefill_8192"]
+        print(json.dumps({"metric": "Kozipel prefill tokens/s (width 2560, 8192-token prompt)", "value": head["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+                          "steps": steps, "warmup": warmup, "ms_per_step": head["ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+                          "dtype": "bf16", "data": "synthetic",
+                          "config": {"model": f"Kozipel, random weights, {layers} layers (parallel and lightning in turn)", "global_batch": 1, "seq_len": 8192,
+                                     "parallelism": "single", "sizes": {str(k): v for k, v in KOZIPEL_SIZES.items()}}, "records": out}), file=json_out, flush=True)
+        return
     for width, (H, R, ff, E, top, ffe, groups, V) in DESIGN_SIZES.items():
         cfg, w = duguzen_random(width, layers, dev)
         m = DuguzenForCausalLM.from_tensors(cfg, w, dev)

@@ -469,6 +469,9 @@ int aria_dyt_stream(const int32_t* ids, const void* table, const void* y, const 
 int aria_act_rows(const void* gate, const void* u, void* act, int64_t M, int64_t n_cols, int64_t ld_in, int64_t ld_act, int relu_gate, int f32,
                   void* stream);
 
+/* ACT [M, I] = max(A gate^T, 0) * (A up^T) in one launch, B [2 I, K] = gate rows, then up rows; K % 64 handled as in aria_gemm_swiglu_bf16, I % 128 == 0. */
+int aria_gemm_relu_glu_bf16(const void* A, const void* B, void* ACT, int64_t M, int64_t N2, int64_t K, int64_t lda, int64_t ldb, int64_t ldact, void* stream);
+
 /* C [M, N] = A [M, K] W^T (W [N, K]) in true 32-bit on the vector ALU.  offsets != NULL: rows offsets[e] .. offsets[e + 1] of A use W + e strideW
  * (int32 [E + 1] on the device).  K % 4 == 0, 16-byte aligned rows. */
 int aria_gemm_f32(const float* A, const float* W, float* C, int64_t M, int64_t N, int64_t K, int64_t lda, int64_t ldw, int64_t ldc,
@@ -601,6 +604,36 @@ int aria_linear_chunks(void* proj, const AriaLinearShape* s, float* state, const
  * between groups (0: shared).  o [T, groups cols], gate rows ldg apart.  cols % 8 == 0; y may be o. */
 int aria_norm_gate(const void* o, const void* gate, int64_t ldg, const float* w, int64_t w_stride, void* y, int64_t T, int64_t groups, int64_t cols, int64_t n,
                    float eps, int silu, int f32, void* stream);
+
+/* A decoder stack of such layers (bf16), for the one-call decode step.  kind 0: one linear-attention mixer whose RMS norm runs over all heads, gated by a
+ * sigmoid; kind 1: chunk-local attention beside a gated linear mixer normed per head and gated by a silu, the half-sum of their normed outputs.  An entry
+ * per layer RUN; `left` / `right`: shapes over ONE projection w_in [ldp, D]; g_off: the linear mixer's output-gate columns. */
+typedef struct {
+    int64_t kind;
+    AriaChunkShape left;
+    AriaLinearShape right;
+    int64_t g_off;
+    const void *w_in, *w_o_left, *w_o;        /* w_o_left [D, H dvp], w_o [D, H dvp] */
+    const float *norm, *out_left, *out_right; /* linear mixer's norm (kind 0: [H dvp], kind 1: [dvp]); norms of the two outputs [D] */
+    void* ring;                               /* chunk cache */
+    float* state;
+    const float* norm2;                       /* [D]; NULL: no feed-forward */
+    int64_t ff;
+    const void *w_gate, *w_up, *w_down;       /* [ff, D], [ff, D], [D, ff]: relu(gate) up */
+    const float* next;                        /* [D] norm of the following run, or the model's final one */
+    int64_t next_embedding;                   /* the embedding output is added in front of the following run */
+} AriaMixLayer;
+typedef struct {
+    int64_t n_runs, D, n, V;                  /* n: true width (norms count n columns); V: rows of the head */
+    float embedding_scale, mult, eps, cap;
+    const float* first;                       /* [D] norm of the first run */
+    const void *embed, *head;
+} AriaMixStack;
+int64_t aria_mix_decode_scratch(const AriaMixStack* stack, const AriaMixLayer* runs, int64_t T, int64_t max_len);
+/* One step of T single tokens of T sequences (seq_rows: 0 .. T, int32 on the device), as aria_latent_decode: logits fp32 [T, V], soft-capped.
+ * ARIA_ERR_UNSUPPORTED: widths beyond the matrix-pipe attention. */
+int aria_mix_decode(const AriaMixStack* stack, const AriaMixLayer* runs, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos,
+                    const int32_t* seq_rows, int64_t max_len, float* logits, void* scratch, int64_t scratch_bytes, void* stream);
 
 #ifdef __cplusplus
 }

@@ -163,6 +163,17 @@ def case_softcap_and_relu_gate(dev, dtype):
     assert rel(got, gu[:, :24].double().clamp_min(0) * gu[:, 24:].double()) < (1e-6 if dtype == f32 else 3e-3)
 
 
+def case_relu_glu(dev, M, ff, K):
+    """The one-launch gated pair against GEMM + elementwise pass (both round gate and up to bf16 first; a long GEMM may sum in another order)."""
+    from aria_amd import ops
+
+    x, w = rnd(M, K, seed=1).to(dev), rnd(2 * ff, K, seed=2, scale=K ** -0.5).to(dev)
+    got, gu = ops.relu_glu(x, w), ops.gemm(x, w)
+    assert rel(got, ops.act_rows(gu[:, ff:], gate=gu[:, :ff], relu=True).cpu().double()) < (1e-7 if K < 1024 else 2e-3)
+    y = x.cpu().double() @ w.cpu().double().T
+    assert rel(got, y[:, :ff].clamp_min(0) * y[:, ff:]) < 1e-2
+
+
 def case_norm_gate(dev, dtype, T=5):
     from aria_amd import ops
 

@@ -28,6 +28,11 @@ def test_softcap_and_relu_gate(dtype):
     C.case_softcap_and_relu_gate(DEV, dtype)
 
 
+@pytest.mark.parametrize("M,ff,K", [(5, 24, 16), (70, 128, 64)])
+def test_relu_glu(M, ff, K):
+    C.case_relu_glu(DEV, M, ff, K)
+
+
 @both
 def test_norm_gate(dtype):
     C.case_norm_gate(DEV, dtype)
