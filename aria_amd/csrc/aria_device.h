@@ -427,6 +427,14 @@ __device__ __forceinline__ float exp2_fast(float x) {
     return __builtin_amdgcn_exp2f(x);
 #endif
 }
+// log2(x) straight on v_log_f32 (x a normal number)
+__device__ __forceinline__ float log2_fast(float x) {
+#ifdef ARIA_EMU
+    return std::log2(x);
+#else
+    return __builtin_amdgcn_logf(x);
+#endif
+}
 __device__ __forceinline__ float rcp_fast(float x) {
 #ifdef ARIA_EMU
     return 1.f / x;

@@ -22,22 +22,30 @@ constexpr int BLK = 64;
 constexpr float RANGE = 216.f;   // in powers of two: +- 2^108 leaves fp32 and bf16 room for the sums
 __device__ const uint32_t linear_zero_page[4] = {};
 
+constexpr int PREP = 512;   // threads of linear_prepare
 template <int DP>
-__global__ __launch_bounds__(256) void linear_prepare_kernel(bf16_t* proj, Lin s, const int32_t* blocks, float* fac, int32_t* marked, float* alpha) {
-    constexpr int PAIRS = DP / 2, NG = 256 / PAIRS, PER = BLK / NG;   // a thread: two channels of PER tokens
+__global__ __launch_bounds__(PREP) void linear_prepare_kernel(bf16_t* proj, Lin s, const int32_t* blocks, float* fac, int32_t* marked, float* alpha) {
+    constexpr int PAIRS = DP / 2, NG = PREP / PAIRS, PER = BLK / NG;   // a thread: two channels of PER tokens
     ARIA_DYN_SMEM(smem);
-    float* sG = reinterpret_cast<float*>(smem);   // [BLK][DP]
-    float* sT = sG + BLK * DP;                    // [NG][DP]
-    float* sM = sT + NG * DP;                     // [4]
-    float* sA = sM + 4;                           // [BLK][rank]
+    float* sT = reinterpret_cast<float*>(smem);   // [NG + 1][DP]: the groups' sums, the first token's value
+    float* sM = sT + (NG + 1) * DP;               // [8]
+    float* sA = sM + 8;                           // [BLK][rank]
     const int t = threadIdx.x, l = t & 63, w = t >> 6, d = 2 * (t % PAIRS), grp = t / PAIRS, h = blockIdx.y;
     const int row0 = blocks[2 * blockIdx.x], n = blocks[2 * blockIdx.x + 1], rank = int(s.rank);
     if (!s.decay) {
-        for (int i = t; i < BLK * rank; i += 256) {
+        for (int i = t; i < BLK * rank; i += PREP) {
             const int tok = i / rank;
             sA[i] = tok < n ? ldf(proj + (long long)(row0 + tok) * s.ldp + s.a_off + i % rank) : 0.f;
         }
         sync();
+    }
+    // this thread's queries and keys, requested before anything is computed (the stores below go to the same rows)
+    uint32_t qw[PER], kw[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const bf16_t* p = proj + (long long)(row0 + min(grp * PER + i, n - 1)) * s.ldp + h * DP + d;
+        qw[i] = *reinterpret_cast<const uint32_t*>(p + s.q_off);
+        kw[i] = *reinterpret_cast<const uint32_t*>(p + s.k_off);
     }
     float z[PER][2];   // log2 of the decay
     if (s.decay) {
@@ -71,21 +79,18 @@ __global__ __launch_bounds__(256) void linear_prepare_kernel(bf16_t* proj, Lin s
 #pragma unroll
         for (int i = 0; i < PER; ++i)
 #pragma unroll
-            for (int c = 0; c < 2; ++c) z[i][c] = (fminf(z[i][c], 0.f) - log1pf(expf(-fabsf(z[i][c])))) * s.inv_tau * 1.4426950408889634f;
+            for (int c = 0; c < 2; ++c) z[i][c] = log2_sigmoid_fast(z[i][c]) * s.inv_tau;
     }
-    float c0 = 0.f, c1 = 0.f;
+    if (grp == 0) {
+        sT[NG * DP + d] = z[0][0];
+        sT[NG * DP + d + 1] = z[0][1];
+    }
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-        const int tok = grp * PER + i;
-        if (tok < n) {
-            c0 += z[i][0];
-            c1 += z[i][1];
-        }
-        sG[tok * DP + d] = c0;
-        sG[tok * DP + d + 1] = c1;
-    }
-    sT[grp * DP + d] = c0;
-    sT[grp * DP + d + 1] = c1;
+    for (int i = 0; i < PER; ++i)   // running sums inside the group
+#pragma unroll
+        for (int c = 0; c < 2; ++c) z[i][c] = (grp * PER + i < n ? z[i][c] : 0.f) + (i ? z[i - 1][c] : 0.f);
+    sT[grp * DP + d] = z[PER - 1][0];
+    sT[grp * DP + d + 1] = z[PER - 1][1];
     sync();
     float o0 = 0.f, o1 = 0.f, last0 = 0.f, last1 = 0.f;
 #pragma unroll
@@ -94,13 +99,14 @@ __global__ __launch_bounds__(256) void linear_prepare_kernel(bf16_t* proj, Lin s
         last0 += sT[g * DP + d];
         last1 += sT[g * DP + d + 1];
     }
-    const float first0 = sG[d], first1 = sG[d + 1];
+    const float first0 = sT[NG * DP + d], first1 = sT[NG * DP + d + 1];
     float drop = fmaxf(first0 - last0, first1 - last1);
     if (!(first0 - last0 <= RANGE) || !(first1 - last1 <= RANGE)) drop = INFINITY;   // (not a number: a decay of zero)
     drop = wave_max_bcast(drop);
     if (l == 0) sM[w] = drop;
     sync();
-    const bool exact = !(fmaxf(fmaxf(sM[0], sM[1]), fmaxf(sM[2], sM[3])) <= RANGE);
+    for (int i = 0; i < PREP / 64; ++i) drop = fmaxf(drop, sM[i]);
+    const bool exact = !(drop <= RANGE);
     const long long bh = (long long)blockIdx.x * s.H + h;
     if (t == 0) marked[bh] = exact;
     const float R0 = 0.5f * (first0 + last0), R1 = 0.5f * (first1 + last1);
@@ -118,65 +124,78 @@ __global__ __launch_bounds__(256) void linear_prepare_kernel(bf16_t* proj, Lin s
         const int tok = grp * PER + i;
         if (tok >= n) continue;
         bf16_t* p = proj + (long long)(row0 + tok) * s.ldp + h * DP + d;
-        const uint32_t qw = *reinterpret_cast<const uint32_t*>(p + s.q_off), kw = *reinterpret_cast<const uint32_t*>(p + s.k_off);
-        float q0 = bflo(qw), q1 = bfhi(qw), k0 = bflo(kw), k1 = bfhi(kw);
+        float q0 = bflo(qw[i]), q1 = bfhi(qw[i]), k0 = bflo(kw[i]), k1 = bfhi(kw[i]);
         if (s.silu) q0 = silu_fast(q0), q1 = silu_fast(q1), k0 = silu_fast(k0), k1 = silu_fast(k1);
         q0 *= s.q_scale;
         q1 *= s.q_scale;
         if (exact) {
             float* a = alpha + ((long long)(row0 + tok) * s.H + h) * DP + d;
-            a[0] = exp2f(z[i][0]);
-            a[1] = exp2f(z[i][1]);
+#pragma unroll
+            for (int c = 0; c < 2; ++c)
+                a[c] = s.decay ? s.decay[2 * h] : exp2f(gate_log2(s, proj + (long long)(row0 + tok) * s.ldp + s.a_off, h * DP + d + c));
         } else {
-            const float e0 = sG[tok * DP + d] + o0 - R0, e1 = sG[tok * DP + d + 1] + o1 - R1;
-            q0 *= exp2f(e0);
-            q1 *= exp2f(e1);
-            k0 *= exp2f(-e0);
-            k1 *= exp2f(-e1);
+            const float e0 = z[i][0] + o0 - R0, e1 = z[i][1] + o1 - R1;
+            q0 *= exp2_fast(e0);
+            q1 *= exp2_fast(e1);
+            k0 *= exp2_fast(-e0);
+            k1 *= exp2_fast(-e1);
         }
         *reinterpret_cast<uint32_t*>(p + s.q_off) = pack2bf(q0, q1);
         *reinterpret_cast<uint32_t*>(p + s.k_off) = pack2bf(k0, k1);
     }
     if (s.silu) {
         const int vc = int(s.dvp) >> 3;
-        for (int i = t; i < n * vc; i += 256) {
-            bf16_t* p = proj + (long long)(row0 + i / vc) * s.ldp + s.v_off + h * s.dvp + (i % vc) * 8;
-            float v[8];
-            ld8(p, v);
+        for (int i0 = t; i0 < n * vc; i0 += 4 * PREP) {
+            u32x4 x[4];
+            bf16_t* p[4];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) v[e] = silu_fast(v[e]);
-            st8(p, v);
+            for (int u = 0; u < 4; ++u) {
+                const int i = min(i0 + PREP * u, n * vc - 1);
+                p[u] = proj + (long long)(row0 + i / vc) * s.ldp + s.v_off + h * s.dvp + (i % vc) * 8;
+                x[u] = ld16(p[u]);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[u][e] = pack2bf(silu_fast(bflo(x[u][e])), silu_fast(bfhi(x[u][e])));
+                if (i0 + PREP * u < n * vc) st16(p[u], x[u]);
+            }
         }
     }
 }
 
-// grid (32 NW-column blocks of the values, heads, chunks), NW waves.  Wave w holds the state's columns 32 w .. + 31 for all DP channels as 32 x 32
-// accumulators [channel][column]; read as the A operand of o^T = S^T q^T their registers are in place (the channel order inside a 16-block follows the
+// A workgroup: 32 NW value columns of a head's chunk, NW DS waves.  Wave w holds the state's columns 32 (w % NW) .. + 31 for its 1 / DS of the DP
+// channels (DS = 2 for 256: the state's registers) as 32 x 32 accumulators [channel][column]; read as the A operand of o^T = S^T q^T their registers are in place (the channel order inside a 16-block follows the
 // accumulator, q^ is read in that order).  The state enters that product as two bf16 numbers, so it is read with 16 bits of mantissa.
-// LDS: q^ and k^ images, v image, scores [64][PP], factors.  Per block three barriers: q^ arrives while the previous block's state is updated, k^ and v
-// while S^T q^T runs.
-template <int DP, int NW>
+// DS = 2: the two waves of a column slice exchange partial sums through LDS, each finishes one half of the block's tokens.
+// LDS: images of q^ (two), k^ and v, scores [64][PP], factors, partial sums; OUT = false: two k^ and v images.  Per block three barriers: q^ is requested a
+// whole block ahead, k^ and v at the end of the block before; k^ is awaited behind S^T q^T, v behind the scores.
+template <int DP, int NW, bool OUT>
 struct ChunkSmem {
-    static constexpr int VB = 32 * NW, PP = 72;
-    static constexpr int Q0 = 0, K0 = TileImg<DP>::BYTES, V0 = 2 * K0, P0 = V0 + TileImg<VB>::BYTES, F0 = P0 + 64 * PP * 2, BYTES = F0 + 2 * 2 * DP * 4;
+    static constexpr int DS = DP > 128 ? 2 : 1, WAVES = NW * DS, VB = 32 * NW, PP = 72, QB = TileImg<DP>::BYTES, VBYTES = TileImg<VB>::BYTES;
+    static constexpr int Q0 = 0, K0 = OUT ? 2 * QB : 0, K_STEP = OUT ? 0 : QB, V0 = K0 + QB + K_STEP, V_STEP = OUT ? 0 : VBYTES, P0 = V0 + VBYTES + V_STEP,
+                         F0 = P0 + (OUT ? 64 * PP * 2 : 0), O0 = F0 + 2 * DP * 4, BYTES = O0 + (OUT && DS == 2 ? WAVES * 4096 : 0);
 };
 template <int DP, int NW, bool OUT>
-__global__ __launch_bounds__(NW * 64) void linear_chunk_kernel(const bf16_t* proj, Lin s, const int32_t* blocks, const int32_t* chunks, const float* fac,
-                                                               const int32_t* marked, const float* alpha, float* states, float* cache, const int32_t* slot,
-                                                               const int32_t* pos, bf16_t* out) {
-    using L = ChunkSmem<DP, NW>;
+__global__ __launch_bounds__(NW * (DP > 128 ? 128 : 64), 2) void linear_chunk_kernel(const bf16_t* proj, Lin s, const int32_t* blocks, const int32_t* chunks, const float* fac,
+                                                               const int32_t* marked, const float* alpha, float* states, float* decays, float* cache,
+                                                               const int32_t* slot, const int32_t* pos, bf16_t* out, int n_chunks) {
+    using L = ChunkSmem<DP, NW, OUT>;
     using QI = TileImg<DP>;
     using VI = TileImg<L::VB>;
-    constexpr int TD = DP / 32, KV_PIECES = DP / 8 / NW + 4;
+    constexpr int DS = L::DS, NWT = L::WAVES, TD = DP / 32 / DS, Q_PIECES = DP / 8 / NWT, V_PIECES = 4 / DS, OT = 2 / DS;   // OT: token halves a wave finishes
     ARIA_DYN_SMEM(smem);
-    char *sQ = smem + L::Q0, *sK = smem + L::K0, *sV = smem + L::V0;
     bf16_t* sP = reinterpret_cast<bf16_t*>(smem + L::P0);
-    float* sF = reinterpret_cast<float*>(smem + L::F0);   // [2][2 DP]
+    float* sF = reinterpret_cast<float*>(smem + L::F0);   // [2][DP]
     const int t = threadIdx.x, l = t & 63, w = first_lane(t >> 6), h2 = l >> 5, c32 = l & 31, q4 = l >> 4, c16 = l & 15;
-    const int v0 = blockIdx.x * L::VB, h = blockIdx.y, c = blockIdx.z;
+    const int ws = w % NW, ds = DS == 2 ? w / NW : 0, td0 = ds * TD;   // this wave's column slice, channel half
+    // workgroup n runs on XCD n % 8: the column blocks of a (head, chunk) share an XCD, whose L2 then holds their q^ and k^
+    const int nvb = (int(s.dvp) + L::VB - 1) / L::VB, group = int(blockIdx.x >> 3) / nvb * 8 + int(blockIdx.x & 7), vb = int(blockIdx.x >> 3) % nvb;
+    if (group >= int(s.H) * n_chunks) return;
+    const int v0 = vb * L::VB, h = group % int(s.H), c = group / int(s.H);
     const int b0 = chunks[4 * c], nb = chunks[4 * c + 1], first = chunks[4 * c + 2], last = chunks[4 * c + 3];
     if (!OUT && last) return;
-    const int vcol = v0 + 32 * w;            // this wave's first column
+    const int vcol = v0 + 32 * ws;           // this wave's first column
     const bool mine = vcol < s.dvp;
     const long long head_state = (long long)s.dp * s.dvp, H = s.H;
     const int r_first = blocks[2 * b0];
@@ -190,62 +209,107 @@ __global__ __launch_bounds__(NW * 64) void linear_chunk_kernel(const bf16_t* pro
 #pragma unroll
         for (int i = 0; i < TD; ++i)
 #pragma unroll
-            for (int r = 0; r < 16; ++r) S[i][r] = src[(long long)(32 * i + acc_row(r, l)) * s.dvp];
+            for (int r = 0; r < 16; ++r) S[i][r] = src[(long long)(32 * (td0 + i) + acc_row(r, l)) * s.dvp];
     }
-    auto dma_rows = [&](const bf16_t* base, int n, char* dst) __attribute__((always_inline)) {   // q^ or k^: DP columns
+    // rows of block j of the chunk: r_first + 64 j .., at most 64
+    const int rows_all = blocks[2 * (b0 + nb - 1)] + blocks[2 * (b0 + nb - 1) + 1] - r_first;
+    unsigned long long marks = 0;            // marked blocks among j & ~63 ..
+    auto load_marks = [&](int j) __attribute__((always_inline)) { marks = ballot(j + l < nb && marked[(long long)(b0 + j + l) * H + h] != 0); };
+    auto is_marked = [&](int j) __attribute__((always_inline)) -> bool { return (marks >> (j & 63)) & 1; };
+    // this lane's chunk of the wave's first DMA piece of an image; later pieces lie a fixed number of rows further on (the swizzle repeats every 16 rows)
+    auto dma_image = [&](auto img, const bf16_t* base, int n, int cols, char* dst) __attribute__((always_inline)) {
+        using I = decltype(img);
+        constexpr int STEP = NWT * 64 / I::CPR;
+        static_assert(STEP % 8 == 0, "");
+        int lane = w * 64 + l;
+        hold(lane);   // (here and below: addresses are cheaper computed again per block than held in registers beside the state)
+        const int row = lane / I::CPR, col = ((lane % I::CPR) ^ I::swz(row)) * 8;
+        const char* at = reinterpret_cast<const char*>(base + (long long)row * s.ldp + col);
+        const char* zero = reinterpret_cast<const char*>(linear_zero_page);
+        const long long step = 2ll * STEP * s.ldp;
 #pragma unroll
-        for (int i = 0; i < DP / 8 / NW; ++i) {
-            const int pc = w + NW * i, ch = pc * 64 + l, row = ch / QI::CPR, col = ((ch % QI::CPR) ^ QI::swz(row)) * 8;
-            const void* src = row < n ? static_cast<const void*>(base + (long long)row * s.ldp + col) : static_cast<const void*>(linear_zero_page);
-            glds16_raw(src, dst + pc * 1024);
+        for (int i = 0; i < 64 / STEP; ++i) {
+            const int x = STEP % 16 && i % 2 ? (I::swz(row + STEP) ^ I::swz(row)) * 8 : 0;   // (steps of 8 rows: every other piece has another swizzle)
+            const int c = x ? ((lane % I::CPR) ^ I::swz(row + STEP)) * 8 : col;
+            const char* src = at + i * step + 2 * (c - col);
+            const bool in = row + STEP * i < n && c < cols;
+            src = in ? src : zero;
+            glds16_raw(src, dst + (w + NWT * i) * 1024);
         }
     };
-    auto dma_q = [&](int b) __attribute__((always_inline)) {
-        dma_rows(proj + (long long)blocks[2 * b] * s.ldp + s.q_off + h * DP, blocks[2 * b + 1], sQ);
+    auto dma_q = [&](int j, int buf) __attribute__((always_inline)) {
+        dma_image(QI(), proj + (long long)(r_first + BLK * j) * s.ldp + s.q_off + h * DP, rows_all - BLK * j, DP, smem + L::Q0 + buf * L::QB);
     };
-    auto dma_kv = [&](int b) __attribute__((always_inline)) {
-        const int n = blocks[2 * b + 1];
-        const bf16_t* rows = proj + (long long)blocks[2 * b] * s.ldp;
-        dma_rows(rows + s.k_off + h * DP, n, sK);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int pc = w + NW * i, ch = pc * 64 + l, row = ch / VI::CPR, col = v0 + ((ch % VI::CPR) ^ VI::swz(row)) * 8;
-            const void* src = row < n && col < s.dvp ? static_cast<const void*>(rows + (long long)row * s.ldp + s.v_off + h * s.dvp + col)
-                                                     : static_cast<const void*>(linear_zero_page);
-            glds16_raw(src, sV + pc * 1024);
-        }
+    auto dma_kv = [&](int j, int buf) __attribute__((always_inline)) {   // (buf: OUT = false has two)
+        const bf16_t* rows = proj + (long long)(r_first + BLK * j) * s.ldp;
+        dma_image(QI(), rows + s.k_off + h * DP, rows_all - BLK * j, DP, smem + L::K0 + buf * L::K_STEP);
+        dma_image(VI(), rows + s.v_off + h * s.dvp + v0, rows_all - BLK * j, int(s.dvp) - v0, smem + L::V0 + buf * L::V_STEP);
     };
     auto barrier = [&]() __attribute__((always_inline)) {   // (LDS-DMA in flight stays in flight)
         wait_lds();
         raw_barrier();
     };
-    f32x4 fnext = f32x4{0.f, 0.f, 0.f, 0.f};
-    auto fetch_f = [&](int b) __attribute__((always_inline)) {
-        if (t < DP / 2) fnext = *reinterpret_cast<const f32x4*>(fac + ((long long)b * H + h) * 3 * DP + 4 * t);
-    };
-    auto park_f = [&](int buf) __attribute__((always_inline)) {
-        if (t < DP / 2) *reinterpret_cast<f32x4*>(sF + buf * 2 * DP + 4 * t) = fnext;
-    };
-    auto scale_rows = [&](f32x16& x, const float* f, int td) __attribute__((always_inline)) {
-#pragma unroll
-        for (int rg = 0; rg < 4; ++rg) {
-            const f32x4 v = *reinterpret_cast<const f32x4*>(f + 32 * td + 8 * rg + 4 * h2);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) x[4 * rg + e] *= v[e];
+    // per-channel factors of a block's start, e^(G_last - R) of the block before times e^R of its own: thread t owns channels 4 t .. 4 t + 3
+    const f32x4 ones = f32x4{1.f, 1.f, 1.f, 1.f};
+    f32x4 f_in = ones, f_out = ones, pending = ones, whole = ones;
+    auto fetch_f = [&](int j) __attribute__((always_inline)) {
+        const float* src = fac + ((long long)(b0 + j) * H + h) * 3 * DP + 4 * t;
+        f_in = f_out = ones;
+        if (t < DP / 4) {
+            if (!is_marked(j)) {
+                f_in = *reinterpret_cast<const f32x4*>(src);
+                f_out = *reinterpret_cast<const f32x4*>(src + DP);
+            }
+            if (!OUT && vb == 0) whole *= *reinterpret_cast<const f32x4*>(src + 2 * DP);
         }
     };
-    fetch_f(b0);
+    auto park_f = [&](int buf) __attribute__((always_inline)) {
+        if (t < DP / 4) *reinterpret_cast<f32x4*>(sF + buf * DP + 4 * t) = pending * f_in;
+        pending = f_out;
+    };
+    auto load_f = [&](f32x4 (&v)[4], const float* f, int td) __attribute__((always_inline)) {
+#pragma unroll
+        for (int rg = 0; rg < 4; ++rg) v[rg] = *reinterpret_cast<const f32x4*>(f + 32 * (td0 + td) + 8 * rg + 4 * h2);
+    };
+    auto scale_rows = [&](f32x16& x, const f32x4 (&v)[4]) __attribute__((always_inline)) {
+#pragma unroll
+        for (int rg = 0; rg < 4; ++rg)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[4 * rg + e] *= v[rg][e];
+    };
+    auto scale_all = [&](const float* f) __attribute__((always_inline)) {
+#pragma unroll
+        for (int td = 0; td < TD; ++td) {
+            f32x4 v[4];
+            load_f(v, f, td);
+            scale_rows(S[td], v);
+            sched_fence();
+        }
+    };
+    // LDS addresses of the fragment reads: a lane's base with the chunk index as an exclusive-or (a row's bytes in front of the chunk field are zeros, and
+    // the swizzle of a row repeats every 16 rows)
+    const int tr = 4 * h2 + (c16 >> 2), tc = 16 * ((l >> 4) & 1) + 4 * (l & 3);   // TileImg::columns' row and column at (0, 0)
+    const int q_lane = L::Q0 + c32 * QI::ROW + 8 * h2 + (QI::swz(c32) << 4);                                  // B operand of S^T q^T, chunk 0
+    const int t0_lane = L::K0 + tr * QI::ROW + (((tc >> 3) ^ QI::swz(tr)) << 4) + (tc & 7) * 2;               // transposing read of k^, channels 0 ..
+    const int t1_lane = L::K0 + (tr + 8) * QI::ROW + (((tc >> 3) ^ QI::swz(tr + 8)) << 4) + (tc & 7) * 2;
+    const int s_lane = c16 * QI::ROW + ((q4 ^ QI::swz(c16)) << 4);                                            // score fragments, relative to an image
+    load_marks(0);
+    fetch_f(0);
     if (OUT) {
-        for (int i = t; i < 64 * L::PP / 8; i += NW * 64) st16(sP + i * 8, zero16());   // (tiles above the diagonal stay zero)
-        dma_q(b0);
+        for (int i = t; i < 64 * L::PP / 8; i += NWT * 64) st16(sP + i * 8, zero16());   // (tiles above the diagonal stay zero)
+        dma_q(0, 0);
     }
-    dma_kv(b0);
+    dma_kv(0, 0);
     park_f(0);
     for (int j = 0; j < nb; ++j) {
-        const int b = b0 + j, row0 = blocks[2 * b], n = blocks[2 * b + 1];
-        const float* f = sF + (j & 1) * 2 * DP;
+        const int row0 = r_first + BLK * j, n = min(BLK, rows_all - BLK * j);
+        const float* f = sF + (j & 1) * DP;
         const bool more = j + 1 < nb;
-        if (marked[(long long)b * H + h]) {   // (workgroup-uniform) token by token: decays from alpha, q, k, v as they lie in proj
+        const bool exact = is_marked(j);
+        if (((j + 1) & 63) == 0) load_marks(j + 1);
+        if (exact) {   // (workgroup-uniform) token by token: decays from alpha, q, k, v as they lie in proj
+            barrier();
+            scale_all(f);
             for (int i = 0; i < n; ++i) {
                 const bf16_t* p = proj + (long long)(row0 + i) * s.ldp;
                 const float* a = alpha + ((long long)(row0 + i) * H + h) * DP;
@@ -255,34 +319,64 @@ __global__ __launch_bounds__(NW * 64) void linear_chunk_kernel(const bf16_t* pro
                 for (int td = 0; td < TD; ++td)
 #pragma unroll
                     for (int r = 0; r < 16; ++r) {
-                        const int d = 32 * td + acc_row(r, l);
+                        const int d = 32 * (td0 + td) + acc_row(r, l);
                         S[td][r] = a[d] * S[td][r] + ldf(p + s.k_off + h * DP + d) * v;
                         if (OUT) o += S[td][r] * ldf(p + s.q_off + h * DP + d);
+                        if ((r & 3) == 3) sched_fence();   // (four channels' operands at a time: the registers are the state's)
                     }
                 if (OUT) {
                     o += shfl_xor(o, 32);
-                    if (mine && h2 == 0) stf(out + ((long long)(row0 + i) * H + h) * s.dvp + vcol + c32, o);
+                    if (DS == 2) {   // (the halves' sums meet in LDS, alternating places)
+                        float* sO = reinterpret_cast<float*>(smem + L::O0) + (i & 1) * NWT * 64;
+                        if (ds == 1) sO[ws * 64 + l] = o;
+                        barrier();
+                        if (ds == 0) o += sO[ws * 64 + l];
+                    }
+                    if (mine && h2 == 0 && ds == 0) stf(out + ((long long)(row0 + i) * H + h) * s.dvp + vcol + c32, o);
                 }
             }
             wait_vm<0>();
             barrier();
             if (more) {
-                fetch_f(b + 1);
-                if (OUT) dma_q(b + 1);
-                dma_kv(b + 1);
+                fetch_f(j + 1);
+                if (OUT) dma_q(j + 1, (j + 1) & 1);
+                dma_kv(j + 1, (j + 1) & 1);
                 park_f((j + 1) & 1);
             }
             continue;
         }
         f32x16 o[2];
         if (OUT) {
-            wait_vm<KV_PIECES>();   // q^ has landed (k^ and v, requested after it, may be in flight)
+            wait_vm<Q_PIECES + V_PIECES>();   // q^ has landed (k^ and v, requested after it, may be in flight)
             barrier();
+            if (more) dma_q(j + 1, (j + 1) & 1);
             o[0] = zero_acc();
             o[1] = zero_acc();
+            int ql = q_lane + (j & 1) * L::QB;
+            hold(ql);
+            s16x8 qf[2][4];   // [buffer][16-channel half, token half]: the next 32 channels are requested in front of this step's products
+            auto load_q = [&](int td, s16x8 (&x)[4]) __attribute__((always_inline)) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int ch = 4 * (td0 + td) + 2 * (i >> 1);
+                    const s16x4 x0 = *reinterpret_cast<const s16x4*>(smem + (ql ^ (ch << 4)) + 32 * (i & 1) * QI::ROW);
+                    const s16x4 x1 = *reinterpret_cast<const s16x4*>(smem + (ql ^ ((ch + 1) << 4)) + 32 * (i & 1) * QI::ROW);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        x[i][e] = x0[e];
+                        x[i][4 + e] = x1[e];
+                    }
+                }
+            };
+            f32x4 fv[4];
+            load_f(fv, f, 0);
+            load_q(0, qf[0]);
 #pragma unroll
             for (int td = 0; td < TD; ++td) {
-                scale_rows(S[td], f, td);
+                if (td + 1 < TD) load_q(td + 1, qf[(td + 1) & 1]);
+                sched_fence();
+                scale_rows(S[td], fv);
+                if (td + 1 < TD) load_f(fv, f, td + 1);
 #pragma unroll
                 for (int u = 0; u < 2; ++u) {
                     const s16x8 hi = pack_frag(S[td], u);
@@ -290,36 +384,57 @@ __global__ __launch_bounds__(NW * 64) void linear_chunk_kernel(const bf16_t* pro
 #pragma unroll
                     for (int e = 0; e < 8; ++e) rest[8 * u + e] = S[td][8 * u + e] - bf2f(bf16_t(hi[e]));
                     const s16x8 lo = pack_frag(rest, u);
-                    const int ch = (32 * td + 16 * u) >> 3;
 #pragma unroll
                     for (int tt = 0; tt < 2; ++tt) {
-                        const int row = 32 * tt + c32;
-                        const char* base = sQ + row * QI::ROW + 8 * h2;
-                        const s16x4 x0 = *reinterpret_cast<const s16x4*>(base + ((ch ^ QI::swz(row)) << 4));
-                        const s16x4 x1 = *reinterpret_cast<const s16x4*>(base + (((ch + 1) ^ QI::swz(row)) << 4));
-                        s16x8 qf;
-#pragma unroll
-                        for (int e = 0; e < 4; ++e) {
-                            qf[e] = x0[e];
-                            qf[4 + e] = x1[e];
-                        }
-                        o[tt] = mfma32(hi, qf, o[tt]);
-                        o[tt] = mfma32(lo, qf, o[tt]);
+                        o[tt] = mfma32(hi, qf[td & 1][2 * u + tt], o[tt]);
+                        o[tt] = mfma32(lo, qf[td & 1][2 * u + tt], o[tt]);
                     }
                 }
+                sched_fence();
+            }
+            if (DS == 2) {   // the other half's partial sums of this wave's tokens, and its own of the other's
+                f32x4* give = reinterpret_cast<f32x4*>(smem + L::O0 + w * 4096) + l;
+#pragma unroll
+                for (int rg = 0; rg < 4; ++rg) {
+                    f32x4 v;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[e] = ds ? o[0][4 * rg + e] : o[1][4 * rg + e];
+                    give[64 * rg] = v;
+                }
+#pragma unroll
+                for (int r = 0; r < 16; ++r) o[0][r] = ds ? o[1][r] : o[0][r];
             }
         }
-        wait_vm<0>();
+        if (OUT) {   // k^ has landed (v and the next q^ may be in flight)
+            if (more)
+                wait_vm<V_PIECES + Q_PIECES>();
+            else
+                wait_vm<V_PIECES>();
+        } else {
+            wait_vm<0>();
+        }
         barrier();
+        if (!OUT && more) dma_kv(j + 1, (j + 1) & 1);
+        if (OUT && DS == 2) {
+            const f32x4* take = reinterpret_cast<const f32x4*>(smem + L::O0 + (ws + (1 - ds) * NW) * 4096) + l;
+#pragma unroll
+            for (int rg = 0; rg < 4; ++rg) {
+                const f32x4 v = take[64 * rg];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) o[0][4 * rg + e] += v[e];
+            }
+        }
         if (OUT) {   // scores: 16 x 16 tiles (a, b) of the lower triangle, rows = keys 4 q4 + r, columns = queries
-            for (int x = w; x < 10; x += NW) {
+            for (int x = w; x < 10; x += NWT) {
                 const int a = x < 1 ? 0 : x < 3 ? 1 : x < 6 ? 2 : 3, kb = x - a * (a + 1) / 2;
                 f32x4 sc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
-                const int kr = 16 * kb + c16, qr = 16 * a + c16;
+                int sl = s_lane;
+                hold(sl);
+                const int qr = 16 * a + c16;
 #pragma unroll
                 for (int kk = 0; kk < DP / 32; ++kk) {
-                    const s16x8 ka = *reinterpret_cast<const s16x8*>(sK + kr * QI::ROW + (((4 * kk + q4) ^ QI::swz(kr)) << 4));
-                    const s16x8 qb = *reinterpret_cast<const s16x8*>(sQ + qr * QI::ROW + (((4 * kk + q4) ^ QI::swz(qr)) << 4));
+                    const s16x8 ka = *reinterpret_cast<const s16x8*>(smem + L::K0 + 16 * kb * QI::ROW + (sl ^ (kk << 6)));
+                    const s16x8 qb = *reinterpret_cast<const s16x8*>(smem + L::Q0 + (j & 1) * L::QB + 16 * a * QI::ROW + (sl ^ (kk << 6)));
                     sc[kk & 1] = mfma16(ka, qb, sc[kk & 1]);
                 }
                 float p[4];
@@ -327,18 +442,24 @@ __global__ __launch_bounds__(NW * 64) void linear_chunk_kernel(const bf16_t* pro
                 for (int r = 0; r < 4; ++r) p[r] = a == kb && 4 * q4 + r > c16 ? 0.f : sc[0][r] + sc[1][r];
                 *reinterpret_cast<u32x2*>(sP + qr * L::PP + 16 * kb + 4 * q4) = u32x2{pack2bf(p[0], p[1]), pack2bf(p[2], p[3])};
             }
-            barrier();   // scores complete; every wave is done with q^
-            if (more) dma_q(b + 1);
+            if (more)
+                wait_vm<Q_PIECES>();   // v has landed
+            else
+                wait_vm<0>();
+            barrier();   // scores complete
         }
-        if (more) fetch_f(b + 1);
+        const char* sV = smem + L::V0 + (j & 1) * L::V_STEP;
+        if (more) fetch_f(j + 1);
         s16x8 vf[4];
 #pragma unroll
-        for (int jb = 0; jb < 4; ++jb) vf[jb] = VI::columns(sV, 16 * jb, 32 * w, l);
+        for (int jb = 0; jb < 4; ++jb) vf[jb] = VI::columns(sV, 16 * jb, 32 * ws, l);
         if (OUT) {
 #pragma unroll
-            for (int tt = 0; tt < 2; ++tt)
+            for (int i = 0; i < OT; ++i) {
+                const int tt = DS == 2 ? ds : i;
 #pragma unroll
-                for (int jb = 0; jb < 2 + 2 * tt; ++jb) {
+                for (int jb = 0; jb < 4; ++jb) {
+                    if (jb >= 2 && tt == 0) break;   // (the first half of the tokens sees the first half of the keys)
                     const bf16_t* src = sP + (32 * tt + c32) * L::PP + 16 * jb + 4 * h2;
                     const s16x4 x0 = *reinterpret_cast<const s16x4*>(src), x1 = *reinterpret_cast<const s16x4*>(src + 8);
                     s16x8 pf;
@@ -347,40 +468,65 @@ __global__ __launch_bounds__(NW * 64) void linear_chunk_kernel(const bf16_t* pro
                         pf[e] = x0[e];
                         pf[4 + e] = x1[e];
                     }
-                    o[tt] = mfma32(vf[jb], pf, o[tt]);
+                    o[i] = mfma32(vf[jb], pf, o[i]);
                 }
-#pragma unroll
-            for (int tt = 0; tt < 2; ++tt)
                 if (mine && 32 * tt + c32 < n) {
                     bf16_t* dst = out + ((long long)(row0 + 32 * tt + c32) * H + h) * s.dvp + vcol + 4 * h2;
 #pragma unroll
                     for (int rg = 0; rg < 4; ++rg)
                         *reinterpret_cast<u32x2*>(dst + 8 * rg) =
-                            u32x2{pack2bf(o[tt][4 * rg], o[tt][4 * rg + 1]), pack2bf(o[tt][4 * rg + 2], o[tt][4 * rg + 3])};
+                            u32x2{pack2bf(o[i][4 * rg], o[i][4 * rg + 1]), pack2bf(o[i][4 * rg + 2], o[i][4 * rg + 3])};
                 }
+            }
         }
+        if (!OUT) scale_all(f);
+        int t0 = t0_lane + (j & 1) * L::K_STEP, t1 = t1_lane + (j & 1) * L::K_STEP;
+        hold(t0);
+        hold(t1);
+        s16x8 kf[2][4];
+        auto load_k = [&](int td, s16x8 (&x)[4]) __attribute__((always_inline)) {
+#pragma unroll
+            for (int jb = 0; jb < 4; ++jb) {
+                const s16x4 x0 = ds_read_tr16(reinterpret_cast<const bf16_t*>(smem + (t0 ^ ((td0 + td) << 6)) + 16 * jb * QI::ROW));
+                const s16x4 x1 = ds_read_tr16(reinterpret_cast<const bf16_t*>(smem + (t1 ^ ((td0 + td) << 6)) + 16 * jb * QI::ROW));
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    x[jb][e] = x0[e];
+                    x[jb][4 + e] = x1[e];
+                }
+            }
+        };
+        load_k(0, kf[0]);
 #pragma unroll
         for (int td = 0; td < TD; ++td) {
-            if (!OUT) scale_rows(S[td], f, td);
+            if (td + 1 < TD) load_k(td + 1, kf[(td + 1) & 1]);
+            sched_fence();
 #pragma unroll
-            for (int jb = 0; jb < 4; ++jb) S[td] = mfma32(QI::columns(sK, 16 * jb, 32 * td, l), vf[jb], S[td]);
-            scale_rows(S[td], f + DP, td);
+            for (int jb = 0; jb < 4; ++jb) S[td] = mfma32(kf[td & 1][jb], vf[jb], S[td]);
+            sched_fence();
         }
         if (more) park_f((j + 1) & 1);
-        barrier();   // every wave is done with k^, v and (OUT = false) the factors' other half
-        if (more) dma_kv(b + 1);
+        if (OUT) barrier();   // every wave is done with k^ and v (OUT = false: the next block's first barrier says so)
+        if (OUT && more) dma_kv(j + 1, 0);
     }
+    if (!OUT || last) {   // what the last block left to the next one
+        f_in = ones;
+        park_f(nb & 1);
+        barrier();
+        scale_all(sF + (nb & 1) * DP);
+    }
+    if (!OUT && t < DP / 4 && vb == 0) *reinterpret_cast<f32x4*>(decays + ((long long)(c + 1) * H + h) * DP + 4 * t) = whole;
     if (!mine || (OUT && !last)) return;
     float* dst = OUT ? slot_state : states + ((long long)(c + 1) * H + h) * head_state + vcol + c32;
 #pragma unroll
     for (int i = 0; i < TD; ++i)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) dst[(long long)(32 * i + acc_row(r, l)) * s.dvp] = S[i][r];
+        for (int r = 0; r < 16; ++r) dst[(long long)(32 * (td0 + i) + acc_row(r, l)) * s.dvp] = S[i][r];
 }
 
-// first states of the chunks: states[c] holds chunk c - 1's state from zero; on return the state in front of chunk c.  A thread: four columns of one
+// first states of the chunks: states[c] and decays[c] hold chunk c - 1's state from zero and decay; on return states[c] is the state in front of chunk c.  A thread: four columns of one
 // channel, all chunks of a sequence.
-__global__ __launch_bounds__(256) void linear_scan_kernel(Lin s, const int32_t* blocks, const int32_t* chunks, const int32_t* seqs, const float* fac, float* states,
+__global__ __launch_bounds__(256) void linear_scan_kernel(Lin s, const int32_t* blocks, const int32_t* chunks, const int32_t* seqs, const float* decays, float* states,
                                                           const float* cache, const int32_t* slot, const int32_t* pos) {
     const int i = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y, c0 = seqs[2 * blockIdx.z], nc = seqs[2 * blockIdx.z + 1];
     const long long head_state = s.dp * s.dvp, H = s.H;
@@ -390,15 +536,24 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(Lin s, const int32_t* 
     if (pos[r0] > 0) x = *reinterpret_cast<const f32x4*>(cache + ((long long)slot[r0] * H + h) * head_state + 4 * i);
     float* at = states + ((long long)c0 * H + h) * head_state + 4 * i;
     *reinterpret_cast<f32x4*>(at) = x;
-    for (int c = c0; c + 1 < c0 + nc; ++c) {
-        at += H * head_state;
-        const f32x4 own = *reinterpret_cast<const f32x4*>(at);
-        float a = 1.f;
-        const int b0 = chunks[4 * c], nb = chunks[4 * c + 1];
-        for (int b = b0; b < b0 + nb; ++b) a *= fac[(((long long)b * H + h) * 3 + 2) * s.dp + d];
+    constexpr int AHEAD = 4;
+    const long long step = H * head_state;
+    for (int c = 1; c < nc; c += AHEAD) {
+        f32x4 own[AHEAD];
+        float a[AHEAD];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) x[e] = a * x[e] + own[e];
-        *reinterpret_cast<f32x4*>(at) = x;
+        for (int u = 0; u < AHEAD; ++u) {
+            const int k = min(c + u, nc - 1);
+            own[u] = *reinterpret_cast<const f32x4*>(at + k * step);
+            a[u] = decays[((long long)(c0 + k) * H + h) * s.dp + d];
+        }
+#pragma unroll
+        for (int u = 0; u < AHEAD; ++u) {
+            if (c + u >= nc) break;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[e] = a[u] * x[e] + own[u][e];
+            *reinterpret_cast<f32x4*>(at + (c + u) * step) = x;
+        }
     }
 }
 
@@ -445,7 +600,7 @@ int shape_ok(const Lin* s) {
 }
 
 struct ChunkScratch {
-    float *fac, *alpha, *states;
+    float *fac, *alpha, *states, *decays;
     int32_t* marked;
     int64_t bytes;
 };
@@ -461,6 +616,7 @@ ChunkScratch layout(const Lin& s, int64_t T, int64_t n_blocks, int64_t n_chunks,
     z.marked = reinterpret_cast<int32_t*>(take(4 * n_blocks * s.H));
     z.alpha = reinterpret_cast<float*>(take(4 * T * s.H * s.dp));
     z.states = reinterpret_cast<float*>(take(4 * n_chunks * s.H * s.dp * s.dvp));
+    z.decays = reinterpret_cast<float*>(take(4 * n_chunks * s.H * s.dp));
     z.bytes = at;
     return z;
 }
@@ -477,25 +633,27 @@ struct ChunkArgs {
 };
 template <int DP, int NW>
 int launch_chunks(const ChunkArgs& a) {
-    using L = ChunkSmem<DP, NW>;
+    using L = ChunkSmem<DP, NW, true>;
     const Lin& s = a.s;
-    const dim3 grid(unsigned((s.dvp + L::VB - 1) / L::VB), unsigned(s.H), unsigned(a.n_chunks)), block(NW * 64);
+    const int64_t nvb = (s.dvp + L::VB - 1) / L::VB;
+    const dim3 grid(unsigned(8 * nvb * ((s.H * a.n_chunks + 7) / 8))), block(L::WAVES * 64);
     if (a.n_chunks > a.n_seq) {
-        ARIA_LAUNCH((linear_chunk_kernel<DP, NW, false>), grid, block, size_t(L::BYTES), a.stream, (const bf16_t*)a.proj, s, a.blocks, a.chunks,
-                    (const float*)a.z.fac, (const int32_t*)a.z.marked, (const float*)a.z.alpha, a.z.states, a.state, a.slot, a.pos, a.out);
+        ARIA_LAUNCH((linear_chunk_kernel<DP, NW, false>), grid, block, size_t(ChunkSmem<DP, NW, false>::BYTES), a.stream, (const bf16_t*)a.proj, s, a.blocks,
+                    a.chunks, (const float*)a.z.fac, (const int32_t*)a.z.marked, (const float*)a.z.alpha, a.z.states, a.z.decays, a.state, a.slot, a.pos, a.out,
+                    int(a.n_chunks));
         const int64_t n4 = s.dp * s.dvp / 4;
         ARIA_LAUNCH(linear_scan_kernel, dim3(unsigned((n4 + 255) / 256), unsigned(s.H), unsigned(a.n_seq)), dim3(256), 0, a.stream, s, a.blocks, a.chunks,
-                    a.seqs, (const float*)a.z.fac, a.z.states, (const float*)a.state, a.slot, a.pos);
+                    a.seqs, (const float*)a.z.decays, a.z.states, (const float*)a.state, a.slot, a.pos);
     }
     ARIA_LAUNCH((linear_chunk_kernel<DP, NW, true>), grid, block, size_t(L::BYTES), a.stream, (const bf16_t*)a.proj, s, a.blocks, a.chunks, (const float*)a.z.fac,
-                (const int32_t*)a.z.marked, (const float*)a.z.alpha, a.z.states, a.state, a.slot, a.pos, a.out);
+                (const int32_t*)a.z.marked, (const float*)a.z.alpha, a.z.states, a.z.decays, a.state, a.slot, a.pos, a.out, int(a.n_chunks));
     return aria_check_launch();
 }
 template <int DP>
 int run_chunks(const ChunkArgs& a) {
-    const size_t lds = size_t(BLK * DP + (256 / (DP / 2)) * DP + 4 + BLK * a.s.rank) * 4;
+    const size_t lds = size_t((PREP / (DP / 2) + 1) * DP + 8 + BLK * a.s.rank) * 4;
     if (lds > 160 * 1024) return ARIA_ERR_UNSUPPORTED;
-    ARIA_LAUNCH((linear_prepare_kernel<DP>), dim3(unsigned(a.n_blocks), unsigned(a.s.H)), dim3(256), lds, a.stream, a.proj, a.s, a.blocks, a.z.fac, a.z.marked,
+    ARIA_LAUNCH((linear_prepare_kernel<DP>), dim3(unsigned(a.n_blocks), unsigned(a.s.H)), dim3(PREP), lds, a.stream, a.proj, a.s, a.blocks, a.z.fac, a.z.marked,
                 a.z.alpha);
     return a.s.dvp <= 64 ? launch_chunks<DP, 2>(a) : launch_chunks<DP, 4>(a);
 }

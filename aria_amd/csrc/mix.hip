@@ -102,12 +102,17 @@ __global__ __launch_bounds__(256) void mix_finish_kernel(const float* part_o, co
         const float wt = f / wave_sum_bcast(sum * f);   // lane = split
         const float* po = part_o + ((long long)tok * splits * H + h) * dvp;
         float acc[4] = {0.f, 0.f, 0.f, 0.f};
-        for (int j = 0; j < splits; ++j) {              // (a split without rows left its slab unwritten: skipped, not multiplied)
-            const float wj = shfl(wt, j);
-            if (wj != 0.f) {
+        for (int j = 0; j < splits; j += 8) {           // (a split without rows left its slab unwritten: selected away, not multiplied)
+            float x[8][4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i)
-                    if (l + 64 * i < dvp) acc[i] += wj * po[(long long)j * H * dvp + l + 64 * i];
+            for (int u = 0; u < 8; ++u)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) x[u][i] = po[(long long)min(j + u, splits - 1) * H * dvp + min(l + 64 * i, dvp - 1)];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) {
+                const float wj = j + u < splits ? shfl(wt, j + u) : 0.f;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[i] += wj != 0.f ? wj * x[u][i] : 0.f;
             }
         }
 #pragma unroll
@@ -151,7 +156,7 @@ Scratch layout(const AriaMixStack& st, const AriaMixLayer* L, int64_t T, int64_t
         const AriaLinearShape& r = L[i].right;
         ldp = std::max(ldp, r.ldp);
         lo = std::max(lo, r.H * r.dvp);
-        ls = std::max(ls, r.H * ((r.dvp + 15) / 16));
+        ls = std::max(ls, r.H * step_blocks(r, T));
         if (L[i].norm2) act = std::max(act, L[i].ff);
         if (L[i].kind) {
             const Chunk& s = L[i].left;
@@ -208,9 +213,9 @@ int64_t aria_mix_decode_scratch(const AriaMixStack* st, const AriaMixLayer* runs
     return layout(*st, runs, T, max_len, nullptr).bytes;
 }
 
-int aria_mix_decode(const AriaMixStack* st, const AriaMixLayer* L, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos,
-                    const int32_t* seq_rows, int64_t max_len, float* logits, void* scratch, int64_t scratch_bytes, void* stream) {
-    if (!st || !L || !ids || !slot || !pos || !seq_rows || !logits || !scratch || T < 0 || max_len <= 0 || st->n_runs <= 0) return ARIA_ERR_INVALID;
+int aria_mix_decode(const AriaMixStack* st, const AriaMixLayer* L, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos, int64_t max_len,
+                    float* logits, void* scratch, int64_t scratch_bytes, void* stream) {
+    if (!st || !L || !ids || !slot || !pos || !logits || !scratch || T < 0 || max_len <= 0 || st->n_runs <= 0) return ARIA_ERR_INVALID;
     if (T == 0) return ARIA_OK;
     if ((st->D & 7) || (reinterpret_cast<uintptr_t>(scratch) & 15)) return ARIA_ERR_ALIGN;
     const Scratch z = layout(*st, L, T, max_len, static_cast<char*>(scratch));
@@ -244,10 +249,10 @@ int aria_mix_decode(const AriaMixStack* st, const AriaMixLayer* L, int64_t T, co
         const RowsIn in = input(y.w_in, nullptr, r.ldp);
         if (y.kind == 0) {
             rc = launch_rows(RowsPair{{in, in}}, 1, T, StoreRows{{z.proj, z.proj}, (long long)r.ldp}, stream);
-            if (rc == ARIA_OK) rc = launch_step<bf16_t>(z.proj, r, y.state, slot, pos, seq_rows, T, z.lo, StepOut{z.lsums, y.norm, (long long)y.g_off}, stream);
+            if (rc == ARIA_OK) rc = launch_step<bf16_t>(z.proj, r, y.state, slot, pos, nullptr, T, z.lo, StepOut{z.lsums, y.norm, (long long)y.g_off}, stream);
             RowsIn o{bf(y.w_o), nullptr, z.lo, (long long)(r.H * r.dvp), int(r.H * r.dvp), int(D)};
             o.sq = z.lsums;
-            o.sq_n = int(r.H * ((r.dvp + 15) / 16));
+            o.sq_n = int(r.H * step_blocks(r, T));
             o.inv_n = 1.f / float(r.H * r.dv);
             o.eps = st->eps;
             if (rc == ARIA_OK) rc = launch_rows(RowsPair{{o, o}}, 1, T, residual(!y.norm2), stream);
@@ -260,7 +265,7 @@ int aria_mix_decode(const AriaMixStack* st, const AriaMixLayer* L, int64_t T, co
             const TileAttn ta{z.proj + s.q_off, (long long)s.ldp, int(s.dq), bf(y.ring), (long long)(s.G * s.cap * cw), (long long)(s.cap * cw), cw, int(s.dq), int(s.dq),
                               int(s.dvp), int(s.H), int(s.H / s.G), int(std::min<int64_t>(s.size, INT32_MAX)), s.scale};
             if (rc == ARIA_OK) rc = launch_tile_attn(ta, slot, pos, z.part_o, z.part_ml, T, ns, stream);
-            if (rc == ARIA_OK) rc = launch_step<bf16_t>(z.proj, r, y.state, slot, pos, seq_rows, T, z.lo, StepOut{}, stream);
+            if (rc == ARIA_OK) rc = launch_step<bf16_t>(z.proj, r, y.state, slot, pos, nullptr, T, z.lo, StepOut{}, stream);
             if (rc != ARIA_OK) break;
             ARIA_LAUNCH(mix_finish_kernel, dim3(unsigned((T * (s.H + r.H) + 3) / 4)), dim3(256), 0, stream, (const float*)z.part_o, (const float*)z.part_ml, int(ns),
                         int(s.H), int(s.dvp), z.ao, z.lo, (const bf16_t*)z.proj, r, (long long)y.g_off, y.norm, st->eps, int(T));

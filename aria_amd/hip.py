@@ -122,7 +122,7 @@ SIGNATURES = {
     "aria_linear_chunks_scratch": [P, I64, I64, I64],
     "aria_linear_chunks": [P, P, P, P, P, P, I64, P, I64, P, I64, P, I64, P, I64, P],
     "aria_mix_decode_scratch": [P, P, I64, I64],
-    "aria_mix_decode": [P, P, I64, P, P, P, P, I64, P, P, I64, P],
+    "aria_mix_decode": [P, P, I64, P, P, P, I64, P, P, I64, P],
     "aria_norm_gate": [P, P, I64, P, I64, P, I64, I64, I64, I64, F32, I32, I32, P],
 }
 

@@ -220,7 +220,6 @@ class _DecodeTables:
         logits = torch.empty((T, self.rows), dtype=f32, device=self.device)
         for t in (batch.ids, batch.slot, batch.pos):
             assert t.dtype == torch.int32 and t.is_contiguous() and t.numel() == T
-        assert batch.cu.dtype == torch.int32 and batch.cu.is_contiguous() and batch.cu.numel() == T + 1
-        lib.call("aria_mix_decode", stack, runs, T, batch.ids.data_ptr(), batch.slot.data_ptr(), batch.pos.data_ptr(), batch.cu.data_ptr(), batch.max_len,
+        lib.call("aria_mix_decode", stack, runs, T, batch.ids.data_ptr(), batch.slot.data_ptr(), batch.pos.data_ptr(), batch.max_len,
                  logits.data_ptr(), self.scratch.data_ptr(), self.scratch.numel(), ops._stream(logits))
         return logits[:, :self.vocab]

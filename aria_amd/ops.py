@@ -1247,7 +1247,15 @@ def linear_step(shape, proj: torch.Tensor, state: torch.Tensor, batch) -> torch.
     return out
 
 
-LINEAR_BLOCK = 64   # rows of a matrix-pipe step of aria_linear_chunks
+LINEAR_BLOCK = 64         # rows of a matrix-pipe step of aria_linear_chunks
+LINEAR_WORKGROUPS = 256   # compute units: a launch should fill them once (a workgroup: a chunk, a head, 128 value columns)
+
+
+def linear_chunking(shape, lengths) -> int:
+    """Blocks per chunk: the fewest with which every workgroup of a launch is resident at once (two a compute unit up to 128 channels)."""
+    per_chunk = LINEAR_WORKGROUPS * (2 if shape.dp <= 128 else 1) // (shape.H * -(-shape.dvp // 128))
+    counts = [-(-n // LINEAR_BLOCK) for n in lengths]
+    return next((k for k in range(1, 64) if sum(-(-c // k) for c in counts) <= per_chunk), 64)
 
 
 def linear_chunks(shape, proj: torch.Tensor, state: torch.Tensor, batch) -> torch.Tensor:
@@ -1256,9 +1264,7 @@ def linear_chunks(shape, proj: torch.Tensor, state: torch.Tensor, batch) -> torc
 
     T = _chk_rows(_chk(proj), shape.ldp, batch)
     _chk_state(shape, state, batch)
-    # about one workgroup per compute unit: chunks x heads x 128-column blocks of the values
-    rows = max(1, T * shape.H * ((shape.dvp + 127) // 128) // 256)
-    blocks, chunks, seqs = batch.linear_tables(LINEAR_BLOCK, max(1, -(-rows // LINEAR_BLOCK)))
+    blocks, chunks, seqs = batch.linear_tables(LINEAR_BLOCK, linear_chunking(shape, batch.lengths))
     lib, ref = hip.get_lib(), ctypes.byref(shape)
     nb, nc, ns = blocks.shape[0], chunks.shape[0], seqs.shape[0]
     scratch = torch.empty(int(lib.cdll.aria_linear_chunks_scratch(ref, T, nb, nc)), dtype=torch.uint8, device=proj.device)

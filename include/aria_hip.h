@@ -630,10 +630,10 @@ typedef struct {
     const void *embed, *head;
 } AriaMixStack;
 int64_t aria_mix_decode_scratch(const AriaMixStack* stack, const AriaMixLayer* runs, int64_t T, int64_t max_len);
-/* One step of T single tokens of T sequences (seq_rows: 0 .. T, int32 on the device), as aria_latent_decode: logits fp32 [T, V], soft-capped.
+/* One step of T single tokens of T sequences, as aria_latent_decode: logits fp32 [T, V], soft-capped.
  * ARIA_ERR_UNSUPPORTED: widths beyond the matrix-pipe attention. */
-int aria_mix_decode(const AriaMixStack* stack, const AriaMixLayer* runs, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos,
-                    const int32_t* seq_rows, int64_t max_len, float* logits, void* scratch, int64_t scratch_bytes, void* stream);
+int aria_mix_decode(const AriaMixStack* stack, const AriaMixLayer* runs, int64_t T, const int32_t* ids, const int32_t* slot, const int32_t* pos, int64_t max_len,
+                    float* logits, void* scratch, int64_t scratch_bytes, void* stream);
 
 #ifdef __cplusplus
 }
