@@ -150,6 +150,13 @@ struct Scratch {
     int64_t bytes;
 };
 int64_t keys_of(const Chunk& s, int64_t max_len) { return std::min(s.size, max_len); }
+int64_t splits_of(const Chunk& s, int64_t T, int64_t max_len) { return tile_attn_splits(s.dq + s.dvp, s.H, s.H / s.G, T, keys_of(s, max_len)); }
+bool tile_shape_ok(const Chunk& s) { return tile_attn_class(s.dq, s.dvp, s.dq + s.dvp) && s.dvp <= 256; }
+TileAttn tile_args(const Chunk& s, const bf16_t* proj, const void* ring) {
+    const int cw = int(s.dq + s.dvp);
+    return TileAttn{proj + s.q_off, (long long)s.ldp, int(s.dq), static_cast<const bf16_t*>(ring), (long long)(s.G * s.cap * cw), (long long)(s.cap * cw), cw, int(s.dq),
+                    int(s.dq), int(s.dvp), int(s.H), int(s.H / s.G), int(std::min<int64_t>(s.size, INT32_MAX)), s.scale};
+}
 Scratch layout(const AriaMixStack& st, const AriaMixLayer* L, int64_t T, int64_t max_len, char* base) {
     int64_t ldp = 0, ao = 0, lo = 0, ls = 0, act = 0, po = 0, ml = 0;
     for (int64_t i = 0; i < st.n_runs; ++i) {
@@ -160,7 +167,7 @@ Scratch layout(const AriaMixStack& st, const AriaMixLayer* L, int64_t T, int64_t
         if (L[i].norm2) act = std::max(act, L[i].ff);
         if (L[i].kind) {
             const Chunk& s = L[i].left;
-            const int64_t ns = tile_attn_splits(s.dq + s.dvp, s.H, s.H / s.G, T, keys_of(s, max_len));
+            const int64_t ns = splits_of(s, T, max_len);
             ao = std::max(ao, s.H * s.dvp);
             po = std::max(po, ns * s.H * s.dvp);
             ml = std::max(ml, ns * s.H * 2);
@@ -200,13 +207,35 @@ int layer_ok(const AriaMixLayer& y, int64_t max_len) {
     if (!y.w_o_left || !y.out_left || !y.out_right || !y.ring || s.H <= 0 || s.G <= 0 || s.H % s.G || s.size <= 0 || keys_of(s, max_len) > s.cap || s.ldp != r.ldp ||
         s.q_off + s.H * s.dq > s.ldp || s.k_off + s.G * s.dq > s.ldp || s.v_off + s.G * s.dvp > s.ldp || (s.q_off & 7) || (s.dq & 7) || (s.dvp & 7))
         return ARIA_ERR_INVALID;
-    if (!tile_attn_class(s.dq, s.dvp, s.dq + s.dvp) || s.dvp > 256) return ARIA_ERR_UNSUPPORTED;
-    return ARIA_OK;
+    return tile_shape_ok(s) ? ARIA_OK : ARIA_ERR_UNSUPPORTED;
 }
 
 }  // namespace
 
 extern "C" {
+
+int64_t aria_chunk_decode_scratch(const AriaChunkShape* s, int64_t T, int64_t max_len) {
+    if (!s || T <= 0 || max_len <= 0 || s->H <= 0 || s->G <= 0 || !tile_shape_ok(*s)) return 0;
+    return 4 * T * splits_of(*s, T, max_len) * s->H * (s->dvp + 2);
+}
+
+int aria_chunk_decode(const void* proj, const void* cache, const AriaChunkShape* s, const int32_t* slot, const int32_t* pos, int64_t max_len, void* out, int64_t T,
+                      void* scratch, int64_t scratch_bytes, void* stream) {
+    if (!proj || !cache || !s || !slot || !pos || !out || !scratch || T < 0 || max_len <= 0 || s->H <= 0 || s->G <= 0 || s->H % s->G || s->size <= 0 ||
+        keys_of(*s, max_len) > s->cap || s->q_off + s->H * s->dq > s->ldp)
+        return ARIA_ERR_INVALID;
+    if ((s->ldp & 7) || (s->q_off & 7) || (reinterpret_cast<uintptr_t>(proj) & 15) || (reinterpret_cast<uintptr_t>(cache) & 15)) return ARIA_ERR_ALIGN;
+    if (!tile_shape_ok(*s) || T > 65535) return ARIA_ERR_UNSUPPORTED;
+    if (T == 0) return ARIA_OK;
+    if (scratch_bytes < aria_chunk_decode_scratch(s, T, max_len)) return ARIA_ERR_INVALID;
+    const int64_t ns = splits_of(*s, T, max_len);
+    float *po = static_cast<float*>(scratch), *ml = po + T * ns * s->H * s->dvp;
+    if (const int rc = launch_tile_attn(tile_args(*s, static_cast<const bf16_t*>(proj), cache), slot, pos, po, ml, T, ns, stream)) return rc;
+    ARIA_LAUNCH(mix_finish_kernel, dim3(unsigned((T * s->H + 3) / 4)), dim3(256), 0, stream, (const float*)po, (const float*)ml, int(ns), int(s->H), int(s->dvp),
+                static_cast<bf16_t*>(out), static_cast<bf16_t*>(nullptr), static_cast<const bf16_t*>(nullptr), AriaLinearShape{}, 0ll,
+                static_cast<const float*>(nullptr), 0.f, int(T));
+    return aria_check_launch();
+}
 
 int64_t aria_mix_decode_scratch(const AriaMixStack* st, const AriaMixLayer* runs, int64_t T, int64_t max_len) {
     if (!st || !runs || T <= 0 || max_len <= 0) return 0;
@@ -259,12 +288,9 @@ int aria_mix_decode(const AriaMixStack* st, const AriaMixLayer* L, int64_t T, co
             scaled = false;
         } else {
             const Chunk& s = y.left;
-            const int64_t keys = keys_of(s, max_len), ns = tile_attn_splits(s.dq + s.dvp, s.H, s.H / s.G, T, keys);
+            const int64_t ns = splits_of(s, T, max_len);
             rc = launch_rows(RowsPair{{in, in}}, 1, T, StoreRowsAndCache{z.proj, static_cast<bf16_t*>(y.ring), s, slot, pos}, stream);
-            const int cw = int(s.dq + s.dvp);
-            const TileAttn ta{z.proj + s.q_off, (long long)s.ldp, int(s.dq), bf(y.ring), (long long)(s.G * s.cap * cw), (long long)(s.cap * cw), cw, int(s.dq), int(s.dq),
-                              int(s.dvp), int(s.H), int(s.H / s.G), int(std::min<int64_t>(s.size, INT32_MAX)), s.scale};
-            if (rc == ARIA_OK) rc = launch_tile_attn(ta, slot, pos, z.part_o, z.part_ml, T, ns, stream);
+            if (rc == ARIA_OK) rc = launch_tile_attn(tile_args(s, z.proj, y.ring), slot, pos, z.part_o, z.part_ml, T, ns, stream);
             if (rc == ARIA_OK) rc = launch_step<bf16_t>(z.proj, r, y.state, slot, pos, nullptr, T, z.lo, StepOut{}, stream);
             if (rc != ARIA_OK) break;
             ARIA_LAUNCH(mix_finish_kernel, dim3(unsigned((T * (s.H + r.H) + 3) / 4)), dim3(256), 0, stream, (const float*)z.part_o, (const float*)z.part_ml, int(ns),

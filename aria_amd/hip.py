@@ -24,7 +24,8 @@ ERRORS = {
 P, I64, I32, F32 = c_void_p, c_int64, c_int, c_float
 RESTYPES = {"aria_gemm_workspace_bytes": c_int64, "aria_decode_scratch_bytes": c_int64, "aria_decode_graph_create": c_void_p,
             "aria_decode_graph_destroy": None, "aria_decode_attn_workspace_bytes": c_int64,
-            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64, "aria_linear_chunks_scratch": c_int64, "aria_mix_decode_scratch": c_int64}  # everything else returns an int status
+            "aria_latent_decode_scratch": c_int64, "aria_latent_splits": c_int64, "aria_linear_chunks_scratch": c_int64, "aria_mix_decode_scratch": c_int64,
+            "aria_chunk_decode_scratch": c_int64}  # everything else returns an int status
 
 # name -> argtypes (all return int).  Kept in one table so tests can check that the shared
 # library exports every symbol the header declares.
@@ -117,6 +118,8 @@ SIGNATURES = {
     "aria_rms_stream": [P, I64, I64, I32, P],
     "aria_softcap": [P, I64, F32, P],
     "aria_chunk_attn_any": [P, P, P, P, P, P, P, P, I64, I32, P],
+    "aria_chunk_decode_scratch": [P, I64, I64],
+    "aria_chunk_decode": [P, P, P, P, P, I64, P, I64, P, I64, P],
     "aria_chunk_rows": [P, P, P, P, P, P, P, I64, I32, P],
     "aria_linear_step": [P, P, P, P, P, P, I64, P, I32, P],
     "aria_linear_chunks_scratch": [P, I64, I64, I64],

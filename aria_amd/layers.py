@@ -230,6 +230,8 @@ class ChunkAttention(nn.Module):
             q, k, v = (proj[:, g[n]:] for n in ("q_off", "k_off", "v_off"))
             o = ops.attention_varlen(q, k, v, cu, longest, g["H"], g["dq"], g["dvp"], g["scale"], kv_heads=g["G"])
             ops.chunk_rows(s, proj, cache.rows, batch)
+        elif batch.longest == 1 and self.flash:
+            o = ops.chunk_attention_decode(s, proj, cache.rows, batch)
         else:
             o = ops.chunk_attention_any(s, proj, cache.rows, batch)
         return ops.linear_any(o, self.w_o)

@@ -1218,6 +1218,19 @@ def chunk_attention_any(shape, proj: torch.Tensor, cache: torch.Tensor, batch) -
     return out
 
 
+def chunk_attention_decode(shape, proj: torch.Tensor, cache: torch.Tensor, batch) -> torch.Tensor:
+    """One token per sequence in bf16: its key and value into the cache, then attention over the chunk's rows on the matrix pipe.  -> [T, H dvp]"""
+    import ctypes
+
+    T, ref, lib = _chk_rows(_chk(proj), shape.ldp, batch), ctypes.byref(shape), hip.get_lib()
+    assert batch.longest == 1
+    chunk_rows(shape, proj, cache, batch)
+    scratch = torch.empty(int(lib.cdll.aria_chunk_decode_scratch(ref, T, batch.max_len)), dtype=torch.uint8, device=proj.device)
+    out = torch.empty((T, shape.H * shape.dvp), dtype=bf16, device=proj.device)
+    lib.call("aria_chunk_decode", _p(proj), _p(cache), ref, _p(batch.slot), _p(batch.pos), batch.max_len, _p(out), T, _p(scratch), scratch.numel(), _stream(proj))
+    return out
+
+
 def _chk_ring(shape, cache: torch.Tensor, proj: torch.Tensor, batch) -> None:
     if cache.shape[1:] != (shape.G, shape.cap, shape.dq + shape.dvp) or not cache.is_contiguous() or cache.dtype != proj.dtype:
         raise ValueError("the cache does not fit the shape")

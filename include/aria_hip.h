@@ -571,6 +571,11 @@ typedef struct {
  * cache, the call's own from proj (call aria_chunk_rows afterwards). */
 int aria_chunk_attn_any(const void* proj, const void* cache, const AriaChunkShape* s, const int32_t* slot, const int32_t* pos, const int32_t* seq,
                         const int32_t* cu, void* out, int64_t T, int f32, void* stream);
+/* Single tokens in bf16 on the matrix pipe, their keys and values already in the cache (aria_chunk_rows): out [T, H dvp].  max_len >= the largest position
+ * + 1.  dq, dvp multiples of 32 that add up to a multiple of 64, dq <= 320, dvp <= 256 (else ARIA_ERR_UNSUPPORTED, scratch size 0). */
+int64_t aria_chunk_decode_scratch(const AriaChunkShape* s, int64_t T, int64_t max_len);
+int aria_chunk_decode(const void* proj, const void* cache, const AriaChunkShape* s, const int32_t* slot, const int32_t* pos, int64_t max_len, void* out, int64_t T,
+                      void* scratch, int64_t scratch_bytes, void* stream);
 /* Writes the call's keys and values to the cache (of the positions that share a row, the last one). */
 int aria_chunk_rows(const void* proj, void* cache, const AriaChunkShape* s, const int32_t* slot, const int32_t* pos, const int32_t* seq, const int32_t* cu,
                     int64_t T, int f32, void* stream);

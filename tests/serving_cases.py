@@ -1,4 +1,4 @@
-"""The serving layer: the scheduler driving a gptfast (Aria) decoder and Duguzen alike, the command line, the trace runner.  Shared by
+"""The serving layer: the scheduler driving a gptfast (Aria) decoder, Duguzen and Kozipel alike, the command line, the trace runner.  Shared by
 tests/test_emu_serving.py (CPU) and tests/test_gpu_serving.py (hardware)."""
 import io
 import json
@@ -6,6 +6,7 @@ import os
 
 import torch
 
+from tests import kozipel_cases as K
 from tests import latent_cases as L
 
 bf16, f32 = torch.bfloat16, torch.float32
@@ -70,21 +71,25 @@ def case_gptfast_generate(dev):
             assert float(row.max() - row[t]) <= 0.05 * float(row.std())
 
 
-def write_model(tmp, name="equal", seed=12):
+DESIGNS = {"duguzen": (L, "equal"), "kozipel": (K, "last")}   # cases module, configuration
+
+
+def write_model(tmp, design="duguzen", seed=12):
     from safetensors.torch import save_file
 
-    cfg = L.CONFIGS[name]
-    w = L.checkpoint(cfg, seed=seed)
+    cases, name = DESIGNS[design]
+    cfg = cases.CONFIGS[name]
+    w = cases.checkpoint(cfg, seed=seed)
     (tmp / "config.json").write_text(json.dumps(cfg))
     save_file(w, str(tmp / "model.safetensors"))
     return cfg, w
 
 
-def case_command_line(dev, tmp):
+def case_command_line(dev, tmp, design="duguzen"):
     from aria_amd import inference as I
     from aria_amd import registry, serving
 
-    cfg, _ = write_model(tmp)
+    cfg, _ = write_model(tmp, design)
     a = I.parse_arguments(["--base_model_path", str(tmp), "--prompt_ids", "5,17,3", "--prompt_ids", "9", "--max_new_tokens", "3", "--temperature", "0",
                            "--dtype", "float32"])
     got = I.generate_ids(a, dev)
@@ -92,17 +97,19 @@ def case_command_line(dev, tmp):
     assert got == serving.generate(m, [[5, 17, 3], [9]], 3, temperature=0) and all(0 <= t < cfg["vocab"] for g in got for t in g)
 
 
-def case_trace_run(dev, tmp, dtype="float32"):
+def case_trace_run(dev, tmp, dtype="float32", design="duguzen"):
     """Steps in, logits out: the files, the order of rows, ``done`` lines, requests that end, a second batch, and the values against the oracle."""
     import numpy as np
 
     from aria_amd import trace_run
-    from oracle import latent_oracle as O
 
-    cfg, w = write_model(tmp)
+    cases = DESIGNS[design][0]
+    O = cases.O
+    cfg, w = write_model(tmp, design)
     out = tmp / "out"
     out.mkdir()
-    a, b, c = ([int(t) for t in L.clear_tokens(cfg, w, n, seed=n)] for n in (6, 4, 3))
+    draw = L.clear_tokens if cases is L else (lambda cfg, w, n, seed: L.tokens(cfg, n, seed))
+    a, b, c = ([int(t) for t in draw(cfg, w, n, seed=n)] for n in (6, 4, 3))
     steps = [dict(step=0, entries=[dict(id="a", tokens=a[:5], want=[0, 4]), dict(id="b", tokens=b[:2], want=[])], end=[]),
              dict(step=1, entries=[dict(id="b", tokens=[b[2]], want=[]), dict(id="a", tokens=[a[5]], want=[])], end=["a"]),
              dict(step=2, entries=[dict(id="b", tokens=[b[3]], want=[0])], end=["b"]),
@@ -115,7 +122,7 @@ def case_trace_run(dev, tmp, dtype="float32"):
     want = {0: O.forward(cfg, w, a)[[0, 4]], 2: O.forward(cfg, w, b)[[3]], 3: O.forward(cfg, w, c)[[2, 1]]}
     for n, x in want.items():
         got = torch.from_numpy(np.fromfile(out / f"{n}.f32", dtype="<f4").reshape(x.shape).copy())
-        assert L.logit_err(got, x) < (5e-5 if dtype == "float32" else L.model_tol(cfg, w, [a, b, c], bf16)), n
+        assert L.logit_err(got, x) < (5e-5 if dtype == "float32" else cases.model_tol(cfg, w, [a, b, c], bf16)), n
 
 
 def case_registry():
@@ -126,5 +133,6 @@ def case_registry():
     assert registry.architecture({"architecture": "Duguzen"}) == "Duguzen"
     assert registry.architecture({"architectures": ["AriaForConditionalGeneration"]}) == registry.architecture({"model_type": "aria"})
     assert registry.resolve({"architecture": "Duguzen"})[1].__name__ == "DuguzenForCausalLM"
+    assert registry.resolve({"architecture": "Kozipel"})[1].__name__ == "KozipelForCausalLM"
     with pytest.raises(ValueError):
         registry.architecture({"architecture": "nothing"})

@@ -23,12 +23,17 @@ def test_gptfast_generate():
     C.case_gptfast_generate(DEV)
 
 
-def test_command_line(tmp_path):
-    C.case_command_line(DEV, tmp_path)
+designs = pytest.mark.parametrize("design", sorted(C.DESIGNS))
 
 
-def test_trace_run(tmp_path):
-    C.case_trace_run(DEV, tmp_path)
+@designs
+def test_command_line(tmp_path, design):
+    C.case_command_line(DEV, tmp_path, design)
+
+
+@designs
+def test_trace_run(tmp_path, design):
+    C.case_trace_run(DEV, tmp_path, design=design)
 
 
 def test_registry():

@@ -30,18 +30,24 @@ def test_gptfast_generate():
     C.case_gptfast_generate(DEV)
 
 
-def test_command_line(tmp_path):
-    C.case_command_line(DEV, tmp_path)
+designs = pytest.mark.parametrize("design", sorted(C.DESIGNS))
 
 
+@designs
+def test_command_line(tmp_path, design):
+    C.case_command_line(DEV, tmp_path, design)
+
+
+@designs
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_trace_run(tmp_path, dtype):
-    C.case_trace_run(DEV, tmp_path, dtype)
+def test_trace_run(tmp_path, dtype, design):
+    C.case_trace_run(DEV, tmp_path, dtype, design)
 
 
-def test_trace_run_program(tmp_path):
+@designs
+def test_trace_run_program(tmp_path, design):
     """bin/trace_run as a program: a step a line, an answer before the next."""
-    C.write_model(tmp_path)
+    cfg, _ = C.write_model(tmp_path, design)
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
     p = subprocess.Popen([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", "bfloat16", "--out", str(tmp_path),
                           "--max-tokens", "8"], stdin=subprocess.PIPE, stdout=subprocess.PIPE, text=True)
@@ -50,7 +56,7 @@ def test_trace_run_program(tmp_path):
             p.stdin.write(json.dumps(dict(step=n, entries=[dict(id="x", tokens=toks, want=[0])], end=["x"] if n == 2 else [])) + "\n")
             p.stdin.flush()
             assert p.stdout.readline().strip() == f"done {n}"
-            assert os.path.getsize(tmp_path / f"{n}.f32") == 4 * 32
+            assert os.path.getsize(tmp_path / f"{n}.f32") == 4 * cfg["vocab"]
         p.stdin.close()
         assert p.wait(timeout=60) == 0
     finally:
