@@ -229,8 +229,7 @@ __global__ __launch_bounds__(NW * (DP > 128 ? 128 : 64), 2) void linear_chunk_ke
         const long long step = 2ll * STEP * s.ldp;
 #pragma unroll
         for (int i = 0; i < 64 / STEP; ++i) {
-            const int x = STEP % 16 && i % 2 ? (I::swz(row + STEP) ^ I::swz(row)) * 8 : 0;   // (steps of 8 rows: every other piece has another swizzle)
-            const int c = x ? ((lane % I::CPR) ^ I::swz(row + STEP)) * 8 : col;
+            const int c = STEP % 16 && i % 2 ? ((lane % I::CPR) ^ I::swz(row + STEP)) * 8 : col;   // (steps of 8 rows: every other piece has another swizzle)
             const char* src = at + i * step + 2 * (c - col);
             const bool in = row + STEP * i < n && c < cols;
             src = in ? src : zero;

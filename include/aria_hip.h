@@ -596,9 +596,9 @@ typedef struct {
 int aria_linear_step(const void* proj, const AriaLinearShape* s, float* state, const int32_t* slot, const int32_t* pos, const int32_t* cu, int64_t n_seq,
                      void* out, int f32, void* stream);
 
-/* Whole prompts and long portions in bf16 on the matrix pipe: dp 64, 128 or 256, dvp a multiple of 64 (else ARIA_ERR_UNSUPPORTED).  The sequences are cut into
- * runs of up to 64 rows, blocks[i] = (first row, rows), and consecutive runs of a sequence form chunks, chunks[i] = (first run, runs, 1 for the
- * first chunk of its sequence, 1 for the last); seqs[i] = (first chunk, chunks).  int32 on the device.  Rewrites the q and k (silu: and v) columns of
+/* Whole prompts and long portions in bf16 on the matrix pipe: dp 64, 128 or 256, dvp a multiple of 64 (else ARIA_ERR_UNSUPPORTED).  Every sequence is cut
+ * into blocks of 64 rows (its last one: the rest), blocks[i] = (first row, rows), and consecutive blocks of a sequence form chunks, chunks[i] = (first block,
+ * blocks, 1 for the first chunk of its sequence, 1 for the last); seqs[i] = (first chunk, chunks).  int32 on the device.  Rewrites the q and k (silu: and v) columns of
  * proj.  scratch: aria_linear_chunks_scratch bytes, 16-byte aligned. */
 int64_t aria_linear_chunks_scratch(const AriaLinearShape* s, int64_t T, int64_t n_blocks, int64_t n_chunks);
 int aria_linear_chunks(void* proj, const AriaLinearShape* s, float* state, const int32_t* slot, const int32_t* pos, const int32_t* blocks, int64_t n_blocks,

@@ -93,6 +93,19 @@ def test_model_long_unequal_prompts(dtype, name):
 
 
 @both
+def test_model_sixteen_requests(dtype):
+    C.case_model(DEV, dtype, "many", lens=tuple(1 + 5 * i % 17 for i in range(16)), tail=4)
+
+
+@both
+@pytest.mark.parametrize("dim", [40, 128, 250, 400, 700])
+def test_recurrence_of_many_sequences(dtype, dim):
+    """whole state lines a workgroup (and, past 512 channels, half ones)"""
+    C.case_mixer(DEV, dtype, "gated", C.right(heads=8, dim=dim, vdim=72, tau=16.0), (2, 3, 1) * 14, tail=2)
+    C.case_mixer(DEV, dtype, "lightning", C.lightning(heads=8, dim=dim, vdim=72, decay=[0.5 + 0.06 * i for i in range(8)])["mixer"], (2, 3, 1) * 14, tail=2)
+
+
+@both
 def test_portions(dtype):
     C.case_portions(DEV, dtype)
     C.case_portions(DEV, dtype, "wide", n=205)
